@@ -616,7 +616,7 @@ def main():
             from docagents_amd.parallel.xgmi_allreduce import verify_and_time
             block("xgmi_allreduce", lambda: verify_and_time(None, dev))
 
-        # last: on ranks sharing one GPU (a rehearsal) the search streams' high-priority queues,
+        # last: on ranks sharing one GPU (a rehearsal) the search streams' queues,
         # once used, slowed every later block 2-3x (profiles/r5/rank8_gloo/serving_search_order/)
         def serving_search():
             """The serving transports side by side: the owner-routed plane (host TCP, the default) and

@@ -14,8 +14,8 @@ from docagents_amd.ops import reference as R  # noqa: E402
 
 if os.environ.get("DA_LIB"):
     import ctypes
-    K._LIB_PATH = Path(os.environ["DA_LIB"])
-    _probe = ctypes.CDLL(str(K._LIB_PATH))  # an older library lacks newer exports: do not bind those
+    K._LIB_OVERRIDE = Path(os.environ["DA_LIB"])
+    _probe = ctypes.CDLL(str(K._LIB_OVERRIDE))  # an older library lacks newer exports: do not bind those
     K._SIGS = {n: a for n, a in K._SIGS.items() if hasattr(_probe, n)}
 
 

@@ -9,7 +9,7 @@ Three lanes per replica, each a thread with its own HIP stream, so latency-criti
 queues behind a decode tick or an admission prefill:
   * the GPU thread: the continuous scheduler's ticks, summaries, ingest embeds, index mutations;
   * the fast lane: query-sized embeds (the question of ``embed`` / ``embed_search``), on a
-    high-priority stream with its own kernel workspace;
+    stream of its own with its own kernel workspace;
   * the search plane (parallel/search_plane.py): a scan worker with its own stream serving this
     rank's shard to every replica; searches are routed to the shards that own their documents.
 
@@ -253,7 +253,7 @@ class EngineServer:
                  admit_wait_s: float = 0.15, admit_hold_frac: float = 0.25):
         self.group, self.log = group, log
         self.urls = urls or []  # every replica's listen URL (topology RPC), replica order
-        # the fast lane: query-sized embeds on their own thread / high-priority stream / workspace
+        # the fast lane: query-sized embeds on their own thread / stream / workspace
         self.fast_embed_max = fast_embed_max
         # lanes = (main, fast) streams of a CU partition (ops/streams.py serving_lanes), or None
         main_stream, fast_stream = (lanes or (None, None))[:2]
@@ -375,7 +375,7 @@ class EngineServer:
         return [extract_summary(t) for t in val]
 
     def _fast_embed(self, texts, preprocess: bool) -> np.ndarray:
-        """Runs on the fast-lane thread: the encoder on a high-priority stream with its own kernel
+        """Runs on the fast-lane thread: the encoder on a stream of its own with its own kernel
         workspace, so it co-runs with the GPU thread's decode tick instead of queueing behind it."""
         e = self.group.engine
         faults.maybe_fail("engine.embed")
@@ -384,7 +384,7 @@ class EngineServer:
         from ..ops import kernels as K
         if self._fast_stream is None:
             torch.cuda.set_device(e.device)
-            self._fast_stream = torch.cuda.Stream(device=e.device, priority=-1)
+            self._fast_stream = torch.cuda.Stream(device=e.device)
         with torch.cuda.stream(self._fast_stream), K.workspace_role("fast"):
             return e.embed(texts, preprocess, out_dtype=torch.float32).cpu().numpy()
 

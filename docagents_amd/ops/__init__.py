@@ -24,7 +24,7 @@ def get_ops(device):
     dev = torch.device(device)
     if dev.type == "cuda":
         from . import kernels
-        kernels.lib()  # fail loudly if the HIP library is missing
+        kernels.lib()  # loading a part fails loudly if its library is missing
         return kernels
     from . import reference
     return reference

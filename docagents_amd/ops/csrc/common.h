@@ -1,7 +1,7 @@
 // Shared device helpers for the gfx950 (CDNA4, MI355X) kernel library.
 //
 // Everything here is written for 64-lane wavefronts and the gfx950 MFMA
-// operand layouts documented in /opt/skills/guides/cdna_hip_programming.md §3:
+// operand layouts:
 //   mfma_f32_16x16x32_bf16:  A lane l -> A[l&15][8*(l>>4)+j],  B lane l -> B[8*(l>>4)+j][l&15]
 //                            C lane l -> C[4*(l>>4)+i][l&15]   (i = 0..3)
 //   mfma_f32_32x32x16_bf16:  A lane l -> A[l&31][8*(l>>5)+j],  B lane l -> B[8*(l>>5)+j][l&31]
@@ -200,9 +200,8 @@ __device__ __forceinline__ float gelu_erf(float x) {
 // scale / fma / fixup sequence per element): every caller rounds the result to bf16.
 __device__ __forceinline__ float silu(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 
-// Bijective XCD-aware remap of a flat workgroup id (cdna_hip_programming.md §5,
-// "XCD swizzle must be bijective"): blocks that share an XCD (b % 8) get a
-// contiguous range of logical tile ids so neighbouring tiles share that XCD's L2.
+// Bijective XCD-aware remap of a flat workgroup id (bijective for any count): blocks that share
+// an XCD (b % 8) get a contiguous range of logical tile ids, so neighbouring tiles share its L2.
 __device__ __forceinline__ int xcd_remap(int bid, int nwg) {
   const int xcd = bid & 7, q = nwg >> 3, r = nwg & 7;
   const int base = (xcd < r) ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q;

@@ -2,7 +2,7 @@
 //
 //   C[M, N] = epi( A[M, K] · W[N, K]^T )       (nn.Linear layout: both operands K-contiguous)
 //
-// Design (MI355X-first, see /opt/skills/guides/cdna_hip_programming.md §5):
+// Design (MI355X-first):
 //  * v_mfma_f32_16x16x32_bf16, 4 waves per workgroup, each wave owns a (BM/WM)x(BN/WN) sub-tile
 //    indexed by fragment repeat (acc[FM][FN]), never by wave position.
 //  * BK = 64, double-buffered LDS with register-staged prefetch (issue global loads for tile t+1

@@ -1,4 +1,4 @@
-"""ctypes bindings for the gfx950 kernel library (``_da_kernels.so``).
+"""ctypes bindings for the gfx950 kernel library (``_da_*.so``, see ``build``).
 
 Every wrapper validates shapes / dtypes / contiguity / device on the host BEFORE launching (a
 mis-shaped launch of a hand-written kernel can fault the GPU), launches on PyTorch's current HIP
@@ -17,12 +17,11 @@ from pathlib import Path
 
 import torch
 
-_LIB = None
 _LOCK = threading.Lock()
 # DA_KERNELS_DEBUG=1: the -DDA_DEBUG build (device asserts: bounds / shape preconditions inside the
 # kernels; python -m docagents_amd.ops.build --debug) instead of the -O3 library
 _DEBUG = os.environ.get("DA_KERNELS_DEBUG", "0") == "1"
-_LIB_PATH = Path(__file__).resolve().parent / ("_da_kernels_debug.so" if _DEBUG else "_da_kernels.so")
+_LIB_OVERRIDE: Path | None = None  # one library with every launcher, instead of the parts (A/B runs)
 
 EPI_NONE, EPI_BIAS, EPI_GELU, EPI_SWIGLU, EPI_RESID = 0, 1, 2, 3, 4
 EPI_ROPE = 6  # gemm8p only: QKV + RoPE + KV-cache write
@@ -91,7 +90,14 @@ _SIGS = {
     "da_layernorm_f16": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p],
     "da_bert_embed_ln_f16": [c_void_p] * 9 + [c_int, c_int, c_float, c_void_p],
     "da_pool_l2norm_f16": [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p],
+    "da_topk_dense_ws": [c_int] * 4,
+    "da_topk_stream_ws": [c_int] * 4,
 }
+# the library part (build.py) of each launcher that is not in "kernels"; da_gemm* are in "gemm"
+_PART_OF = {n: "token" for n in (
+    "da_quant_fp8_rows", "da_rmsnorm", "da_swiglu_interleaved", "da_layernorm", "da_layernorm_q", "da_layernorm_f16",
+    "da_bert_embed_ln", "da_bert_embed_ln_q", "da_bert_embed_ln_f16", "da_embed", "da_pool_l2norm", "da_pool_l2norm_f16",
+    "da_rope_cache", "da_sample", "da_sample_partial", "da_sample_chunked", "da_sample_finalize")}
 
 
 class KernelLibraryMissing(RuntimeError):
@@ -102,39 +108,61 @@ class KernelError(RuntimeError):
     pass
 
 
-def lib() -> ctypes.CDLL:
-    """Load (building on first use if sources are newer) the kernel library."""
-    global _LIB
-    if _LIB is not None:
-        return _LIB
+class _Kernels:
+    """The launchers of every part; a part is built (if its sources are newer) and loaded at the first
+    use of one of its launchers."""
+
+    def __getattr__(self, name: str):
+        if not name.startswith("da_"):
+            raise AttributeError(name)
+        load_part(_part_of(name))
+        return self.__dict__.get(name) or getattr(_LOADED[_part_of(name)], name)
+
+
+_LIB = _Kernels()
+_LOADED: dict[str, ctypes.CDLL] = {}
+
+
+def _part_of(name: str) -> str:
+    return _PART_OF.get(name) or ("gemm" if name.startswith("da_gemm") else "kernels")
+
+
+def load_part(part: str) -> None:
     with _LOCK:
-        if _LIB is not None:
-            return _LIB
-        if os.environ.get("DA_BUILD_ON_IMPORT", "1") == "1":
+        if part in _LOADED:
+            return
+        from .build import build, lib_path
+        path = _LIB_OVERRIDE or lib_path(part, _DEBUG)
+        if _LIB_OVERRIDE is None and os.environ.get("DA_BUILD_ON_IMPORT", "1") == "1":
             try:
-                from .build import build
-                build(debug=_DEBUG)
+                build(debug=_DEBUG, parts=(part,))
             except Exception as e:  # noqa: BLE001 - fall through to the explicit check below
-                if not _LIB_PATH.exists():
-                    raise KernelLibraryMissing(f"cannot build {_LIB_PATH}: {e}") from e
-        if not _LIB_PATH.exists():
-            raise KernelLibraryMissing(f"{_LIB_PATH} not built; run python -m docagents_amd.ops.build")
+                if not path.exists():
+                    raise KernelLibraryMissing(f"cannot build {path}: {e}") from e
+        if not path.exists():
+            raise KernelLibraryMissing(f"{path} not built; run python -m docagents_amd.ops.build")
         import torch.cuda  # noqa: F401 - make sure torch's HIP runtime is loaded first
-        L = ctypes.CDLL(str(_LIB_PATH))
+        L = ctypes.CDLL(str(path))
         for name, argt in _SIGS.items():
-            fn = getattr(L, name)
-            fn.argtypes = argt
-            fn.restype = c_int
-        L.da_topk_dense_ws.argtypes = [c_int, c_int, c_int, c_int]
-        L.da_topk_dense_ws.restype = c_size_t
-        L.da_topk_stream_ws.argtypes = [c_int, c_int, c_int, c_int]
-        L.da_topk_stream_ws.restype = c_size_t
-        _LIB = L
-        return L
+            if _part_of(name) == part:
+                fn = getattr(L, name)
+                fn.argtypes = argt
+                fn.restype = c_size_t if name.endswith("_ws") else c_int
+                _LIB.__dict__[name] = fn
+        _LOADED[part] = L
+
+
+def lib(parts=()) -> _Kernels:
+    """The kernel launchers; ``parts`` are loaded now, any other at the first use of its launchers."""
+    for p in parts:
+        if p not in _LOADED:
+            load_part(p)
+    return _LIB
 
 
 def available() -> bool:
-    return torch.cuda.is_available() and _LIB_PATH.exists()
+    from .build import PARTS, lib_path
+    return torch.cuda.is_available() and all(lib_path(p, _DEBUG).exists() for p in PARTS)
 
 
 def _ptr(t):

@@ -171,7 +171,7 @@ class CollectiveSearchPlane:
         if self.device.type == "cuda":
             torch.cuda.set_device(self.device)
             if self.stream is None:
-                self.stream = torch.cuda.Stream(device=self.device, priority=-1)
+                self.stream = torch.cuda.Stream(device=self.device)
         take: list[_Pending] = []
         wait = self.idle_s
         try:

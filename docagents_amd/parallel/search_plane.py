@@ -290,7 +290,7 @@ class SearchPlane:
                  retry_s: float = 1.0, connect_timeout_s: float = 2.0, send_timeout_s: float = 5.0):
         self.index, self.rank, self.world = index, rank, max(1, world)
         self.device = torch.device(device) if device is not None else getattr(index, "device", torch.device("cpu"))
-        self.stream = stream  # None: a high-priority stream created by the scan worker
+        self.stream = stream  # None: a stream created by the scan worker
         self.owner = owner or (lambda d: owner_of(d, self.world))
         self.host, self.port = host, port
         self.timeout_s, self.max_rows = timeout_s, max_rows
@@ -609,7 +609,7 @@ class SearchPlane:
         if self.device.type == "cuda":
             torch.cuda.set_device(self.device)
             if self.stream is None:
-                self.stream = torch.cuda.Stream(device=self.device, priority=-1)
+                self.stream = torch.cuda.Stream(device=self.device)
         while not self._stop:
             take = self._take()
             if not take:

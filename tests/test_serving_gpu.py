@@ -47,7 +47,7 @@ def test_decode_fast_embed_and_search_plane_co_run_exactly():
             res.update((t, (a, c)) for t, a, c in o)
         return [res[i] for i in range(12)]
 
-    fast = torch.cuda.Stream(priority=-1)
+    fast = torch.cuda.Stream()
 
     def embeds():
         with torch.cuda.stream(fast), K.workspace_role("fast"):

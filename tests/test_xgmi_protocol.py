@@ -17,7 +17,9 @@ import time
 import numpy as np
 import pytest
 
-from docagents_amd.ops.build import LIB
+from docagents_amd.ops.build import lib_path
+
+LIB = lib_path("kernels")
 
 TPB = 256
 
