@@ -39,7 +39,7 @@ _ENGINES = {}
 
 def local_engine(cfg: Config):
     """One in-process Engine per config (LLM_PROVIDER=local)."""
-    key = (cfg.embed_arch, cfg.llm_arch)
+    key = (cfg.embed_arch, cfg.llm_arch, cfg.llm_dtype)
     if key not in _ENGINES:
         import torch
         from .engine.engine import Engine
@@ -49,6 +49,7 @@ def local_engine(cfg: Config):
                                summary_max_new=cfg.summary_max_new_tokens, index_kind=cfg.index_kind,
                                ivf_lists=cfg.ivf_lists, ivf_probes=cfg.ivf_probes,
                                enc_dtype="fp8" if cfg.dtype == "fp8" else "bf16",
+                               llm_dtype=cfg.llm_dtype,
                                max_seq=4096 if dev == "cuda" else 1024)
     return _ENGINES[key]
 

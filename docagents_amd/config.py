@@ -51,6 +51,7 @@ class Config:
     llm_arch: str = field(default="phi3-mini", metadata={"env": "LLM_ARCH"})
     embed_dim: int = field(default=0, metadata={"env": "EMBED_DIM"})  # 0 -> encoder hidden size
     dtype: str = field(default="bf16", metadata={"env": "DTYPE"})
+    llm_dtype: str = field(default="bf16", metadata={"env": "LLM_DTYPE"})  # decoder: bf16, or fp32 where it has it
     tp_size: int = field(default=1, metadata={"env": "TP_SIZE"})
     index_shards: int = field(default=1, metadata={"env": "INDEX_SHARDS"})
     index_kind: str = field(default="flat", metadata={"env": "INDEX_KIND"})
@@ -133,16 +134,19 @@ class Config:
     def replace(self, **kw) -> "Config":
         return dataclasses.replace(self, **kw)
 
-    # engine compute dtypes (the encoder's; the decoder is bf16): bf16 everywhere; fp16 encoder
+    # engine compute dtypes (the encoder's; LLM_DTYPE is the decoder's): bf16 everywhere; fp16 encoder
     # (f16 MFMA GEMMs + flash, fp16 LayerNorm); fp8 (OCP e4m3) encoder GEMMs.
     # Anything else is refused at startup, never run as something else.
     ENGINE_DTYPES = ("bf16", "fp16", "fp8")
+    LLM_DTYPES = ("bf16", "fp32")
 
     def validate_engine(self) -> "Config":
         """Startup check of the engine keys whose wrong value would otherwise silently run a
         different configuration (the engine process calls it before touching the GPU)."""
         if self.dtype not in self.ENGINE_DTYPES:
             raise ValueError(f"DTYPE={self.dtype!r} is not supported (choose one of {', '.join(self.ENGINE_DTYPES)})")
+        if self.llm_dtype not in self.LLM_DTYPES:
+            raise ValueError(f"LLM_DTYPE={self.llm_dtype!r} is not supported (choose one of {', '.join(self.LLM_DTYPES)})")
         if self.index_kind not in ("flat", "ivfflat"):
             raise ValueError(f"INDEX_KIND={self.index_kind!r} is not supported (flat | ivfflat)")
         if self.tp_size < 1:

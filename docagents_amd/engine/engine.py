@@ -20,7 +20,8 @@ import torch
 
 from ..models.bert import BertEncoder, pack_for_encoder
 from ..models.configs import decoder_config, encoder_config
-from ..models.llama import LlamaDecoder, TPContext
+from ..models import make_decoder
+from ..models.llama import TPContext
 from ..models.tokenizer import ChatFormat, decoder_tokenizer, encoder_tokenizer
 from ..ops import h2d
 from ..text.preprocess import extract_summary, preprocess_text
@@ -42,7 +43,8 @@ class Engine:
                  max_new_tokens: int = 64, summary_max_new: int = 128, index_kind: str = "flat",
                  ivf_lists: int = 100, ivf_probes: int = 1, load_llm: bool = True, load_encoder: bool = True,
                  use_graphs: bool = True, embed_max_tokens: int = 65536, enc_dtype: str = "bf16",
-                 share_prefix: bool = True, overlap_waves: bool = False, kv_cache_gb: float = 0.0):
+                 share_prefix: bool = True, overlap_waves: bool = False, kv_cache_gb: float = 0.0,
+                 llm_dtype: str = "bf16"):
         self.device = torch.device(device)
         self.lock = threading.RLock()      # the decoder / generator (one GPU thread drives it)
         self.enc_lock = threading.RLock()  # the encoder: the fast embed lane and the batcher share it
@@ -64,7 +66,7 @@ class Engine:
         self.decoder = None
         self.gen = None
         if load_llm:
-            self.decoder = LlamaDecoder(self.dec_cfg, self.device, seed=seed, tp=tp)
+            self.decoder = make_decoder(self.dec_cfg, self.device, seed=seed, tp=tp, dtype=llm_dtype)
             if max_batch <= 0:
                 max_batch = self.auto_batch(max_seq, overlap_waves, kv_gb=kv_cache_gb)
             # + 1 dummy slot (padded graph rows) + 2 prompt-head slots (ContinuousScheduler heads)
@@ -88,10 +90,9 @@ class Engine:
         (batch + 4 slots x max_seq, this rank's kv heads) fits ``kv_gb`` GB, or the device's free
         HBM after the weights less AUTO_RESERVE_BYTES. Phi-3-mini on an MI355X: 128 (213 GB of
         KV); Llama-3-70B on one GPU: 16. CPU: 64."""
-        from ..models.llama import KVCache
         if self.device.type != "cuda" and kv_gb <= 0:
             return 64
-        per = KVCache.bytes_for(self.dec_cfg, 1, min(max_seq, self.dec_cfg.max_pos), self.decoder.tp.size)
+        per = self.decoder.cache_bytes(1, max_seq)
         if kv_gb > 0:
             budget = int(kv_gb * 1e9)
         else:

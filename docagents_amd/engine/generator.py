@@ -10,7 +10,6 @@ every few steps. The reference's equivalent is one OpenAI chat call per request
 from __future__ import annotations
 
 import collections
-import math
 import threading
 import time
 from types import SimpleNamespace
@@ -18,7 +17,7 @@ from types import SimpleNamespace
 import numpy as np
 import torch
 
-from ..models.llama import DecodeState, LlamaDecoder, pack_prompts
+from ..models.llama import DecodeState, decode_workspace_bytes, pack_prompts
 from ..ops import h2d
 
 
@@ -37,13 +36,13 @@ class GenResult:
 
 
 class Generator:
-    def __init__(self, model: LlamaDecoder, max_batch: int = 64, max_seq: int = 4096, temperature: float = 0.2,
+    def __init__(self, model, max_batch: int = 64, max_seq: int = 4096, temperature: float = 0.2,
                  seed: int = 0, eos=(), use_graphs: bool = True, max_prefill_tokens: int = 65536,
                  check_every: int = 16, share_prefix: bool = True, min_shared_prefix: int = 64):
         self.model = model
         # prompts of one wave that start with the same tokens (the Answer / Summarize system prompt:
         # ~260 tokens of every QA prompt) prefill that head once; see _generate_wave
-        self.share_prefix, self.min_shared_prefix = share_prefix, min_shared_prefix
+        self.share_prefix, self.min_shared_prefix = share_prefix and model.prefix_sharing, min_shared_prefix
         self.max_batch = max_batch
         self.temperature, self.seed = temperature, seed
         self.eos = tuple(e for e in eos if e is not None)[:4]
@@ -57,7 +56,7 @@ class Generator:
             # one extra slot: the dummy slot for padded rows of a bucket
             model.alloc_cache(max_batch + 1, max_seq)
         self.cache = model.cache
-        self.dummy_slot = self.cache.acquire(1)[0]
+        self.dummy_slot = self.cache.acquire(1, [1])[0]
         self.head = None  # {"tokens", "P", "slot"}: the last wave's shared prompt head, kept in its own slot
         self.states: dict[tuple, DecodeState] = {}
         self.stats = {"prefill_s": 0.0, "decode_s": 0.0, "prefill_tokens": 0, "decode_steps": 0, "decode_tokens": 0,
@@ -67,15 +66,9 @@ class Generator:
         self.sync_phases = False
         if self.is_cuda:
             from ..ops import kernels
-            kernels.reserve_workspace(self.workspace_bytes(model.cfg, model.hl, model.tp.size, max_batch,
-                                                           self.cache.max_seq), model.device)
+            kernels.reserve_workspace(model.workspace_bytes(max_batch, self.cache.max_seq), model.device)
 
-    @staticmethod
-    def workspace_bytes(cfg, heads_local: int, tp: int, max_batch: int, max_seq: int) -> int:
-        """The shared split-KV / split-K workspace a generator reserves (parallel/hbm_plan.py)."""
-        nsplit = math.ceil(max_seq / 256)
-        return max(max_batch * heads_local * nsplit * (cfg.head_dim + 2) * 4,
-                   8 * max_batch * max(cfg.ffn * 2 // tp, cfg.vocab) * 4)
+    workspace_bytes = staticmethod(decode_workspace_bytes)
 
     def close(self):
         """Give this generator's KV slots (the padded rows' dummy slot, a kept prompt-head slot) back
@@ -112,7 +105,11 @@ class Generator:
         # warm up on a side stream (allocator + lazy init), then capture one step
         s = torch.cuda.Stream()
         s.wait_stream(torch.cuda.current_stream())
-        saved = [t.clone() for t in (st.tokens, st.pos, st.lens, st.active, st.hist, st.conf)]
+        kept = (st.tokens, st.pos, st.lens, st.active, st.hist, st.conf, st.slot)
+        saved = [t.clone() for t in kept]
+        if self.model.stateful_step:  # the warm-up steps advance the spare slot, not the rows' sequences
+            st.slot.fill_(self.dummy_slot)
+            st.pos.zero_(); st.active.zero_()
         with torch.cuda.stream(s):
             for _ in range(2):
                 self.model.decode_step(st)
@@ -120,7 +117,7 @@ class Generator:
         g = torch.cuda.CUDAGraph()
         with torch.cuda.graph(g):
             self.model.decode_step(st)
-        for t, v in zip((st.tokens, st.pos, st.lens, st.active, st.hist, st.conf), saved):
+        for t, v in zip(kept, saved):
             t.copy_(v)
         st.graph = g
 
@@ -167,7 +164,7 @@ class Generator:
             t0 = time.perf_counter()
             to = lambda a: h2d(a, dev)  # noqa: E731
             logits = m.prefill(to(flat), to(pos), to(slot_tok), to(cu), int(lens.max()), to(last), prefix=prefix,
-                               local_logits=True)
+                               local_logits=True, lens=lens.tolist())
             r0, r1 = row0 + i, row0 + j
             m.sample(logits, self.temperature, self.seed, 0, out_tok=st.tokens[r0:r1], out_lp=st.lp[r0:r1],
                      conf=st.conf[r0:r1], active=st.active[r0:r1], ctr=st.pos[r0:r1], pos=st.pos[r0:r1],
@@ -178,9 +175,19 @@ class Generator:
 
     def generate(self, prompts: list[list[int]], max_new: int) -> list[GenResult]:
         out: list[GenResult] = []
-        for s in range(0, len(prompts), self.max_batch):
-            out.extend(self._generate_wave(prompts[s:s + self.max_batch], max_new))
+        s = 0
+        while s < len(prompts):
+            n = self._wave_size(prompts[s:s + self.max_batch], max_new)
+            out.extend(self._generate_wave(prompts[s:s + n], max_new))
+            s += n
         return out
+
+    def _wave_size(self, prompts, max_new: int) -> int:
+        """How many of the prompts the cache can hold at once (at least one: it then fails by itself)."""
+        n = len(prompts)
+        while n > 1 and not self.cache.fits([len(p) + max(1, max_new) for p in prompts[:n]]):
+            n -= 1
+        return n
 
     def _generate_wave(self, prompts, max_new: int) -> list[GenResult]:
         if not prompts:
@@ -202,13 +209,14 @@ class Generator:
         n = len(prompts)
         max_new = max(1, max_new)
         for p in prompts:
-            if len(p) + max_new > self.cache.max_seq:
-                raise ValueError(f"prompt of {len(p)} tokens + {max_new} new exceeds the context ({self.cache.max_seq})")
+            if len(p) + max_new > self.cache.capacity():
+                raise ValueError(f"prompt of {len(p)} tokens + {max_new} new exceeds the context "
+                                 f"({self.cache.capacity()})")
             if len(p) == 0:
                 raise ValueError("empty prompt")
         B = min(_bucket(n), self.max_batch) if self.use_graphs else n
         st = self._state(B, max_new, lane)
-        slots = self.cache.acquire(n)
+        slots = self.cache.acquire(n, [len(p) + max_new for p in prompts])
         try:
             self.stats["calls"] += 1
             plen = np.asarray([len(p) for p in prompts], dtype=np.int32)
@@ -478,9 +486,9 @@ class ContinuousScheduler:
         max_new = max(1, min(int(max_new), self.cap))
         if not prompt:
             raise ValueError("empty prompt")
-        if len(prompt) + max_new > self.gen.cache.max_seq:
+        if len(prompt) + max_new > self.gen.cache.capacity():
             raise ValueError(f"prompt of {len(prompt)} tokens + {max_new} new exceeds the context "
-                             f"({self.gen.cache.max_seq})")
+                             f"({self.gen.cache.capacity()})")
         self.pending.append((list(prompt), max_new, tag))
 
     def busy(self) -> bool:
@@ -630,6 +638,8 @@ class ContinuousScheduler:
             p = self.pending[0]
             if take and tot + len(p[0]) > self.max_admit_tokens:
                 break
+            if not self.gen.cache.fits([len(t[0]) + t[1] for t in [*take, p]]):
+                break  # waits for running sequences to give their share of the cache back
             take.append(self.pending.popleft())
             tot += len(p[0])
         if not take:
@@ -647,7 +657,7 @@ class ContinuousScheduler:
         order = sorted(range(len(take)), key=lambda i: (hs[i] is None, id(hs[i])))
         take, hs = [take[i] for i in order], [hs[i] for i in order]
         n, rows = len(take), free[:len(take)]
-        slots = self.gen.cache.acquire(n)
+        slots = self.gen.cache.acquire(n, [len(t[0]) + t[1] for t in take])
         prompts = [t[0] for t in take]
         plen = np.asarray([len(p) for p in prompts], dtype=np.int32)
         budget = np.asarray([t[1] for t in take], dtype=np.int32)

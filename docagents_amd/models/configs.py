@@ -1,10 +1,13 @@
-"""Model architectures (random-init weights of these shapes; no network for checkpoints).
+"""Model architectures: presets (random-init weights of these shapes) and checkpoint folders.
 
 Encoders (BGE / E5 class, BERT layers) replace OpenAI text-embedding-3-* (SURVEY.md §2.4 N1/N2);
-decoders (Phi-3-mini / Llama-3) replace gpt-4o-mini for Summarize / Answer (N6/N7).
+decoders (Phi-3-mini / Llama-3 / Binupel) replace gpt-4o-mini for Summarize / Answer (N6/N7). A decoder is
+named by a preset or by a folder with ``config.json`` and ``*.safetensors``, whose "architecture" picks the
+parser (``ARCHITECTURES``) and thereby the model class (``models.make_decoder``).
 """
 from __future__ import annotations
 
+import os
 from dataclasses import dataclass
 
 
@@ -60,6 +63,125 @@ class DecoderConfig:
         return self.layers * 2 * self.kv_heads * self.head_dim * dtype_bytes
 
 
+# ---------------------------------------------------------------------- decoders of mixed layers
+@dataclass(frozen=True)
+class GatedRecurrence:
+    """Griffin's recurrent block: real-gated linear recurrent unit behind a short convolution."""
+    width: int
+    blocks: int   # equal parts of the channels with gate matrices of their own
+    conv: int     # taps
+
+    def param_count(self, h: int) -> int:
+        w = self.width
+        return 3 * h * w + w * (2 + self.conv + 1 + 1 + 2) + 2 * w * (w // self.blocks)
+
+
+@dataclass(frozen=True)
+class SigmoidAttention:
+    """Causal attention with unnormalised sigmoid weights, normed queries and keys, values = keys."""
+    heads: int
+    kv_heads: int
+    dim: int
+    scale: float
+    q_temp: tuple[float, float] | None = None  # (coef, every)
+
+    def param_count(self, h: int) -> int:
+        return h * (2 * self.heads + self.kv_heads) * self.dim + 2 * self.dim + self.heads * (1 + h)
+
+
+@dataclass(frozen=True)
+class SelectiveScan:
+    """Mamba (selective state space) block."""
+    inner: int
+    state: int
+    dt_rank: int
+    conv: int
+
+    def param_count(self, h: int) -> int:
+        n = self.inner
+        return 3 * h * n + n * (self.conv + 3 + 2 * self.dt_rank + 3 * self.state)
+
+
+@dataclass(frozen=True)
+class HybridLayer:
+    mixer: GatedRecurrence | SigmoidAttention | SelectiveScan
+    ff: int = 0                     # 0: no feed-forward
+    weights_of: int | None = None   # use that layer's tensors (with a state of its own)
+
+
+@dataclass(frozen=True)
+class HybridConfig:
+    """A decoder whose layers mix different sequence mixers: fp32 residual stream with the norm after the sum
+    (x <- norm(alpha x + sublayer(x))), token shift ahead of every mixer, gated-relu feed-forwards."""
+    name: str
+    vocab: int
+    hidden: int
+    spec: tuple[HybridLayer, ...]
+    alpha: float
+    eps: float
+    max_pos: int = 1 << 20   # positions enter only through the query temperature: bounds the page table
+    path: str = ""           # checkpoint folder ("": random init)
+
+    @property
+    def layers(self) -> int:
+        return len(self.spec)
+
+    def param_count(self) -> int:
+        h = self.hidden
+        own = [s for s in self.spec if s.weights_of is None]
+        return 2 * self.vocab * h + h + sum(s.mixer.param_count(h) + 3 * h * s.ff + h * (3 if s.ff else 2) for s in own)
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2) -> int:
+        att = [s.mixer for s in self.spec if isinstance(s.mixer, SigmoidAttention)]
+        return sum(a.kv_heads * (a.dim * dtype_bytes + 4) for a in att)
+
+
+def _binupel_mixer(kind: str, m: dict):
+    if kind == "rglru":
+        if m["width"] % m["blocks"]:
+            raise ValueError(f"rglru: blocks={m['blocks']} must divide width={m['width']}")
+        return GatedRecurrence(m["width"], m["blocks"], m["conv"])
+    if kind == "attention":
+        if m["heads"] % m["kv_heads"]:
+            raise ValueError(f"attention: kv_heads={m['kv_heads']} must divide heads={m['heads']}")
+        if m.get("vdim", m["dim"]) != m["dim"]:
+            raise ValueError(f"attention: the values are the keys, vdim={m['vdim']} must equal dim={m['dim']}")
+        t = m.get("q_temp")
+        return SigmoidAttention(m["heads"], m["kv_heads"], m["dim"], float(m["scale"]),
+                                (float(t["coef"]), float(t["every"])) if t else None)
+    if kind == "mamba1":
+        return SelectiveScan(m["inner"], m["state"], m["dt_rank"], m["conv"])
+    raise ValueError(f"unknown mixer {kind!r} (rglru, attention, mamba1)")
+
+
+def binupel_config(c: dict, name: str, path: str = "") -> HybridConfig:
+    """The parsed ``config.json`` of a Binupel checkpoint."""
+    spec = []
+    for i, layer in enumerate(c["layers"]):
+        mlp, src = layer.get("mlp"), layer.get("weights_of")
+        if mlp and mlp.get("kind", "dense") != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r} (dense)")
+        spec.append(HybridLayer(_binupel_mixer(layer["type"], layer["mixer"]), mlp["ff"] if mlp else 0, src))
+    for i, s in enumerate(spec):
+        if s.weights_of is not None:
+            j = s.weights_of
+            if not 0 <= j < len(spec) or spec[j].weights_of is not None:
+                raise ValueError(f"layer {i}: weights_of={j} names no layer with tensors of its own")
+            if (spec[j].mixer, spec[j].ff) != (s.mixer, s.ff):
+                raise ValueError(f"layer {i} differs from layer {j}, whose weights it uses")
+    return HybridConfig(name, c["vocab"], c["width"], tuple(spec), float(c["postln_alpha"]), float(c["norm"]["eps"]),
+                        path=path)
+
+
+ARCHITECTURES = {"Binupel": binupel_config}
+
+
+def _binupel(name: str, hidden: int, ff: int, vocab: int, groups: int, rec: GatedRecurrence, att: SigmoidAttention,
+             ssm: SelectiveScan) -> HybridConfig:
+    layer = [HybridLayer(m, ff) for m in (rec, att, ssm, ssm)]
+    return HybridConfig(name, vocab, hidden, tuple(layer * groups), alpha=2.0, eps=1e-6)
+
+
 ENCODERS = {
     "bge-small": EncoderConfig("bge-small", hidden=384, layers=12, heads=12, ffn=1536),
     "bge-base": EncoderConfig("bge-base"),
@@ -83,6 +205,12 @@ DECODERS = {
     # the GPU decode-attention kernels take
     "tiny-dec-tp8": DecoderConfig("tiny-dec-tp8", vocab=32064, hidden=1024, layers=2, heads=16, kv_heads=8,
                                   ffn=1024, max_pos=4096, rope_theta=500000.0),
+    # Binupel at Llama-3-8B's width, feed-forward, attention shape and vocabulary (8 x [recurrence,
+    # attention, 2 x scan]: 8.0 G parameters), and a miniature
+    "binupel-8b": _binupel("binupel-8b", 4096, 14336, 128256, 8, GatedRecurrence(4096, 16, 4),
+                           SigmoidAttention(32, 8, 128, 128 ** -0.5, (0.1, 8192)), SelectiveScan(8192, 16, 256, 4)),
+    "tiny-binupel": _binupel("tiny-binupel", 256, 512, 32064, 1, GatedRecurrence(320, 5, 4),
+                             SigmoidAttention(8, 2, 32, 32 ** -0.5, (0.1, 64)), SelectiveScan(448, 16, 24, 4)),
 }
 
 ALIASES = {"text-embedding-3-large": "bge-large", "text-embedding-3-small": "bge-base",
@@ -96,8 +224,27 @@ def encoder_config(name: str) -> EncoderConfig:
     return ENCODERS[name]
 
 
-def decoder_config(name: str) -> DecoderConfig:
+def decoder_dtypes(cfg) -> tuple[str, ...]:
+    """The precisions a decoder runs in."""
+    return ("bf16", "fp32") if isinstance(cfg, HybridConfig) else ("bf16",)
+
+
+def checkpoint_config(path: str):
+    """The configuration in a checkpoint folder's ``config.json``."""
+    from .checkpoint import read_config
+    c = read_config(path)
+    arch = c.get("architecture")
+    if arch not in ARCHITECTURES:
+        raise ValueError(f"{path}: unknown architecture {arch!r}; known: {sorted(ARCHITECTURES)}")
+    return ARCHITECTURES[arch](c, os.path.basename(os.path.abspath(path)), os.path.abspath(path))
+
+
+def decoder_config(name: str) -> DecoderConfig | HybridConfig:
+    """A preset's configuration, or that of a checkpoint folder."""
+    from .checkpoint import is_checkpoint
     name = ALIASES.get(name, name)
-    if name not in DECODERS:
-        raise ValueError(f"unknown decoder arch {name!r}; choose from {sorted(DECODERS)}")
-    return DECODERS[name]
+    if name in DECODERS:
+        return DECODERS[name]
+    if is_checkpoint(name):
+        return checkpoint_config(name)
+    raise ValueError(f"unknown decoder arch {name!r}; choose from {sorted(DECODERS)} or name a checkpoint folder")

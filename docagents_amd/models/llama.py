@@ -188,6 +188,13 @@ def random_weights(cfg: DecoderConfig, device, seed: int = 0, tp_rank: int = 0, 
     return w
 
 
+def decode_workspace_bytes(cfg: DecoderConfig, heads_local: int, tp: int, max_batch: int, max_seq: int) -> int:
+    """The shared split-KV / split-K workspace a generator reserves (parallel/hbm_plan.py)."""
+    nsplit = -(-max_seq // 256)
+    return max(max_batch * heads_local * nsplit * (cfg.head_dim + 2) * 4,
+               8 * max_batch * max(cfg.ffn * 2 // tp, cfg.vocab) * 4)
+
+
 class KVCache:
     """Contiguous per-slot KV cache: k/v [layers][slots, Hkv_local, max_seq, D] (one allocation)."""
 
@@ -198,13 +205,21 @@ class KVCache:
                                device=device)
         self.free = list(range(slots - 1, -1, -1))
 
+    def fits(self, tokens: list[int]) -> bool:
+        """Whether sequences of these lengths can be admitted together now (a slot holds any length)."""
+        return len(tokens) <= len(self.free)
+
+    def capacity(self) -> int:
+        """The longest sequence the cache could hold."""
+        return self.max_seq
+
     def k(self, layer):
         return self.buf[layer, 0]
 
     def v(self, layer):
         return self.buf[layer, 1]
 
-    def acquire(self, n: int) -> list[int]:
+    def acquire(self, n: int, tokens: list[int] | None = None) -> list[int]:
         if n > len(self.free):
             raise RuntimeError(f"KV cache exhausted: want {n} slots, {len(self.free)} free")
         return [self.free.pop() for _ in range(n)]
@@ -220,6 +235,8 @@ class KVCache:
 class LlamaDecoder:
     unit_gains = False  # set by _fold_norm_gains
     layer_hook = None   # prefill: called with the layer index before each layer (stream steering)
+    prefix_sharing = True   # prompts may attend to a shared head in another slot
+    stateful_step = False   # running a decode step twice leaves a sequence as running it once
 
     def __init__(self, cfg: DecoderConfig, device="cuda", seed: int = 0, tp: TPContext | None = None,
                  weights: dict | None = None):
@@ -259,6 +276,22 @@ class LlamaDecoder:
         max_seq = min(max_seq, self.cfg.max_pos)
         self.cache = KVCache(self.cfg, slots, max_seq, self.tp.size, self.device)
         return self.cache
+
+    def cache_bytes(self, slots: int, max_seq: int) -> int:
+        return KVCache.bytes_for(self.cfg, slots, min(max_seq, self.cfg.max_pos), self.tp.size)
+
+    def workspace_bytes(self, max_batch: int, max_seq: int) -> int:
+        return decode_workspace_bytes(self.cfg, self.hl, self.tp.size, max_batch, max_seq)
+
+    def decode_buffers(self, B: int) -> dict:
+        """Static buffers of a decode state; tuples are shared as they are by views of fewer rows."""
+        c, b16 = self.cfg, dict(dtype=torch.bfloat16, device=self.device)
+        return {"x": torch.zeros(B, c.hidden, **b16), "h": torch.zeros(B, c.hidden, **b16),
+                "qkv": torch.zeros(B, (self.hl + 2 * self.kl) * c.head_dim, **b16),
+                "attn": torch.zeros(B, self.hl * c.head_dim, **b16),
+                "logits": torch.zeros(B, c.vocab // self.tp.size, **b16),  # this rank's slice
+                # gemm_dk deferred-norm partial sums [parts, 64]
+                "ssq": tuple(torch.zeros(512 * 64, dtype=torch.float32, device=self.device) for _ in range(2))}
 
     # ------------------------------------------------------------- shared layer body
     def _attn_out_and_mlp(self, L, a, x):
@@ -308,7 +341,7 @@ class LlamaDecoder:
     # ------------------------------------------------------------- prefill
     def prefill(self, ids: torch.Tensor, pos: torch.Tensor, slot_tok: torch.Tensor, cu: torch.Tensor,
                 max_seqlen: int, last_idx: torch.Tensor, prefix: tuple[int, int] | None = None,
-                local_logits: bool = False) -> torch.Tensor:
+                local_logits: bool = False, lens=None) -> torch.Tensor:
         """Packed causal prefill; writes the KV cache; returns logits [B, V] of each sequence's last token
         (local_logits: this rank's vocab slice [B, V/t], the input of ``sample``).
         prefix = (slot, P): every sequence continues a shared P-token head already in ``slot``'s cache
@@ -474,8 +507,8 @@ class LlamaDecoder:
 class DecodeState:
     """Static device buffers for a batch bucket of B sequences (HIP-graph friendly)."""
 
-    def __init__(self, model: LlamaDecoder, B: int, max_new: int, temperature: float, seed: int, eos=()):
-        c, dev = model.cfg, model.device
+    def __init__(self, model, B: int, max_new: int, temperature: float, seed: int, eos=()):
+        dev = model.device
         i32 = dict(dtype=torch.int32, device=dev)
         self.B = B
         self.tokens = torch.zeros(B, **i32)
@@ -488,14 +521,7 @@ class DecodeState:
         self.hist = torch.full((B, max(1, max_new)), -1, **i32)
         self.conf = torch.zeros(B, 2, dtype=torch.float32, device=dev)
         self.lp = torch.zeros(B, dtype=torch.float32, device=dev)
-        h = c.hidden
-        self.x = torch.zeros(B, h, dtype=torch.bfloat16, device=dev)
-        self.h = torch.zeros(B, h, dtype=torch.bfloat16, device=dev)
-        self.qkv = torch.zeros(B, (model.hl + 2 * model.kl) * c.head_dim, dtype=torch.bfloat16, device=dev)
-        self.attn = torch.zeros(B, model.hl * c.head_dim, dtype=torch.bfloat16, device=dev)
-        self.logits = torch.zeros(B, c.vocab // model.tp.size, dtype=torch.bfloat16, device=dev)  # this rank's slice
-        # gemm_dk deferred-norm partial sums [parts, 64] (a tuple: shared as-is by row views)
-        self.ssq = tuple(torch.zeros(512 * 64, dtype=torch.float32, device=dev) for _ in range(2))
+        self.__dict__.update(model.decode_buffers(B))
         self.temperature, self.seed, self.eos = temperature, seed, tuple(eos)[:4]
         self.graph = None
 

@@ -5,6 +5,7 @@ parallel) and the objects of a part are linked into that part's shared library n
 
     gemm     _da_gemm.so      matrix products
     token    _da_token.so     norms, embeddings, pooling, RoPE, samplers
+    hybrid   _da_hybrid.so    recurrent mixers, paged attention, 32-bit residual stream, fp32 products
     kernels  _da_kernels.so   everything else (attention, vector search, collectives, runtime)
 
 A process loads (and, in a checkout without built libraries, compiles) only the parts it calls. The
@@ -35,6 +36,7 @@ ARCH = os.environ.get("DA_OFFLOAD_ARCH", "gfx950")
 _PART_SOURCES = {
     "gemm": ("gemm.hip", "gemm256.hip", "gemm4w.hip", "gemm8p.hip", "gemm_dk.hip"),
     "token": ("norm.hip", "rope_sample.hip"),
+    "hybrid": ("gemm_any.hip", "paged_attn.hip", "recurrent.hip", "stream_norm.hip"),
 }
 PARTS = (*_PART_SOURCES, "kernels")
 

@@ -200,6 +200,9 @@ __device__ __forceinline__ float gelu_erf(float x) {
 // scale / fma / fixup sequence per element): every caller rounds the result to bf16.
 __device__ __forceinline__ float silu(float x) { return x * __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 
+// The activation of a gated feed-forward's gate half (uniform flag): silu or relu.
+__device__ __forceinline__ float gate_act(float g, int relu) { return relu ? fmaxf(g, 0.f) : silu(g); }
+
 // Bijective XCD-aware remap of a flat workgroup id (bijective for any count): blocks that share
 // an XCD (b % 8) get a contiguous range of logical tile ids, so neighbouring tiles share its L2.
 __device__ __forceinline__ int xcd_remap(int bid, int nwg) {

@@ -9,6 +9,7 @@ enum Epi : int {
   EPI_SWIGLU = 3,     // W rows interleaved in 16-row (gate, up) groups; out N/2 = silu(g)*u
   EPI_RESID = 4,      // bias (optional) + residual add
   EPI_PARTIAL = 5,    // fp32 split-K partial to workspace
+  EPI_REGLU = 7,      // launchers only: EPI_SWIGLU's layout with relu(g)*u (args carry relu = 1)
   EPI_ROPE = 6,       // QKV projection: RoPE (interleaved pairs) on q / k, k / v written to the KV cache
 };
 
@@ -28,6 +29,7 @@ struct GemmArgs {
   const float* sa; const float* sw;  // fp8 path: per-row (A) and per-output-channel (W) scales
   const bf16_t* gamma; float eps;    // GEMV only: fused RMSNorm of the input row (gamma != null)
   RopeArgs rope;                     // EPI_ROPE only
+  int relu;   // EPI_SWIGLU: the gate's activation is relu, not silu
   int group;  // gemm8p: row tiles per grouped-M band of the tile order (0: the default, 4)
 };
 

@@ -172,7 +172,7 @@ gemm_bf16_kernel(GemmArgs p) {
 #pragma unroll
       for (int e = 0; e < 8; e += 2) {
         float g0 = srow[e], g1 = srow[e + 1], u0 = srow[16 + e], u1 = srow[16 + e + 1];
-        packed[e / 2] = pack_bf2(silu(g0) * u0, silu(g1) * u1);
+        packed[e / 2] = pack_bf2(gate_act(g0, p.relu) * u0, gate_act(g1, p.relu) * u1);
       }
       *(u32x4_t*)(p.C + (size_t)gm * p.ldc + gout) = u32x4_t{packed[0], packed[1], packed[2], packed[3]};
     }
@@ -228,7 +228,7 @@ __global__ void __launch_bounds__(256)
 gemm_splitk_reduce(const float* __restrict__ ws, int splits, int M, int N, int epi,
                    const bf16_t* __restrict__ bias, const bf16_t* __restrict__ resid, int ldr,
                    bf16_t* __restrict__ C, int ldc, const float* __restrict__ ssq_in = nullptr, int parts = 0,
-                   int norm_k = 1, float eps = 0.f) {
+                   int norm_k = 1, float eps = 0.f, int relu = 0) {
   const int nout = (epi == EPI_SWIGLU) ? N / 2 : N;
   const int chunks = nout / 8;
   const size_t total = (size_t)M * chunks;
@@ -247,7 +247,7 @@ gemm_splitk_reduce(const float* __restrict__ ws, int splits, int M, int N, int e
       sum_rows8(ws + (size_t)m * N + gc, splits, (size_t)M * N, g);
       sum_rows8(ws + (size_t)m * N + gc + 16, splits, (size_t)M * N, u);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) v[e] = silu(g[e] * inv) * (u[e] * inv);
+      for (int e = 0; e < 8; ++e) v[e] = gate_act(g[e] * inv, relu) * (u[e] * inv);
     } else {
       sum_rows8(ws + (size_t)m * N + oc, splits, (size_t)M * N, v);
 #pragma unroll
@@ -379,7 +379,7 @@ gemv_kernel(GemmArgs p) {
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
       const int o = g * 16 + 2 * t + j;
-      if (o < p.N / 2) p.C[o] = f2bf(silu(acc[j]) * acc[2 + j]);
+      if (o < p.N / 2) p.C[o] = f2bf(gate_act(acc[j], p.relu) * acc[2 + j]);
     }
   } else {
 #pragma unroll
@@ -590,6 +590,8 @@ DA_EXPORT int da_gemm_dk_splitk(const void* A, int lda, const void* W, void* C, 
   hipStream_t s = (hipStream_t)stream;
   if (M < 1 || M > 64 || K % 64 || N % 16 || lda % 8 || ldc % 8 || !ws || splits < 2 || (K / 64) % splits)
     return (int)hipErrorInvalidValue;
+  const int relu = epi == EPI_REGLU;
+  if (relu) epi = EPI_SWIGLU;
   if (epi == EPI_SWIGLU && N % 32) return (int)hipErrorInvalidValue;
   if (epi == EPI_RESID && (!resid || ldr % 8 || ssq_in)) return (int)hipErrorInvalidValue;
   if (ssq_out && (epi != EPI_RESID || N % 512)) return (int)hipErrorInvalidValue;
@@ -611,7 +613,7 @@ DA_EXPORT int da_gemm_dk_splitk(const void* A, int lda, const void* W, void* C, 
   const int blocks = (int)((work + 255) / 256);
   gemm_splitk_reduce<<<blocks, 256, 0, s>>>((const float*)ws, splits, M, N, epi, (const bf16_t*)bias,
                                              (const bf16_t*)resid, ldr, (bf16_t*)C, ldc, ssq_in, ssq_parts, norm_k,
-                                             eps);
+                                             eps, relu);
   DA_LAUNCH_CHECK();
 }
 
@@ -642,6 +644,8 @@ DA_EXPORT int da_gemm_bf16(const void* A, int lda, const void* W, void* C, int l
                            const void* rms_gamma, float rms_eps, void* stream) {
   hipStream_t s = (hipStream_t)stream;
   if (K % 64 || N % 8 || lda % 8 || ldc % 8) return (int)hipErrorInvalidValue;
+  const int relu = epi == EPI_REGLU;
+  if (relu) epi = EPI_SWIGLU;
   if (epi == EPI_SWIGLU && N % 32) return (int)hipErrorInvalidValue;
   if (splits < 1) splits = 1;
   if ((K / 64) % splits) return (int)hipErrorInvalidValue;
@@ -650,7 +654,7 @@ DA_EXPORT int da_gemm_bf16(const void* A, int lda, const void* W, void* C, int l
   a.A = (const bf16_t*)A; a.W = (const bf16_t*)W; a.C = (bf16_t*)C;
   a.bias = (const bf16_t*)bias; a.resid = (const bf16_t*)resid; a.ws = (float*)ws;
   a.M = M; a.N = N; a.K = K; a.lda = lda; a.ldc = ldc; a.ldr = ldr; a.k_per_split = K / splits;
-  a.gamma = (const bf16_t*)rms_gamma; a.eps = rms_eps;
+  a.gamma = (const bf16_t*)rms_gamma; a.eps = rms_eps; a.relu = relu;
   if ((rms_gamma || rms_eps > 0.f) && tile != 6) return (int)hipErrorInvalidValue;  // fused RMSNorm: GEMV only
   if (tile == 0) {
     // decode-sized M: 32x128 / 64x128 weight-streaming tiles (+ split-K, chosen by the caller);
@@ -686,6 +690,6 @@ DA_EXPORT int da_gemm_bf16(const void* A, int lda, const void* W, void* C, int l
   int blocks = (int)((work + 255) / 256);
   if (blocks > 4096) blocks = 4096;
   gemm_splitk_reduce<<<blocks, 256, 0, s>>>((const float*)ws, splits, M, N, epi, a.bias, a.resid, ldr,
-                                             a.C, ldc);
+                                             a.C, ldc, nullptr, 0, 1, 0.f, relu);
   DA_LAUNCH_CHECK();
 }

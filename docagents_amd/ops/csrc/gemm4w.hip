@@ -291,7 +291,7 @@ gemm4w_kernel(GemmArgs p) {
       for (int q = 0; q < 4; ++q) {
         float v[4];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = silu(acc[i][2 * q][e]) * acc[i][2 * q + 1][e];
+        for (int e = 0; e < 4; ++e) v[e] = gate_act(acc[i][2 * q][e], p.relu) * acc[i][2 * q + 1][e];
         *(u32x2_t*)(st + (i * 16 + fr) * SROW4 + (q * 16 + fg * 4) * 2) =
             u32x2_t{T::pack2(v[0], v[1]), T::pack2(v[2], v[3])};
       }

@@ -297,7 +297,7 @@ gemm8p_kernel(GemmArgs p) {
           for (int i = 0; i < MI; ++i) {
             float v[4];
 #pragma unroll
-            for (int q = 0; q < 4; ++q) v[q] = silu(acc[ih][jh_][i][0][q]) * acc[ih][jh_][i][1][q];
+            for (int q = 0; q < 4; ++q) v[q] = gate_act(acc[ih][jh_][i][0][q], p.relu) * acc[ih][jh_][i][1][q];
             *(u32x2_t*)(st + (ih * QR + i * 16 + efr) * SROW + (jh_ * 16 + efg * 4) * 2) =
                 u32x2_t{T::pack2(v[0], v[1]), T::pack2(v[2], v[3])};
           }

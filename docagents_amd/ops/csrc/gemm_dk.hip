@@ -31,6 +31,7 @@ struct DkArgs {
   float* ssq_out;       // EPI_RESID (nullable): [gridDim.x][64] sums of squares of this tile's output rows
   int M, N, K, lda, ldc, ldr, ssq_parts, norm_k;
   float eps;
+  int relu;  // EPI_SWIGLU: the gate's activation is relu, not silu
   int rb;  // row blocks of BM rows: 1, or 2 (M > BM; workgroup pairs share an XCD)
 };
 
@@ -211,7 +212,7 @@ gemm_dk_kernel(DkArgs p) {
         const float gt = red[0][m][gc + e] + red[1][m][gc + e] + red[2][m][gc + e] + red[3][m][gc + e];
         const float up = red[0][m][gc + 16 + e] + red[1][m][gc + 16 + e] + red[2][m][gc + 16 + e] +
                          red[3][m][gc + 16 + e];
-        v[e] = silu(gt) * up;
+        v[e] = gate_act(gt, p.relu) * up;
       }
       const int oc = n0 / 2 + 16 * g + 8 * hh;
       if (m < Mb && oc < p.N / 2) {  // a ragged last tile (N % BN == 32) holds one gate/up group
@@ -327,6 +328,8 @@ DA_EXPORT int da_gemm_dk(const void* A, int lda, const void* W, void* C, int ldc
                          const void* resid, int ldr, int M, int N, int K, int epi, const float* ssq_in, int ssq_parts,
                          int norm_k, float eps, float* ssq_out, void* stream) {
   if (M < 1 || M > 64 || K % 256 || N % 16 || lda % 8 || ldc % 8) return (int)hipErrorInvalidValue;
+  const int relu = epi == EPI_REGLU;
+  if (relu) epi = EPI_SWIGLU;
   if (epi == EPI_SWIGLU && N % 32) return (int)hipErrorInvalidValue;
   if (epi == EPI_RESID && (!resid || ldr % 8)) return (int)hipErrorInvalidValue;
   if (ssq_out && epi != EPI_RESID) return (int)hipErrorInvalidValue;
@@ -336,7 +339,7 @@ DA_EXPORT int da_gemm_dk(const void* A, int lda, const void* W, void* C, int ldc
   a.bias = (const bf16_t*)bias; a.resid = (const bf16_t*)resid;
   a.ssq_in = ssq_in; a.ssq_out = ssq_out;
   a.M = M; a.N = N; a.K = K; a.lda = lda; a.ldc = ldc; a.ldr = ldr;
-  a.ssq_parts = ssq_parts; a.norm_k = norm_k; a.eps = eps;
+  a.ssq_parts = ssq_parts; a.norm_k = norm_k; a.eps = eps; a.relu = relu;
   const bool norm = ssq_in != nullptr;
   hipStream_t s = (hipStream_t)stream;
   a.rb = 1;

@@ -65,7 +65,7 @@ rope_cache_kernel(bf16_t* __restrict__ qkv, const int* __restrict__ pos, const i
   }
 }
 
-// One workgroup per row of logits [B, V] (bf16). temperature <= 0 -> greedy.
+// One workgroup per row of logits [B, V] (bf16 or fp32). temperature <= 0 -> greedy.
 // Device-side decode bookkeeping so one decode step is graph-capturable (no host round trip):
 //   ctr[b]   : per-row RNG counter (the row's position); null -> `step`
 //   out_tok  : sampled token (also the next step's input token)
@@ -75,7 +75,7 @@ rope_cache_kernel(bf16_t* __restrict__ qkv, const int* __restrict__ pos, const i
 //   pos/lens : advanced by one for active rows
 //   hist     : hist[b * hist_ld + (pos[b] - start[b])] = tok (generation history)
 struct SampleArgs {
-  const bf16_t* logits; int V, ld; float temperature; unsigned seed, step;
+  const void* logits; int V, ld; float temperature; unsigned seed, step;
   const int* ctr; int* out_tok; float* out_lp; float* conf; int* active; int* pos; int* lens;
   int* hist; const int* start; int hist_ld; int eos0, eos1, eos2, eos3;
 };
@@ -103,21 +103,25 @@ __device__ __forceinline__ void sample_bookkeep(const SampleArgs& a, int b, int 
   if (stop && a.active) a.active[b] = 0;
 }
 
+__device__ __forceinline__ float logit_f(bf16_t x) { return bf2f(x); }
+__device__ __forceinline__ float logit_f(float x) { return x; }
+
+template <typename L>
 __global__ void __launch_bounds__(1024)
 sample_kernel(SampleArgs a) {
   __shared__ float redf[16];
   __shared__ float bestv[16];
   __shared__ int besti[16];
   const int b = blockIdx.x;
-  const bf16_t* row = a.logits + (size_t)b * a.ld;
-  const int V = a.V;
+  const L* row = (const L*)a.logits + (size_t)b * a.ld;
+  const int V = a.V, V8 = sizeof(L) == 2 ? V / 8 : 0;  // fp32 rows: the scalar loop below
   const float temperature = a.temperature;
   const float invT = temperature > 0.f ? 1.f / temperature : 0.f;
   const unsigned rs = a.ctr ? (unsigned)a.ctr[b] : a.step;
   const unsigned rkey = rs * 131071u + (unsigned)b;
   float mx = -INFINITY, bv = -INFINITY;
   int bi = 0;
-  for (int c = threadIdx.x; c < V / 8; c += blockDim.x) {
+  for (int c = threadIdx.x; c < V8; c += blockDim.x) {
     u32x4_t u = *(const u32x4_t*)(row + c * 8);
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
@@ -129,8 +133,8 @@ sample_kernel(SampleArgs a) {
       if (score > bv) { bv = score; bi = v; }
     }
   }
-  for (int v = (V / 8) * 8 + threadIdx.x; v < V; v += blockDim.x) {  // tail
-    const float x = bf2f(row[v]);
+  for (int v = V8 * 8 + threadIdx.x; v < V; v += blockDim.x) {  // tail
+    const float x = logit_f(row[v]);
     mx = fmaxf(mx, x);
     float score = x;
     if (temperature > 0.f) score = x * invT - __logf(-__logf(u01(a.seed, rkey, (unsigned)v)));
@@ -146,14 +150,14 @@ sample_kernel(SampleArgs a) {
   if (lane == 0) { bestv[wid] = bv; besti[wid] = bi; }
   const float gmax = block_max(mx, redf);  // contains __syncthreads
   float s = 0.f;
-  for (int v = threadIdx.x; v < V; v += blockDim.x) s += __expf(bf2f(row[v]) - gmax);
+  for (int v = threadIdx.x; v < V; v += blockDim.x) s += __expf(logit_f(row[v]) - gmax);
   s = block_sum(s, redf);
   if (threadIdx.x == 0) {
     float fv = bestv[0];
     int fi = besti[0];
     for (int i = 1; i < nw; ++i)
       if (bestv[i] > fv || (bestv[i] == fv && besti[i] < fi)) { fv = bestv[i]; fi = besti[i]; }
-    sample_bookkeep(a, b, fi, bf2f(row[fi]) - gmax - __logf(s));
+    sample_bookkeep(a, b, fi, logit_f(row[fi]) - gmax - __logf(s));
   }
 }
 
@@ -222,15 +226,16 @@ sample_partial_kernel(const bf16_t* __restrict__ logits, int V, int ld, int v0, 
 // index, ties to the lower index), the logprob's log-sum-exp combined per chunk.
 constexpr int SAMPLE_CL = 1024;  // vocabulary entries per chunk: 4 per thread, kept in registers
 
+template <typename L>
 __global__ void __launch_bounds__(256)
-sample_chunk_kernel(const bf16_t* __restrict__ logits, int V, int ld, float temperature, unsigned seed,
+sample_chunk_kernel(const L* __restrict__ logits, int V, int ld, float temperature, unsigned seed,
                     unsigned step, const int* __restrict__ ctr, float* __restrict__ stats) {
   __shared__ float redf[16];
   __shared__ float bestv[16];
   __shared__ int besti[16];
   const int c = blockIdx.x, b = blockIdx.y, NC = gridDim.x;
   const int v0 = c * SAMPLE_CL;
-  const bf16_t* row = logits + (size_t)b * ld;
+  const L* row = logits + (size_t)b * ld;
   const float invT = temperature > 0.f ? 1.f / temperature : 0.f;
   const unsigned rs = ctr ? (unsigned)ctr[b] : step;
   const unsigned rkey = rs * 131071u + (unsigned)b;
@@ -239,7 +244,7 @@ sample_chunk_kernel(const bf16_t* __restrict__ logits, int V, int ld, float temp
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int v = v0 + threadIdx.x + 256 * i;
-    xs[i] = v < V ? bf2f(row[v]) : -INFINITY;
+    xs[i] = v < V ? logit_f(row[v]) : -INFINITY;
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i) {  // ascending v per thread: ties keep the lower index
@@ -273,7 +278,7 @@ sample_chunk_kernel(const bf16_t* __restrict__ logits, int V, int ld, float temp
     o[1] = __int_as_float(fi);
     o[2] = lmax;
     o[3] = sacc;
-    o[4] = bf2f(row[fi]);
+    o[4] = logit_f(row[fi]);
     o[5] = o[6] = o[7] = 0.f;
   }
 }
@@ -336,13 +341,17 @@ DA_EXPORT int da_sample_finalize(const void* gathered, int B, int ranks, void* o
 DA_EXPORT int da_sample_chunked(const void* logits, int B, int V, int ld, float temperature, unsigned seed,
                                 unsigned step, const void* ctr, void* ws, void* out_tok, void* out_lp, void* conf,
                                 void* active, void* pos, void* lens, void* hist, const void* start, int hist_ld,
-                                int eos0, int eos1, int eos2, int eos3, void* stream) {
+                                int eos0, int eos1, int eos2, int eos3, int f32, void* stream) {
   if (hist && (!pos || !start)) return (int)hipErrorInvalidValue;
   if (V <= 0 || ld < V || !ws) return (int)hipErrorInvalidValue;
   if (B == 0) return 0;
   const int NC = (V + SAMPLE_CL - 1) / SAMPLE_CL;
-  sample_chunk_kernel<<<dim3(NC, B), 256, 0, (hipStream_t)stream>>>((const bf16_t*)logits, V, ld, temperature,
-                                                                     seed, step, (const int*)ctr, (float*)ws);
+  if (f32)
+    sample_chunk_kernel<float><<<dim3(NC, B), 256, 0, (hipStream_t)stream>>>(
+        (const float*)logits, V, ld, temperature, seed, step, (const int*)ctr, (float*)ws);
+  else
+    sample_chunk_kernel<bf16_t><<<dim3(NC, B), 256, 0, (hipStream_t)stream>>>(
+        (const bf16_t*)logits, V, ld, temperature, seed, step, (const int*)ctr, (float*)ws);
   const hipError_t e = hipGetLastError();
   if (e != hipSuccess) return (int)e;
   SampleArgs a{};
@@ -367,16 +376,17 @@ DA_EXPORT int da_rope_cache(void* qkv, const void* pos, const void* slot, const 
 
 DA_EXPORT int da_sample(const void* logits, int B, int V, int ld, float temperature, unsigned seed, unsigned step,
                         const void* ctr, void* out_tok, void* out_lp, void* conf, void* active, void* pos, void* lens,
-                        void* hist, const void* start, int hist_ld, int eos0, int eos1, int eos2, int eos3,
+                        void* hist, const void* start, int hist_ld, int eos0, int eos1, int eos2, int eos3, int f32,
                         void* stream) {
   if (ld % 8) return (int)hipErrorInvalidValue;
   if (hist && (!pos || !start)) return (int)hipErrorInvalidValue;
   if (B == 0) return 0;
   SampleArgs a;
-  a.logits = (const bf16_t*)logits; a.V = V; a.ld = ld; a.temperature = temperature; a.seed = seed; a.step = step;
+  a.logits = logits; a.V = V; a.ld = ld; a.temperature = temperature; a.seed = seed; a.step = step;
   a.ctr = (const int*)ctr; a.out_tok = (int*)out_tok; a.out_lp = (float*)out_lp; a.conf = (float*)conf;
   a.active = (int*)active; a.pos = (int*)pos; a.lens = (int*)lens; a.hist = (int*)hist; a.start = (const int*)start;
   a.hist_ld = hist_ld; a.eos0 = eos0; a.eos1 = eos1; a.eos2 = eos2; a.eos3 = eos3;
-  sample_kernel<<<B, 1024, 0, (hipStream_t)stream>>>(a);
+  if (f32) sample_kernel<float><<<B, 1024, 0, (hipStream_t)stream>>>(a);
+  else sample_kernel<bf16_t><<<B, 1024, 0, (hipStream_t)stream>>>(a);
   DA_LAUNCH_CHECK();
 }

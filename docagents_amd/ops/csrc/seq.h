@@ -1,0 +1,57 @@
+// Shared pieces of the kernels that run a batch of sequence portions against per-sequence state.
+#pragma once
+#include "common.h"
+
+// A step's batch: B portions packed row after row. Portion b is rows cu[b] .. cu[b + 1] - 1 of the
+// packed matrices, the tokens at positions pos0[b], pos0[b] + 1, ... of the sequence that owns state
+// slot slot[b]; seq[t] is the portion of packed row t. A portion at position 0 starts its sequence:
+// whatever its slot holds from an earlier owner is not read.
+struct SeqMeta {
+  const int* cu; const int* slot; const int* pos0; const int* seq;
+  int T, B;
+};
+
+// Chunks of CHUNK tokens for the recurrences: chunk i is tokens [CHUNK * ck[2i+1], + CHUNK) of portion
+// ck[2i]; base[b] is the number of chunks of the portions before b.
+struct ChunkMeta {
+  const int* ck; const int* base;
+  int n;
+};
+constexpr int CHUNK = 64;
+constexpr int PAGE = 64;  // tokens per cache page
+
+// Activation storage: bf16 (the serving precision) or fp32; arithmetic is fp32 either way.
+template <typename T> struct Act;
+template <> struct Act<bf16_t> {
+  __device__ static __forceinline__ float to_f(bf16_t v) { return bf2f(v); }
+  __device__ static __forceinline__ bf16_t from_f(float v) { return f2bf(v); }
+  __device__ static __forceinline__ f32x4_t load4(const bf16_t* p) {
+    const u32x2_t u = *(const u32x2_t*)p;
+    return f32x4_t{__uint_as_float(u[0] << 16), __uint_as_float(u[0] & 0xffff0000u), __uint_as_float(u[1] << 16),
+                   __uint_as_float(u[1] & 0xffff0000u)};
+  }
+  __device__ static __forceinline__ void store4(bf16_t* p, const f32x4_t& v) {
+    *(u32x2_t*)p = u32x2_t{pack_bf2(v[0], v[1]), pack_bf2(v[2], v[3])};
+  }
+  __device__ static __forceinline__ f32x2_t load2(const bf16_t* p) {
+    const unsigned u = *(const unsigned*)p;
+    return f32x2_t{__uint_as_float(u << 16), __uint_as_float(u & 0xffff0000u)};
+  }
+  __device__ static __forceinline__ void store2(bf16_t* p, float a, float b) { *(unsigned*)p = pack_bf2(a, b); }
+};
+template <> struct Act<float> {
+  __device__ static __forceinline__ float to_f(float v) { return v; }
+  __device__ static __forceinline__ float from_f(float v) { return v; }
+  __device__ static __forceinline__ f32x4_t load4(const float* p) { return *(const f32x4_t*)p; }
+  __device__ static __forceinline__ void store4(float* p, const f32x4_t& v) { *(f32x4_t*)p = v; }
+  __device__ static __forceinline__ f32x2_t load2(const float* p) { return *(const f32x2_t*)p; }
+  __device__ static __forceinline__ void store2(float* p, float a, float b) { *(f32x2_t*)p = f32x2_t{a, b}; }
+};
+
+__device__ __forceinline__ float sigmoid32(float x) { return 1.f / (1.f + expf(-x)); }
+__device__ __forceinline__ float softplus32(float x) { return x > 20.f ? x + expf(-x) : log1pf(expf(x)); }
+__device__ __forceinline__ float silu32(float x) { return x / (1.f + expf(-x)); }
+__device__ __forceinline__ float gelu_tanh32(float x) {
+  // 0.5 (1 + tanh(z)) = sigmoid(2 z)
+  return x * sigmoid32(1.5957691216057308f * (x + 0.044715f * x * x * x));
+}

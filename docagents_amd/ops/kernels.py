@@ -25,6 +25,8 @@ _LIB_OVERRIDE: Path | None = None  # one library with every launcher, instead of
 
 EPI_NONE, EPI_BIAS, EPI_GELU, EPI_SWIGLU, EPI_RESID = 0, 1, 2, 3, 4
 EPI_ROPE = 6  # gemm8p only: QKV + RoPE + KV-cache write
+EPI_REGLU = 7  # EPI_SWIGLU with relu in place of silu
+GATED = (EPI_SWIGLU, EPI_REGLU)
 
 c_longlong = ctypes.c_longlong
 c_void_p, c_int, c_float, c_uint, c_size_t = (ctypes.c_void_p, ctypes.c_int, ctypes.c_float,
@@ -50,7 +52,7 @@ _SIGS = {
     "da_pool_l2norm": [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p],
     "da_rope_cache": [c_void_p] * 6 + [c_int] * 6 + [c_void_p],
     "da_sample": [c_void_p, c_int, c_int, c_int, c_float, c_uint, c_uint] + [c_void_p] * 9
-                 + [c_int] * 5 + [c_void_p],
+                 + [c_int] * 6 + [c_void_p],
     "da_flash_attn_v2": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_int,
                          c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_void_p, c_longlong,
                          c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p],
@@ -73,7 +75,7 @@ _SIGS = {
     "da_kmeans_accum": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p],
     "da_sample_partial": [c_void_p, c_int, c_int, c_int, c_int, c_float, c_uint, c_uint, c_void_p, c_void_p, c_void_p],
     "da_sample_chunked": [c_void_p, c_int, c_int, c_int, c_float, c_uint, c_uint] + [c_void_p] * 10
-                         + [c_int] * 5 + [c_void_p],
+                         + [c_int] * 6 + [c_void_p],
     "da_sample_finalize": [c_void_p, c_int, c_int] + [c_void_p] * 8 + [c_int] * 5 + [c_void_p],
     "da_stream_create_cumask": [c_uint, ctypes.POINTER(c_uint), ctypes.POINTER(c_void_p)],
     "da_stream_get_cumask": [c_void_p, c_uint, ctypes.POINTER(c_uint)],
@@ -231,7 +233,7 @@ def _workspace(nbytes: int, device) -> torch.Tensor:
 
 def gemv_fusable(M: int, N: int, K: int, epi: int = EPI_NONE) -> bool:
     """True when gemm() runs the batch-1 GEMV (which can also fuse the input RMSNorm)."""
-    return M == 1 and K % 512 == 0 and N % 4 == 0 and (epi != EPI_SWIGLU or N % 32 == 0)
+    return M == 1 and K % 512 == 0 and N % 4 == 0 and (epi not in GATED or N % 32 == 0)
 
 
 def gemm(a: torch.Tensor, w: torch.Tensor, bias=None, epi: int = EPI_NONE, resid=None, out=None,
@@ -249,8 +251,8 @@ def gemm(a: torch.Tensor, w: torch.Tensor, bias=None, epi: int = EPI_NONE, resid
     _req(a.stride(1) == 1 and a.stride(0) % 8 == 0 and a.stride(0) >= K, "a must be row-major, 16-B aligned rows")
     _req(w.is_contiguous(), "w must be contiguous")
     _req(a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0, "operands must be 16-B aligned")
-    nout = N // 2 if epi == EPI_SWIGLU else N
-    if epi == EPI_SWIGLU:
+    nout = N // 2 if epi in GATED else N
+    if epi in GATED:
         _req(N % 32 == 0, "SwiGLU needs N % 32 == 0")
     if out is None:
         out = torch.empty((M, nout), dtype=torch.bfloat16, device=a.device)
@@ -305,7 +307,7 @@ DK_SPLITK_ABOVE = 32
 def dk_fusable(M: int, N: int, K: int, epi: int = EPI_NONE) -> bool:
     """True when gemm() runs a decode-sized product on gemm_dk (no split-K)."""
     return (DECODE_DK and 2 <= M <= DK_MAX_M and K % 256 == 0 and N % 16 == 0
-            and epi in (EPI_NONE, EPI_BIAS, EPI_RESID, EPI_SWIGLU) and (epi != EPI_SWIGLU or N % 32 == 0))
+            and epi in (EPI_NONE, EPI_BIAS, EPI_RESID, *GATED) and (epi not in GATED or N % 32 == 0))
 
 
 def _dk_splitk(M: int, N: int) -> bool:
@@ -345,7 +347,7 @@ def gemm_dk(a, w, epi: int = EPI_NONE, bias=None, resid=None, out=None, norm_in=
     _req(1 <= M <= 64 and K % 256 == 0 and N % 16 == 0 and w.shape[1] == K, f"gemm_dk shape M={M} N={N} K={K}")
     _req(a.stride(1) == 1 and a.stride(0) % 8 == 0 and w.is_contiguous(), "gemm_dk layout")
     _req(a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0, "operands must be 16-B aligned")
-    nout = N // 2 if epi == EPI_SWIGLU else N
+    nout = N // 2 if epi in GATED else N
     if out is None:
         out = torch.empty((M, nout), dtype=torch.bfloat16, device=a.device)
     _req(out.shape == (M, nout) and out.stride(1) == 1 and out.stride(0) % 8 == 0, "bad out")
@@ -834,8 +836,12 @@ def _sample_ws(nfloats: int, device) -> torch.Tensor:
 
 def sample(logits, temperature: float, seed: int, step: int = 0, out_tok=None, out_lp=None, conf=None,
            active=None, ctr=None, pos=None, lens=None, hist=None, start=None, eos=()):
-    """Fused temperature sampler (see rope_sample.hip). Returns (tokens, logprobs)."""
-    _bf16_cuda(logits, "logits")
+    """Fused temperature sampler over bf16 or fp32 logits (see rope_sample.hip). Returns (tokens, logprobs)."""
+    f32 = int(logits.dtype == torch.float32)
+    if f32:
+        _req(logits.is_cuda, "logits must be on GPU")
+    else:
+        _bf16_cuda(logits, "logits")
     B, V = logits.shape
     _req(logits.stride(1) == 1 and logits.stride(0) % 8 == 0, "logits layout")
     dev = logits.device
@@ -861,12 +867,12 @@ def sample(logits, temperature: float, seed: int, step: int = 0, out_tok=None, o
         _check(lib().da_sample_chunked(_ptr(logits), B, V, logits.stride(0), float(temperature), seed & 0xffffffff,
                                        step & 0xffffffff, _ptr(ctr), _ptr(ws), _ptr(out_tok), _ptr(out_lp),
                                        _ptr(conf), _ptr(active), _ptr(pos), _ptr(lens), _ptr(hist), _ptr(start),
-                                       hist_ld, e[0], e[1], e[2], e[3], _stream()), "sample_chunked")
+                                       hist_ld, e[0], e[1], e[2], e[3], f32, _stream()), "sample_chunked")
         return out_tok, out_lp
     _check(lib().da_sample(_ptr(logits), B, V, logits.stride(0), float(temperature), seed & 0xffffffff,
                            step & 0xffffffff, _ptr(ctr), _ptr(out_tok), _ptr(out_lp), _ptr(conf), _ptr(active),
                            _ptr(pos), _ptr(lens), _ptr(hist), _ptr(start), hist_ld, e[0], e[1], e[2], e[3],
-                           _stream()), "sample")
+                           f32, _stream()), "sample")
     return out_tok, out_lp
 
 
@@ -1115,3 +1121,8 @@ def pool_l2norm_f16(h, cu_seqlens, mode: int = 0, out32=None, out16=None):
     _check(lib().da_pool_l2norm_f16(_ptr(h), _ptr(cu_seqlens), B, D, mode, _ptr(out32), _ptr(out16), _stream()),
            "pool_l2norm_f16")
     return out32 if out32 is not None else out16
+
+
+# the batch-of-portions ops (recurrent mixers, paged attention, 32-bit residual stream)
+from .seq_kernels import (causal_conv, gated_scan, gemm_any, rglru_gates, selective_scan,  # noqa: E402,F401
+                          sigmoid_attn, stream_final, stream_step)

@@ -14,6 +14,8 @@ import torch.nn.functional as F
 
 EPI_NONE, EPI_BIAS, EPI_GELU, EPI_SWIGLU, EPI_RESID = 0, 1, 2, 3, 4
 EPI_ROPE = 6  # gemm8p only: QKV + RoPE + KV-cache write
+EPI_REGLU = 7  # EPI_SWIGLU with relu in place of silu
+GATED = (EPI_SWIGLU, EPI_REGLU)
 
 
 def gemv_fusable(M, N, K, epi=EPI_NONE):
@@ -32,10 +34,10 @@ def _epilogue(y, N, bias, epi, resid, out):
         y = y + bias.float()
     if epi == EPI_GELU:
         y = F.gelu(y)
-    elif epi == EPI_SWIGLU:
+    elif epi in GATED:
         yy = y.view(y.shape[0], N // 32, 2, 16)
         g, u = yy[:, :, 0, :], yy[:, :, 1, :]
-        y = (F.silu(g) * u).reshape(y.shape[0], N // 2)
+        y = ((F.silu(g) if epi == EPI_SWIGLU else F.relu(g)) * u).reshape(y.shape[0], N // 2)
     elif epi == EPI_RESID:
         y = y + resid.float()
     y = y.to(torch.bfloat16)
@@ -481,7 +483,7 @@ DK_SPLITK_ABOVE = 32
 
 def dk_fusable(M, N, K, epi=EPI_NONE):
     return (DECODE_DK and 2 <= M <= DK_MAX_M and K % 256 == 0 and N % 16 == 0
-            and epi in (EPI_NONE, EPI_BIAS, EPI_RESID, EPI_SWIGLU) and (epi != EPI_SWIGLU or N % 32 == 0))
+            and epi in (EPI_NONE, EPI_BIAS, EPI_RESID, *GATED) and (epi not in GATED or N % 32 == 0))
 
 
 def dk_parts(N, M=0):
@@ -536,3 +538,8 @@ def flash_attn_f16(q, k, v, cu_seqlens, max_seqlen, H, Hkv, D, causal=False, sca
         out.copy_(y)
         return out
     return y
+
+
+# the batch-of-portions ops (recurrent mixers, paged attention, 32-bit residual stream)
+from .seq_reference import (causal_conv, gated_scan, gemm_any, rglru_gates, selective_scan,  # noqa: E402,F401
+                            sigmoid_attn, stream_final, stream_step)

@@ -1,0 +1,65 @@
+"""The batch of one step: portions of sequences packed row after row, each against its own state slot."""
+from __future__ import annotations
+
+from dataclasses import dataclass, replace
+
+import numpy as np
+import torch
+
+from . import h2d
+
+CHUNK = 64  # tokens per chunk of a recurrence (csrc/seq.h)
+PAGE = 64   # tokens per cache page (csrc/seq.h)
+
+
+@dataclass
+class SeqBatch:
+    """Portion b is packed rows ``cu[b] .. cu[b + 1]``: the tokens at positions ``pos0[b]``, ... of the
+    sequence in state slot ``slot[b]``; ``seq[t]`` is row t's portion (all int32, on the device)."""
+    cu: torch.Tensor
+    slot: torch.Tensor
+    pos0: torch.Tensor
+    seq: torch.Tensor
+    T: int                 # packed rows
+    B: int                 # portions
+    max_len: int           # longest portion
+    max_ctx: int           # bound on position + 1 over the batch (sets split counts: a host number)
+    singles: bool = True   # a portion of one token may be in the batch
+    table: torch.Tensor | None = None  # int32 [slots, pages of a slot]: the cache's page table
+    ck: torch.Tensor | None = None     # int32 [n_chunks, 2]: (portion, chunk of it)
+    base: torch.Tensor | None = None   # int32 [B]: chunks of the portions before b
+    n_chunks: int = 0                  # 0: every portion fits one chunk
+
+    def on(self, table) -> "SeqBatch":
+        return replace(self, table=table)
+
+
+def pack_batch(lens, slots, pos0, device, ids=None):
+    """Host lists -> (SeqBatch, token ids on the device or None): one host-to-device copy."""
+    lens = np.asarray(lens, dtype=np.int64)
+    B, T = len(lens), int(lens.sum())
+    if B == 0 or lens.min() < 1:
+        raise ValueError("a batch needs portions of at least one token")
+    cu = np.zeros(B + 1, dtype=np.int32)
+    np.cumsum(lens, out=cu[1:])
+    parts = [cu, np.asarray(slots, dtype=np.int32), np.asarray(pos0, dtype=np.int32),
+             np.repeat(np.arange(B, dtype=np.int32), lens)]
+    n = 0
+    if lens.max() > CHUNK:
+        per = -(-lens // CHUNK)
+        n = int(per.sum())
+        base = np.cumsum(per) - per
+        ck = np.stack([np.repeat(np.arange(B), per), np.arange(n) - np.repeat(base, per)], axis=1)
+        parts += [ck.astype(np.int32).ravel(), base.astype(np.int32)]
+    if ids is not None:
+        parts.append(np.asarray(ids, dtype=np.int32))
+    flat = h2d(np.concatenate(parts), device)
+    out, at = [], 0
+    for p in parts:
+        out.append(flat[at:at + len(p)])
+        at += len(p)
+    m = SeqBatch(out[0], out[1], out[2], out[3], T, B, int(lens.max()), int((lens + parts[2]).max()),
+                 bool((lens == 1).any()))
+    if n:
+        m.ck, m.base, m.n_chunks = out[4].view(n, 2), out[5], n
+    return m, (out[-1] if ids is not None else None)

@@ -1,0 +1,240 @@
+"""Bindings of the batch-of-portions kernels (``csrc/stream_norm.hip``, ``recurrent.hip``,
+``paged_attn.hip``, ``gemm_any.hip``). Re-exported by ``kernels``; the fp32 oracles with the same
+signatures are in ``seq_reference``. Activations are bf16, or fp32 in the fp32 precision; the residual
+stream, recurrent state, decays, step sizes and attention weights are fp32 in both."""
+from __future__ import annotations
+
+
+import torch
+
+from . import kernels as K
+from .kernels import _check, _ptr, _req, _stream, c_float, c_int, c_longlong, c_void_p, lib
+from .seq_batch import PAGE, SeqBatch
+
+_META = [c_void_p] * 4 + [c_int] * 2
+K._SIGS.update({
+    "da_gemm_any": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p] + [c_int] * 6 + [c_longlong] * 4
+                   + [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p],
+    "da_stream_step": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_float, c_float, c_int, c_int]
+                      + [c_void_p] * 5 + _META + [c_int, c_int, c_void_p],
+    "da_stream_final": [c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_void_p, c_int, c_int, c_void_p],
+    "da_causal_conv": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int] + _META
+                      + [c_int, c_void_p],
+    "da_selective_scan": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_int]
+                         + [c_void_p] * 4 + [c_int] * 3 + [c_void_p, c_int, c_void_p, c_int]
+                         + [c_void_p] * 4 + [c_int] + _META + [c_int, c_void_p],
+    "da_gated_scan": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p,
+                      c_int] + [c_void_p] * 4 + [c_int] + _META + [c_int, c_void_p],
+    "da_sigmoid_attn": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float,
+                        c_float, c_float, K.ctypes.c_double] + [c_int] * 4 + [c_void_p, c_int, c_void_p] + [c_int] * 4
+                       + _META + [c_int, c_void_p],
+})
+K._PART_OF.update({n: "hybrid" for n in ("da_gemm_any", "da_stream_step", "da_stream_final", "da_causal_conv",
+                                         "da_selective_scan", "da_gated_scan", "da_sigmoid_attn")})
+
+ACTS = (torch.bfloat16, torch.float32)
+ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_RGLRU = 0, 1, 2, 3
+
+
+def _act(t, name, dtype=None):
+    _req(t.is_cuda and t.dtype in ACTS and (dtype is None or t.dtype == dtype), f"{name}: bf16 / fp32 on the GPU")
+    _req(t.stride(-1) == 1 and t.data_ptr() % 16 == 0, f"{name} layout")
+    return int(t.dtype == torch.float32)
+
+
+def _f32(t, name, numel=None):
+    _req(t.is_cuda and t.dtype == torch.float32 and t.is_contiguous(), f"{name} must be contiguous fp32 on GPU")
+    _req(numel is None or t.numel() == numel, f"{name}: {t.numel()} elements, want {numel}")
+
+
+def _meta(m: SeqBatch):
+    for t, n, name in ((m.cu, m.B + 1, "cu"), (m.slot, m.B, "slot"), (m.pos0, m.B, "pos0"), (m.seq, m.T, "seq")):
+        _req(t.is_cuda and t.dtype == torch.int32 and t.is_contiguous() and t.numel() >= n, f"batch {name}")
+    return [_ptr(m.cu), _ptr(m.slot), _ptr(m.pos0), _ptr(m.seq), m.T, m.B]
+
+
+def _chunks(m: SeqBatch):
+    if m.n_chunks:
+        _req(m.ck.dtype == torch.int32 and m.ck.numel() == 2 * m.n_chunks and m.base.numel() == m.B, "batch chunks")
+    return [_ptr(m.ck), _ptr(m.base), m.n_chunks]
+
+
+def gemm_any(a, w, bias=None, epi: int = ANY_NONE):
+    """fp32 [M, N'] = epi(a[M, K] @ w[N, K]^T + bias), a and w both bf16 or both fp32, bias fp32; any M and
+    N, K a multiple of 16 bytes. ANY_SOFTPLUS: softplus; ANY_REGLU: w rows interleaved by 16 (gate, up)."""
+    f32 = _act(a, "a")
+    _act(w, "w", a.dtype)
+    M, Kd = a.shape
+    N = w.shape[0]
+    _req(w.is_contiguous() and w.shape[1] >= 1 and Kd == w.shape[1] and epi in (ANY_NONE, ANY_SOFTPLUS, ANY_REGLU), "gemm_any")
+    if bias is not None:
+        _f32(bias, "bias", N)
+    out = torch.empty((M, N // 2 if epi == ANY_REGLU else N), dtype=torch.float32, device=a.device)
+    _check(lib().da_gemm_any(_ptr(a), a.stride(0), _ptr(w), _ptr(out), out.stride(0), _ptr(bias), M, N, Kd, f32, epi, 1, 0,
+                             0, 0, 0, None, 0, None, None, None, 0, _stream()), "gemm_any")
+    return out
+
+
+def rglru_gates(u, w, bias, lam):
+    """Gated linear recurrence, block-diagonal gates: u [T, blocks * bw], w [blocks, 2 bw, bw] (rows of the
+    recurrence and input gates interleaved by 16), bias fp32 [blocks, 2 bw], lam fp32 [C] (the log decay at
+    an open recurrence gate) -> (decay, drive) fp32 [T, C]: decay = exp(lam r), drive = sqrt(1 - decay^2) i u."""
+    f32 = _act(u, "u")
+    _act(w, "w", u.dtype)
+    blocks, bw2, bw = w.shape
+    T, C = u.shape
+    _req(w.is_contiguous() and bw2 == 2 * bw and blocks * bw == C and bw % 16 == 0, "gate weights [blocks, 2 bw, bw]")
+    _f32(bias, "bias", blocks * bw2)
+    _f32(lam, "lam", C)
+    decay = torch.empty((T, C), dtype=torch.float32, device=u.device)
+    drive = torch.empty_like(decay)
+    _check(lib().da_gemm_any(_ptr(u), u.stride(0), _ptr(w), None, 0, _ptr(bias), T, bw2, bw, f32, ANY_RGLRU, blocks, bw,
+                             bw2 * bw, 0, bw2, _ptr(u), u.stride(0), _ptr(lam), _ptr(decay), _ptr(drive), C, _stream()),
+           "rglru_gates")
+    return decay, drive
+
+
+def stream_step(m: SeqBatch, dim: int, eps: float = 0.0, alpha: float = 1.0, ids=None, table=None, x=None, y=None,
+                w=None, mu=None, prev=None, save=None, want_x: bool = True, want_h: bool = True, act=None):
+    """One update of the fp32 residual stream: x' = table[ids], or RMSNorm(alpha x + y) w over ``dim`` of the
+    padded columns; h = x' or, with mu / prev (state [slots, Dp]), x' + (x'_previous token - x') mu, in the
+    activation type. save: state [slots, Dp] that receives each portion's last row of x. -> (x', h)."""
+    src = table if ids is not None else y
+    f32 = _act(src, "table / y", act)
+    Dp = src.shape[1]
+    dev = src.device
+    _req(src.is_contiguous() and Dp % 4 == 0 and dim <= Dp <= 16384, "stream columns")
+    if ids is not None:
+        _req(ids.dtype == torch.int32 and ids.is_contiguous() and ids.numel() >= m.T and ids.is_cuda, "ids")
+    else:
+        _f32(x, "x", m.T * Dp)
+        _f32(w, "w", Dp)
+        _req(y.shape[0] == m.T, "y rows")
+    if mu is not None:
+        _f32(mu, "mu", Dp)
+        _f32(prev, "prev")
+    if save is not None:
+        _f32(save, "save")
+    xo = torch.empty((m.T, Dp), dtype=torch.float32, device=dev) if want_x else None
+    ho = torch.empty((m.T, Dp), dtype=src.dtype, device=dev) if want_h else None
+    rows = 1 if m.T <= 1024 else 4
+    _check(lib().da_stream_step(_ptr(ids), _ptr(table), 0 if table is None else table.shape[0], _ptr(x), _ptr(y), _ptr(w),
+                                float(alpha), float(eps), dim, Dp, _ptr(xo), _ptr(ho), _ptr(mu), _ptr(prev), _ptr(save),
+                                *_meta(m), rows, f32, _stream()), "stream_step")
+    return xo, ho
+
+
+def stream_final(x, w, eps: float, dim: int, act, rows=None):
+    """RMSNorm of the (selected: rows int64) stream rows in the activation type."""
+    _f32(x, "x")
+    _f32(w, "w", x.shape[1])
+    if rows is not None:
+        _req(rows.dtype == torch.int64 and rows.is_contiguous() and rows.is_cuda, "rows int64")
+    n = x.shape[0] if rows is None else rows.numel()
+    y = torch.empty((n, x.shape[1]), dtype=act, device=x.device)
+    _check(lib().da_stream_final(_ptr(x), _ptr(rows), _ptr(w), float(eps), dim, x.shape[1], _ptr(y), n,
+                                 int(act == torch.float32), _stream()), "stream_final")
+    return y
+
+
+def causal_conv(x, w, bias, state, m: SeqBatch, silu: bool):
+    """Per-channel causal convolution over each portion: x [T, C] (row view), w fp32 [taps, C] (last row: the
+    current token), bias fp32 [C], state [slots, taps - 1, C] (read only; the recurrence replaces it)."""
+    f32 = _act(x, "x")
+    taps, C = w.shape
+    _f32(w, "w")
+    _f32(bias, "bias", C)
+    _req(x.shape == (m.T, C) and x.stride(0) % 4 == 0 and C % 4 == 0, "conv input")
+    _req(state.dtype == x.dtype and state.is_contiguous() and state.shape[1:] == (taps - 1, C), "conv state")
+    y = torch.empty((m.T, C), dtype=x.dtype, device=x.device)
+    _check(lib().da_causal_conv(_ptr(x), x.stride(0), _ptr(w), _ptr(bias), _ptr(state), _ptr(y), C, C, taps, int(silu),
+                                *_meta(m), f32, _stream()), "causal_conv")
+    return y
+
+
+def _conv_args(conv_x, conv_state, C, dtype):
+    _act(conv_x, "conv_x", dtype)
+    _req(conv_state.dtype == dtype and conv_state.is_contiguous() and conv_state.shape[2] == C, "conv state")
+    return [_ptr(conv_x), conv_x.stride(0), _ptr(conv_state), conv_state.shape[1] + 1]
+
+
+def selective_scan(x, dt, bc, off_b: int, off_c: int, z, A, D, state, conv_x, conv_state, m: SeqBatch):
+    """Mamba's recurrence: x, z [T, C]; dt fp32 [T, C]; B and C rows at columns off_b / off_c of bc; A fp32
+    [C, N] = log2(e) * (negative rates); D fp32 [C]; state fp32 [slots, C, N], updated, as is conv_state (from
+    the convolution's inputs conv_x). -> (S C + D x) silu(z) in the activation type."""
+    f32 = _act(x, "x")
+    _act(z, "z", x.dtype)
+    _act(bc, "bc", x.dtype)
+    C, N = A.shape
+    for t, n, k in ((A, "A", C * N), (D, "D", C), (dt, "dt", m.T * C), (state, "state", None)):
+        _f32(t, n, k)
+    _req(x.shape == (m.T, C) and z.shape == (m.T, C) and state.shape[1:] == (C, N) and N <= 512
+         and max(off_b, off_c) + N <= bc.shape[1] and bc.shape[0] == m.T, "selective_scan shapes")
+    y = torch.empty((m.T, C), dtype=x.dtype, device=x.device)
+    cs = cd = None
+    if m.n_chunks:
+        cs = torch.empty((m.n_chunks + m.B, C, N), dtype=torch.float32, device=x.device)
+        cd = torch.empty((m.n_chunks + m.B, C), dtype=torch.float32, device=x.device)
+    _check(lib().da_selective_scan(_ptr(x), x.stride(0), _ptr(dt), C, _ptr(bc), bc.stride(0), off_b, off_c, _ptr(z),
+                                   z.stride(0), _ptr(A), _ptr(D), _ptr(state), _ptr(y), C, C, N,
+                                   *_conv_args(conv_x, conv_state, C, x.dtype), _ptr(cs), _ptr(cd), *_chunks(m), *_meta(m),
+                                   f32, _stream()), "selective_scan")
+    return y
+
+
+def gated_scan(decay, drive, gate, state, conv_x, conv_state, m: SeqBatch):
+    """S <- decay S + drive per channel (fp32 [T, C]), state fp32 [slots, C] updated (and conv_state, see
+    ``selective_scan``) -> S gelu_tanh(gate) in gate's type."""
+    f32 = _act(gate, "gate")
+    C = state.shape[1]
+    for t, n, k in ((decay, "decay", m.T * C), (drive, "drive", m.T * C), (state, "state", None)):
+        _f32(t, n, k)
+    _req(gate.shape == (m.T, C), "gate [T, C]")
+    y = torch.empty((m.T, C), dtype=gate.dtype, device=gate.device)
+    cs = cd = None
+    if m.n_chunks:
+        cs = torch.empty((m.n_chunks + m.B, C), dtype=torch.float32, device=gate.device)
+        cd = torch.empty_like(cs)
+    _check(lib().da_gated_scan(_ptr(decay), _ptr(drive), _ptr(gate), gate.stride(0), _ptr(state), _ptr(y), C, C,
+                               *_conv_args(conv_x, conv_state, C, gate.dtype), _ptr(cs), _ptr(cd), *_chunks(m), *_meta(m),
+                               f32, _stream()), "gated_scan")
+    return y
+
+
+def _attn_split(B: int, G: int, qtiles: int, max_ctx: int):
+    """(splits, pages per split) of the single-token kernel: ~1024 workgroups, >= 4 pages (one per wave) each."""
+    pages = -(-max_ctx // PAGE)
+    want = max(1, min(-(-1024 // (B * G * qtiles)), -(-pages // 4)))
+    pps = -(-pages // want)
+    return -(-pages // pps), pps
+
+
+def sigmoid_attn(qkg, kc, kr, pb, qk_w, m: SeqBatch, H: int, G: int, dim: int, scale: float, eps: float, temp=None):
+    """Attention with unnormalised sigmoid weights, values = keys: qkg [T, (H + G) D + >= H] (overwritten: the
+    queries are prepared in place), pages kc [pages, G, 64, D] / kr fp32 [pages, G, 64] through m.table, pb fp32
+    [H] added to the scores, qk_w fp32 [D] = query norm weight * key norm weight, temp = (coef, every) of the
+    query temperature 1 + coef ln(floor((p + 1) / every) + 1). Every head's output is multiplied by the sigmoid
+    of its gate column. -> [T, H D]."""
+    f32 = _act(qkg, "qkg")
+    D = kc.shape[3]
+    _act(kc, "kc", qkg.dtype)
+    _f32(kr, "kr")
+    _f32(pb, "pb", H)
+    _f32(qk_w, "qk_w", D)
+    _req(qkg.shape[0] == m.T and qkg.shape[1] >= (H + G) * D + H and qkg.stride(0) % 8 == 0, "qkg columns")
+    _req(kc.is_contiguous() and kc.shape[1:3] == (G, PAGE) and kr.shape == kc.shape[:3] and D % 32 == 0, "pages")
+    t = m.table
+    _req(t is not None and t.is_cuda and t.dtype == torch.int32 and t.is_contiguous() and t.dim() == 2, "page table")
+    _req(m.max_ctx <= t.shape[1] * PAGE, f"context {m.max_ctx} exceeds the page table ({t.shape[1]} pages)")
+    out = torch.empty((m.T, H * D), dtype=qkg.dtype, device=qkg.device)
+    nsplit, pps = _attn_split(m.B, G, -(-(H // G) // 16), m.max_ctx)
+    part = None
+    if not f32 and m.singles and nsplit > 1:
+        part = torch.empty((m.B, H, nsplit, D), dtype=torch.float32, device=qkg.device)
+    coef, every = temp if temp else (0.0, 0.0)
+    _check(lib().da_sigmoid_attn(_ptr(qkg), qkg.stride(0), _ptr(kc), _ptr(kr), _ptr(t), t.shape[1], kc.shape[0], _ptr(pb),
+                                 _ptr(qk_w), float(scale), float(eps), float(coef), float(every), H, G, D, dim, _ptr(out),
+                                 out.stride(0), _ptr(part), nsplit if part is not None else 1,
+                                 pps if part is not None else -(-m.max_ctx // PAGE), m.max_len, int(m.singles), *_meta(m),
+                                 f32, _stream()), "sigmoid_attn")
+    return out

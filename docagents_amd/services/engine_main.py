@@ -108,7 +108,7 @@ def main(argv=None) -> int:
                  temperature=cfg.temperature, max_new_tokens=cfg.max_new_tokens,
                  summary_max_new=cfg.summary_max_new_tokens, index_kind=cfg.index_kind, ivf_lists=cfg.ivf_lists,
                  ivf_probes=cfg.ivf_probes, max_seq=4096 if dev.type == "cuda" else 1024,
-                 enc_dtype=cfg.dtype)
+                 enc_dtype=cfg.dtype, llm_dtype=cfg.llm_dtype)
     if cfg.engine_admit_tokens > 0:
         eng.admit_tokens = cfg.engine_admit_tokens
     if cfg.engine_continuous and dev.type == "cuda" and eng.gen is not None:
