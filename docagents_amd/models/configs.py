@@ -206,8 +206,8 @@ DECODERS = {
     "tiny-dec-tp8": DecoderConfig("tiny-dec-tp8", vocab=32064, hidden=1024, layers=2, heads=16, kv_heads=8,
                                   ffn=1024, max_pos=4096, rope_theta=500000.0),
     # Binupel at Llama-3-8B's width, feed-forward, attention shape and vocabulary (8 x [recurrence,
-    # attention, 2 x scan]: 8.0 G parameters), and a miniature
-    "binupel-8b": _binupel("binupel-8b", 4096, 14336, 128256, 8, GatedRecurrence(4096, 16, 4),
+    # attention, 2 x scan]: 9.1 G parameters), and a miniature
+    "binupel-9b": _binupel("binupel-9b", 4096, 14336, 128256, 8, GatedRecurrence(4096, 16, 4),
                            SigmoidAttention(32, 8, 128, 128 ** -0.5, (0.1, 8192)), SelectiveScan(8192, 16, 256, 4)),
     "tiny-binupel": _binupel("tiny-binupel", 256, 512, 32064, 1, GatedRecurrence(320, 5, 4),
                              SigmoidAttention(8, 2, 32, 32 ** -0.5, (0.1, 64)), SelectiveScan(448, 16, 24, 4)),

@@ -1,0 +1,632 @@
+"""The Binupel decoder against its plain implementation (tests/binupel_oracle.py): each mechanism alone, whole
+models, portions of prompts, batches, slots and pages that change hands, and generation through the
+framework's generator, scheduler and engine."""
+import json
+import math
+
+import numpy as np
+import pytest
+import torch
+
+import binupel_oracle as oracle
+from binupel_cases import (CONFIGS, CPU, GPU16, GPU32, TOL, WHERE, att, build, check, checkpoint, config, expect, rec,
+                           row_errors, run, tokens, weights)
+from docagents_amd.engine.generator import ContinuousScheduler, Generator
+from docagents_amd.engine.replay import replay
+from docagents_amd.models import make_decoder
+from docagents_amd.models.checkpoint import load_weights, read_safetensors
+from docagents_amd.models.configs import DECODERS, HybridConfig, binupel_config, checkpoint_config, decoder_config
+from docagents_amd.models.state import LayerState, StateCache
+from docagents_amd.ops import get_ops
+from docagents_amd.ops.seq_batch import PAGE, pack_batch
+
+@pytest.fixture(autouse=True, scope="module")
+def one_thread():
+    """The plain implementation's many tiny operations run faster without a thread pool."""
+    n = torch.get_num_threads()
+    torch.set_num_threads(1)
+    yield
+    torch.set_num_threads(n)
+
+
+ACT = {"fp32": torch.float32, "bf16": torch.bfloat16}
+
+
+def close(got, want, dtype, scale=1.0):
+    got, want = got.double().cpu(), want.double()
+    tol = {"fp32": 2e-5, "bf16": 1.5e-2}[dtype] * scale
+    err = (got - want).abs().max() / want.abs().max()
+    assert err < tol, f"off by {float(err):.3g} of the largest value"
+
+
+def rand(seed, *shape, std=1.0):
+    return std * torch.randn(shape, generator=torch.Generator().manual_seed(seed))
+
+
+class Portions:
+    """Three sequences of unequal lengths, fed to an op in portions; want() is the oracle's whole sequences."""
+
+    def __init__(self, device, dtype, lens=(150, 3, 70), cuts=((2, 64, 70, 1, 13), (1, 2), (66, 1, 3))):
+        self.device, self.act, self.lens, self.cuts = device, ACT[dtype], lens, cuts
+        self.slots = [2, 0, 3]
+
+    def __iter__(self):
+        """(batch, rows of every sequence in it as (sequence, first, last))"""
+        at = [0] * len(self.lens)
+        for k in range(max(len(c) for c in self.cuts)):
+            ids = [i for i, c in enumerate(self.cuts) if k < len(c)]
+            n = [self.cuts[i][k] for i in ids]
+            m, _ = pack_batch(n, [self.slots[i] for i in ids], [at[i] for i in ids], self.device)
+            spans = [(i, at[i], at[i] + c) for i, c in zip(ids, n)]
+            for i, c in zip(ids, n):
+                at[i] += c
+            yield m, spans
+
+    def pack(self, seqs, spans):
+        return torch.cat([seqs[i][a:b] for i, a, b in spans]).to(self.device, self.act).contiguous()
+
+    def stored(self, seqs):
+        """What an op sees of values kept in the activation type."""
+        return [s.to(self.act).double() for s in seqs]
+
+    def state(self, *shape, dtype=None):
+        """Slots that hold another sequence's leftovers."""
+        return torch.full((4, *shape), 7.0, dtype=dtype or torch.float32, device=self.device)
+
+
+# ---------------------------------------------------------------------------------- mechanisms alone
+@pytest.mark.parametrize("device,dtype", WHERE)
+def test_stream_norm_and_token_shift(device, dtype):
+    P = Portions(device, dtype)
+    dim, Dp, alpha, eps = 90, 128, 1.3, 0.02
+    pad = lambda t: torch.nn.functional.pad(t, (0, Dp - dim))  # noqa: E731
+    xs, ys = [rand(1 + i, n, dim) for i, n in enumerate(P.lens)], [rand(11 + i, n, dim) for i, n in enumerate(P.lens)]
+    w, mu = rand(5, dim), rand(6, dim)
+    prev, save = P.state(Dp), P.state(Dp)
+    to = lambda t: pad(t).float().to(device).contiguous()  # noqa: E731
+    ops = get_ops(device)
+    for m, spans in P:
+        x = torch.cat([xs[i][a:b] for i, a, b in spans])
+        y = P.pack([pad(s) for s in ys], spans)
+        got_x, h = ops.stream_step(m, dim, eps=eps, alpha=alpha, x=to(x), y=y, w=to(w), mu=to(mu), prev=prev, save=save,
+                                   act=P.act)
+        row = 0
+        for i, a, b in spans:
+            full = oracle.rms(alpha * xs[i].double() + P.stored(ys)[i], w.double(), eps)
+            close(got_x[row:row + b - a, :dim], full[a:b], "fp32")
+            assert not got_x[row:row + b - a, dim:].any()
+            close(h[row:row + b - a, :dim], oracle.token_shift(full, mu.double())[a:b], dtype)
+            assert torch.equal(save[P.slots[i], :dim].cpu(), xs[i][b - 1])
+            prev[P.slots[i], :dim] = full[b - 1].float().to(device)  # what the next norm would save
+            prev[P.slots[i], dim:] = 0
+            row += b - a
+
+
+@pytest.mark.parametrize("taps", [1, 2, 3, 4, 7])
+@pytest.mark.parametrize("device,dtype", WHERE)
+def test_causal_conv(device, dtype, taps):
+    P = Portions(device, dtype)
+    C, ops = 68, get_ops(device)
+    xs, w, b = [rand(i, n, C) for i, n in enumerate(P.lens)], rand(8, taps, C), rand(9, C)
+    state = P.state(taps - 1, C, dtype=P.act)
+    f = lambda t: t.float().to(device).contiguous()  # noqa: E731
+    for silu in (False, True):
+        state.fill_(7.0)
+        for m, spans in P:
+            x = P.pack(xs, spans)
+            got = ops.causal_conv(x, f(w), f(b), state, m, silu)
+            # a recurrence that decays at once (and so outputs nothing) keeps the convolution's inputs
+            zero = torch.zeros(m.T, C, device=device)
+            ops.gated_scan(zero, zero, x, torch.zeros(4, C, device=device), x, state, m)
+            row = 0
+            for i, a, e in spans:
+                want = oracle.causal_conv(P.stored(xs)[i], w.double().t(), b.double())
+                want = want * torch.sigmoid(want) if silu else want
+                close(got[row:row + e - a], want[a:e], dtype)
+                row += e - a
+
+
+@pytest.mark.parametrize("blocks,bw", [(1, 64), (5, 16), (2, 96)])
+@pytest.mark.parametrize("device,dtype", WHERE)
+def test_gated_recurrence(device, dtype, blocks, bw):
+    """Gates and scan; one channel forgets at once, one almost never (a = exp(-1e-3) at an open gate)."""
+    P = Portions(device, dtype)
+    C, ops = blocks * bw, get_ops(device)
+    us, gs = [rand(i, n, C) for i, n in enumerate(P.lens)], [rand(20 + i, n, C) for i, n in enumerate(P.lens)]
+    q = lambda t: t.to(P.act).double()  # noqa: E731
+    w = {"ra": q(rand(3, blocks, bw, bw, std=bw ** -0.5)), "ri": q(rand(4, blocks, bw, bw, std=bw ** -0.5)),
+         "ra.b": rand(5, blocks, bw).double(), "ri.b": rand(6, blocks, bw).double()}
+    lam = rand(7, C).double() - 2
+    lam[0], lam[-1] = 9.0, -9.0
+    inter = lambda a, b, *s: torch.stack([a.reshape(blocks, bw // 16, 16, *s), b.reshape(blocks, bw // 16, 16, *s)], 2)  # noqa: E731
+    gw = inter(w["ra"], w["ri"], bw).reshape(blocks, 2 * bw, bw).to(device, P.act).contiguous()
+    gb = inter(w["ra.b"], w["ri.b"]).reshape(blocks, 2 * bw).float().to(device).contiguous()
+    state, conv = P.state(C), P.state(0, C, dtype=P.act)
+    for m, spans in P:
+        u, g = P.pack(us, spans), P.pack(gs, spans)
+        decay, drive = ops.rglru_gates(u, gw, gb, (-8 * oracle.softplus(lam)).float().to(device))
+        got = ops.gated_scan(decay, drive, g, state, g, conv, m)
+        row = 0
+        for i, a, b in spans:
+            uu = P.stored(us)[i]
+            r, gi = oracle.rglru_gates(uu, w, "", blocks)
+            s = oracle.rglru_scan(uu, r, gi, lam)
+            close(got[row:row + b - a], (s * oracle.gelu_tanh(P.stored(gs)[i]))[a:b], dtype)
+            close(state[P.slots[i]], s[b - 1], "fp32", 3)
+            row += b - a
+
+
+@pytest.mark.parametrize("N", [1, 4, 8, 16, 20, 33, 64])
+@pytest.mark.parametrize("device,dtype", WHERE)
+def test_selective_scan(device, dtype, N):
+    P = Portions(device, dtype)
+    C, ops = 68, get_ops(device)
+    off_b, off_c, ld = 3, 3 + N, 8 * math.ceil((3 + 2 * N) / 8)
+    xs, zs, dts = [[rand(10 * k + i, n, C) for i, n in enumerate(P.lens)] for k in range(3)]
+    bcs = [rand(50 + i, n, ld) for i, n in enumerate(P.lens)]
+    dts = [0.3 * d.abs() for d in dts]
+    A, D = -torch.exp(rand(60, C, N)).double(), rand(61, C).double()
+    A[0] = -30.0      # forgets within a token
+    A[-1] = -1e-3     # remembers everything
+    state, conv = P.state(C, N), P.state(0, C, dtype=P.act)
+    f = lambda t: t.float().to(device).contiguous()  # noqa: E731
+    for m, spans in P:
+        x, z, bc = P.pack(xs, spans), P.pack(zs, spans), P.pack(bcs, spans)
+        dt = f(torch.cat([dts[i][a:b] for i, a, b in spans]))
+        got = ops.selective_scan(x, dt, bc, off_b, off_c, z, f(A * math.log2(math.e)), f(D), state, x, conv, m)
+        row = 0
+        for i, a, b in spans:
+            bc64 = P.stored(bcs)[i]
+            y = oracle.mamba1_scan(P.stored(xs)[i], dts[i].double(), bc64[:, off_b:off_b + N], bc64[:, off_c:off_c + N], A, D)
+            zz = P.stored(zs)[i]
+            close(got[row:row + b - a], (y * zz * torch.sigmoid(zz))[a:b], dtype)
+            row += b - a
+
+
+@pytest.mark.parametrize("epi", [0, 1, 2])
+@pytest.mark.parametrize("M,N,K", [(1, 32, 64), (3, 96, 40), (70, 160, 264), (200, 64, 16)])
+@pytest.mark.parametrize("device,dtype", WHERE)
+def test_product_of_any_size_keeps_fp32(device, dtype, M, N, K, epi):
+    a, w, b = rand(1, M, K).to(ACT[dtype]), rand(2, N, K, std=K ** -0.5).to(ACT[dtype]), rand(3, N)
+    y = a.double() @ w.double().t() + b.double()
+    if epi == 1:
+        y = oracle.softplus(y)
+    elif epi == 2:
+        yy = y.view(M, N // 32, 2, 16)
+        y = (torch.relu(yy[:, :, 0]) * yy[:, :, 1]).reshape(M, N // 2)
+    close(get_ops(device).gemm_any(a.to(device), w.to(device), b.to(device), epi), y, "fp32")
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("M", [1, 5, 40, 100, 300, 700])
+@pytest.mark.parametrize("N,K", [(512, 512), (96, 192)])
+def test_relu_gated_epilogue_of_every_product_route(M, N, K):
+    a, w = rand(1, M, K).bfloat16(), rand(2, N, K, std=K ** -0.5).bfloat16()
+    yy = (a.double() @ w.double().t()).view(M, N // 32, 2, 16)
+    want = (torch.relu(yy[:, :, 0]) * yy[:, :, 1]).reshape(M, N // 2)
+    close(get_ops("cuda").gemm(a.cuda(), w.cuda(), epi=7), want, "bf16")
+
+
+def paged(device, act, slots, pages, G, D, seed=0):
+    """(keys, 1 / rms, table) of a pool with shuffled pages full of leftovers."""
+    order = np.random.default_rng(seed).permutation(slots * pages).reshape(slots, pages).astype(np.int32)
+    kc = torch.full((slots * pages, G, PAGE, D), 5.0, dtype=act, device=device)
+    kr = torch.full((slots * pages, G, PAGE), 3.0, device=device)
+    return kc, kr, torch.from_numpy(order).to(device)
+
+
+def attend(ops, device, act, seqs, spans_by_step, H, G, dim, D, scale, eps, pb, qn, kn, temp, slots=4):
+    """Feed (q, k, gate) sequences in portions; rows per sequence in order."""
+    pages = max(-(-len(s[0]) // PAGE) for s in seqs)
+    kc, kr, table = paged(device, act, slots, pages, G, D)
+    out = [[] for _ in seqs]
+    padh = lambda t: torch.nn.functional.pad(t, (0, D - dim)).flatten(1)  # noqa: E731
+    qk_w = torch.nn.functional.pad(qn * kn, (0, D - dim)).float().to(device)
+    for spans in spans_by_step:
+        m, _ = pack_batch([b - a for _, a, b in spans], [i for i, _, _ in spans], [a for _, a, _ in spans], device)
+        rows = torch.cat([torch.cat([padh(seqs[i][0][a:b]), padh(seqs[i][1][a:b]), seqs[i][2][a:b]], 1) for i, a, b in spans])
+        rows = torch.nn.functional.pad(rows, (0, -rows.shape[1] % 8)).to(device, act).contiguous()
+        y = ops.sigmoid_attn(rows, kc, kr, pb.float().to(device), qk_w, m.on(table), H, G, dim, scale, eps, temp)
+        y = y.float().cpu().view(-1, H, D)
+        assert not y[:, :, dim:].any()
+        row = 0
+        for i, a, b in spans:
+            out[i].append(y[row:row + b - a, :, :dim])
+            row += b - a
+    return [torch.cat(o) for o in out]
+
+
+def attend_oracle(q, k, gate, H, G, dim, scale, eps, pb, qn, kn, temp):
+    q, k, gate = q.double(), k.double(), gate.double()
+    t = oracle.query_temperature(range(len(q)), None if temp is None else {"coef": temp[0], "every": temp[1]})
+    o = oracle.sigmoid_attention(oracle.rms(q, qn.double(), eps) * t[:, None, None], oracle.rms(k, kn.double(), eps), k,
+                                 scale, pb.double())
+    return o * torch.sigmoid(gate)[:, :, None]
+
+
+@pytest.mark.parametrize("H,G,dim,D", [(4, 2, 32, 32), (2, 2, 50, 64), (6, 1, 96, 96), (20, 1, 128, 128), (3, 3, 180, 192),
+                                       (4, 1, 256, 256), (2, 1, 290, 320)])
+@pytest.mark.parametrize("device,dtype", WHERE)
+def test_sigmoid_attention(device, dtype, H, G, dim, D):
+    act = ACT[dtype]
+    lens = (200, 7, 131)
+    seqs = [tuple(t.to(act) for t in (rand(i, n, H, dim), 2 * rand(10 + i, n, G, dim), rand(20 + i, n, H)))
+            for i, n in enumerate(lens)]
+    pb, qn, kn = rand(31, H) - 2, 1 + 0.3 * rand(32, dim), 1 + 0.3 * rand(33, dim)
+    kw = dict(H=H, G=G, dim=dim, scale=1.3 * dim ** -0.5, eps=1e-3, pb=pb, qn=qn, kn=kn, temp=(0.7, 30))
+    steps = [[(0, 0, 63), (1, 0, 1), (2, 0, 131)], [(0, 63, 66), (1, 1, 7)], [(0, 66, 198)], [(0, 198, 199)], [(0, 199, 200)]]
+    got = attend(get_ops(device), device, act, seqs, steps, D=D, **kw)
+    for s, g in zip(seqs, got):
+        close(g, attend_oracle(*s, **kw), dtype)
+
+
+@pytest.mark.parametrize("device,dtype", WHERE)
+@pytest.mark.parametrize("decoded", [False, True])
+def test_one_key_stands_out(device, dtype, decoded):
+    """Queries aligned with one key each (the first tokens, page borders, their own place, far away), a bias
+    under which no other key counts: the output is that key, times the gate."""
+    act, H, G, dim, n = ACT[dtype], 2, 1, 64, 400
+    pairs = {399: 0, 398: 1, 397: 63, 396: 64, 395: 127, 394: 128, 393: 393, 392: 391, 391: 319, 320: 320, 319: 0, 64: 63,
+             63: 63, 127: 64, 128: 0, 192: 191, 0: 0, 1: 0}
+    k = rand(2, n, G, dim)
+    q = rand(3, n, H, dim)
+    for i, j in pairs.items():
+        q[i] = k[j] * torch.tensor([[2.0], [0.5]])
+    q, k, gate = q.to(act), k.to(act), rand(4, n, H).to(act)
+    kw = dict(H=H, G=G, dim=dim, scale=0.6, eps=1e-6, pb=torch.tensor([-24.0, -23.0]), qn=torch.ones(dim),
+              kn=torch.ones(dim), temp=None)
+    cut = [0, *range(380, n + 1)] if decoded else [0, n]
+    steps = [[(0, a, b)] for a, b in zip(cut, cut[1:])]
+    got, = attend(get_ops(device), device, act, [(q, k, gate)], steps, D=64, **kw)
+    close(got, attend_oracle(q, k, gate, **kw), dtype)
+    for i, j in pairs.items():
+        want = k[j].float() * torch.sigmoid(gate[i].float())[:, None]
+        assert (got[i] - want).abs().max() < 0.03 * want.abs().max() + 0.02, (i, j)
+
+
+@pytest.mark.parametrize("every", [1, 7, 64, 2.5])
+def test_query_temperature_steps(every):
+    """A weight of the temperature's steps alone: one key, whose score is scale * temp * dim."""
+    n, dim = 140, 32
+    k = torch.ones(n, 1, dim)
+    kw = dict(H=1, G=1, dim=dim, scale=0.01, eps=0.0, pb=torch.zeros(1), qn=torch.ones(dim), kn=torch.ones(dim),
+              temp=(0.9, every))
+    got, = attend(get_ops("cpu"), "cpu", torch.float32, [(k.clone(), k, torch.zeros(n, 1))], [[(0, 0, n)]], D=32, **kw)
+    t = [1 + 0.9 * math.log(math.floor((p + 1) / every) + 1) for p in range(n)]
+    want = [0.5 * (p + 1) / (1 + math.exp(-0.32 * t[p])) for p in range(n)]
+    assert np.allclose(got[:, 0, 0].numpy(), want, rtol=1e-5)
+
+
+# ---------------------------------------------------------------------------------- whole models
+@pytest.mark.parametrize("device,dtype", WHERE)
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_prompts_and_layers(tmp_path, name, device, dtype):
+    model, cfg, w = build(tmp_path, name, device, dtype, seed=1)
+    req = {n: tokens(cfg, n, n) for n in (1, 2, 65, 150)}
+    got = run(model, req, [[(n, n)] for n in req])
+    for n in req:
+        check(got[n], expect(cfg, w, req[n]), dtype, f"{name}: prompt of {n}")
+
+
+@pytest.mark.parametrize("device,dtype", WHERE)
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+@pytest.mark.parametrize("cuts", [(2,), (3, 64, 1, 29), (64, 65, 1), (63, 1, 2, 1, 130)])
+def test_portions_equal_the_whole(tmp_path, name, device, dtype, cuts):
+    model, cfg, w = build(tmp_path, name, device, dtype, seed=2)
+    n = 40 if cuts == (2,) else 197
+    req = {"a": tokens(cfg, n, 5)}
+    sched, left, k = [], n, 0
+    while left:
+        c = min(left, cuts[k % len(cuts)])
+        sched.append([("a", c)])
+        left, k = left - c, k + 1
+    got = run(model, req, sched)["a"]
+    check(got, expect(cfg, w, req["a"]), dtype, f"{name} in {cuts}")
+
+
+@pytest.mark.parametrize("device,dtype", WHERE)
+@pytest.mark.parametrize("name", ["odd", "wide"])
+def test_token_by_token_equals_the_prompt(tmp_path, name, device, dtype):
+    model, cfg, w = build(tmp_path, name, device, dtype, seed=3)
+    req = {"a": tokens(cfg, 140, 6)}
+    check(run(model, req, [[("a", 1)]] * 140)["a"], expect(cfg, w, req["a"]), dtype, name)
+
+
+def mixed_schedule(lens, seed):
+    """Up to four live requests a step, portions of 2..70 beside single tokens, requests left out of steps."""
+    rng = np.random.default_rng(seed)
+    left, live, todo, sched = dict(lens), [], list(lens), []
+    while todo or live:
+        while len(live) < 4 and todo and (not live or rng.random() < 0.6):
+            live.append(todo.pop(0))
+        step = []
+        for i in live:
+            if rng.random() < 0.8:
+                c = min(left[i], 1 if rng.random() < 0.5 else int(rng.integers(2, 70)))
+                step.append((i, c))
+                left[i] -= c
+        live = [i for i in live if left[i]]
+        if step:
+            sched.append(step)
+    return sched
+
+
+@pytest.mark.parametrize("device,dtype", WHERE)
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_mixed_batches_reuse_slots_and_pages(tmp_path, name, device, dtype):
+    """Nine requests through four slots and a pool that could not hold them all: every position equals the
+    request alone."""
+    model, cfg, w = build(tmp_path, name, device, dtype, seed=4)
+    lens = {f"r{i}": n for i, n in enumerate((130, 5, 66, 1, 200, 64, 31, 90, 128))}
+    req = {i: tokens(cfg, n, 50 + n) for i, n in lens.items()}
+    got = run(model, req, mixed_schedule(lens, 7), max_seq=256, pool=4 * 200 + 64)
+    for i in req:
+        check(got[i], expect(cfg, w, req[i]), dtype, f"{name}: {i} of {lens[i]} tokens")
+
+
+@pytest.mark.parametrize("device,dtype", [CPU, GPU32, GPU16])
+def test_long_decoding_across_pages(tmp_path, device, dtype):
+    model, cfg, w = build(tmp_path, "odd", device, dtype, seed=5)
+    req = {"a": tokens(cfg, 330, 8), "b": tokens(cfg, 300, 9)}
+    sched = [[("a", 60), ("b", 31)]] + [[("a", 1), ("b", 1)]] * 269 + [[("a", 1)]]
+    got = run(model, req, sched)
+    for i in req:
+        check(got[i], expect(cfg, w, req[i]), dtype, i)
+
+
+@pytest.mark.parametrize("device,dtype", WHERE)
+def test_a_slots_earlier_owner_leaves_no_trace(tmp_path, device, dtype):
+    """The same request before and after others used its slot and pages: equal to the last bit."""
+    model, cfg, _ = build(tmp_path, "odd", device, dtype, seed=6)
+    a, b = tokens(cfg, 90, 1), tokens(cfg, 90, 2)
+    got = run(model, {"a": a, "b": b, "c": a}, [[("a", 90)], [("b", 90)], [("c", 90)]], slots=1)
+    assert torch.equal(got["a"], got["c"]) and not torch.equal(got["a"], got["b"])
+
+
+def test_layers_that_share_weights_keep_states_of_their_own(tmp_path):
+    model, cfg, w = build(tmp_path, "ones", "cpu", "fp32", seed=7)
+    plain = json.loads(json.dumps(cfg))
+    pw = dict(w)
+    for i, layer in enumerate(plain["layers"]):
+        j = layer.pop("weights_of", None)
+        if j is not None:
+            pw.update({f"l{i}{k[len(f'l{j}'):]}": v for k, v in w.items() if k.startswith(f"l{j}.")})
+    t = tokens(cfg, 70, 3)
+    assert torch.equal(expect(cfg, w, t), expect(plain, pw, t))
+    check(run(model, {"a": t}, [[("a", 33)], [("a", 37)]])["a"], expect(plain, pw, t), "fp32")
+
+
+# ---------------------------------------------------------------------------------- generation
+def greedy(cfg, w, prompt, n):
+    t = list(prompt)
+    for _ in range(n):
+        t.append(int(oracle.forward(cfg, w, t)[0][-1].argmax()))
+    return t[len(prompt):]
+
+
+def sharp(w):
+    w["head"] = w["head"] * 4  # far from ties
+
+
+@pytest.mark.parametrize("device,dtype", [CPU, GPU32])
+def test_greedy_generation_through_generator_and_scheduler(tmp_path, device, dtype):
+    """Generator waves and the continuous scheduler (its graphs on the GPU), both on a cache too small for all
+    requests at once, produce the plain implementation's tokens."""
+    model, cfg, w = build(tmp_path, "odd", device, dtype, seed=8, edit=sharp)
+    prompts = [tokens(cfg, n, 70 + n) for n in (3, 40, 70, 1, 66, 12, 29)]
+    want = [greedy(cfg, w, p, 9) for p in prompts]
+    model.alloc_cache(6, 128, tokens=6 * 64)
+    g = Generator(model, max_batch=4, max_seq=128, temperature=0.0)
+    assert [r.tokens for r in g.generate(prompts, 9)] == want
+    sch = ContinuousScheduler(g, B=4, max_new_cap=16, chunk_steps=3)
+    assert [r.tokens for r in sch.run_all(prompts, 9)] == want
+    assert sch.run_all(prompts[:1], 4)[0].tokens == want[0][:4]
+    g.close()
+    assert len(model.cache.free) == 6 and len(model.cache.free_pages) == model.cache.pages
+
+
+@pytest.mark.gpu
+def test_decode_graphs_replay_the_eager_steps(tmp_path):
+    """bf16: captured decode steps against eager ones over several waves with eager work in between."""
+    model, cfg, _ = build(tmp_path, "wide", "cuda", "bf16", seed=9, edit=sharp)
+    model.alloc_cache(10, 256)
+    eager = Generator(model, max_batch=4, max_seq=256, temperature=0.0, use_graphs=False)
+    graph = Generator(model, max_batch=4, max_seq=256, temperature=0.0, use_graphs=True)
+    for wave in range(3):
+        prompts = [tokens(cfg, n, 90 + n + wave) for n in (5, 80, 17, 64)]
+        a = [r.tokens for r in eager.generate(prompts, 20)]
+        torch.cuda.synchronize()
+        assert a == [r.tokens for r in graph.generate(prompts, 20)]
+
+
+def test_scheduler_admits_what_the_pool_holds(tmp_path):
+    model, cfg, _ = build(tmp_path, "ones", "cpu", "fp32", seed=10)
+    model.alloc_cache(9, 256, tokens=5 * 64)  # the spare slot's page and four more
+    g = Generator(model, max_batch=8, max_seq=256, temperature=0.0)
+    sch = ContinuousScheduler(g, B=8, max_new_cap=8)
+    with pytest.raises(ValueError, match="exceeds the context"):
+        sch.submit(tokens(cfg, 400, 0), 8)
+    for n in (100, 100, 20):
+        sch.submit(tokens(cfg, n, n), 8, n)
+    sch.tick(steps=1)
+    assert sch.n_active == 2 and len(sch.pending) == 1
+    done = {}
+    while sch.busy():
+        done.update(sch.tick())
+    assert sorted(done) == [20, 100] and len(model.cache.free_pages) == 4
+
+
+def test_engine_serves_a_preset_and_a_checkpoint(tmp_path):
+    from docagents_amd.engine.engine import Engine
+    e = Engine("tiny-enc", "tiny-binupel", "cpu", max_batch=4, max_seq=512, max_new_tokens=4, summary_max_new=4,
+               use_graphs=False)
+    assert isinstance(e.dec_cfg, HybridConfig) and e.describe()["decoder"] == "tiny-binupel"
+    (text, conf), = e.answer_many([("q?", [[10, 11, 12]], 0.9)], 4)
+    assert isinstance(text, str) and 0 < conf <= 0.9
+    out, busy = e.cb_tick([(1, ("q?", [[10, 11, 12]], 0.9))])
+    while busy:
+        o, busy = e.cb_tick([])
+        out += o
+    assert out[0][1] == text  # the scheduler and the wave path agree
+    assert e.auto_batch(512, kv_gb=36 * e.decoder.cache_bytes(1, 512) / 1e9) == 32
+    cfg = config(64, 1000, [(att(2, 1, 32), 64), (rec(64, 2, 4), 64)])
+    path = checkpoint(tmp_path, cfg, weights(cfg, 3))
+    e = Engine("tiny-enc", path, "cpu", max_batch=2, max_seq=256, max_new_tokens=4, use_graphs=False, llm_dtype="fp32")
+    r, = e.gen.generate([[5, 6, 7]], 4)
+    assert r.n_tokens >= 1
+    from docagents_amd.config import Config
+    with pytest.raises(ValueError, match="LLM_DTYPE"):
+        Config(llm_dtype="fp64").validate_engine()
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["bf16", "fp32"])
+def test_engine_on_the_gpu(dtype):
+    from docagents_amd.engine.engine import Engine
+    e = Engine("tiny-enc", "tiny-binupel", "cuda", max_batch=4, max_seq=512, max_new_tokens=8, summary_max_new=8,
+               temperature=0.0, llm_dtype=dtype)
+    items = [(f"question {i}?", [list(range(10, 30 + 40 * i))], 0.9) for i in range(6)]
+    wave = e.answer_many(items, 8)
+    out, busy = e.cb_tick(list(enumerate(items)))
+    while busy:
+        o, busy = e.cb_tick([])
+        out += o
+    if dtype == "fp32":  # bf16: another batch size is another product kernel, near-ties may fall differently
+        assert [t for _, t, _ in sorted(out)] == [t for t, _ in wave]
+    assert len(out) == 6
+
+
+# ---------------------------------------------------------------------------------- replay
+def test_trace_replay_writes_the_wanted_rows(tmp_path):
+    model, cfg, w = build(tmp_path, "odd", "cpu", "fp32", seed=11)
+    a, b = tokens(cfg, 80, 1), tokens(cfg, 9, 2)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:70], "want": [0, 69]}, {"id": "b", "tokens": b, "want": [8]}],
+              "end": ["b"]},
+             {"step": 1, "entries": [{"id": "a", "tokens": a[70:71], "want": []}], "end": []},
+             {"step": 2, "entries": [{"id": "a", "tokens": a[71:], "want": [8]}], "end": ["a"]}]
+    done = []
+    replay(model, 192, [json.dumps(s) for s in steps], str(tmp_path), done.append)
+    assert done == [0, 1, 2] and not (tmp_path / "1.f32").exists()
+    ea, eb = expect(cfg, w, a), expect(cfg, w, b)
+    read = lambda n: torch.from_numpy(np.fromfile(tmp_path / f"{n}.f32", dtype="<f4")).view(-1, cfg["vocab"])  # noqa: E731
+    check(read(0), torch.stack([ea[0], ea[69], eb[8]]), "fp32")
+    check(read(2), ea[79:], "fp32")
+    for bad in ([{"id": "x", "tokens": [cfg["vocab"]], "want": []}], [{"id": "x", "tokens": [1], "want": [1]}],
+                [{"id": "x", "tokens": [], "want": []}]):
+        with pytest.raises(ValueError):
+            replay(model, 192, [json.dumps({"step": 0, "entries": bad, "end": []})], str(tmp_path), done.append)
+
+
+@pytest.mark.gpu
+def test_trace_command(tmp_path):
+    import os
+    import subprocess
+    import sys
+    cfg = CONFIGS["wide"]
+    w = weights(cfg, 12)
+    (tmp_path / "m").mkdir(), (tmp_path / "o").mkdir()
+    t = tokens(cfg, 100, 4)
+    steps = [{"step": 0, "entries": [{"id": "q", "tokens": t[:97], "want": [96]}], "end": []},
+             {"step": 1, "entries": [{"id": "q", "tokens": t[97:98], "want": [0]}], "end": []},
+             {"step": 2, "entries": [{"id": "q", "tokens": t[98:], "want": [1]}], "end": ["q"]}]
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    r = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model",
+                        checkpoint(tmp_path / "m", cfg, w), "--dtype", "float32", "--out", str(tmp_path / "o"),
+                        "--max-tokens", "100"], input="".join(json.dumps(s) + "\n" for s in steps), text=True,
+                       capture_output=True, timeout=100)
+    assert r.returncode == 0 and r.stdout.split() == "done 0 done 1 done 2".split(), r.stderr[-2000:]
+    got = torch.cat([torch.from_numpy(np.fromfile(tmp_path / "o" / f"{n}.f32", dtype="<f4")).view(1, -1) for n in range(3)])
+    check(got, expect(cfg, w, t)[[96, 97, 99]], "fp32")
+
+
+# ---------------------------------------------------------------------------------- configuration, loading, state
+def test_registry_and_configuration(tmp_path):
+    assert isinstance(decoder_config("binupel-9b"), HybridConfig)
+    assert 9.0e9 < DECODERS["binupel-9b"].param_count() < 9.2e9
+    cfg = CONFIGS["odd"]
+    c = decoder_config(checkpoint(tmp_path, cfg, weights(cfg)))
+    assert c.layers == 7 and c.spec[4].weights_of == 1 and c.spec[4].ff == 100 and c.spec[0].ff == 0
+    assert c.param_count() == sum(v.numel() for v in weights(cfg).values())
+    assert c.kv_bytes_per_token() == 2 * 3 * (40 * 2 + 4)
+    edit = lambda **kw: {**json.loads(json.dumps(cfg)), **kw}  # noqa: E731
+    for change in (lambda c: c["layers"][0].update(type="rwkv"), lambda c: c["layers"][1]["mixer"].update(vdim=39),
+                   lambda c: c["layers"][1]["mlp"].update(kind="moe"), lambda c: c["layers"][4].update(weights_of=5),
+                   lambda c: c["layers"][4].update(mlp=None), lambda c: c["layers"][1]["mixer"].update(kv_heads=4)):
+        bad = edit()
+        change(bad)
+        with pytest.raises((ValueError, KeyError)):
+            binupel_config(bad, "bad")
+    (tmp_path / "config.json").write_text(json.dumps(edit(architecture="Unheard")))
+    with pytest.raises(ValueError, match="unknown architecture"):
+        checkpoint_config(str(tmp_path))
+    with pytest.raises(ValueError, match="unknown decoder arch"):
+        decoder_config(str(tmp_path / "missing"))
+    with pytest.raises(ValueError, match="not supported"):
+        make_decoder(decoder_config("tiny-dec"), "cpu", dtype="fp32")
+
+
+def test_checkpoint_reading(tmp_path):
+    from safetensors.torch import save_file
+    w = {"a": rand(1, 3, 5).bfloat16(), "b": rand(2, 7), "c": torch.arange(4, dtype=torch.int32)}
+    save_file(w, str(tmp_path / "x.safetensors"), metadata={"k": "v"})
+    got = load_weights(tmp_path)
+    assert set(got) == set(w) and all(torch.equal(got[k], w[k]) and got[k].dtype == w[k].dtype for k in w)
+    data = (tmp_path / "x.safetensors").read_bytes()
+    (tmp_path / "short.safetensors").write_bytes(data[:-1])
+    with pytest.raises(ValueError):
+        read_safetensors(tmp_path / "short.safetensors")
+    (tmp_path / "head.safetensors").write_bytes((1 << 40).to_bytes(8, "little") + b"{}")
+    with pytest.raises(ValueError):
+        read_safetensors(tmp_path / "head.safetensors")
+    cfg = CONFIGS["ones"]
+    w = weights(cfg)
+    w.pop("l1.mix.lam")
+    with pytest.raises(ValueError, match="l1.mix.lam"):
+        make_decoder(binupel_config(cfg, "x"), "cpu", weights=w)
+
+
+def test_state_cache_ownership():
+    spec = [LayerState({"s": ((3,), torch.float32)}, {"k": ((2, PAGE, 4), torch.bfloat16)})]
+    c = StateCache(spec, 3, 256, "cpu", tokens=6 * 64)
+    assert c.pages == 6 and c.layers[0]["s"].shape == (3, 3) and c.layers[0]["k"].shape == (6, 2, 64, 4)
+    assert StateCache.bytes_for(spec, 3, 256, 6 * 64) == 3 * 12 + 6 * 2 * 64 * 4 * 2
+    a, b = c.acquire(2, [65, 1])
+    assert len(c.owned[a]) == 2 and len(c.owned[b]) == 1 and c.table[a, :2].tolist() == c.owned[a]
+    assert not set(c.owned[a]) & set(c.owned[b])
+    assert c.fits([192]) and not c.fits([193]) and not c.fits([1, 1])
+    with pytest.raises(RuntimeError, match="exhausted"):
+        c.acquire(1, [256])
+    c.extend([b], [64])
+    assert len(c.owned[b]) == 1
+    c.extend([b], [256])
+    with pytest.raises(ValueError):
+        c.extend([a], [257])
+    with pytest.raises(RuntimeError, match="exhausted"):
+        c.extend([a], [192])
+    c.release([a])
+    assert c.fits([128]) and sorted(c.free_pages + c.owned[b]) == list(range(6))
+
+
+def test_batch_packing():
+    m, ids = pack_batch([1, 130, 64], [2, 0, 1], [9, 0, 5], "cpu", list(range(195)))
+    assert m.cu.tolist() == [0, 1, 131, 195] and (m.T, m.B, m.max_len, m.max_ctx, m.singles) == (195, 3, 130, 130, True)
+    assert m.ck.tolist() == [[0, 0], [1, 0], [1, 1], [1, 2], [2, 0]] and m.base.tolist() == [0, 1, 4]
+    assert ids.tolist() == list(range(195)) and m.seq.tolist() == [0] + [1] * 130 + [2] * 64
+    assert pack_batch([64, 2], [0, 1], [0, 0], "cpu")[0].n_chunks == 0
+    with pytest.raises(ValueError):
+        pack_batch([2, 0], [0, 1], [0, 0], "cpu")
+
+
+def test_a_wrong_mechanism_shows():
+    """The tolerance is sharp: small mistakes planted in the plain implementation exceed it by far."""
+    cfg = CONFIGS["odd"]
+    w = weights(cfg, 1)
+    t = tokens(cfg, 100, 1)
+    right = expect(cfg, w, t)
+    for name, edit in {"taps": lambda w: w.update({"l0.mix.conv": w["l0.mix.conv"].flip(1)}),
+                       "bias": lambda w: w.update({"l1.mix.pb": w["l1.mix.pb"] + 0.5}),
+                       "shift": lambda w: w.update({"l2.shift": w["l2.shift"] * 0}),
+                       "gates": lambda w: w.update({"l2.mix.ra": w["l2.mix.ri"], "l2.mix.ri": w["l2.mix.ra"]})}.items():
+        bad = dict(w)
+        edit(bad)
+        assert row_errors(expect(cfg, bad, t), right).max() > 3 * TOL["bf16"], name
