@@ -197,6 +197,12 @@ def main():
     ap.add_argument("--tp70b-batches", default="1,16", help="tp_decode_70b: decode batches timed")
     ap.add_argument("--tp70b-arch", default="llama3-70b",
                     help="tp_decode_70b's decoder (tests: a miniature of the same TP = 8 layout on CPU ranks)")
+    ap.add_argument("--decoders", default="",
+                    help="comma-separated decoder archs: instead of the QA workload, time their prefill and decode "
+                         "at full layer width side by side (bench/decoder_layers.py), one JSON line")
+    ap.add_argument("--decoder-prefills", default="1x2048,8x2048,1x8192", help="--decoders: prompts x tokens")
+    ap.add_argument("--decoder-rows", default="1,16,64", help="--decoders: decode batch sizes")
+    ap.add_argument("--decoder-context", type=int, default=2048, help="--decoders: tokens before the decoded ones")
     ap.add_argument("--block-budget-s", type=float, default=360.0,
                     help="N > 1: wall budget of each multi-GPU block; past it every rank ends the run and rank 0 "
                          "prints the JSON line with the blocks done so far (a hung collective cannot eat the headline)")
@@ -215,6 +221,19 @@ def main():
     dev = info.device
     if dev.type != "cuda" and not a.cpu_rehearsal:
         raise SystemExit("bench.py needs a GPU (run it through gpurun)")
+    if a.decoders:
+        sys.path.insert(0, os.path.join(os.path.dirname(os.path.abspath(__file__)), "bench"))
+        import decoder_layers
+        rows = []
+        for arch in a.decoders.split(","):
+            rows.append(decoder_layers.run(
+                arch, [tuple(map(int, p.split("x"))) for p in a.decoder_prefills.split(",")],
+                [int(b) for b in a.decoder_rows.split(",")], a.decoder_context, a.steps, a.warmup, a.seed))
+            log(info, json.dumps(rows[-1]))
+            torch.cuda.empty_cache()
+        print(json.dumps({"decoders": rows, "steps": a.steps, "warmup": a.warmup, "dtype": "bf16",
+                          "data": "synthetic, random-init weights"}), flush=True)
+        return
     sync = torch.cuda.synchronize if dev.type == "cuda" else (lambda: None)
     t_setup = time.perf_counter()
     TP = a.tp

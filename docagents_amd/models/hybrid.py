@@ -63,10 +63,13 @@ class Linear:
         self.bias = None if bias is None else bias.to(act).contiguous()
         self.gated = relu_gated
 
-    def __call__(self, x, out=None):
+    def __call__(self, x, out=None, partial: bool = False):
+        """partial: the consumer also takes fp32 split-K partials [splits, M, N]."""
         if self.act == torch.float32:
             y = self.ops.gemm_any(x, self.w, self.bias, ANY_REGLU if self.gated else ANY_NONE)
             return y if out is None else out.copy_(y)
+        if partial and self.ops.partials_fit(x.shape[0], *self.w.shape):
+            return self.ops.gemm_partials(x, self.w)
         epi = EPI_REGLU if self.gated else (EPI_NONE if self.bias is None else EPI_BIAS)
         return self.ops.gemm(x, self.w, bias=self.bias, epi=epi, out=out)
 
@@ -116,7 +119,7 @@ class RecurrenceMixer:
         gate, x = yx[:, :C], yx[:, C:]
         u = o.causal_conv(x, self.conv_w, self.conv_b, st["conv"], m, silu=False)
         decay, drive = o.rglru_gates(u, self.gate_w, self.gate_b, self.lam)
-        return self.out(o.gated_scan(decay, drive, gate, st["rec"], x, st["conv"], m))
+        return self.out(o.gated_scan(decay, drive, gate, st["rec"], x, st["conv"], m), partial=True)
 
 
 class AttentionMixer:
@@ -152,7 +155,7 @@ class AttentionMixer:
         s = self.s
         a = self.ops.sigmoid_attn(self.proj(h), st["k"], st["k_rms"], self.pb, self.qk_w, m, s.heads, s.kv_heads, s.dim,
                                   s.scale, self.eps, s.q_temp)
-        return self.out(a)
+        return self.out(a, partial=True)
 
 
 class ScanMixer:
@@ -191,7 +194,7 @@ class ScanMixer:
         low = self.low(xc)
         dt = o.gemm_any(low[:, :self.dt_k], self.dt_w, self.dt_b, ANY_SOFTPLUS)
         y = o.selective_scan(xc, dt, low, s.dt_rank, s.dt_rank + s.state, z, self.A, self.D, st["ssm"], x, st["conv"], m)
-        return self.out(y)
+        return self.out(y, partial=True)
 
 
 MIXERS = {GatedRecurrence: RecurrenceMixer, SigmoidAttention: AttentionMixer, SelectiveScan: ScanMixer}
@@ -335,7 +338,7 @@ class HybridDecoder:
             after = {} if L.gate_up else shift[i + 1]
             x, h = o.stream_step(m, c.hidden, x=x, y=y, w=L.norm1, save=st[i]["shift"], **after, **kw)
             if L.gate_up:
-                x, h = o.stream_step(m, c.hidden, x=x, y=L.down(L.gate_up(h)), w=L.norm2, **shift[i + 1], **kw)
+                x, h = o.stream_step(m, c.hidden, x=x, y=L.down(L.gate_up(h), partial=True), w=L.norm2, **shift[i + 1], **kw)
         return x
 
     def _logits(self, x, rows=None, out=None):

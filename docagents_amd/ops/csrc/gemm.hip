@@ -617,6 +617,23 @@ DA_EXPORT int da_gemm_dk_splitk(const void* A, int lda, const void* W, void* C, 
   DA_LAUNCH_CHECK();
 }
 
+// A . W^T left as `splits` fp32 partials [splits][M][N] in ws (splits = 1: the product itself) for a consumer
+// that sums them in its own pass. Decode-sized tiles: 2 = 64x128, 3 = 32x128, 9 = 128x64.
+DA_EXPORT int da_gemm_partials(const void* A, int lda, const void* W, int M, int N, int K, int tile, int splits,
+                               void* ws, void* stream) {
+  if (M < 1 || K % 64 || N % 8 || lda % 8 || splits < 1 || (K / 64) % splits || !ws) return (int)hipErrorInvalidValue;
+  GemmArgs a{};
+  a.A = (const bf16_t*)A; a.W = (const bf16_t*)W; a.ws = (float*)ws;
+  a.M = M; a.N = N; a.K = K; a.lda = lda; a.ldc = N; a.k_per_split = K / splits;
+  hipStream_t s = (hipStream_t)stream;
+  switch (tile) {
+    case 2: return launch_decode_tile<64, 128>(a, EPI_PARTIAL, splits, s);
+    case 3: return launch_decode_tile<32, 128>(a, EPI_PARTIAL, splits, s);
+    case 9: return launch_tile<128, 64, 2, 2, 4>(a, EPI_PARTIAL, splits, s);
+    default: return (int)hipErrorInvalidValue;
+  }
+}
+
 // Prefill QKV projection with RoPE + KV-cache write fused into the epilogue (gemm8p EPI_ROPE);
 // M >= 256 (the phase-split kernel), N == (H + 2 Hkv) * D, D % 8 == 0. kv_out = 0: the k / v
 // columns of C are left unwritten (cache only).

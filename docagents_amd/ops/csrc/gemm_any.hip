@@ -128,8 +128,8 @@ __global__ void __launch_bounds__(256) gemm_any_kernel(AnyArgs p) {
           const int ch = z * (p.N / 2) + col;
           const float la = p.lam[ch] * sigmoid32(x);  // log of the decay, <= 0
           const float u = Act<T>::to_f(((const T*)p.u)[(size_t)m * p.ldu + ch]);
-          p.decay[(size_t)m * p.ldg + ch] = expf(la);
-          p.drive[(size_t)m * p.ldg + ch] = sqrtf(-expm1f(2.f * la)) * sigmoid32(y) * u;
+          p.decay[(size_t)m * p.ldg + ch] = exp32(la);
+          p.drive[(size_t)m * p.ldg + ch] = __builtin_amdgcn_sqrtf(one_minus_exp32(2.f * la)) * sigmoid32(y) * u;
         }
       }
   } else {

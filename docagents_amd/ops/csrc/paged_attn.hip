@@ -41,37 +41,67 @@ struct PrepArgs {
   int dim;                      // columns a head really has
 };
 
-// One wave per (token, head): queries are normalised and scaled in place, keys go to their page.
-template <typename T>
-__global__ void __launch_bounds__(256) attn_prep_kernel(PrepArgs p) {
+// A head per group of `lanes` lanes (a power of two >= D / 8, at most a wave), 8 columns per lane and
+// step: queries are normalised and scaled in place, keys go to their page. STEPS * 8 * lanes >= D.
+template <typename T, int STEPS>
+__global__ void __launch_bounds__(256) attn_prep_kernel(PrepArgs p, int lanes) {
   const AttnArgs& a = p.a;
-  const int t = blockIdx.x, h = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (h >= a.H + a.G) return;
+  const int per = 256 / lanes, heads = a.H + a.G;
+  const int item = blockIdx.x * per + threadIdx.x / lanes, l = threadIdx.x % lanes;
+  const bool live = item < a.m.T * heads;
+  const int it = live ? item : a.m.T * heads - 1, t = it / heads, h = it % heads;
   const int b = a.m.seq[t], pos = a.m.pos0[b] + t - a.m.cu[b];
   T* row = (T*)a.qkg + (size_t)t * a.ld + (size_t)h * a.D;
+  f32x4_t v[STEPS][2];
   float ss = 0.f;
-  for (int d = lane * 2; d < a.D; d += 128) {
-    const f32x2_t v = Act<T>::load2(row + d);
-    ss = fmaf(v[0], v[0], fmaf(v[1], v[1], ss));
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i) {
+    const int d = (i * lanes + l) * 8;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      v[i][j] = d < a.D ? Act<T>::load4(row + d + 4 * j) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss = fmaf(v[i][j][e], v[i][j][e], ss);
+    }
   }
-  const float inv = 1.f / sqrtf(wave_sum(ss) / p.dim + p.eps);
+  for (int o = lanes >> 1; o > 0; o >>= 1) ss += __shfl_xor(ss, o, 64);
+  if (!live) return;
+  const float inv = 1.f / sqrtf(ss / p.dim + p.eps);
+  T* dst = row;
+  float f = 1.f;
   if (h < a.H) {
-    float f = inv * p.scale;
+    f = inv * p.scale;
     if (p.temp_every > 0.) f *= fmaf(p.temp_coef, logf((float)(floor((double)(pos + 1) / p.temp_every) + 1.)), 1.f);
-    for (int d = lane * 2; d < a.D; d += 128) {
-      const f32x2_t v = Act<T>::load2(row + d), w = Act<float>::load2(p.qk_w + d);
-      Act<T>::store2(row + d, v[0] * (f * w[0]), v[1] * (f * w[1]));
-    }
   } else {
-    const int pg = page_of(a, a.m.slot[b], pos / PAGE);
-    const size_t kr = ((size_t)pg * a.G + h - a.H) * PAGE + pos % PAGE;
-    T* dst = (T*)a.kc + kr * a.D;
-    for (int d = lane * 2; d < a.D; d += 128) {
-      const f32x2_t v = Act<T>::load2(row + d);
-      Act<T>::store2(dst + d, v[0], v[1]);
-    }
-    if (lane == 0) a.kr[kr] = inv;
+    const size_t kr = ((size_t)page_of(a, a.m.slot[b], pos / PAGE) * a.G + h - a.H) * PAGE + pos % PAGE;
+    dst = (T*)a.kc + kr * a.D;
+    if (l == 0) a.kr[kr] = inv;
   }
+#pragma unroll
+  for (int i = 0; i < STEPS; ++i) {
+    const int d = (i * lanes + l) * 8;
+    if (d >= a.D) continue;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      f32x4_t x = v[i][j];
+      if (h < a.H) {
+        const f32x4_t w = *(const f32x4_t*)(p.qk_w + d + 4 * j);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x[e] *= f * w[e];
+      }
+      Act<T>::store4(dst + d + 4 * j, x);
+    }
+  }
+}
+
+template <typename T>
+static void launch_prep(const PrepArgs& p, hipStream_t s) {
+  int lanes = 4;
+  while (lanes < 64 && lanes * 8 < p.a.D) lanes *= 2;
+  const int per = 256 / lanes;
+  const unsigned grid = ((size_t)p.a.m.T * (p.a.H + p.a.G) + per - 1) / per;
+  if (p.a.D <= lanes * 8) attn_prep_kernel<T, 1><<<grid, 256, 0, s>>>(p, lanes);
+  else attn_prep_kernel<T, 2><<<grid, 256, 0, s>>>(p, lanes);
 }
 
 // ------------------------------------------------------------------------------- any size, fp32 arithmetic
@@ -153,8 +183,6 @@ template <int D> struct MA {
 __device__ __forceinline__ unsigned split_lo(unsigned hi, float a, float b) {
   return pack_bf2(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
 }
-
-constexpr float LOG2E = 1.4426950408889634f;
 
 template <int D>
 __global__ void __launch_bounds__(256, D <= 128 ? 2 : 1) sigmoid_attn_kernel(AttnArgs a, int skip_single) {
@@ -484,7 +512,7 @@ DA_EXPORT int da_sigmoid_attn(void* qkg, int ld, void* kc, void* kr, const void*
                               double temp_every, int H, int G, int D, int dim, void* out, int ldo, void* part,
                               int nsplit, int pps, int max_len, int singles, const void* cu, const void* slot,
                               const void* pos0, const void* seq, int T, int B, int f32, void* stream) {
-  if (T < 1 || B < 1 || B > 65535 || G < 1 || H % G || D < 32 || D % 32 || D > 768 || dim < 1 || dim > D || ld % 8 ||
+  if (T < 1 || B < 1 || B > 65535 || G < 1 || H % G || D < 32 || D % 32 || D > 768 || (long long)T * (H + G) > 0x7fffffffll || dim < 1 || dim > D || ld % 8 ||
       ldo % 8 || max_pages < 1 || pages < 1 || max_len < 1 || nsplit < 1 || pps < 1 || (nsplit > 1 && !part))
     return (int)hipErrorInvalidValue;
   AttnArgs a{qkg, ld, kc, (float*)kr, (const int*)table, max_pages, pages, (const float*)pb, out, ldo, H, G, D,
@@ -492,12 +520,11 @@ DA_EXPORT int da_sigmoid_attn(void* qkg, int ld, void* kc, void* kr, const void*
              pps};
   PrepArgs p{a, (const float*)qk_w, scale, eps, temp_coef, temp_every, dim};
   hipStream_t s = (hipStream_t)stream;
-  const dim3 pg(T, (H + G + 3) / 4);
   if (f32) {
-    attn_prep_kernel<float><<<pg, 256, 0, s>>>(p);
+    launch_prep<float>(p, s);
     return launch_any_d<float>(a, max_len, s);
   }
-  attn_prep_kernel<bf16_t><<<pg, 256, 0, s>>>(p);
+  launch_prep<bf16_t>(p, s);
   if (!mfma_dim(D)) return launch_any_d<bf16_t>(a, max_len, s);
   switch (D) {
     case 32: return launch_mfma<32>(a, max_len, singles, s);

@@ -5,9 +5,9 @@
 //    y_c = (sum_n S[c, n] C_n + D_c x_c) * silu(z_c).
 // 3) gated linear recurrence: S_c <- a_c S_c + d_c, y_c = S_c * gelu(g_c).
 //
-// Both recurrences run in fp32 in one of two ways. Short portions (decode, up to CHUNK tokens): one
-// launch, a thread walks its channel's tokens from the stored state. Longer ones are cut into chunks of
-// CHUNK tokens: (a) every chunk but a portion's last runs from zero (the first: from the stored state)
+// Both recurrences run in fp32 in one of two ways. Short portions (decode, up to one chunk), and
+// longer ones where the sequences alone fill the chip: one launch, a thread walks its channel's tokens from the
+// stored state. Else the portions are cut into chunks: (a) every chunk but a portion's last runs from zero (the first: from the stored state)
 // and leaves its end state and its total decay, (b) one pass over the chunks turns those into each
 // chunk's start state, (c) every chunk runs again from its start state and writes its outputs. Chunks of
 // all portions fill the chip, and a token's arithmetic differs between the two ways by rounding only.
@@ -35,8 +35,6 @@ __device__ __forceinline__ void conv_state_store(const ConvState& s, const SeqMe
 }
 
 // ------------------------------------------------------------------------------- convolution
-constexpr int CONV_RUN = 8;  // consecutive tokens of a thread
-
 struct ConvArgs {
   const void* x; const float* w; const float* bias; const void* state; void* y;  // w [taps][C]
   int ldx, ldy, C, taps;
@@ -52,7 +50,7 @@ __device__ __forceinline__ f32x4_t conv_input(const ConvArgs& a, int t, int k, i
   return Act<T>::load4((const T*)a.state + ((size_t)a.m.slot[b] * (a.taps - 1) + (a.taps - 1 + j - k)) * a.C + c);
 }
 
-template <typename T, int TAPS, int SILU>
+template <typename T, int TAPS, int SILU, int CONV_RUN>  // CONV_RUN: consecutive tokens of a thread
 __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
   const int c = (blockIdx.x * 64 + (threadIdx.x & 63)) * 4;
   const int t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * CONV_RUN;
@@ -67,27 +65,43 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
     Act<T>::store4((T*)a.y + (size_t)t * a.ldy + c, v);
   };
   if constexpr (TAPS > 0) {
-    f32x4_t w[TAPS], win[TAPS];  // win[TAPS - 1] is the current token's input
+    // the run's inputs and the taps - 1 before it, all loads issued together
+    f32x4_t w[TAPS], x[CONV_RUN + TAPS - 1];
 #pragma unroll
     for (int k = 0; k < TAPS; ++k) w[k] = *(const f32x4_t*)(a.w + (size_t)k * a.C + c);
-    int b = -1;
-    for (int t = t0; t < t1; ++t) {
-      const int bt = a.m.seq[t];
-      if (bt != b) {
-        b = bt;
+    const int b0 = a.m.seq[t0], b1 = a.m.seq[t1 - 1];
+    if (b0 == b1) {
+      const int s0 = a.m.cu[b0];
+      const T* st = (const T*)a.state + (size_t)a.m.slot[b0] * (TAPS - 1) * a.C + c;
+      const bool stored = a.m.pos0[b0] != 0;
 #pragma unroll
-        for (int k = 1; k < TAPS; ++k) win[TAPS - 1 - k] = conv_input<T>(a, t, k, c);
-      } else {
-#pragma unroll
-        for (int k = 0; k + 1 < TAPS; ++k) win[k] = win[k + 1];
+      for (int i = 0; i < CONV_RUN + TAPS - 1; ++i) {
+        const int t = min(t0 + i - (TAPS - 1), t1 - 1);
+        x[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        if (t >= s0) x[i] = Act<T>::load4((const T*)a.x + (size_t)t * a.ldx + c);
+        else if (stored) x[i] = Act<T>::load4(st + (size_t)(TAPS - 1 + t - s0) * a.C);
       }
-      win[TAPS - 1] = Act<T>::load4((const T*)a.x + (size_t)t * a.ldx + c);
-      f32x4_t v = bias;
 #pragma unroll
-      for (int k = 0; k < TAPS; ++k)
+      for (int i = 0; i < CONV_RUN; ++i) {
+        if (t0 + i >= t1) break;
+        f32x4_t v = bias;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = fmaf(w[k][e], win[k][e], v[e]);
-      emit(t, v);
+        for (int k = 0; k < TAPS; ++k)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] = fmaf(w[k][e], x[i + k][e], v[e]);
+        emit(t0 + i, v);
+      }
+    } else {  // a portion ends inside the run
+      for (int t = t0; t < t1; ++t) {
+        f32x4_t v = bias;
+#pragma unroll
+        for (int k = 0; k < TAPS; ++k) {
+          const f32x4_t xk = conv_input<T>(a, t, TAPS - 1 - k, c);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] = fmaf(w[k][e], xk[e], v[e]);
+        }
+        emit(t, v);
+      }
     }
   } else {
     for (int t = t0; t < t1; ++t) {
@@ -103,12 +117,12 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
   }
 }
 
-template <typename T>
+template <typename T, int CONV_RUN>
 static int launch_conv(const ConvArgs& a, int silu, hipStream_t s) {
   const dim3 grid((a.C / 4 + 63) / 64, (a.m.T + 4 * CONV_RUN - 1) / (4 * CONV_RUN)), block(256);
 #define CONV_CASE(K)                                                      \
-  if (silu) causal_conv_kernel<T, K, 1><<<grid, block, 0, s>>>(a);        \
-  else causal_conv_kernel<T, K, 0><<<grid, block, 0, s>>>(a);
+  if (silu) causal_conv_kernel<T, K, 1, CONV_RUN><<<grid, block, 0, s>>>(a);        \
+  else causal_conv_kernel<T, K, 0, CONV_RUN><<<grid, block, 0, s>>>(a);
   switch (a.taps) {
     case 2: CONV_CASE(2) break;
     case 3: CONV_CASE(3) break;
@@ -120,13 +134,15 @@ static int launch_conv(const ConvArgs& a, int silu, hipStream_t s) {
 }
 
 DA_EXPORT int da_causal_conv(const void* x, int ldx, const void* w, const void* bias, const void* state, void* y,
-                             int ldy, int C, int taps, int silu, const void* cu, const void* slot, const void* pos0,
+                             int ldy, int C, int taps, int silu, int max_len, const void* cu, const void* slot, const void* pos0,
                              const void* seq, int T, int B, int f32, void* stream) {
-  if (T < 1 || B < 1 || C < 4 || C % 4 || ldx % 4 || ldy % 4 || taps < 1 || (T + 31) / 32 > 65535)
+  if (T < 1 || B < 1 || C < 4 || C % 4 || ldx % 4 || ldy % 4 || taps < 1 || (T + 3) / 4 > 65535 * 8)
     return (int)hipErrorInvalidValue;
   ConvArgs a{x, (const float*)w, (const float*)bias, state, y, ldx, ldy, C, taps,
              SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B}};
-  return f32 ? launch_conv<float>(a, silu, (hipStream_t)stream) : launch_conv<bf16_t>(a, silu, (hipStream_t)stream);
+  hipStream_t s = (hipStream_t)stream;
+  if (max_len == 1 && T < 4096) return f32 ? launch_conv<float, 1>(a, silu, s) : launch_conv<bf16_t, 1>(a, silu, s);
+  return f32 ? launch_conv<float, 8>(a, silu, s) : launch_conv<bf16_t, 8>(a, silu, s);
 }
 
 // ------------------------------------------------------------------------------- phases
@@ -142,7 +158,7 @@ template <int PHASE>
 __device__ __forceinline__ ScanSpan scan_span(const SeqMeta& m, const ChunkMeta& ch, int g) {
   if constexpr (PHASE == SCAN_DIRECT) return ScanSpan{g, m.cu[g], m.cu[g + 1], 0, true, m.cu[g] == m.cu[g + 1]};
   const int b = ch.ck[2 * g], k = ch.ck[2 * g + 1];
-  const int t0 = m.cu[b] + k * CHUNK, t1 = min(t0 + CHUNK, m.cu[b + 1]);
+  const int t0 = m.cu[b] + k * ch.len, t1 = min(t0 + ch.len, m.cu[b + 1]);
   const bool last = t1 == m.cu[b + 1];
   return ScanSpan{b, t0, t1, k, last, PHASE == SCAN_LOCAL && last};
 }
@@ -163,6 +179,34 @@ struct SelArgs {
 
 constexpr int SEL_TT = 16;  // tokens whose B, C rows are staged together
 
+// NS consecutive floats n0 .. of a row of N, zero past its end (vector accesses where rows are 16-byte aligned).
+template <int NS>
+__device__ __forceinline__ void row_load(float (&v)[NS], const float* p, int n0, int N) {
+  if (N % 4 == 0) {
+#pragma unroll
+    for (int i = 0; i < NS; i += 4) {
+      const f32x4_t x = n0 + i < N ? *(const f32x4_t*)(p + n0 + i) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[i + e] = x[e];
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < NS; ++i) v[i] = n0 + i < N ? p[n0 + i] : 0.f;
+  }
+}
+template <int NS>
+__device__ __forceinline__ void row_store(float* p, const float (&v)[NS], int n0, int N) {
+  if (N % 4 == 0) {
+#pragma unroll
+    for (int i = 0; i < NS; i += 4)
+      if (n0 + i < N) *(f32x4_t*)(p + n0 + i) = f32x4_t{v[i], v[i + 1], v[i + 2], v[i + 3]};
+  } else {
+#pragma unroll
+    for (int i = 0; i < NS; ++i)
+      if (n0 + i < N) p[n0 + i] = v[i];
+  }
+}
+
 // A channel's N states live in `lanes` neighbouring lanes, NS each. Dynamic LDS: SEL_TT rows of B | C.
 template <typename T, int NS, int PHASE>
 __global__ void __launch_bounds__(256) sel_scan_kernel(SelArgs a) {
@@ -175,27 +219,16 @@ __global__ void __launch_bounds__(256) sel_scan_kernel(SelArgs a) {
   const int cc = live ? c : a.C - 1;
   float S[NS], A[NS];
   float* st = a.state + ((size_t)a.m.slot[sp.b] * a.C + cc) * a.N;
+  row_load<NS>(A, a.A + (size_t)cc * a.N, n0, a.N);
 #pragma unroll
-  for (int i = 0; i < NS; ++i) {
-    A[i] = n0 + i < a.N ? a.A[(size_t)cc * a.N + n0 + i] : 0.f;
-    S[i] = 0.f;
-  }
+  for (int i = 0; i < NS; ++i) S[i] = 0.f;
   const bool stored = a.m.pos0[sp.b] != 0;
   if (PHASE == SCAN_FINAL && !sp.only()) {
-    const float* cs = a.chunk_state + (chunk_row(a.ch, sp.b, sp.k) * a.C + cc) * a.N;
-#pragma unroll
-    for (int i = 0; i < NS; ++i)
-      if (n0 + i < a.N) S[i] = cs[n0 + i];
+    row_load<NS>(S, a.chunk_state + (chunk_row(a.ch, sp.b, sp.k) * a.C + cc) * a.N, n0, a.N);
   } else if (sp.k == 0) {
-#pragma unroll
-    for (int i = 0; i < NS; ++i)
-      if (stored && n0 + i < a.N) S[i] = st[n0 + i];
-    if constexpr (PHASE == SCAN_LOCAL) {
-      float* cs = a.chunk_state + (chunk_row(a.ch, sp.b, 0) * a.C + cc) * a.N;
-#pragma unroll
-      for (int i = 0; i < NS; ++i)
-        if (live && n0 + i < a.N) cs[n0 + i] = S[i];
-    }
+    if (stored) row_load<NS>(S, st, n0, a.N);
+    if constexpr (PHASE == SCAN_LOCAL)
+      if (live) row_store<NS>(a.chunk_state + (chunk_row(a.ch, sp.b, 0) * a.C + cc) * a.N, S, n0, a.N);
   }
   const float Dc = a.D[cc];
   float sdt = 0.f;
@@ -244,15 +277,10 @@ __global__ void __launch_bounds__(256) sel_scan_kernel(SelArgs a) {
   if (!live) return;
   if constexpr (PHASE == SCAN_LOCAL) {
     const size_t row = chunk_row(a.ch, sp.b, sp.k + 1);
-    float* cs = a.chunk_state + (row * a.C + c) * a.N;
-#pragma unroll
-    for (int i = 0; i < NS; ++i)
-      if (n0 + i < a.N) cs[n0 + i] = S[i];
+    row_store<NS>(a.chunk_state + (row * a.C + c) * a.N, S, n0, a.N);
     if (g == 0) a.chunk_dt[row * a.C + c] = sdt;
   } else if (sp.last) {
-#pragma unroll
-    for (int i = 0; i < NS; ++i)
-      if (n0 + i < a.N) st[n0 + i] = S[i];
+    row_store<NS>(st, S, n0, a.N);
     if (g == 0) conv_state_store<T>(a.conv, a.m, sp.b, c);
   }
 }
@@ -262,7 +290,7 @@ __global__ void __launch_bounds__(256) sel_scan_kernel(SelArgs a) {
 __global__ void __launch_bounds__(256) sel_carry_kernel(SelArgs a) {
   const int i = blockIdx.x * 256 + threadIdx.x, b = blockIdx.y;
   if (i >= a.C * a.N) return;
-  const int n = (a.m.cu[b + 1] - a.m.cu[b] + CHUNK - 1) / CHUNK;
+  const int n = (a.m.cu[b + 1] - a.m.cu[b] + a.ch.len - 1) / a.ch.len;
   const int c = i / a.N;
   const size_t row = chunk_row(a.ch, b, 0), CN = (size_t)a.C * a.N;
   if (n < 3) return;  // rows 0 and 1 are final
@@ -306,22 +334,23 @@ DA_EXPORT int da_selective_scan(const void* x, int ldx, const void* dt, int lddt
                                 int offC, const void* z, int ldz, const void* A, const void* D, void* state, void* y,
                                 int ldy, int C, int N, const void* conv_x, int ld_conv, void* conv_state, int taps,
                                 void* chunk_state, void* chunk_dt, const void* ck, const void* base, int n_chunks,
-                                const void* cu, const void* slot, const void* pos0, const void* seq, int T, int B,
+                                int chunk, int max_len, const void* cu, const void* slot, const void* pos0, const void* seq, int T, int B,
                                 int f32, void* stream) {
-  if (T < 1 || B < 1 || B > 65535 || C < 1 || N < 1 || N > 512 || taps < 1 || n_chunks < 0 || n_chunks > 65535)
+  if (T < 1 || B < 1 || B > 65535 || C < 1 || N < 1 || N > 512 || taps < 1 || n_chunks < 0 || n_chunks > 65535 || (n_chunks && chunk < 1))
     return (int)hipErrorInvalidValue;
   if (n_chunks && (!ck || !base || !chunk_state || !chunk_dt)) return (int)hipErrorInvalidValue;
-  const int ns = N <= 4 ? 4 : (N % 16 == 0 ? 16 : 8);
+  // single tokens: four states a lane, so the states' rows are read and written in whole lines
+  const int ns = N <= 4 || (max_len <= 4 && N <= 256) ? 4 : 8;
   int lanes = 1;
   while (lanes * ns < N) lanes *= 2;
   SelArgs a{x, (const float*)dt, bc, z, (const float*)A, (const float*)D, (float*)state, y, (float*)chunk_state,
             (float*)chunk_dt, ldx, lddt, ldbc, ldz, ldy, offB, offC, C, N, lanes,
             ConvState{conv_x, ld_conv, conv_state, taps, C},
             SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B},
-            ChunkMeta{(const int*)ck, (const int*)base, n_chunks}};
+            ChunkMeta{(const int*)ck, (const int*)base, n_chunks, chunk}};
   hipStream_t s = (hipStream_t)stream;
-  if (f32) return ns == 4 ? launch_sel<float, 4>(a, s) : ns == 8 ? launch_sel<float, 8>(a, s) : launch_sel<float, 16>(a, s);
-  return ns == 4 ? launch_sel<bf16_t, 4>(a, s) : ns == 8 ? launch_sel<bf16_t, 8>(a, s) : launch_sel<bf16_t, 16>(a, s);
+  if (f32) return ns == 4 ? launch_sel<float, 4>(a, s) : launch_sel<float, 8>(a, s);
+  return ns == 4 ? launch_sel<bf16_t, 4>(a, s) : launch_sel<bf16_t, 8>(a, s);
 }
 
 // ------------------------------------------------------------------------------- gated recurrence
@@ -378,7 +407,7 @@ __global__ void __launch_bounds__(256) gru_scan_kernel(GruArgs a) {
 
 __global__ void __launch_bounds__(256) gru_carry_kernel(GruArgs a) {
   const int c = blockIdx.x * 256 + threadIdx.x, b = blockIdx.y;
-  const int n = (a.m.cu[b + 1] - a.m.cu[b] + CHUNK - 1) / CHUNK;
+  const int n = (a.m.cu[b + 1] - a.m.cu[b] + a.ch.len - 1) / a.ch.len;
   if (c >= a.C || n < 3) return;
   const size_t row = chunk_row(a.ch, b, 0);
   float s = a.chunk_state[(row + 1) * a.C + c];
@@ -415,14 +444,14 @@ static int launch_gru(const GruArgs& a, hipStream_t s) {
 DA_EXPORT int da_gated_scan(const void* decay, const void* drive, const void* gate, int ldg, void* state, void* y,
                             int ldy, int C, const void* conv_x, int ld_conv, void* conv_state, int taps,
                             void* chunk_state, void* chunk_decay, const void* ck, const void* base, int n_chunks,
-                            const void* cu, const void* slot, const void* pos0, const void* seq, int T, int B, int f32,
+                            int chunk, const void* cu, const void* slot, const void* pos0, const void* seq, int T, int B, int f32,
                             void* stream) {
-  if (T < 1 || B < 1 || B > 65535 || C < 1 || taps < 1 || n_chunks < 0 || n_chunks > 65535)
+  if (T < 1 || B < 1 || B > 65535 || C < 1 || taps < 1 || n_chunks < 0 || n_chunks > 65535 || (n_chunks && chunk < 1))
     return (int)hipErrorInvalidValue;
   if (n_chunks && (!ck || !base || !chunk_state || !chunk_decay)) return (int)hipErrorInvalidValue;
   GruArgs a{(const float*)decay, (const float*)drive, gate, (float*)state, y, (float*)chunk_state,
             (float*)chunk_decay, ldg, ldy, C, ConvState{conv_x, ld_conv, conv_state, taps, C},
             SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B},
-            ChunkMeta{(const int*)ck, (const int*)base, n_chunks}};
+            ChunkMeta{(const int*)ck, (const int*)base, n_chunks, chunk}};
   return f32 ? launch_gru<float>(a, (hipStream_t)stream) : launch_gru<bf16_t>(a, (hipStream_t)stream);
 }

@@ -11,13 +11,12 @@ struct SeqMeta {
   int T, B;
 };
 
-// Chunks of CHUNK tokens for the recurrences: chunk i is tokens [CHUNK * ck[2i+1], + CHUNK) of portion
-// ck[2i]; base[b] is the number of chunks of the portions before b.
+// Chunks of `len` tokens for the recurrences: chunk i is tokens [len * ck[2i+1], + len) of portion ck[2i];
+// base[b] is the number of chunks of the portions before b.
 struct ChunkMeta {
   const int* ck; const int* base;
-  int n;
+  int n, len;
 };
-constexpr int CHUNK = 64;
 constexpr int PAGE = 64;  // tokens per cache page
 
 // Activation storage: bf16 (the serving precision) or fp32; arithmetic is fp32 either way.
@@ -48,9 +47,39 @@ template <> struct Act<float> {
   __device__ static __forceinline__ void store2(float* p, float a, float b) { *(f32x2_t*)p = f32x2_t{a, b}; }
 };
 
-__device__ __forceinline__ float sigmoid32(float x) { return 1.f / (1.f + expf(-x)); }
-__device__ __forceinline__ float softplus32(float x) { return x > 20.f ? x + expf(-x) : log1pf(expf(x)); }
-__device__ __forceinline__ float silu32(float x) { return x / (1.f + expf(-x)); }
+// Elementary functions good to a few fp32 ulp on the hardware's 1-ulp exp2 / log2 / rcp / sqrt (the library
+// forms spend most of their instructions on cases that cannot occur here: the epilogues and scans that
+// use these run at their instruction count).
+constexpr float LOG2E = 1.4426950408889634f;
+// e^x, x <= 88: the part of x * log2(e) that fp32 drops is put back (first order).
+__device__ __forceinline__ float exp32(float x) {
+  x = fminf(x, 88.f);
+  const float t = x * LOG2E;
+  const float lo = fmaf(x, 1.925963033500e-8f, fmaf(x, LOG2E, -t));
+  const float e = __builtin_amdgcn_exp2f(t);
+  return fmaf(e, lo * 0.6931471805599453f, e);
+}
+__device__ __forceinline__ float sigmoid32(float x) { return __builtin_amdgcn_rcpf(1.f + exp32(-x)); }
+// log(1 + e^x) = max(x, 0) + log1p(e), e = e^-|x|; log1p(e) = log(u) e / (u - 1) with u = fl(1 + e), which
+// cancels the rounding of u (Goldberg, "What every computer scientist should know about floating-point
+// arithmetic", 1991, theorem 4).
+__device__ __forceinline__ float softplus32(float x) {
+  const float e = exp32(-fabsf(x)), u = 1.f + e, d = u - 1.f;
+  const float l = __builtin_amdgcn_logf(u) * 0.6931471805599453f;
+  return fmaxf(x, 0.f) + (d == 0.f ? e : l * e * __builtin_amdgcn_rcpf(d));
+}
+// 1 - e^y for y <= 0: the series of the exponential where the difference would cancel.
+__device__ __forceinline__ float one_minus_exp32(float y) {
+  float p = fmaf(y, 1.f / 8.f, 1.f);
+  p = fmaf(p * y, 1.f / 7.f, 1.f);
+  p = fmaf(p * y, 1.f / 6.f, 1.f);
+  p = fmaf(p * y, 1.f / 5.f, 1.f);
+  p = fmaf(p * y, 1.f / 4.f, 1.f);
+  p = fmaf(p * y, 1.f / 3.f, 1.f);
+  p = fmaf(p * y, 1.f / 2.f, 1.f);
+  return y > -0.4f ? -y * p : 1.f - exp32(y);
+}
+__device__ __forceinline__ float silu32(float x) { return x * sigmoid32(x); }
 __device__ __forceinline__ float gelu_tanh32(float x) {
   // 0.5 (1 + tanh(z)) = sigmoid(2 z)
   return x * sigmoid32(1.5957691216057308f * (x + 0.044715f * x * x * x));

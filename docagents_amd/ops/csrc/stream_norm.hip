@@ -7,8 +7,9 @@
 #include "seq.h"
 
 struct StreamArgs {
-  const int* ids; const void* table; int vocab;             // EMBED: x' = table[ids]
+  const int* ids; const void* table; int vocab;             // embedding: x' = table[ids]
   const float* x; const void* y; const float* w; float alpha, eps;
+  int splits;                                               // y is the sum of `splits` fp32 [T][Dp] partials
   int D, Dp;                                                // columns, padded columns (row stride)
   float* x_out; void* h_out;
   const float* mu; const float* prev;                       // token shift: mu [Dp], state [slots][Dp]
@@ -17,86 +18,108 @@ struct StreamArgs {
   int rows;                                                 // consecutive tokens per workgroup
 };
 
-template <typename T, int NCH, bool EMBED>
+enum StreamSrc : int { SRC_EMBED = 0, SRC_Y = 1, SRC_PARTIALS = 2 };
+
+// A thread holds NCH 4-column pieces of a row. The next row's loads are issued before this row's sum.
+template <typename T, int NCH, int SRC>
 __global__ void __launch_bounds__(256) stream_kernel(StreamArgs a) {
   __shared__ float red[16];
   const int nt = blockDim.x, nc = a.Dp / 4;
-  f32x4_t cur[NCH], prv[NCH];
+  f32x4_t nx[NCH], cur[NCH], prv[NCH];
 
-  auto row_of = [&](int t, f32x4_t (&v)[NCH]) {
-    if constexpr (EMBED) {
-      const int id = min(max(a.ids[t], 0), a.vocab - 1);
+  auto col = [&](int i) { return (int)threadIdx.x + i * nt; };  // this thread's i-th piece
+  auto fetch = [&](int t) {  // alpha x + y of row t (embedding: the row itself) into nx
+    const size_t src = SRC == SRC_EMBED ? min(max(a.ids[t], 0), a.vocab - 1) : t;
 #pragma unroll
-      for (int i = 0; i < NCH; ++i) {
-        const int c = threadIdx.x + i * nt;
-        v[i] = c < nc ? Act<T>::load4((const T*)a.table + (size_t)id * a.Dp + c * 4) : f32x4_t{0.f, 0.f, 0.f, 0.f};
-      }
-    } else {
-      float ss = 0.f;
+    for (int i = 0; i < NCH; ++i) {
+      const int c = min(col(i), nc - 1) * 4;
+      if constexpr (SRC == SRC_EMBED) {
+        nx[i] = Act<T>::load4((const T*)a.table + src * a.Dp + c);
+      } else {
+        f32x4_t y;
+        if constexpr (SRC == SRC_Y) {
+          y = Act<T>::load4((const T*)a.y + src * a.Dp + c);
+        } else {
+          y = f32x4_t{0.f, 0.f, 0.f, 0.f};
+          const float* p = (const float*)a.y + src * a.Dp + c;
+          const size_t st = (size_t)a.m.T * a.Dp;
+          for (int s0 = 0; s0 < a.splits; s0 += 4) {
+            f32x4_t v[4];
 #pragma unroll
-      for (int i = 0; i < NCH; ++i) {
-        const int c = threadIdx.x + i * nt;
-        v[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-        if (c < nc) {
-          const f32x4_t x = *(const f32x4_t*)(a.x + (size_t)t * a.Dp + c * 4);
-          const f32x4_t y = Act<T>::load4((const T*)a.y + (size_t)t * a.Dp + c * 4);
+            for (int s = 0; s < 4; ++s) v[s] = *(const f32x4_t*)(p + min(s0 + s, a.splits - 1) * st);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            v[i][e] = fmaf(a.alpha, x[e], y[e]);
-            ss = fmaf(v[i][e], v[i][e], ss);
+            for (int s = 0; s < 4; ++s)
+#pragma unroll
+              for (int e = 0; e < 4; ++e) y[e] += s0 + s < a.splits ? v[s][e] : 0.f;
           }
         }
-      }
-      const float inv = 1.f / sqrtf(block_sum(ss, red) / a.D + a.eps);
+        const f32x4_t x = *(const f32x4_t*)(a.x + src * a.Dp + c);
 #pragma unroll
-      for (int i = 0; i < NCH; ++i) {
-        const int c = threadIdx.x + i * nt;
-        if (c < nc) {
-          const f32x4_t w = *(const f32x4_t*)(a.w + c * 4);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) v[i][e] *= inv * w[e];
-        }
+        for (int e = 0; e < 4; ++e) nx[i][e] = fmaf(a.alpha, x[e], y[e]);
       }
     }
   };
+  auto normed = [&](f32x4_t (&v)[NCH]) {  // v = the fetched row, normalised; then nx is free
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NCH; ++i) {
+      v[i] = nx[i];
+      if (SRC != SRC_EMBED && col(i) < nc)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = fmaf(v[i][e], v[i][e], ss);
+    }
+    return ss;
+  };
+  auto scale = [&](f32x4_t (&v)[NCH], float ss) {
+    if constexpr (SRC == SRC_EMBED) return;
+    const float inv = 1.f / sqrtf(block_sum(ss, red) / a.D + a.eps);
+#pragma unroll
+    for (int i = 0; i < NCH; ++i) {
+      const f32x4_t w = *(const f32x4_t*)(a.w + min(col(i), nc - 1) * 4);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[i][e] *= inv * w[e];
+    }
+  };
 
-  const int t0 = blockIdx.x * a.rows;
-  for (int t = t0; t < min(t0 + a.rows, a.m.T); ++t) {
-    const int b = a.m.seq[t], s0 = a.m.cu[b];
-    if (a.mu) {
-      if (t == s0) {
-        const bool start = a.m.pos0[b] == 0;
-        const float* p = a.prev + (size_t)a.m.slot[b] * a.Dp;
+  const int t0 = blockIdx.x * a.rows, t1 = min(t0 + a.rows, a.m.T);
+  const bool redo = a.mu && t0 != a.m.cu[a.m.seq[t0]];  // the row before the first one is a neighbour's
+  fetch(redo ? t0 - 1 : t0);
+  if (redo) {
+    const float ss = normed(prv);
+    fetch(t0);
+    scale(prv, ss);
+  }
+  for (int t = t0; t < t1; ++t) {
+    const int b = a.m.seq[t];
+    if (a.mu && t == a.m.cu[b]) {
+      const bool start = a.m.pos0[b] == 0;
+      const float* p = a.prev + (size_t)a.m.slot[b] * a.Dp;
 #pragma unroll
-        for (int i = 0; i < NCH; ++i) {
-          const int c = threadIdx.x + i * nt;
-          prv[i] = (!start && c < nc) ? *(const f32x4_t*)(p + c * 4) : f32x4_t{0.f, 0.f, 0.f, 0.f};
-        }
-      } else if (t == t0) {
-        row_of(t - 1, prv);
-      } else {
-#pragma unroll
-        for (int i = 0; i < NCH; ++i) prv[i] = cur[i];
+      for (int i = 0; i < NCH; ++i) {
+        prv[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        if (!start) prv[i] = *(const f32x4_t*)(p + min(col(i), nc - 1) * 4);
       }
     }
-    row_of(t, cur);
+    const float ss = normed(cur);
+    if (t + 1 < t1) fetch(t + 1);
+    scale(cur, ss);
     const bool keep = a.save && t + 1 == a.m.cu[b + 1];
 #pragma unroll
     for (int i = 0; i < NCH; ++i) {
-      const int c = threadIdx.x + i * nt;
-      if (c >= nc) continue;
-      if (a.x_out) *(f32x4_t*)(a.x_out + (size_t)t * a.Dp + c * 4) = cur[i];
+      const int c = col(i) * 4;
+      if (c >= a.Dp) continue;
+      if (a.x_out) *(f32x4_t*)(a.x_out + (size_t)t * a.Dp + c) = cur[i];
       if (a.h_out) {
         f32x4_t h = cur[i];
         if (a.mu) {
-          const f32x4_t mu = *(const f32x4_t*)(a.mu + c * 4);
+          const f32x4_t mu = *(const f32x4_t*)(a.mu + c);
 #pragma unroll
           for (int e = 0; e < 4; ++e) h[e] = fmaf(prv[i][e] - cur[i][e], mu[e], cur[i][e]);
         }
-        Act<T>::store4((T*)a.h_out + (size_t)t * a.Dp + c * 4, h);
+        Act<T>::store4((T*)a.h_out + (size_t)t * a.Dp + c, h);
       }
-      if (keep)
-        *(f32x4_t*)(a.save + (size_t)a.m.slot[b] * a.Dp + c * 4) = *(const f32x4_t*)(a.x + (size_t)t * a.Dp + c * 4);
+      if (keep) *(f32x4_t*)(a.save + (size_t)a.m.slot[b] * a.Dp + c) = *(const f32x4_t*)(a.x + (size_t)t * a.Dp + c);
+      prv[i] = cur[i];
     }
   }
 }
@@ -124,37 +147,40 @@ stream_final_kernel(const float* __restrict__ x, const long long* __restrict__ r
   }
 }
 
-template <typename T, bool EMBED>
+template <typename T, int SRC>
 static int launch_stream(const StreamArgs& a, hipStream_t s) {
   const int nc = a.Dp / 4;
   const int nt = nc >= 256 ? 256 : (nc + 63) / 64 * 64;
   const int nch = (nc + nt - 1) / nt;
   const dim3 grid((a.m.T + a.rows - 1) / a.rows), block(nt);
-  if (nch <= 1) stream_kernel<T, 1, EMBED><<<grid, block, 0, s>>>(a);
-  else if (nch <= 2) stream_kernel<T, 2, EMBED><<<grid, block, 0, s>>>(a);
-  else if (nch <= 4) stream_kernel<T, 4, EMBED><<<grid, block, 0, s>>>(a);
-  else if (nch <= 8) stream_kernel<T, 8, EMBED><<<grid, block, 0, s>>>(a);
-  else if (nch <= 16) stream_kernel<T, 16, EMBED><<<grid, block, 0, s>>>(a);
+  if (nch <= 1) stream_kernel<T, 1, SRC><<<grid, block, 0, s>>>(a);
+  else if (nch <= 2) stream_kernel<T, 2, SRC><<<grid, block, 0, s>>>(a);
+  else if (nch <= 4) stream_kernel<T, 4, SRC><<<grid, block, 0, s>>>(a);
+  else if (nch <= 8) stream_kernel<T, 8, SRC><<<grid, block, 0, s>>>(a);
+  else if (nch <= 16) stream_kernel<T, 16, SRC><<<grid, block, 0, s>>>(a);
   else return (int)hipErrorInvalidValue;
   DA_LAUNCH_CHECK();
 }
 
 // x' = norm(alpha x + y) (ids null) or table[ids] (embedding rows in the activation type); outputs
-// and state as in StreamArgs, any of x_out / h_out / mu / save null. D % 4 == 0 columns of Dp.
-DA_EXPORT int da_stream_step(const void* ids, const void* table, int vocab, const void* x, const void* y,
+// and state as in StreamArgs, any of x_out / h_out / mu / save null. splits > 0: y holds that many fp32
+// partials. D of Dp columns, Dp % 4 == 0.
+DA_EXPORT int da_stream_step(const void* ids, const void* table, int vocab, const void* x, const void* y, int splits,
                              const void* w, float alpha, float eps, int D, int Dp, void* x_out, void* h_out,
                              const void* mu, const void* prev, void* save, const void* cu, const void* slot,
                              const void* pos0, const void* seq, int T, int B, int rows, int f32, void* stream) {
-  if (T < 1 || B < 1 || rows < 1 || Dp % 4 || D < 1 || D > Dp || !cu || !slot || !pos0 || !seq || x_out == x)
+  if (T < 1 || B < 1 || rows < 1 || Dp % 4 || D < 1 || D > Dp || !cu || !slot || !pos0 || !seq || splits < 0)
     return (int)hipErrorInvalidValue;
-  if (ids ? (!table || vocab < 1 || save) : (!x || !y || !w)) return (int)hipErrorInvalidValue;
+  if (ids ? (!table || vocab < 1 || save) : (!x || !y || !w || x_out == x)) return (int)hipErrorInvalidValue;
   if (mu && (!prev || prev == save)) return (int)hipErrorInvalidValue;
-  StreamArgs a{(const int*)ids, table, vocab, (const float*)x, y, (const float*)w, alpha, eps, D, Dp, (float*)x_out,
-               h_out, (const float*)mu, (const float*)prev, (float*)save,
+  StreamArgs a{(const int*)ids, table, vocab, (const float*)x, y, (const float*)w, alpha, eps, splits, D, Dp,
+               (float*)x_out, h_out, (const float*)mu, (const float*)prev, (float*)save,
                SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B}, rows};
   hipStream_t s = (hipStream_t)stream;
-  if (f32) return ids ? launch_stream<float, true>(a, s) : launch_stream<float, false>(a, s);
-  return ids ? launch_stream<bf16_t, true>(a, s) : launch_stream<bf16_t, false>(a, s);
+  if (f32) return ids ? launch_stream<float, SRC_EMBED>(a, s)
+                      : splits ? launch_stream<float, SRC_PARTIALS>(a, s) : launch_stream<float, SRC_Y>(a, s);
+  return ids ? launch_stream<bf16_t, SRC_EMBED>(a, s)
+             : splits ? launch_stream<bf16_t, SRC_PARTIALS>(a, s) : launch_stream<bf16_t, SRC_Y>(a, s);
 }
 
 DA_EXPORT int da_stream_final(const void* x, const void* rows, const void* w, float eps, int D, int Dp, void* y,

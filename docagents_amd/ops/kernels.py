@@ -1124,5 +1124,5 @@ def pool_l2norm_f16(h, cu_seqlens, mode: int = 0, out32=None, out16=None):
 
 
 # the batch-of-portions ops (recurrent mixers, paged attention, 32-bit residual stream)
-from .seq_kernels import (causal_conv, gated_scan, gemm_any, rglru_gates, selective_scan,  # noqa: E402,F401
-                          sigmoid_attn, stream_final, stream_step)
+from .seq_kernels import (causal_conv, gated_scan, gemm_any, gemm_partials, partials_fit,  # noqa: E402,F401
+                          rglru_gates, selective_scan, sigmoid_attn, stream_final, stream_step)

@@ -1,14 +1,14 @@
 """The batch of one step: portions of sequences packed row after row, each against its own state slot."""
 from __future__ import annotations
 
-from dataclasses import dataclass, replace
+from dataclasses import dataclass, field, replace
 
 import numpy as np
 import torch
 
 from . import h2d
 
-CHUNK = 64  # tokens per chunk of a recurrence (csrc/seq.h)
+CHUNK = 64  # a recurrence's chunks are multiples of this many tokens
 PAGE = 64   # tokens per cache page (csrc/seq.h)
 
 
@@ -26,12 +26,31 @@ class SeqBatch:
     max_ctx: int           # bound on position + 1 over the batch (sets split counts: a host number)
     singles: bool = True   # a portion of one token may be in the batch
     table: torch.Tensor | None = None  # int32 [slots, pages of a slot]: the cache's page table
-    ck: torch.Tensor | None = None     # int32 [n_chunks, 2]: (portion, chunk of it)
-    base: torch.Tensor | None = None   # int32 [B]: chunks of the portions before b
-    n_chunks: int = 0                  # 0: every portion fits one chunk
+    lens: np.ndarray | None = None     # the portions' lengths (host); None: single tokens
+    _chunks: dict = field(default_factory=dict)
 
     def on(self, table) -> "SeqBatch":
         return replace(self, table=table)
+
+    def chunk_len(self, waves: int, fill: int = 2048) -> int:
+        """Tokens per chunk of a recurrence whose portions take ``waves`` waves each when walked from end to
+        end: as long as the chip is filled (``fill`` waves); 0 when the portions alone do that, or are short."""
+        if self.max_len <= CHUNK:
+            return 0
+        want = -(-fill * self.max_len // max(1, waves * self.T))  # chunks of the longest portion
+        return 0 if want <= 1 else max(CHUNK, -(-self.max_len // (want * CHUNK)) * CHUNK)
+
+    def chunks(self, n: int):
+        """(int32 [chunks, 2]: portion and chunk of it, int32 [B]: chunks of the portions before b, chunks) of
+        n tokens each."""
+        if n not in self._chunks:
+            per = -(-self.lens // n)
+            base = np.cumsum(per) - per
+            tot = int(per.sum())
+            ck = np.stack([np.repeat(np.arange(self.B), per), np.arange(tot) - np.repeat(base, per)], axis=1)
+            flat = h2d(np.concatenate([ck.ravel(), base]).astype(np.int32), self.cu.device)
+            self._chunks[n] = (flat[:2 * tot].view(tot, 2), flat[2 * tot:], tot)
+        return self._chunks[n]
 
 
 def pack_batch(lens, slots, pos0, device, ids=None):
@@ -44,13 +63,6 @@ def pack_batch(lens, slots, pos0, device, ids=None):
     np.cumsum(lens, out=cu[1:])
     parts = [cu, np.asarray(slots, dtype=np.int32), np.asarray(pos0, dtype=np.int32),
              np.repeat(np.arange(B, dtype=np.int32), lens)]
-    n = 0
-    if lens.max() > CHUNK:
-        per = -(-lens // CHUNK)
-        n = int(per.sum())
-        base = np.cumsum(per) - per
-        ck = np.stack([np.repeat(np.arange(B), per), np.arange(n) - np.repeat(base, per)], axis=1)
-        parts += [ck.astype(np.int32).ravel(), base.astype(np.int32)]
     if ids is not None:
         parts.append(np.asarray(ids, dtype=np.int32))
     flat = h2d(np.concatenate(parts), device)
@@ -59,7 +71,5 @@ def pack_batch(lens, slots, pos0, device, ids=None):
         out.append(flat[at:at + len(p)])
         at += len(p)
     m = SeqBatch(out[0], out[1], out[2], out[3], T, B, int(lens.max()), int((lens + parts[2]).max()),
-                 bool((lens == 1).any()))
-    if n:
-        m.ck, m.base, m.n_chunks = out[4].view(n, 2), out[5], n
+                 bool((lens == 1).any()), lens=lens)
     return m, (out[-1] if ids is not None else None)

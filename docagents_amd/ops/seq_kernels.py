@@ -15,16 +15,17 @@ _META = [c_void_p] * 4 + [c_int] * 2
 K._SIGS.update({
     "da_gemm_any": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p] + [c_int] * 6 + [c_longlong] * 4
                    + [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p],
-    "da_stream_step": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_float, c_float, c_int, c_int]
+    "da_gemm_partials": [c_void_p, c_int, c_void_p] + [c_int] * 5 + [c_void_p, c_void_p],
+    "da_stream_step": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_float, c_float, c_int, c_int]
                       + [c_void_p] * 5 + _META + [c_int, c_int, c_void_p],
     "da_stream_final": [c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_void_p, c_int, c_int, c_void_p],
-    "da_causal_conv": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int] + _META
+    "da_causal_conv": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int] + _META
                       + [c_int, c_void_p],
     "da_selective_scan": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_int]
                          + [c_void_p] * 4 + [c_int] * 3 + [c_void_p, c_int, c_void_p, c_int]
-                         + [c_void_p] * 4 + [c_int] + _META + [c_int, c_void_p],
+                         + [c_void_p] * 4 + [c_int] * 3 + _META + [c_int, c_void_p],
     "da_gated_scan": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p,
-                      c_int] + [c_void_p] * 4 + [c_int] + _META + [c_int, c_void_p],
+                      c_int] + [c_void_p] * 4 + [c_int] * 2 + _META + [c_int, c_void_p],
     "da_sigmoid_attn": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float,
                         c_float, c_float, K.ctypes.c_double] + [c_int] * 4 + [c_void_p, c_int, c_void_p] + [c_int] * 4
                        + _META + [c_int, c_void_p],
@@ -53,10 +54,15 @@ def _meta(m: SeqBatch):
     return [_ptr(m.cu), _ptr(m.slot), _ptr(m.pos0), _ptr(m.seq), m.T, m.B]
 
 
-def _chunks(m: SeqBatch):
-    if m.n_chunks:
-        _req(m.ck.dtype == torch.int32 and m.ck.numel() == 2 * m.n_chunks and m.base.numel() == m.B, "batch chunks")
-    return [_ptr(m.ck), _ptr(m.base), m.n_chunks]
+def _scratch(m: SeqBatch, waves: int, device, *shapes):
+    """Arguments of a chunked recurrence: fp32 scratch [chunks + B, *shape] each, the chunk list, its length and
+    the chunk length (no scratch and no chunks where the portions are walked from end to end)."""
+    n = m.chunk_len(waves)
+    if n == 0:
+        return [], [None] * len(shapes) + [None, None, 0, 0]
+    ck, base, tot = m.chunks(n)
+    ws = [torch.empty((tot + m.B, *s), dtype=torch.float32, device=device) for s in shapes]
+    return ws, [*map(_ptr, ws), _ptr(ck), _ptr(base), tot, n]
 
 
 def gemm_any(a, w, bias=None, epi: int = ANY_NONE):
@@ -73,6 +79,28 @@ def gemm_any(a, w, bias=None, epi: int = ANY_NONE):
     _check(lib().da_gemm_any(_ptr(a), a.stride(0), _ptr(w), _ptr(out), out.stride(0), _ptr(bias), M, N, Kd, f32, epi, 1, 0,
                              0, 0, 0, None, 0, None, None, None, 0, _stream()), "gemm_any")
     return out
+
+
+def partials_fit(M: int, N: int, Kd: int) -> bool:
+    """Whether a decode-sized product would run as split-K partials + a reduce launch (see ``kernels.gemm``): then
+    a consumer that sums the partials itself saves that launch and a rounding."""
+    return 1 < M <= 128 and not (M <= K.DK_SPLITK_ABOVE and Kd % 256 == 0)
+
+
+def gemm_partials(a, w):
+    """bf16 a[M, K] @ w[N, K]^T as fp32 partials [splits, M, N] (their sum is the product), in the shared workspace:
+    valid until the next product."""
+    K._bf16_cuda(a, "a"); K._bf16_cuda(w, "w")
+    M, Kd = a.shape
+    N = w.shape[0]
+    _req(w.shape[1] == Kd and Kd % 64 == 0 and N % 8 == 0 and M <= 128 and w.is_contiguous() and a.stride(1) == 1
+         and a.stride(0) % 8 == 0 and a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0, "gemm_partials operands")
+    tile = 9 if M > 64 else K._decode_tile(M)
+    splits = K._auto_splits(M, N, Kd)
+    ws = K._workspace(splits * M * N * 4, a.device)
+    _check(lib().da_gemm_partials(_ptr(a), a.stride(0), _ptr(w), M, N, Kd, tile, splits, _ptr(ws), _stream()),
+           "gemm_partials")
+    return ws[:splits * M * N * 4].view(torch.float32).view(splits, M, N)
 
 
 def rglru_gates(u, w, bias, lam):
@@ -97,29 +125,33 @@ def rglru_gates(u, w, bias, lam):
 def stream_step(m: SeqBatch, dim: int, eps: float = 0.0, alpha: float = 1.0, ids=None, table=None, x=None, y=None,
                 w=None, mu=None, prev=None, save=None, want_x: bool = True, want_h: bool = True, act=None):
     """One update of the fp32 residual stream: x' = table[ids], or RMSNorm(alpha x + y) w over ``dim`` of the
-    padded columns; h = x' or, with mu / prev (state [slots, Dp]), x' + (x'_previous token - x') mu, in the
+    padded columns (y [T, Dp], or its fp32 partials
+    [splits, T, Dp] from ``gemm_partials``); h = x' or, with mu / prev (state [slots, Dp]), x' + (x'_previous token - x') mu, in the
     activation type. save: state [slots, Dp] that receives each portion's last row of x. -> (x', h)."""
     src = table if ids is not None else y
-    f32 = _act(src, "table / y", act)
-    Dp = src.shape[1]
+    f32 = _act(src, "table / y", None if src.dim() == 3 else act)
+    Dp = src.shape[-1]
     dev = src.device
+    splits = src.shape[0] if src.dim() == 3 else 0
+    if splits:
+        f32 = int(act == torch.float32)
     _req(src.is_contiguous() and Dp % 4 == 0 and dim <= Dp <= 16384, "stream columns")
     if ids is not None:
         _req(ids.dtype == torch.int32 and ids.is_contiguous() and ids.numel() >= m.T and ids.is_cuda, "ids")
     else:
         _f32(x, "x", m.T * Dp)
         _f32(w, "w", Dp)
-        _req(y.shape[0] == m.T, "y rows")
+        _req(y.shape[-2] == m.T and (not splits or y.dtype == torch.float32), "y rows")
     if mu is not None:
         _f32(mu, "mu", Dp)
         _f32(prev, "prev")
     if save is not None:
         _f32(save, "save")
     xo = torch.empty((m.T, Dp), dtype=torch.float32, device=dev) if want_x else None
-    ho = torch.empty((m.T, Dp), dtype=src.dtype, device=dev) if want_h else None
-    rows = 1 if m.T <= 1024 else 4
-    _check(lib().da_stream_step(_ptr(ids), _ptr(table), 0 if table is None else table.shape[0], _ptr(x), _ptr(y), _ptr(w),
-                                float(alpha), float(eps), dim, Dp, _ptr(xo), _ptr(ho), _ptr(mu), _ptr(prev), _ptr(save),
+    ho = torch.empty((m.T, Dp), dtype=act or src.dtype, device=dev) if want_h else None
+    rows = 1 if m.T <= 2048 or mu is None else 8
+    _check(lib().da_stream_step(_ptr(ids), _ptr(table), 0 if table is None else table.shape[0], _ptr(x), _ptr(y), splits,
+                                _ptr(w), float(alpha), float(eps), dim, Dp, _ptr(xo), _ptr(ho), _ptr(mu), _ptr(prev), _ptr(save),
                                 *_meta(m), rows, f32, _stream()), "stream_step")
     return xo, ho
 
@@ -148,7 +180,7 @@ def causal_conv(x, w, bias, state, m: SeqBatch, silu: bool):
     _req(state.dtype == x.dtype and state.is_contiguous() and state.shape[1:] == (taps - 1, C), "conv state")
     y = torch.empty((m.T, C), dtype=x.dtype, device=x.device)
     _check(lib().da_causal_conv(_ptr(x), x.stride(0), _ptr(w), _ptr(bias), _ptr(state), _ptr(y), C, C, taps, int(silu),
-                                *_meta(m), f32, _stream()), "causal_conv")
+                                m.max_len, *_meta(m), f32, _stream()), "causal_conv")
     return y
 
 
@@ -171,14 +203,12 @@ def selective_scan(x, dt, bc, off_b: int, off_c: int, z, A, D, state, conv_x, co
     _req(x.shape == (m.T, C) and z.shape == (m.T, C) and state.shape[1:] == (C, N) and N <= 512
          and max(off_b, off_c) + N <= bc.shape[1] and bc.shape[0] == m.T, "selective_scan shapes")
     y = torch.empty((m.T, C), dtype=x.dtype, device=x.device)
-    cs = cd = None
-    if m.n_chunks:
-        cs = torch.empty((m.n_chunks + m.B, C, N), dtype=torch.float32, device=x.device)
-        cd = torch.empty((m.n_chunks + m.B, C), dtype=torch.float32, device=x.device)
+    ws, chunk = _scratch(m, C * -(-N // 8) // 64, x.device, (C, N), (C,))
     _check(lib().da_selective_scan(_ptr(x), x.stride(0), _ptr(dt), C, _ptr(bc), bc.stride(0), off_b, off_c, _ptr(z),
                                    z.stride(0), _ptr(A), _ptr(D), _ptr(state), _ptr(y), C, C, N,
-                                   *_conv_args(conv_x, conv_state, C, x.dtype), _ptr(cs), _ptr(cd), *_chunks(m), *_meta(m),
-                                   f32, _stream()), "selective_scan")
+                                   *_conv_args(conv_x, conv_state, C, x.dtype), *chunk, m.max_len, *_meta(m), f32,
+                                   _stream()), "selective_scan")
+    del ws
     return y
 
 
@@ -191,13 +221,11 @@ def gated_scan(decay, drive, gate, state, conv_x, conv_state, m: SeqBatch):
         _f32(t, n, k)
     _req(gate.shape == (m.T, C), "gate [T, C]")
     y = torch.empty((m.T, C), dtype=gate.dtype, device=gate.device)
-    cs = cd = None
-    if m.n_chunks:
-        cs = torch.empty((m.n_chunks + m.B, C), dtype=torch.float32, device=gate.device)
-        cd = torch.empty_like(cs)
+    ws, chunk = _scratch(m, C // 64, gate.device, (C,), (C,))
     _check(lib().da_gated_scan(_ptr(decay), _ptr(drive), _ptr(gate), gate.stride(0), _ptr(state), _ptr(y), C, C,
-                               *_conv_args(conv_x, conv_state, C, gate.dtype), _ptr(cs), _ptr(cd), *_chunks(m), *_meta(m),
-                               f32, _stream()), "gated_scan")
+                               *_conv_args(conv_x, conv_state, C, gate.dtype), *chunk, *_meta(m), f32, _stream()),
+           "gated_scan")
+    del ws
     return y
 
 

@@ -36,6 +36,14 @@ def gemm_any(a, w, bias=None, epi: int = ANY_NONE):
     return y
 
 
+def partials_fit(M: int, N: int, K: int) -> bool:
+    return False
+
+
+def gemm_partials(a, w):
+    return (a.float() @ w.float().t())[None]
+
+
 def rglru_gates(u, w, bias, lam):
     blocks, _, bw = w.shape
     ub = u.float().view(-1, blocks, bw)
@@ -48,6 +56,8 @@ def rglru_gates(u, w, bias, lam):
 def stream_step(m: SeqBatch, dim: int, eps: float = 0.0, alpha: float = 1.0, ids=None, table=None, x=None, y=None,
                 w=None, mu=None, prev=None, save=None, want_x: bool = True, want_h: bool = True, act=None):
     act = act or (table if ids is not None else y).dtype
+    if y is not None and y.dim() == 3:
+        y = y.sum(0)
     if ids is not None:
         xo = table[ids.long()].float()
     else:
