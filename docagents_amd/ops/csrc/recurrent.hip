@@ -11,7 +11,8 @@
 // and leaves its end state and its total decay, (b) one pass over the chunks turns those into each
 // chunk's start state, (c) every chunk runs again from its start state and writes its outputs. Chunks of
 // all portions fill the chip, and a token's arithmetic differs between the two ways by rounding only.
-// The convolution's state is replaced by the recurrence's launch: its own launch still reads it.
+// The convolution's state is replaced by the recurrence's launch, as its own launch still reads it (in
+// batches of single tokens a thread's reads are its own: there the convolution replaces it).
 #include "seq.h"
 
 struct ConvState {
@@ -23,21 +24,30 @@ struct ConvState {
 // portion is shorter; one thread per channel, old entries are read before they are overwritten).
 template <typename T>
 __device__ __forceinline__ void conv_state_store(const ConvState& s, const SeqMeta& m, int b, int c) {
+  if (!s.state) return;
   const int s0 = m.cu[b], n = m.cu[b + 1] - s0, keep = s.taps - 1;
   const bool start = m.pos0[b] == 0;
   T* st = (T*)s.state + (size_t)m.slot[b] * keep * s.C + c;
   const T* x = (const T*)s.x + c;
-  for (int i = 0; i < keep; ++i) {
-    const int j = n - keep + i;
-    st[(size_t)i * s.C] = j >= 0 ? x[(size_t)(s0 + j) * s.ldx]
-                                 : (start ? Act<T>::from_f(0.f) : st[(size_t)(i + n) * s.C]);
+  constexpr int U = 4;
+  for (int i0 = 0; i0 < keep; i0 += U) {
+    T v[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int i = min(i0 + u, keep - 1), j = n - keep + i;
+      v[u] = j >= 0 ? x[(size_t)(s0 + j) * s.ldx] : (start ? Act<T>::from_f(0.f) : st[(size_t)(i + n) * s.C]);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (i0 + u < keep) st[(size_t)(i0 + u) * s.C] = v[u];
   }
 }
 
 // ------------------------------------------------------------------------------- convolution
 struct ConvArgs {
-  const void* x; const float* w; const float* bias; const void* state; void* y;  // w [taps][C]
+  const void* x; const float* w; const float* bias; void* state; void* y;  // w [taps][C]
   int ldx, ldy, C, taps;
+  int update;  // single tokens only: replace the state
   SeqMeta m;
 };
 
@@ -60,7 +70,7 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
   auto emit = [&](int t, f32x4_t v) {
     if constexpr (SILU) {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] = silu32(v[e]);
+      for (int e = 0; e < 4; ++e) v[e] = act_silu<T>(v[e]);
     }
     Act<T>::store4((T*)a.y + (size_t)t * a.ldy + c, v);
   };
@@ -91,6 +101,11 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
           for (int e = 0; e < 4; ++e) v[e] = fmaf(w[k][e], x[i + k][e], v[e]);
         emit(t0 + i, v);
       }
+      if (CONV_RUN == 1 && a.update) {
+        T* w0 = (T*)a.state + (size_t)a.m.slot[b0] * (TAPS - 1) * a.C + c;
+#pragma unroll
+        for (int i = 0; i + 1 < TAPS; ++i) Act<T>::store4(w0 + (size_t)i * a.C, x[i + 1]);
+      }
     } else {  // a portion ends inside the run
       for (int t = t0; t < t1; ++t) {
         f32x4_t v = bias;
@@ -113,6 +128,11 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
         for (int e = 0; e < 4; ++e) v[e] = fmaf(w[e], x[e], v[e]);
       }
       emit(t, v);
+      if (a.update) {
+        T* st = (T*)a.state + (size_t)a.m.slot[a.m.seq[t]] * (a.taps - 1) * a.C + c;
+        for (int k = a.taps - 2; k >= 0; --k)  // oldest first
+          Act<T>::store4(st + (size_t)(a.taps - 2 - k) * a.C, conv_input<T>(a, t, k, c));
+      }
     }
   }
 }
@@ -133,15 +153,17 @@ static int launch_conv(const ConvArgs& a, int silu, hipStream_t s) {
   DA_LAUNCH_CHECK();
 }
 
-DA_EXPORT int da_causal_conv(const void* x, int ldx, const void* w, const void* bias, const void* state, void* y,
+// max_len: longest portion; batches of single tokens (max_len == 1) also replace the state.
+DA_EXPORT int da_causal_conv(const void* x, int ldx, const void* w, const void* bias, void* state, void* y,
                              int ldy, int C, int taps, int silu, int max_len, const void* cu, const void* slot, const void* pos0,
                              const void* seq, int T, int B, int f32, void* stream) {
-  if (T < 1 || B < 1 || C < 4 || C % 4 || ldx % 4 || ldy % 4 || taps < 1 || (T + 3) / 4 > 65535 * 8)
+  if (T < 1 || B < 1 || C < 4 || C % 4 || ldx % 4 || ldy % 4 || taps < 1 || max_len < 1 ||
+      (T + 3) / 4 > (max_len == 1 ? 65535 : 65535 * 8))
     return (int)hipErrorInvalidValue;
-  ConvArgs a{x, (const float*)w, (const float*)bias, state, y, ldx, ldy, C, taps,
+  ConvArgs a{x, (const float*)w, (const float*)bias, state, y, ldx, ldy, C, taps, max_len == 1,
              SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B}};
   hipStream_t s = (hipStream_t)stream;
-  if (max_len == 1 && T < 4096) return f32 ? launch_conv<float, 1>(a, silu, s) : launch_conv<bf16_t, 1>(a, silu, s);
+  if (max_len == 1) return f32 ? launch_conv<float, 1>(a, silu, s) : launch_conv<bf16_t, 1>(a, silu, s);
   return f32 ? launch_conv<float, 8>(a, silu, s) : launch_conv<bf16_t, 8>(a, silu, s);
 }
 
@@ -171,13 +193,12 @@ struct SelArgs {
   const float* A; const float* D;                                 // A [C][N] = log2(e) * (negative rates)
   float* state; void* y;                                          // state [slots][C][N]
   float* chunk_state; float* chunk_dt;                            // [chunks + B][C][N], [chunks + B][C]
-  int ldx, lddt, ldbc, ldz, ldy, offB, offC, C, N, lanes;         // lanes of a channel (power of two)
+  int ldx, lddt, ldbc, ldz, ldy, offB, offC, C, N;
+  int lanes, tile;                                                // lanes of a channel (power of two)
   ConvState conv;
   SeqMeta m;
   ChunkMeta ch;
 };
-
-constexpr int SEL_TT = 16;  // tokens whose B, C rows are staged together
 
 // NS consecutive floats n0 .. of a row of N, zero past its end (vector accesses where rows are 16-byte aligned).
 template <int NS>
@@ -207,10 +228,12 @@ __device__ __forceinline__ void row_store(float* p, const float (&v)[NS], int n0
   }
 }
 
-// A channel's N states live in `lanes` neighbouring lanes, NS each. Dynamic LDS: SEL_TT rows of B | C.
+// A channel's N states live in `lanes` neighbouring lanes, NS each. B and C rows are staged `tile` tokens at a time in dynamic LDS
+// ([tile][2][lanes * NS] fp32); the step sizes, inputs and gates of the next U tokens are in flight while
+// the current ones are added.
 template <typename T, int NS, int PHASE>
 __global__ void __launch_bounds__(256) sel_scan_kernel(SelArgs a) {
-  extern __shared__ float sbc[];  // [SEL_TT][2][lanes * NS]
+  extern __shared__ __attribute__((aligned(16))) float sbc[];
   const ScanSpan sp = scan_span<PHASE>(a.m, a.ch, blockIdx.y);
   if (sp.idle) return;
   const int G = a.lanes, NP = G * NS, cpb = 256 / G;
@@ -236,41 +259,64 @@ __global__ void __launch_bounds__(256) sel_scan_kernel(SelArgs a) {
   const T* zp = (const T*)a.z + cc;
   const float* dp = a.dt + cc;
   constexpr int U = 4;
-  for (int tb = sp.t0; tb < sp.t1; tb += SEL_TT) {
-    const int nt = min(SEL_TT, sp.t1 - tb);
+  float dt[U], x[U], z[U];
+  auto fetch = [&](int t) {  // tokens past the span change nothing: step size and input 0
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const size_t tt = min(t + u, sp.t1 - 1);
+      const float in = t + u < sp.t1 ? 1.f : 0.f;
+      dt[u] = dp[tt * a.lddt] * in;
+      x[u] = Act<T>::to_f(xp[tt * a.ldx]) * in;
+      z[u] = PHASE == SCAN_LOCAL ? 0.f : Act<T>::to_f(zp[tt * a.ldz]);
+    }
+  };
+  fetch(sp.t0);
+  for (int tb = sp.t0; tb < sp.t1; tb += a.tile) {  // tile % U == 0
+    const int nt = min(a.tile, (sp.t1 - tb + U - 1) / U * U);
     __syncthreads();
     for (int i = threadIdx.x; i < nt * 2 * NP; i += 256) {
       const int r = i / (2 * NP), q = i % (2 * NP), n = q % NP;
-      sbc[i] = n < a.N ? Act<T>::to_f(((const T*)a.bc)[(size_t)(tb + r) * a.ldbc + (q < NP ? a.offB : a.offC) + n]) : 0.f;
+      const size_t t = min(tb + r, sp.t1 - 1);
+      sbc[i] = n < a.N ? Act<T>::to_f(((const T*)a.bc)[t * a.ldbc + (q < NP ? a.offB : a.offC) + n]) : 0.f;
     }
     __syncthreads();
     for (int r0 = 0; r0 < nt; r0 += U) {
-      float dt[U], x[U], z[U];
+      float d_[U], x_[U], z_[U], y[U];
 #pragma unroll
       for (int u = 0; u < U; ++u) {
-        const size_t t = tb + min(r0 + u, nt - 1);
-        dt[u] = dp[t * a.lddt];
-        x[u] = Act<T>::to_f(xp[t * a.ldx]);
-        z[u] = PHASE == SCAN_LOCAL ? 0.f : Act<T>::to_f(zp[t * a.ldz]);
+        d_[u] = dt[u];
+        x_[u] = x[u];
+        z_[u] = z[u];
       }
+      fetch(tb + r0 + U);
+      // straight-line over the U tokens: their exponentials and LDS reads overlap the states' chains
 #pragma unroll
       for (int u = 0; u < U; ++u) {
-        if (r0 + u >= nt) break;
         const float* br = sbc + (r0 + u) * 2 * NP + n0;
-        const float dx = dt[u] * x[u];
-        float y = 0.f;
+        const float dx = d_[u] * x_[u];
+        y[u] = 0.f;
 #pragma unroll
-        for (int i = 0; i < NS; ++i) {
-          S[i] = fmaf(__builtin_amdgcn_exp2f(dt[u] * A[i]), S[i], dx * br[i]);
-          if constexpr (PHASE != SCAN_LOCAL) y = fmaf(S[i], br[NP + i], y);
+        for (int i = 0; i < NS; i += 4) {
+          const f32x4_t B = *(const f32x4_t*)(br + i);
+          f32x4_t C{0.f, 0.f, 0.f, 0.f};
+          if constexpr (PHASE != SCAN_LOCAL) C = *(const f32x4_t*)(br + NP + i);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            S[i + e] = fmaf(__builtin_amdgcn_exp2f(d_[u] * A[i + e]), S[i + e], dx * B[e]);
+            if constexpr (PHASE != SCAN_LOCAL) y[u] = fmaf(S[i + e], C[e], y[u]);
+          }
         }
-        if constexpr (PHASE == SCAN_LOCAL) {
-          sdt += dt[u];
-        } else {
-          for (int o = 1; o < G; o <<= 1) y += __shfl_xor(y, o, 64);
-          if (live && g == 0)
-            ((T*)a.y)[(size_t)(tb + r0 + u) * a.ldy + c] = Act<T>::from_f(fmaf(Dc, x[u], y) * silu32(z[u]));
-        }
+        sdt += d_[u];
+      }
+      if constexpr (PHASE != SCAN_LOCAL) {
+        for (int o = 1; o < G; o <<= 1)
+#pragma unroll
+          for (int u = 0; u < U; ++u) y[u] += __shfl_xor(y[u], o, 64);
+        if (live && g == 0)
+#pragma unroll
+          for (int u = 0; u < U; ++u)
+            if (tb + r0 + u < sp.t1)
+              ((T*)a.y)[(size_t)(tb + r0 + u) * a.ldy + c] = Act<T>::from_f(fmaf(Dc, x_[u], y[u]) * act_silu<T>(z_[u]));
       }
     }
   }
@@ -317,7 +363,7 @@ template <typename T, int NS>
 static int launch_sel(const SelArgs& a, hipStream_t s) {
   const int cpb = 256 / a.lanes;
   const unsigned gx = (a.C + cpb - 1) / cpb;
-  const size_t lds = (size_t)SEL_TT * 2 * a.lanes * NS * 4;
+  const size_t lds = (size_t)a.tile * 2 * a.lanes * NS * 4;
   if (a.ch.n == 0) {
     sel_scan_kernel<T, NS, SCAN_DIRECT><<<dim3(gx, a.m.B), 256, lds, s>>>(a);
   } else {
@@ -343,8 +389,9 @@ DA_EXPORT int da_selective_scan(const void* x, int ldx, const void* dt, int lddt
   const int ns = N <= 4 || (max_len <= 4 && N <= 256) ? 4 : 8;
   int lanes = 1;
   while (lanes * ns < N) lanes *= 2;
+  const int tile = min(64, max(16, 2048 / (lanes * ns)));  // at most 64 KB of LDS
   SelArgs a{x, (const float*)dt, bc, z, (const float*)A, (const float*)D, (float*)state, y, (float*)chunk_state,
-            (float*)chunk_dt, ldx, lddt, ldbc, ldz, ldy, offB, offC, C, N, lanes,
+            (float*)chunk_dt, ldx, lddt, ldbc, ldz, ldy, offB, offC, C, N, lanes, tile,
             ConvState{conv_x, ld_conv, conv_state, taps, C},
             SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B},
             ChunkMeta{(const int*)ck, (const int*)base, n_chunks, chunk}};
@@ -378,8 +425,8 @@ __global__ void __launch_bounds__(256) gru_scan_kernel(GruArgs a) {
     if constexpr (PHASE == SCAN_LOCAL) a.chunk_state[chunk_row(a.ch, sp.b, 0) * a.C + c] = s;
   }
   constexpr int U = 8;
-  for (int t0 = sp.t0; t0 < sp.t1; t0 += U) {
-    float d[U], v[U], g[U];
+  float d[U], v[U], g[U];
+  auto fetch = [&](int t0) {
 #pragma unroll
     for (int u = 0; u < U; ++u) {
       const size_t t = min(t0 + u, sp.t1 - 1);
@@ -387,13 +434,23 @@ __global__ void __launch_bounds__(256) gru_scan_kernel(GruArgs a) {
       v[u] = a.drive[t * a.C + c];
       g[u] = PHASE == SCAN_LOCAL ? 0.f : Act<T>::to_f(((const T*)a.gate)[t * a.ldg + c]);
     }
+  };
+  fetch(sp.t0);
+  for (int t0 = sp.t0; t0 < sp.t1; t0 += U) {
+    float o[U];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
-      if (t0 + u >= sp.t1) break;
-      s = fmaf(d[u], s, v[u]);
-      if constexpr (PHASE == SCAN_LOCAL) p *= d[u];
-      else ((T*)a.y)[(size_t)(t0 + u) * a.ldy + c] = Act<T>::from_f(s * gelu_tanh32(g[u]));
+      if (t0 + u < sp.t1) {
+        s = fmaf(d[u], s, v[u]);
+        if constexpr (PHASE == SCAN_LOCAL) p *= d[u];
+      }
+      o[u] = s * act_gelu_tanh<T>(g[u]);
     }
+    if (t0 + U < sp.t1) fetch(t0 + U);
+    if constexpr (PHASE != SCAN_LOCAL)
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+        if (t0 + u < sp.t1) ((T*)a.y)[(size_t)(t0 + u) * a.ldy + c] = Act<T>::from_f(o[u]);
   }
   if constexpr (PHASE == SCAN_LOCAL) {
     const size_t row = chunk_row(a.ch, sp.b, sp.k + 1);

@@ -80,7 +80,16 @@ __device__ __forceinline__ float one_minus_exp32(float y) {
   return y > -0.4f ? -y * p : 1.f - exp32(y);
 }
 __device__ __forceinline__ float silu32(float x) { return x * sigmoid32(x); }
+// The same for outputs that are rounded to the activation type anyway: bf16 takes the short forms.
+template <typename T> __device__ __forceinline__ float act_silu(float x) {
+  if constexpr (sizeof(T) == 2) return silu(x);
+  else return silu32(x);
+}
 __device__ __forceinline__ float gelu_tanh32(float x) {
   // 0.5 (1 + tanh(z)) = sigmoid(2 z)
   return x * sigmoid32(1.5957691216057308f * (x + 0.044715f * x * x * x));
+}
+template <typename T> __device__ __forceinline__ float act_gelu_tanh(float x) {
+  if constexpr (sizeof(T) == 4) return gelu_tanh32(x);
+  return x * __builtin_amdgcn_rcpf(1.f + __expf(-1.5957691216057308f * (x + 0.044715f * x * x * x)));
 }

@@ -22,7 +22,7 @@ enum StreamSrc : int { SRC_EMBED = 0, SRC_Y = 1, SRC_PARTIALS = 2 };
 
 // A thread holds NCH 4-column pieces of a row. The next row's loads are issued before this row's sum.
 template <typename T, int NCH, int SRC>
-__global__ void __launch_bounds__(256) stream_kernel(StreamArgs a) {
+__global__ void __launch_bounds__(NCH == 1 ? 1024 : 256) stream_kernel(StreamArgs a) {
   __shared__ float red[16];
   const int nt = blockDim.x, nc = a.Dp / 4;
   f32x4_t nx[NCH], cur[NCH], prv[NCH];
@@ -30,29 +30,34 @@ __global__ void __launch_bounds__(256) stream_kernel(StreamArgs a) {
   auto col = [&](int i) { return (int)threadIdx.x + i * nt; };  // this thread's i-th piece
   auto fetch = [&](int t) {  // alpha x + y of row t (embedding: the row itself) into nx
     const size_t src = SRC == SRC_EMBED ? min(max(a.ids[t], 0), a.vocab - 1) : t;
+    if constexpr (SRC == SRC_PARTIALS) {
+#pragma unroll
+      for (int i = 0; i < NCH; ++i) nx[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      constexpr int U = NCH <= 2 ? 8 : 4;  // partials of every piece in flight together
+      const size_t st = (size_t)a.m.T * a.Dp;
+      for (int s0 = 0; s0 < a.splits; s0 += U) {
+        f32x4_t v[U][NCH];
+#pragma unroll
+        for (int s = 0; s < U; ++s)
+#pragma unroll
+          for (int i = 0; i < NCH; ++i)
+            v[s][i] = *(const f32x4_t*)((const float*)a.y + min(s0 + s, a.splits - 1) * st + src * a.Dp +
+                                        min(col(i), nc - 1) * 4);
+#pragma unroll
+        for (int s = 0; s < U; ++s)
+#pragma unroll
+          for (int i = 0; i < NCH; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) nx[i][e] += s0 + s < a.splits ? v[s][i][e] : 0.f;
+      }
+    }
 #pragma unroll
     for (int i = 0; i < NCH; ++i) {
       const int c = min(col(i), nc - 1) * 4;
       if constexpr (SRC == SRC_EMBED) {
         nx[i] = Act<T>::load4((const T*)a.table + src * a.Dp + c);
       } else {
-        f32x4_t y;
-        if constexpr (SRC == SRC_Y) {
-          y = Act<T>::load4((const T*)a.y + src * a.Dp + c);
-        } else {
-          y = f32x4_t{0.f, 0.f, 0.f, 0.f};
-          const float* p = (const float*)a.y + src * a.Dp + c;
-          const size_t st = (size_t)a.m.T * a.Dp;
-          for (int s0 = 0; s0 < a.splits; s0 += 4) {
-            f32x4_t v[4];
-#pragma unroll
-            for (int s = 0; s < 4; ++s) v[s] = *(const f32x4_t*)(p + min(s0 + s, a.splits - 1) * st);
-#pragma unroll
-            for (int s = 0; s < 4; ++s)
-#pragma unroll
-              for (int e = 0; e < 4; ++e) y[e] += s0 + s < a.splits ? v[s][e] : 0.f;
-          }
-        }
+        const f32x4_t y = SRC == SRC_Y ? Act<T>::load4((const T*)a.y + src * a.Dp + c) : nx[i];
         const f32x4_t x = *(const f32x4_t*)(a.x + src * a.Dp + c);
 #pragma unroll
         for (int e = 0; e < 4; ++e) nx[i][e] = fmaf(a.alpha, x[e], y[e]);
@@ -150,7 +155,8 @@ stream_final_kernel(const float* __restrict__ x, const long long* __restrict__ r
 template <typename T, int SRC>
 static int launch_stream(const StreamArgs& a, hipStream_t s) {
   const int nc = a.Dp / 4;
-  const int nt = nc >= 256 ? 256 : (nc + 63) / 64 * 64;
+  // few rows: a row over as many threads as it has pieces (latency); else 256 threads a row
+  const int most = a.m.T <= 512 ? 1024 : 256, nt = nc >= most ? (nc > 1024 ? 256 : most) : (nc + 63) / 64 * 64;
   const int nch = (nc + nt - 1) / nt;
   const dim3 grid((a.m.T + a.rows - 1) / a.rows), block(nt);
   if (nch <= 1) stream_kernel<T, 1, SRC><<<grid, block, 0, s>>>(a);

@@ -32,7 +32,7 @@ class SeqBatch:
     def on(self, table) -> "SeqBatch":
         return replace(self, table=table)
 
-    def chunk_len(self, waves: int, fill: int = 2048) -> int:
+    def chunk_len(self, waves: int, fill: int) -> int:
         """Tokens per chunk of a recurrence whose portions take ``waves`` waves each when walked from end to
         end: as long as the chip is filled (``fill`` waves); 0 when the portions alone do that, or are short."""
         if self.max_len <= CHUNK:

@@ -54,10 +54,10 @@ def _meta(m: SeqBatch):
     return [_ptr(m.cu), _ptr(m.slot), _ptr(m.pos0), _ptr(m.seq), m.T, m.B]
 
 
-def _scratch(m: SeqBatch, waves: int, device, *shapes):
+def _scratch(m: SeqBatch, waves: int, fill: int, device, *shapes):
     """Arguments of a chunked recurrence: fp32 scratch [chunks + B, *shape] each, the chunk list, its length and
     the chunk length (no scratch and no chunks where the portions are walked from end to end)."""
-    n = m.chunk_len(waves)
+    n = m.chunk_len(waves, fill)
     if n == 0:
         return [], [None] * len(shapes) + [None, None, 0, 0]
     ck, base, tot = m.chunks(n)
@@ -171,7 +171,8 @@ def stream_final(x, w, eps: float, dim: int, act, rows=None):
 
 def causal_conv(x, w, bias, state, m: SeqBatch, silu: bool):
     """Per-channel causal convolution over each portion: x [T, C] (row view), w fp32 [taps, C] (last row: the
-    current token), bias fp32 [C], state [slots, taps - 1, C] (read only; the recurrence replaces it)."""
+    current token), bias fp32 [C], state [slots, taps - 1, C]: the inputs before the portion, replaced here in batches of single tokens and
+    by the recurrence's op otherwise."""
     f32 = _act(x, "x")
     taps, C = w.shape
     _f32(w, "w")
@@ -184,10 +185,12 @@ def causal_conv(x, w, bias, state, m: SeqBatch, silu: bool):
     return y
 
 
-def _conv_args(conv_x, conv_state, C, dtype):
+def _conv_args(conv_x, conv_state, C, dtype, m: SeqBatch):
+    """The recurrence replaces the convolution's state, except where the convolution did (single tokens)."""
     _act(conv_x, "conv_x", dtype)
     _req(conv_state.dtype == dtype and conv_state.is_contiguous() and conv_state.shape[2] == C, "conv state")
-    return [_ptr(conv_x), conv_x.stride(0), _ptr(conv_state), conv_state.shape[1] + 1]
+    keep = conv_state.shape[1]
+    return [_ptr(conv_x), conv_x.stride(0), _ptr(conv_state) if keep and m.max_len > 1 else None, keep + 1]
 
 
 def selective_scan(x, dt, bc, off_b: int, off_c: int, z, A, D, state, conv_x, conv_state, m: SeqBatch):
@@ -203,10 +206,10 @@ def selective_scan(x, dt, bc, off_b: int, off_c: int, z, A, D, state, conv_x, co
     _req(x.shape == (m.T, C) and z.shape == (m.T, C) and state.shape[1:] == (C, N) and N <= 512
          and max(off_b, off_c) + N <= bc.shape[1] and bc.shape[0] == m.T, "selective_scan shapes")
     y = torch.empty((m.T, C), dtype=x.dtype, device=x.device)
-    ws, chunk = _scratch(m, C * -(-N // 8) // 64, x.device, (C, N), (C,))
+    ws, chunk = _scratch(m, C * -(-N // 8) // 64, 2048, x.device, (C, N), (C,))
     _check(lib().da_selective_scan(_ptr(x), x.stride(0), _ptr(dt), C, _ptr(bc), bc.stride(0), off_b, off_c, _ptr(z),
                                    z.stride(0), _ptr(A), _ptr(D), _ptr(state), _ptr(y), C, C, N,
-                                   *_conv_args(conv_x, conv_state, C, x.dtype), *chunk, m.max_len, *_meta(m), f32,
+                                   *_conv_args(conv_x, conv_state, C, x.dtype, m), *chunk, m.max_len, *_meta(m), f32,
                                    _stream()), "selective_scan")
     del ws
     return y
@@ -221,9 +224,9 @@ def gated_scan(decay, drive, gate, state, conv_x, conv_state, m: SeqBatch):
         _f32(t, n, k)
     _req(gate.shape == (m.T, C), "gate [T, C]")
     y = torch.empty((m.T, C), dtype=gate.dtype, device=gate.device)
-    ws, chunk = _scratch(m, C // 64, gate.device, (C,), (C,))
+    ws, chunk = _scratch(m, C // 64, 16384, gate.device, (C,), (C,))
     _check(lib().da_gated_scan(_ptr(decay), _ptr(drive), _ptr(gate), gate.stride(0), _ptr(state), _ptr(y), C, C,
-                               *_conv_args(conv_x, conv_state, C, gate.dtype), *chunk, *_meta(m), f32, _stream()),
+                               *_conv_args(conv_x, conv_state, C, gate.dtype, m), *chunk, *_meta(m), f32, _stream()),
            "gated_scan")
     del ws
     return y
