@@ -247,6 +247,35 @@ def random_weights(cfg: HybridConfig, device="cpu", seed: int = 0) -> dict[str, 
     return out
 
 
+def layer_states(cfg: HybridConfig, act=torch.bfloat16) -> list[LayerState]:
+    """What every layer keeps per sequence: its mixer's state and the token shift's previous row."""
+    shift = {"shift": ((_up(cfg.hidden),), torch.float32)}
+    per = [MIXERS[type(s.mixer)].state(s.mixer, act) for s in cfg.spec]
+    return [LayerState({**p.slot, **shift}, p.page) for p in per]
+
+
+def cache_bytes(cfg: HybridConfig, slots: int, max_seq: int, act=torch.bfloat16) -> int:
+    return StateCache.bytes_for(layer_states(cfg, act), slots, min(max_seq, cfg.max_pos))
+
+
+def decode_workspace_bytes(cfg: HybridConfig, max_batch: int) -> int:
+    """Split-K partials of the decode-sized products: up to 8 splits of the widest, or 256 tiles of 64 x 128."""
+    widest = max(max(v[0] for v in tensor_shapes(cfg).values()), 2 * max(s.ff for s in cfg.spec))
+    return max(64 << 20, 8 * max_batch * _up(widest) * 4)
+
+
+def prefill_bytes_per_token(cfg: HybridConfig) -> int:
+    """Activations of the widest layer while it runs: stream (fp32, two of it), its input and output, and the
+    mixer's or the feed-forward's intermediates."""
+    def mixer(m):
+        if isinstance(m, GatedRecurrence):
+            return RecurrenceMixer.padded(m)[1] * (2 * 2 + 2 + 2 * 4 + 2)
+        if isinstance(m, SelectiveScan):
+            return _up(m.inner) * (2 * 2 + 2 + 4 + 2) + 2 * _up(m.dt_rank + 2 * m.state)
+        return AttentionMixer.padded(m) * 2 * (2 * m.heads + m.kv_heads)
+    return 12 * _up(cfg.hidden) + max(max(mixer(s.mixer), 2 * _up(s.ff)) for s in cfg.spec)
+
+
 class _Layer:
     """One layer's packed weights (shared by the layers that use them)."""
 
@@ -305,23 +334,16 @@ class HybridDecoder:
             raise ValueError(f"{self.cfg.name}: missing tensors {missing[:4]}, wrong shapes {bad[:4]}")
 
     # ------------------------------------------------------------- state
-    def layer_states(self) -> list[LayerState]:
-        shift = {"shift": ((self.hp,), torch.float32)}
-        per = [MIXERS[type(s.mixer)].state(s.mixer, self.act) for s in self.cfg.spec]
-        return [LayerState({**p.slot, **shift}, p.page) for p in per]
-
     def alloc_cache(self, slots: int, max_seq: int, tokens: int | None = None) -> StateCache:
-        self.cache = StateCache(self.layer_states(), slots, min(max_seq, self.cfg.max_pos), self.device, tokens)
+        self.cache = StateCache(layer_states(self.cfg, self.act), slots, min(max_seq, self.cfg.max_pos), self.device,
+                                tokens)
         return self.cache
 
     def cache_bytes(self, slots: int, max_seq: int) -> int:
-        return StateCache.bytes_for(self.layer_states(), slots, min(max_seq, self.cfg.max_pos))
+        return cache_bytes(self.cfg, slots, max_seq, self.act)
 
     def workspace_bytes(self, max_batch: int, max_seq: int) -> int:
-        """Split-K partials of the decode-sized products (16 splits of one 128-column tile row at most)."""
-        widest = max([self.head.w.shape[0]] + [L.gate_up.w.shape[0] for L in self.layers if L.gate_up]
-                     + [L.mixer.proj.w.shape[0] for L in self.layers])
-        return max(64 << 20, 8 * max_batch * widest * 4)
+        return decode_workspace_bytes(self.cfg, max_batch)
 
     # ------------------------------------------------------------- step
     def _forward(self, m: SeqBatch, ids) -> torch.Tensor:

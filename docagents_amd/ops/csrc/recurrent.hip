@@ -386,7 +386,7 @@ DA_EXPORT int da_selective_scan(const void* x, int ldx, const void* dt, int lddt
     return (int)hipErrorInvalidValue;
   if (n_chunks && (!ck || !base || !chunk_state || !chunk_dt)) return (int)hipErrorInvalidValue;
   // single tokens: four states a lane, so the states' rows are read and written in whole lines
-  const int ns = N <= 4 || (max_len <= 4 && N <= 256) ? 4 : 8;
+  const int ns = N <= 4 || (max_len <= 4 && N <= 256 && B < 16) ? 4 : 8;
   int lanes = 1;
   while (lanes * ns < N) lanes *= 2;
   const int tile = min(64, max(16, 2048 / (lanes * ns)));  // at most 64 KB of LDS

@@ -31,7 +31,7 @@ from __future__ import annotations
 
 from dataclasses import dataclass
 
-from ..models.configs import DecoderConfig, EncoderConfig, decoder_config, encoder_config
+from ..models.configs import DecoderConfig, EncoderConfig, HybridConfig, decoder_config, encoder_config
 
 GB = 1e9
 HBM_BYTES = 288 * GB
@@ -45,6 +45,8 @@ TP70B_WORLD = 8              # tp_decode_70b runs at N = 8 (L
 def decoder_weight_bytes(cfg: DecoderConfig, tp: int = 1) -> int:
     """bf16 bytes of one TP rank's decoder weights as ``random_weights`` / ``shard_weights`` lay them
     out: the embedding table whole on every rank, lm_head and every projection split ``tp`` ways."""
+    if isinstance(cfg, HybridConfig):
+        return 2 * cfg.param_count()
     h, d = cfg.hidden, cfg.head_dim
     proj = h * (cfg.heads + 2 * cfg.kv_heads) * d + cfg.heads * d * h + 3 * h * cfg.ffn
     per_layer = proj // tp + 2 * h
@@ -52,16 +54,25 @@ def decoder_weight_bytes(cfg: DecoderConfig, tp: int = 1) -> int:
 
 
 def kv_bytes(cfg: DecoderConfig, slots: int, max_seq: int, tp: int = 1) -> int:
+    if isinstance(cfg, HybridConfig):
+        from ..models.hybrid import cache_bytes
+        return cache_bytes(cfg, slots, max_seq)
     from ..models.llama import KVCache
     return KVCache.bytes_for(cfg, slots, min(max_seq, cfg.max_pos), tp)
 
 
 def workspace_bytes(cfg: DecoderConfig, max_batch: int, max_seq: int, tp: int = 1) -> int:
+    if isinstance(cfg, HybridConfig):
+        from ..models.hybrid import decode_workspace_bytes
+        return decode_workspace_bytes(cfg, max_batch)
     from ..engine.generator import Generator
     return Generator.workspace_bytes(cfg, cfg.heads // tp, tp, max_batch, min(max_seq, cfg.max_pos))
 
 
 def prefill_transient_bytes(cfg: DecoderConfig, tp: int = 1, tokens: int = MAX_PREFILL_TOKENS) -> int:
+    if isinstance(cfg, HybridConfig):
+        from ..models.hybrid import prefill_bytes_per_token
+        return tokens * prefill_bytes_per_token(cfg)
     h, d = cfg.hidden, cfg.head_dim
     per_tok = 3 * h + (cfg.heads + 2 * cfg.kv_heads) * d // tp + cfg.heads * d // tp + 2 * cfg.ffn // tp
     return 2 * tokens * per_tok

@@ -616,6 +616,18 @@ def test_registry_and_configuration(tmp_path):
         make_decoder(decoder_config("tiny-dec"), "cpu", dtype="fp32")
 
 
+def test_hbm_plan_prices_the_allocations():
+    from docagents_amd.models.hybrid import HybridDecoder
+    from docagents_amd.parallel import hbm_plan as HP
+    cfg = decoder_config("tiny-binupel")
+    m = HybridDecoder(cfg, "cpu")
+    c = m.alloc_cache(5, 300)
+    held = sum(t.numel() * t.element_size() for layer in c.layers for t in layer.values())
+    assert HP.kv_bytes(cfg, 5, 300) == held == m.cache_bytes(5, 300)
+    plan = HP.bench_plan(HP.BenchArgs(llm="binupel-9b", batch=64), 1)
+    assert HP.check(plan) == [] and plan["headline"]["decoder_weights"] == 2 * decoder_config("binupel-9b").param_count()
+
+
 def test_checkpoint_reading(tmp_path):
     from safetensors.torch import save_file
     w = {"a": rand(1, 3, 5).bfloat16(), "b": rand(2, 7), "c": torch.arange(4, dtype=torch.int32)}

@@ -9,15 +9,15 @@ pytestmark = pytest.mark.gpu
 
 from docagents_amd.engine.generator import Generator  # noqa: E402
 from docagents_amd.models.configs import decoder_config  # noqa: E402
-from docagents_amd.models.llama import LlamaDecoder  # noqa: E402
+from docagents_amd.models import make_decoder  # noqa: E402
 from docagents_amd.ops import streams as S  # noqa: E402
 
 
-@pytest.mark.parametrize("arch,n,plen", [("tiny-dec", 8, 300), ("phi3-mini", 4, 700)])
+@pytest.mark.parametrize("arch,n,plen", [("tiny-dec", 8, 300), ("phi3-mini", 4, 700), ("tiny-binupel", 8, 300)])
 def test_overlapped_waves_match_sequential(arch, n, plen):
     dev = torch.device("cuda", 0)
     cfg = decoder_config(arch)
-    m = LlamaDecoder(cfg, dev, seed=0)
+    m = make_decoder(cfg, dev, seed=0)
     m.alloc_cache(2 * n + 4, 2048)
     gen = Generator(m, max_batch=n, max_seq=2048, temperature=0.2, seed=3, eos=())
     rng = np.random.default_rng(0)
