@@ -91,6 +91,7 @@ class Config:
     # Python GIL switch interval of the engine process (ms; 0 = interpreter default 5 ms). 0.5 ms
     # measured no better for the query path under load (profiles/r3/stack/*switch*)
     engine_switch_interval_ms: float = field(default=0.0, metadata={"env": "ENGINE_SWITCH_INTERVAL_MS"})
+    engine_prefill_chunk: int = field(default=-1, metadata={"env": "ENGINE_PREFILL_CHUNK"})  # -1 -> the model's; 0 off
     engine_admit_tokens: int = field(default=0, metadata={"env": "ENGINE_ADMIT_TOKENS"})  # 0 -> 4 prefill chunks
     # grouped admission under load (engine/server.py _admit_ready): while >= ENGINE_ADMIT_HOLD_FRAC of
     # the decode rows are busy, arrivals wait until ENGINE_ADMIT_MIN of them (or the free rows) are

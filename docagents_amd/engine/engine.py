@@ -253,7 +253,8 @@ class Engine:
             from .generator import ContinuousScheduler
             self._sched = ContinuousScheduler(self.gen, B=self.gen.max_batch,
                                               max_new_cap=max(self.max_new_tokens, self.summary_max_new),
-                                              max_admit_tokens=getattr(self, "admit_tokens", None))
+                                              max_admit_tokens=getattr(self, "admit_tokens", None),
+                                              prefill_chunk=getattr(self, "prefill_chunk", None))
         return self._sched
 
     def cb_tick(self, new_items, steps: int | None = None, stop=None):

@@ -19,6 +19,7 @@ import torch
 
 from ..models.llama import DecodeState, decode_workspace_bytes, pack_prompts
 from ..ops import h2d
+from ..ops.seq_batch import pack_batch
 
 
 def _bucket(n: int) -> int:
@@ -450,12 +451,20 @@ class ContinuousScheduler:
     stop fires after exactly m tokens with no kernel change. Free rows point at the generator's
     dummy KV slot and stay inactive (the sampler never advances them).
 
+    Models whose step takes any portions of sequences (``portion_steps``) admit a prompt longer than
+    ``prefill_chunk`` tokens portion by portion: while one is being filled, a tick is one mixed step
+    of at most prefill_chunk prompt tokens beside one token of every decoding row, so a long prompt
+    delays the running rows by a portion, not by its whole prefill.
+
     Not thread-safe: ``submit`` and ``tick`` are called from the engine's single GPU thread.
     """
 
     def __init__(self, gen: "Generator", B: int | None = None, max_new_cap: int = 256, chunk_steps: int = 8,
-                 max_admit_tokens: int | None = None, max_heads: int = 2):
+                 max_admit_tokens: int | None = None, max_heads: int = 2, prefill_chunk: int | None = None):
         self.gen, self.m = gen, gen.model
+        # tokens of a prompt portion (0: whole prompts only; None: the model's default)
+        self.prefill_chunk = (self.m.portion_steps if prefill_chunk is None else prefill_chunk) if self.m.portion_steps else 0
+        self.filling: dict[int, list] = {}       # row -> [prompt, tokens already run]
         # Prompt-head cache (automatic prefix caching): a head shared by the prompts of one admission
         # (the Answer system prompt) is prefilled once into a slot of its own and kept; later prompts
         # starting with it prefill only their suffix, and their decode reads the head's keys from
@@ -511,6 +520,8 @@ class ContinuousScheduler:
         arrival waits for at most one step while an unloaded request runs many steps per tick."""
         self.stats["ticks"] += 1
         done = self._admit()
+        if self.filling:
+            return done + self._mixed_step()
         if self.n_active:
             st, k = self._bucket_state(), steps or self.chunk_steps
             k = max(1, min(k, max(left for left in self.left if left is not None)))
@@ -644,6 +655,11 @@ class ContinuousScheduler:
             tot += len(p[0])
         if not take:
             return []
+        if self.prefill_chunk:
+            free = self._start_filling([t for t in take if len(t[0]) > self.prefill_chunk], free)
+            take = [t for t in take if len(t[0]) <= self.prefill_chunk]
+            if not take:
+                return []
         # prompt heads: reuse a cached one, or cache the head this admission's prompts share
         hs = [self._match_head(t[0]) for t in take] if self.max_heads else [None] * len(take)
         if self.max_heads:
@@ -697,8 +713,77 @@ class ContinuousScheduler:
         # a budget of one token (or an immediate EOS) finishes at prefill
         return self._reap(rows)
 
+    def _start_filling(self, take, free) -> list:
+        """Give rows, slots and cache to prompts that run in portions; their rows stay on the spare slot (and
+        inactive) until the last portion. Returns the rows still free."""
+        slots = self.gen.cache.acquire(len(take), [len(p) + b for p, b, _ in take])
+        for r, sl, (p, b, tag) in zip(free, slots, take):
+            self.rows[r] = (tag, sl, int(b), None)
+            self.filling[r] = [p, 0]
+        self.stats["admitted"] += len(take)
+        return free[len(take):]
+
+    def _mixed_step(self) -> list:
+        """One batch: the next portions of the prompts being filled, one token of every decoding row."""
+        st, dev = self.st, self.m.device
+        t0 = time.perf_counter()
+        portions, room = [], self.prefill_chunk
+        for r, (p, at) in self.filling.items():
+            n = min(len(p) - at, room)
+            if n > 0:
+                portions.append((r, at, n))
+                room -= n
+        dec = [r for r, x in enumerate(self.rows) if x is not None and r not in self.filling]
+        fin = [r for r, at, n in portions if at + n == len(self.filling[r][0])]
+        ids = [t for r, at, n in portions for t in self.filling[r][0][at:at + n]]
+        lens = [n for _, _, n in portions] + [1] * len(dec)
+        m, tok = pack_batch(lens, [self.rows[r][1] for r in [x[0] for x in portions] + dec],
+                            [at for _, at, _ in portions] + [0] * len(dec), dev, ids + [0] * len(dec))
+        ends = np.cumsum(lens) - 1
+        want = [int(e) for e, (r, _, _) in zip(ends, portions) if r in fin] + [int(e) for e in ends[len(portions):]]
+        if dec:  # their tokens and positions are on the device
+            di = h2d(np.asarray(dec, dtype=np.int64), dev)
+            tok[len(ids):] = st.tokens.index_select(0, di)
+            m.pos0[len(portions):] = st.pos.index_select(0, di)
+            m.max_ctx = self.gen.cache.max_seq
+        logits = self.m.step(m, tok, h2d(np.asarray(want, dtype=np.int64), dev) if want else None)
+        for r, _, n in portions:
+            self.filling[r][1] += n
+            self.gen.stats["prefill_tokens"] += n
+        if fin:  # these rows start to decode: their first token comes from this step
+            fi = h2d(np.asarray(fin, dtype=np.int64), dev)
+            plen = np.asarray([len(self.filling[r][0]) for r in fin], dtype=np.int32)
+            budget = np.asarray([self.rows[r][2] for r in fin], dtype=np.int32)
+            for name, v in (("pos", plen - 1), ("lens", plen), ("start", plen - 1 - (self.cap - budget)),
+                            ("slot", np.asarray([self.rows[r][1] for r in fin], dtype=np.int32)),
+                            ("active", np.ones(len(fin), dtype=np.int32))):
+                getattr(st, name).index_copy_(0, fi, h2d(v, dev))
+            st.hist.index_fill_(0, fi, -1)
+            st.conf.index_fill_(0, fi, 0.0)
+            for r in fin:
+                del self.filling[r]
+                self.left[r] = self.rows[r][2]
+        live = fin + dec
+        self.stats["mixed_steps"] = self.stats.get("mixed_steps", 0) + 1
+        if not live:
+            return []
+        idx = h2d(np.asarray(live, dtype=np.int64), dev)
+        names = ("tokens", "lp", "conf", "active", "pos", "lens", "hist", "start")
+        s = {n: getattr(st, n).index_select(0, idx) for n in names}
+        self.m.sample(logits, self.gen.temperature, self.gen.seed, 0, out_tok=s["tokens"], out_lp=s["lp"], conf=s["conf"],
+                      active=s["active"], ctr=s["pos"], pos=s["pos"], lens=s["lens"], hist=s["hist"], start=s["start"],
+                      eos=self.gen.eos)
+        for n in names:
+            getattr(st, n).index_copy_(0, idx, s[n])
+        for r in live:
+            self.left[r] = max(0, self.left[r] - 1)
+        self.gen.stats["decode_steps"] += 1
+        out = self._reap(live)
+        self.gen.stats["decode_s"] += time.perf_counter() - t0
+        return out
+
     def _reap(self, rows=None) -> list:
-        rows = [i for i, r in enumerate(self.rows) if r is not None] if rows is None else rows
+        rows = [i for i, r in enumerate(self.rows) if r is not None and i not in self.filling] if rows is None else rows
         if not rows:
             return []
         st = self.st

@@ -296,6 +296,7 @@ class _Layer:
 
 class HybridDecoder:
     prefix_sharing = False  # a prompt head's recurrent state is not shared between sequences
+    portion_steps = 8192    # a step runs any portions; prompts are cut at this many tokens by default
     stateful_step = True    # running a step twice advances a sequence twice (graph warm-up uses a spare slot)
     layer_hook = None       # prefill: called with the layer index before each layer (stream steering)
 

@@ -236,6 +236,7 @@ class LlamaDecoder:
     unit_gains = False  # set by _fold_norm_gains
     layer_hook = None   # prefill: called with the layer index before each layer (stream steering)
     prefix_sharing = True   # prompts may attend to a shared head in another slot
+    portion_steps = 0       # runs whole prompts (or their tails behind a shared head) and single tokens only
     stateful_step = False   # running a decode step twice leaves a sequence as running it once
 
     def __init__(self, cfg: DecoderConfig, device="cuda", seed: int = 0, tp: TPContext | None = None,

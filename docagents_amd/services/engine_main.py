@@ -111,6 +111,8 @@ def main(argv=None) -> int:
                  enc_dtype=cfg.dtype, llm_dtype=cfg.llm_dtype)
     if cfg.engine_admit_tokens > 0:
         eng.admit_tokens = cfg.engine_admit_tokens
+    if cfg.engine_prefill_chunk >= 0:
+        eng.prefill_chunk = cfg.engine_prefill_chunk
     if cfg.engine_continuous and dev.type == "cuda" and eng.gen is not None:
         eng.scheduler.warmup()  # every row bucket's decode graph, before the first request (all TP ranks)
     index_dir = a.index_dir if a.index_dir is not None else cfg.index_dir_path()

@@ -476,6 +476,34 @@ def test_greedy_generation_through_generator_and_scheduler(tmp_path, device, dty
     assert len(model.cache.free) == 6 and len(model.cache.free_pages) == model.cache.pages
 
 
+@pytest.mark.parametrize("device,dtype", [CPU, GPU32])
+@pytest.mark.parametrize("chunk", [2, 16, 65])
+def test_scheduler_runs_prompt_portions_beside_decoding_rows(tmp_path, device, dtype, chunk):
+    """Prompts longer than a portion fill in mixed steps while other rows decode; rows, slots and pages are
+    reused; tokens are the plain implementation's."""
+    model, cfg, w = build(tmp_path, "odd", device, dtype, seed=14, edit=sharp)
+    prompts = [tokens(cfg, n, 30 + n) for n in (3, 70, 17, 1, 66, 2, 100)]
+    want = [greedy(cfg, w, p, 7) for p in prompts]
+    model.alloc_cache(5, 128, tokens=7 * 64)
+    g = Generator(model, max_batch=4, max_seq=128, temperature=0.0)
+    sch = ContinuousScheduler(g, B=4, max_new_cap=8, chunk_steps=2, prefill_chunk=chunk)
+    assert [r.tokens for r in sch.run_all(prompts, 7)] == want
+    assert sch.stats["mixed_steps"] > (100 // chunk) // 2 and not sch.filling
+    # a long prompt arrives while a short one decodes: both advance in every mixed step
+    sch.submit(prompts[0], 7, "short")
+    sch.tick(steps=1)
+    sch.submit(prompts[6], 7, "long")
+    done, before = {}, sch.stats["mixed_steps"]
+    while sch.busy():
+        done.update(sch.tick(steps=1))
+    assert done["short"].tokens == want[0] and done["long"].tokens == want[6]
+    # (a portion of two: the short prompt's second portion comes first)
+    assert sch.stats["mixed_steps"] - before == -(-100 // chunk) + (chunk < 3)
+    assert sorted(model.cache.free_pages) == sorted(set(range(7)) - set(model.cache.owned[g.dummy_slot]))
+    whole = ContinuousScheduler(g, B=4, max_new_cap=8, prefill_chunk=0)
+    assert [r.tokens for r in whole.run_all(prompts, 7)] == want and "mixed_steps" not in whole.stats
+
+
 @pytest.mark.gpu
 def test_decode_graphs_replay_the_eager_steps(tmp_path):
     """bf16: captured decode steps against eager ones over several waves with eager work in between."""
