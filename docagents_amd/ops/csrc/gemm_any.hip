@@ -23,6 +23,66 @@ struct AnyArgs {
   const void* u; const float* lam; float* decay; float* drive; int ldu, ldg;
 };
 
+// Four neighbouring outputs of row m, columns n .. n + 3 (past N: not stored).
+template <int EPI>
+__device__ __forceinline__ void any_block(const AnyArgs& p, int z, int m, int n, f32x4_t v) {
+  if (n >= p.N) return;
+  const float* bias = p.bias ? p.bias + z * p.sBias : nullptr;
+  float* o = (float*)p.C + z * p.sC + (size_t)m * p.ldc + n;
+  const bool vec = (p.N & 3) == 0 && (p.ldc & 3) == 0;
+  if (bias) {
+    if (vec) v += *(const f32x4_t*)(bias + n);
+    else
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] += bias[min(n + e, p.N - 1)];
+  }
+  if constexpr (EPI == ANY_SOFTPLUS)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = softplus32(v[e]);
+  if (vec) {
+    *(f32x4_t*)o = v;
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (n + e < p.N) o[e] = v[e];
+  }
+}
+
+// Gates of four neighbouring channels from ch on: decay and driving term of the recurrence.
+__device__ __forceinline__ void any_gates(const float* lam4, const f32x4_t& x, const f32x4_t& y, const f32x4_t& u,
+                                          f32x4_t& decay, f32x4_t& drive) {
+  const f32x4_t lam = *(const f32x4_t*)lam4;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const float la = lam[e] * sigmoid32(x[e]);  // log of the decay, <= 0
+    decay[e] = exp32(la);
+    drive[e] = __builtin_amdgcn_sqrtf(one_minus_square32(la, decay[e])) * sigmoid32(y[e]) * u[e];
+  }
+}
+
+// Four neighbouring pairs of row m: columns nb + 4 fg .. of a 32-column group and the 16 after them (nb % 32 == 0).
+template <int EPI>
+__device__ __forceinline__ void any_pair(const AnyArgs& p, int z, int m, int nb, int fg, f32x4_t x, f32x4_t y,
+                                         const f32x4_t& u) {
+  if (p.bias) {
+    const float* bias = p.bias + z * p.sBias + nb + 4 * fg;
+    x += *(const f32x4_t*)bias;
+    y += *(const f32x4_t*)(bias + 16);
+  }
+  const int col = nb / 2 + 4 * fg;
+  f32x4_t r, d;
+  if constexpr (EPI == ANY_REGLU) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) r[e] = fmaxf(x[e], 0.f) * y[e];
+    *(f32x4_t*)((float*)p.C + z * p.sC + (size_t)m * p.ldc + col) = r;
+  } else {
+    const int ch = z * (p.N / 2) + col;
+    any_gates(p.lam + ch, x, y, u, r, d);
+    *(f32x4_t*)(p.decay + (size_t)m * p.ldg + ch) = r;
+    *(f32x4_t*)(p.drive + (size_t)m * p.ldg + ch) = d;
+  }
+}
+
 constexpr int ANY_ROWB = 144;
 
 template <typename T, int EPI, int BT>
@@ -110,70 +170,134 @@ __global__ void __launch_bounds__(256) gemm_any_kernel(AnyArgs p) {
   }
 
   // W is the MFMA's first operand: lane (fr, fg) holds row fr, columns 4 fg .. 4 fg + 3 of each 16 x 16 block
-  const float* bias = p.bias ? p.bias + z * p.sBias : nullptr;
-  const f32x4_t zero{0.f, 0.f, 0.f, 0.f};
-  if constexpr (EPI == ANY_REGLU || EPI == ANY_RGLRU) {
 #pragma unroll
-    for (int jp = 0; jp < F / 2; ++jp) {
-      const int nb = n0 + wn * WT + jp * 32;
-      if (nb >= p.N) continue;
-      const int col = nb / 2 + 4 * fg;
-      const f32x4_t b0 = bias ? *(const f32x4_t*)(bias + nb + 4 * fg) : zero;
-      const f32x4_t b1 = bias ? *(const f32x4_t*)(bias + nb + 16 + 4 * fg) : zero;
-      const int ch = z * (p.N / 2) + col;
-      const f32x4_t lam = EPI == ANY_RGLRU ? *(const f32x4_t*)(p.lam + ch) : zero;
+  for (int i = 0; i < F; ++i) {
+    const int m = m0 + wm * WT + i * 16 + fr;
+    if (m >= p.M) continue;
+    if constexpr (EPI == ANY_REGLU || EPI == ANY_RGLRU) {
 #pragma unroll
-      for (int i = 0; i < F; ++i) {
-        const int m = m0 + wm * WT + i * 16 + fr;
-        if (m >= p.M) continue;
-        const f32x4_t x = acc[i][2 * jp] + b0, y = acc[i][2 * jp + 1] + b1;
-        f32x4_t r, d;
-        if constexpr (EPI == ANY_REGLU) {
+      for (int jp = 0; jp < F / 2; ++jp) {
+        const int nb = n0 + wn * WT + jp * 32;
+        if (nb >= p.N) continue;
+        const int ch = z * (p.N / 2) + nb / 2 + 4 * fg;
+        f32x4_t u{0.f, 0.f, 0.f, 0.f};
+        if constexpr (EPI == ANY_RGLRU) u = Act<T>::load4((const T*)p.u + (size_t)m * p.ldu + ch);
+        any_pair<EPI>(p, z, m, nb, fg, acc[i][2 * jp], acc[i][2 * jp + 1], u);
+      }
+    } else {
 #pragma unroll
-          for (int e = 0; e < 4; ++e) r[e] = fmaxf(x[e], 0.f) * y[e];
-          *(f32x4_t*)((float*)p.C + z * p.sC + (size_t)m * p.ldc + col) = r;
-        } else {
-          const f32x4_t u = Act<T>::load4((const T*)p.u + (size_t)m * p.ldu + ch);
+      for (int j = 0; j < F; ++j) any_block<EPI>(p, z, m, n0 + wn * WT + j * 16 + 4 * fg, acc[i][j]);
+    }
+  }
+}
+
+// K up to 256 and many rows (bf16): a workgroup keeps its 64 rows of W in LDS and walks row tiles of A, the
+// next tile's loads in flight during this one's products and epilogue (which costs as much as they do). Results
+// leave through LDS in whole lines (64-byte pieces of rows a power of two apart: 299 us, whole lines 240 us for
+// 16384 x 8192 step sizes).
+template <int EPI>
+__global__ void __launch_bounds__(256) gemm_walk_kernel(AnyArgs p) {
+  extern __shared__ __attribute__((aligned(16))) char sm[];
+  const int rowb = p.K * 2 + 16, pieces = p.K / 8, lp = p.K / 32;  // bytes and 16-byte pieces of a row, per thread
+  char* sW = sm;
+  char* sA = sm + 64 * rowb;
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, wm = wv >> 1, wn = wv & 1;
+  const int fr = lane & 15, fg = lane >> 4;
+  const int n0 = blockIdx.x * 64, z = blockIdx.z, mt = (p.M + 63) / 64;
+  const bf16_t* A = (const bf16_t*)p.A + z * p.sA;
+  const bf16_t* W = (const bf16_t*)p.W + z * p.sW;
+  u32x4_t r[8];
+  auto load = [&](const bf16_t* X, int row0, int rows, int ld) {
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            const float la = lam[e] * sigmoid32(x[e]);  // log of the decay, <= 0
-            r[e] = exp32(la);
-            d[e] = __builtin_amdgcn_sqrtf(one_minus_exp32(2.f * la)) * sigmoid32(y[e]) * u[e];
-          }
-          *(f32x4_t*)(p.decay + (size_t)m * p.ldg + ch) = r;
-          *(f32x4_t*)(p.drive + (size_t)m * p.ldg + ch) = d;
-        }
+    for (int i = 0; i < 8; ++i)
+      if (i < lp) {
+        const int pc = tid + 256 * i;
+        r[i] = *(const u32x4_t*)(X + (size_t)min(row0 + pc / pieces, rows - 1) * ld + pc % pieces * 8);
+      }
+  };
+  auto store = [&](char* s) {
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      if (i < lp) {
+        const int pc = tid + 256 * i;
+        *(u32x4_t*)(s + pc / pieces * rowb + pc % pieces * 16) = r[i];
+      }
+  };
+  load(W, n0, p.N, p.K);
+  store(sW);
+  load(A, blockIdx.y * 64, p.M, p.lda);
+  store(sA);
+  __syncthreads();
+  for (int t = blockIdx.y; t < mt; t += gridDim.y) {
+    if (t + (int)gridDim.y < mt) load(A, (t + gridDim.y) * 64, p.M, p.lda);
+    f32x4_t acc[2][2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int j = 0; j < 2; ++j) acc[i][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int k = 0; k < p.K; k += 32) {
+      bf16x8_t fa[2], fw[2];
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        fa[i] = *(const bf16x8_t*)(sA + (wm * 32 + i * 16 + fr) * rowb + k * 2 + fg * 16);
+        fw[i] = *(const bf16x8_t*)(sW + (wn * 32 + i * 16 + fr) * rowb + k * 2 + fg * 16);
+      }
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i][j] = mfma16(fw[j], fa[i], acc[i][j]);
+    }
+    // staged rows of 64 (gates: 32 decays, 32 driving terms) fp32, in place of the A tile
+    constexpr int SW = 68;
+    const int nb = n0 + wn * 32;
+    f32x4_t v[2][2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int ml = wm * 32 + i * 16 + fr;
+      f32x4_t b0{0.f, 0.f, 0.f, 0.f}, b1 = b0;
+      if (p.bias && nb < p.N) {
+        const float* bias = p.bias + z * p.sBias + nb + 4 * fg;
+        b0 = *(const f32x4_t*)bias;
+        if (nb + 16 < p.N) b1 = *(const f32x4_t*)(bias + 16);
+      }
+      v[i][0] = acc[i][0] + b0;
+      v[i][1] = acc[i][1] + b1;
+      if constexpr (EPI == ANY_RGLRU) {  // the gates' input is this tile of A
+        if (nb < p.N)
+          any_gates(p.lam + z * (p.N / 2) + nb / 2 + 4 * fg, v[i][0], v[i][1],
+                    Act<bf16_t>::load4((const bf16_t*)(sA + ml * rowb) + nb / 2 + 4 * fg), v[i][0], v[i][1]);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 2; ++j)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[i][j][e] = softplus32(v[i][j][e]);
       }
     }
-  } else {
-    float* C = (float*)p.C + z * p.sC;
-    const bool vec = (p.N & 3) == 0 && (p.ldc & 3) == 0;
+    __syncthreads();  // the A tile has been read
+    float* st = (float*)sA;
 #pragma unroll
-    for (int j = 0; j < F; ++j) {
-      const int n = n0 + wn * WT + j * 16 + 4 * fg;
-      if (n >= p.N) continue;
-      f32x4_t b = zero;
-      if (bias)
+    for (int i = 0; i < 2; ++i)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) b[e] = bias[min(n + e, p.N - 1)];
+      for (int j = 0; j < 2; ++j) {
+        const int col = EPI == ANY_RGLRU ? j * 32 + wn * 16 + 4 * fg : wn * 32 + j * 16 + 4 * fg;
+        *(f32x4_t*)(st + (wm * 32 + i * 16 + fr) * SW + col) = v[i][j];
+      }
+    __syncthreads();
 #pragma unroll
-      for (int i = 0; i < F; ++i) {
-        const int m = m0 + wm * WT + i * 16 + fr;
-        if (m >= p.M) continue;
-        f32x4_t v = acc[i][j] + b;
-        if constexpr (EPI == ANY_SOFTPLUS)
-#pragma unroll
-          for (int e = 0; e < 4; ++e) v[e] = softplus32(v[e]);
-        float* o = C + (size_t)m * p.ldc + n;
-        if (vec) {
-          *(f32x4_t*)o = v;
-        } else {
-#pragma unroll
-          for (int e = 0; e < 4; ++e)
-            if (n + e < p.N) o[e] = v[e];
-        }
+    for (int i = 0; i < 4; ++i) {
+      const int row = (tid >> 4) + 16 * i, c = (tid & 15) * 4, m = t * 64 + row;
+      const f32x4_t o = *(const f32x4_t*)(st + row * SW + c);
+      if (m >= p.M) continue;
+      if constexpr (EPI == ANY_RGLRU) {
+        const int cl = n0 / 2 + (c & 31);
+        if (cl < p.N / 2) *(f32x4_t*)((c < 32 ? p.decay : p.drive) + (size_t)m * p.ldg + z * (p.N / 2) + cl) = o;
+      } else {
+        if (n0 + c < p.N) *(f32x4_t*)((float*)p.C + z * p.sC + (size_t)m * p.ldc + n0 + c) = o;
       }
     }
+    __syncthreads();
+    if (t + (int)gridDim.y < mt) store(sA);
+    __syncthreads();
   }
 }
 
@@ -190,6 +314,17 @@ static int launch_any(const AnyArgs& a, int batch, hipStream_t s) {
 }
 template <typename T, int EPI>
 static int launch_any_t(const AnyArgs& a, int batch, hipStream_t s) {
+  if constexpr (sizeof(T) == 2 && (EPI == ANY_SOFTPLUS || EPI == ANY_RGLRU)) {
+    if (a.M >= 1024 && a.K <= 256 && a.K % 32 == 0 && a.N % 16 == 0 && a.ldc % 4 == 0 && (EPI != ANY_RGLRU || (a.A == a.u && a.sA == a.N / 2 && a.K == a.N / 2))) {
+      const int row = a.K * 2 + 16 > 272 ? a.K * 2 + 16 : 272, lds = 64 * (a.K * 2 + 16 + row), nt = (a.N + 63) / 64 * batch, mt = (a.M + 63) / 64;
+      static const hipError_t e = hipFuncSetAttribute((const void*)gemm_walk_kernel<EPI>,
+                                                      hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 528);
+      if (e != hipSuccess) return (int)e;
+      const int walks = mt < (2048 + nt - 1) / nt ? mt : (2048 + nt - 1) / nt;  // ~2048 workgroups
+      gemm_walk_kernel<EPI><<<dim3((a.N + 63) / 64, walks, batch), 256, lds, s>>>(a);
+      DA_LAUNCH_CHECK();
+    }
+  }
   const long tiles = (long)((a.N + 127) / 128) * ((a.M + 127) / 128) * batch;
   return a.N % 128 == 0 && tiles >= 512 ? launch_any<T, EPI, 128>(a, batch, s) : launch_any<T, EPI, 64>(a, batch, s);
 }

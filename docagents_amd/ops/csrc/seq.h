@@ -51,14 +51,8 @@ template <> struct Act<float> {
 // forms spend most of their instructions on cases that cannot occur here: the epilogues and scans that
 // use these run at their instruction count).
 constexpr float LOG2E = 1.4426950408889634f;
-// e^x, x <= 88: the part of x * log2(e) that fp32 drops is put back (first order).
-__device__ __forceinline__ float exp32(float x) {
-  x = fminf(x, 88.f);
-  const float t = x * LOG2E;
-  const float lo = fmaf(x, 1.925963033500e-8f, fmaf(x, LOG2E, -t));
-  const float e = __builtin_amdgcn_exp2f(t);
-  return fmaf(e, lo * 0.6931471805599453f, e);
-}
+// e^x: relative error |x| * 2^-24 from the product's rounding, 1 ulp from the exponential
+__device__ __forceinline__ float exp32(float x) { return __builtin_amdgcn_exp2f(x * LOG2E); }
 __device__ __forceinline__ float sigmoid32(float x) { return __builtin_amdgcn_rcpf(1.f + exp32(-x)); }
 // log(1 + e^x) = max(x, 0) + log1p(e), e = e^-|x|; log1p(e) = log(u) e / (u - 1) with u = fl(1 + e), which
 // cancels the rounding of u (Goldberg, "What every computer scientist should know about floating-point
@@ -68,16 +62,17 @@ __device__ __forceinline__ float softplus32(float x) {
   const float l = __builtin_amdgcn_logf(u) * 0.6931471805599453f;
   return fmaxf(x, 0.f) + (d == 0.f ? e : l * e * __builtin_amdgcn_rcpf(d));
 }
-// 1 - e^y for y <= 0: the series of the exponential where the difference would cancel.
-__device__ __forceinline__ float one_minus_exp32(float y) {
-  float p = fmaf(y, 1.f / 8.f, 1.f);
-  p = fmaf(p * y, 1.f / 7.f, 1.f);
-  p = fmaf(p * y, 1.f / 6.f, 1.f);
-  p = fmaf(p * y, 1.f / 5.f, 1.f);
-  p = fmaf(p * y, 1.f / 4.f, 1.f);
-  p = fmaf(p * y, 1.f / 3.f, 1.f);
-  p = fmaf(p * y, 1.f / 2.f, 1.f);
-  return y > -0.4f ? -y * p : 1.f - exp32(y);
+// 1 - e^(2 y) for y <= 0, given a = e^y: the series of the exponential where the difference would cancel.
+__device__ __forceinline__ float one_minus_square32(float y, float a) {
+  const float x = 2.f * y;
+  float p = fmaf(x, 1.f / 8.f, 1.f);
+  p = fmaf(p * x, 1.f / 7.f, 1.f);
+  p = fmaf(p * x, 1.f / 6.f, 1.f);
+  p = fmaf(p * x, 1.f / 5.f, 1.f);
+  p = fmaf(p * x, 1.f / 4.f, 1.f);
+  p = fmaf(p * x, 1.f / 3.f, 1.f);
+  p = fmaf(p * x, 1.f / 2.f, 1.f);
+  return x > -0.4f ? -x * p : fmaf(-a, a, 1.f);
 }
 __device__ __forceinline__ float silu32(float x) { return x * sigmoid32(x); }
 // The same for outputs that are rounded to the activation type anyway: bf16 takes the short forms.

@@ -126,7 +126,7 @@ def test_causal_conv(device, dtype, taps):
                 row += e - a
 
 
-@pytest.mark.parametrize("blocks,bw", [(1, 64), (5, 16), (2, 96)])
+@pytest.mark.parametrize("blocks,bw", [(1, 64), (5, 16), (2, 96), (3, 256)])
 @pytest.mark.parametrize("device,dtype", WHERE)
 def test_gated_recurrence(device, dtype, blocks, bw):
     """Gates and scan; one channel forgets at once, one almost never (a = exp(-1e-3) at an open gate)."""
@@ -185,7 +185,7 @@ def test_selective_scan(device, dtype, N):
 
 @pytest.mark.parametrize("epi", [0, 1, 2])
 @pytest.mark.parametrize("M,N,K", [(1, 32, 64), (3, 96, 40), (70, 160, 264), (200, 64, 16),
-                                   (2900, 2944, 72)])
+                                   (2900, 2944, 72), (1100, 200, 256)])
 @pytest.mark.parametrize("device,dtype", WHERE)
 def test_product_of_any_size_keeps_fp32(device, dtype, M, N, K, epi):
     if M > 1000 and (device == "cpu" or epi == 2):
@@ -202,7 +202,8 @@ def test_product_of_any_size_keeps_fp32(device, dtype, M, N, K, epi):
 
 @pytest.mark.gpu
 def test_elementary_functions_keep_fp32():
-    """softplus and the gates' decay / drive over their whole range, relative to the value itself."""
+    """softplus and the gates' decay / drive over their whole range, relative to the value itself
+    (an exponential of argument x is good to |x| * 2^-24: 2.6e-6 at 30)."""
     x = torch.cat([torch.linspace(-30, 30, 4001), torch.logspace(-6, 1, 1000), -torch.logspace(-6, 1, 1000)])
     n = len(x)
     a, w = torch.zeros(n, 64), torch.zeros(32, 64)
@@ -210,7 +211,7 @@ def test_elementary_functions_keep_fp32():
     ops = get_ops("cuda")
     got = ops.gemm_any(a.cuda(), w.cuda(), None, 1)[:, 0].double().cpu()
     want = torch.nn.functional.softplus(x.double(), threshold=60)
-    assert ((got - want).abs() / want).max() < 1e-6
+    assert ((got - want).abs() / want).max() < 4e-6
     # r = sigmoid(x) through a block of 16 channels; lam spreads the decays
     u = torch.zeros(n, 16)
     u[:, 0] = x
@@ -223,7 +224,25 @@ def test_elementary_functions_keep_fp32():
     assert ((decay.double().cpu() - la.exp()).abs() / la.exp()).max() < 2e-5
     want = torch.sqrt(-torch.expm1(2 * la[:, 0])) * s * x.double()
     keep = want.abs() > 1e-20
-    assert ((drive[:, 0].double().cpu() - want).abs() / want.abs())[keep].max() < 2e-6
+    assert ((drive[:, 0].double().cpu() - want).abs() / want.abs())[keep].max() < 4e-6
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("blocks,bw", [(3, 64), (2, 256), (4, 48), (2, 320)])
+def test_gates_of_many_rows(blocks, bw):
+    """The row-walking kernel (blocks of 32 .. 256 channels) and the tiled one, against each other's widths."""
+    T, C, ops = 2111, blocks * bw, get_ops("cuda")
+    u = rand(1, T, C).bfloat16()
+    ra, ri = (rand(k, blocks, bw, bw, std=bw ** -0.5).bfloat16() for k in (2, 3))
+    rb, ib, lam = rand(4, blocks, bw), rand(5, blocks, bw), rand(6, C).double() - 2
+    w = torch.stack([ra.view(blocks, bw // 16, 16, bw), ri.view(blocks, bw // 16, 16, bw)], 2).reshape(blocks, 2 * bw, bw)
+    b = torch.stack([rb.view(blocks, bw // 16, 16), ib.view(blocks, bw // 16, 16)], 2).reshape(blocks, 2 * bw)
+    decay, drive = ops.rglru_gates(u.cuda(), w.cuda(), b.cuda(), (-8 * oracle.softplus(lam)).float().cuda())
+    r, i = oracle.rglru_gates(u.double(), {"ra": ra.double(), "ri": ri.double(), "ra.b": rb.double(), "ri.b": ib.double()},
+                              "", blocks)
+    a = torch.exp(-8 * r * oracle.softplus(lam))
+    close(decay, a, "fp32")
+    close(drive, torch.sqrt(1 - a * a) * i * u.double(), "fp32")
 
 
 @pytest.mark.gpu
