@@ -66,7 +66,7 @@ class DecoderConfig:
 # ---------------------------------------------------------------------- decoders of mixed layers
 @dataclass(frozen=True)
 class GatedRecurrence:
-    """Griffin's recurrent block: real-gated linear recurrent unit behind a short convolution."""
+    """Recurrent block in the manner of Griffin: gated diagonal recurrence behind a short convolution, times a branch."""
     width: int
     blocks: int   # equal parts of the channels with gate matrices of their own
     conv: int     # taps
