@@ -463,7 +463,8 @@ class ContinuousScheduler:
                  max_admit_tokens: int | None = None, max_heads: int = 2, prefill_chunk: int | None = None):
         self.gen, self.m = gen, gen.model
         # tokens of a prompt portion (0: whole prompts only; None: the model's default)
-        self.prefill_chunk = (self.m.portion_steps if prefill_chunk is None else prefill_chunk) if self.m.portion_steps else 0
+        most = self.m.portion_steps
+        self.prefill_chunk = min(most, most if prefill_chunk is None else prefill_chunk)
         self.filling: dict[int, list] = {}       # row -> [prompt, tokens already run]
         # Prompt-head cache (automatic prefix caching): a head shared by the prompts of one admission
         # (the Answer system prompt) is prefilled once into a slot of its own and kept; later prompts

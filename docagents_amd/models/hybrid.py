@@ -308,7 +308,8 @@ class HybridDecoder:
         self.ops = get_ops(self.device)
         self.tp = tp or TPContext()
         if self.tp.size != 1:
-            raise ValueError(f"{cfg.name}: tensor parallelism is not supported for decoders of mixed layers (TP={self.tp.size})")
+            raise ValueError(f"{cfg.name}: tensor parallelism is not supported for decoders of mixed layers "
+                             f"(TP={self.tp.size})")
         self.act = act = DTYPES[dtype]
         if weights is None:
             if cfg.path:

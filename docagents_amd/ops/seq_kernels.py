@@ -72,7 +72,7 @@ def gemm_any(a, w, bias=None, epi: int = ANY_NONE):
     _act(w, "w", a.dtype)
     M, Kd = a.shape
     N = w.shape[0]
-    _req(w.is_contiguous() and w.shape[1] >= 1 and Kd == w.shape[1] and epi in (ANY_NONE, ANY_SOFTPLUS, ANY_REGLU), "gemm_any")
+    _req(w.is_contiguous() and Kd == w.shape[1] and epi in (ANY_NONE, ANY_SOFTPLUS, ANY_REGLU), "gemm_any")
     if bias is not None:
         _f32(bias, "bias", N)
     out = torch.empty((M, N // 2 if epi == ANY_REGLU else N), dtype=torch.float32, device=a.device)
@@ -126,8 +126,8 @@ def stream_step(m: SeqBatch, dim: int, eps: float = 0.0, alpha: float = 1.0, ids
                 w=None, mu=None, prev=None, save=None, want_x: bool = True, want_h: bool = True, act=None):
     """One update of the fp32 residual stream: x' = table[ids], or RMSNorm(alpha x + y) w over ``dim`` of the
     padded columns (y [T, Dp], or its fp32 partials
-    [splits, T, Dp] from ``gemm_partials``); h = x' or, with mu / prev (state [slots, Dp]), x' + (x'_previous token - x') mu, in the
-    activation type. save: state [slots, Dp] that receives each portion's last row of x. -> (x', h)."""
+    [splits, T, Dp] from ``gemm_partials``); h = x' or, with mu / prev (state [slots, Dp]),
+    x' + (x'_previous token - x') mu, in the activation type. save: state [slots, Dp] that receives each portion's last row of x. -> (x', h)."""
     src = table if ids is not None else y
     f32 = _act(src, "table / y", None if src.dim() == 3 else act)
     Dp = src.shape[-1]
@@ -171,8 +171,8 @@ def stream_final(x, w, eps: float, dim: int, act, rows=None):
 
 def causal_conv(x, w, bias, state, m: SeqBatch, silu: bool):
     """Per-channel causal convolution over each portion: x [T, C] (row view), w fp32 [taps, C] (last row: the
-    current token), bias fp32 [C], state [slots, taps - 1, C]: the inputs before the portion, replaced here in batches of single tokens and
-    by the recurrence's op otherwise."""
+    current token), bias fp32 [C], state [slots, taps - 1, C]: the inputs before the portion, replaced here in
+    batches of single tokens and by the recurrence's op otherwise."""
     f32 = _act(x, "x")
     taps, C = w.shape
     _f32(w, "w")

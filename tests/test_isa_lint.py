@@ -26,7 +26,7 @@ HOT_NO_SCRATCH = {  # mangled-name prefixes of the kernels the flagship bench ru
                  "_Z18gemm_splitk_reduce", "_Z23splitk_reduce_resid_ssq"],
     "gemm8p.hip": ["_Z13gemm8p_kernelILi6ELi256E", "_Z13gemm8p_kernelILi3ELi256E", "_Z13gemm8p_kernelILi4ELi256E"],
     "gemm_dk.hip": ["_Z14gemm_dk_kernel"],
-    "gemm_any.hip": ["_Z15gemm_any_kernelIt"],
+    "gemm_any.hip": ["_Z15gemm_any_kernelIt", "_Z16gemm_walk_kernel"],
     "paged_attn.hip": ["_Z19sigmoid_attn_kernelILi64E", "_Z19sigmoid_attn_kernelILi128E", "_Z21sigmoid_decode_kernelILi128E",
                        "_Z16attn_prep_kernelIt"],
     "recurrent.hip": ["_Z15sel_scan_kernelItLi8E", "_Z15sel_scan_kernelItLi4E", "_Z15gru_scan_kernelIt",
