@@ -22,9 +22,9 @@ def read_config(path) -> dict:
         return json.load(f)
 
 
-def read_safetensors(path, device="cpu") -> dict[str, torch.Tensor]:
-    """Every tensor of one file: an 8-byte little-endian header length, the JSON header (name -> dtype, shape,
-    data_offsets) and the data."""
+def _open(path):
+    """(mapped bytes, offset of the data, header) of one file: an 8-byte little-endian header length, the JSON
+    header (name -> dtype, shape, data_offsets) and the data."""
     raw = np.memmap(path, dtype=np.uint8, mode="r")
     if raw.size < 8:
         raise ValueError(f"{path}: not a safetensors file")
@@ -32,16 +32,26 @@ def read_safetensors(path, device="cpu") -> dict[str, torch.Tensor]:
     if n > raw.size - 8:
         raise ValueError(f"{path}: header of {n} bytes in a file of {raw.size}")
     head = json.loads(raw[8:8 + n].tobytes())
+    head.pop("__metadata__", None)
+    return raw, 8 + n, head
+
+
+def tensor_shapes(path) -> dict[str, tuple]:
+    """Name -> shape of every tensor of a checkpoint folder (headers only)."""
+    return {name: tuple(t["shape"]) for f in _files(path) for name, t in _open(f)[2].items()}
+
+
+def read_safetensors(path, device="cpu") -> dict[str, torch.Tensor]:
+    """Every tensor of one file."""
+    raw, data, head = _open(path)
     out = {}
     for name, t in head.items():
-        if name == "__metadata__":
-            continue
         if t["dtype"] not in _DTYPES:
             raise ValueError(f"{path}: {name} has dtype {t['dtype']}")
         np_dt, dt = _DTYPES[t["dtype"]]
-        lo, hi = (8 + n + o for o in t["data_offsets"])
+        lo, hi = (data + o for o in t["data_offsets"])
         want = int(np.prod(t["shape"], dtype=np.int64)) * np.dtype(np_dt).itemsize
-        if not 8 + n <= lo <= hi <= raw.size or hi - lo != want:
+        if not data <= lo <= hi <= raw.size or hi - lo != want:
             raise ValueError(f"{path}: {name} has bad offsets")
         a = np.frombuffer(raw[lo:hi].tobytes(), dtype=np_dt).reshape(t["shape"])
         v = torch.from_numpy(a.copy())
@@ -49,11 +59,15 @@ def read_safetensors(path, device="cpu") -> dict[str, torch.Tensor]:
     return out
 
 
-def load_weights(path, device="cpu") -> dict[str, torch.Tensor]:
+def _files(path) -> list[Path]:
     files = sorted(Path(path).glob("*.safetensors"))
     if not files:
         raise FileNotFoundError(f"no *.safetensors in {path}")
+    return files
+
+
+def load_weights(path, device="cpu") -> dict[str, torch.Tensor]:
     out: dict[str, torch.Tensor] = {}
-    for f in files:
+    for f in _files(path):
         out.update(read_safetensors(f, device))
     return out

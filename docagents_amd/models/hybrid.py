@@ -1,26 +1,24 @@
-"""Decoders that mix sequence mixers layer by layer, on the gfx950 kernels (Binupel).
+"""Decoders that mix sequence mixers layer by layer, on the gfx950 kernels (Binupel, Zamitar).
 
-Residual stream x in fp32; per layer, with alpha, the norm weights and the shift mu of the configuration:
+Residual stream x in fp32. Per layer run, in a "postnorm" block (with alpha, the norm weights and the shift mu of the
+configuration):
 
     h  = x + (x_previous - x) mu                token shift (x_previous: the previous token's row, state)
     x  = RMSNorm(alpha x + mixer(h)) w1
     x  = RMSNorm(alpha x + down(relu(gate x) * up x)) w2        where the layer has a feed-forward
 
-Each line's norm, the shift of the next layer's input and the saving of the shift's state are one launch
-(``stream_step``). Mixers:
+and in a "parallel" block (learned column scales s1, s2; layers of the loop begin a pass by adding its vector and,
+from the second pass on, the embedding output):
 
-    gated recurrence   [gate | input] GEMM, causal conv, block-diagonal gates GEMM whose epilogue turns the
-                       gates into decay and drive, scan (+ output gate, + conv state), output GEMM
-    sigmoid attention  [q | k | gates] GEMM, query / key preparation + page write, attention over the paged
-                       keys (values = keys, stored once), output GEMM
-    selective scan     [x | z] GEMM, causal conv + silu, [dt | B | C] GEMM, step-size GEMM with a softplus
-                       epilogue in fp32, scan (+ D x, silu(z), conv state), output GEMM
+    h  = LayerNorm(x) w
+    x  = x + s1 mixer(h) + s2 (down(silu(gate h + b) * (up h + b)) + b)
+
+The sums of a line, the norm that follows them, the shift and the saving of its state are one launch
+(``stream_step``, ``stream_add``). The mixers are in ``mixers``.
 
 A step (``step``) runs any batch of portions of sequences (``SeqBatch``): whole prompts, parts of prompts and
 single tokens side by side, each from the state its slot holds. Prefill and the graph-captured decode step
-are that same step. Weights are packed once at load: projections that share an input are concatenated, and
-every width is zero-padded to what the kernels tile by (norms divide by the true width), so any
-configuration runs on the same kernels. ``dtype`` "fp32" runs everything in true fp32.
+are that same step. ``dtype`` "fp32" runs everything in true fp32.
 """
 from __future__ import annotations
 
@@ -31,188 +29,33 @@ import torch
 from ..ops import get_ops
 from ..ops.reference import interleave_gate_up
 from ..ops.seq_batch import PAGE, SeqBatch, pack_batch
-from .configs import GatedRecurrence, HybridConfig, SelectiveScan, SigmoidAttention
+from .configs import (ChannelDelta, GatedRecurrence, HybridConfig, LatentAttention, SelectiveScan, SigmoidAttention)
+from .mixers import (MIXERS, AttentionMixer, DeltaMixer, LatentMixer, Linear, RecurrenceMixer, _pad, _up)
 from .state import LayerState, StateCache
 
-EPI_NONE, EPI_BIAS, EPI_REGLU = 0, 1, 7
-ANY_NONE, ANY_SOFTPLUS, ANY_REGLU = 0, 1, 2
 DTYPES = {"bf16": torch.bfloat16, "fp32": torch.float32}
-TILE = 64  # K of every product, N of the packed projections
-
-
-def _up(n: int, m: int = TILE) -> int:
-    return -(-n // m) * m
-
-
-def _pad(t: torch.Tensor, *shape: int) -> torch.Tensor:
-    """Zero-padded at the end of every dimension (-1: as it is)."""
-    shape = [s if n < 0 else n for s, n in zip(t.shape, shape)]
-    if list(t.shape) == shape:
-        return t.contiguous()
-    out = torch.zeros(shape, dtype=t.dtype, device=t.device)
-    out[tuple(slice(0, s) for s in t.shape)] = t
-    return out
-
-
-class Linear:
-    """x W^T (+ bias) in the activation type: gemm.hip's kernels in bf16, gemm_any in fp32."""
-
-    def __init__(self, ops, w, act, bias=None, relu_gated: bool = False):
-        self.ops, self.act = ops, act
-        self.w = w.to(act).contiguous()
-        self.bias = None if bias is None else bias.to(act).contiguous()
-        self.gated = relu_gated
-
-    def __call__(self, x, out=None, partial: bool = False):
-        """partial: the consumer also takes fp32 split-K partials [splits, M, N]."""
-        if self.act == torch.float32:
-            y = self.ops.gemm_any(x, self.w, self.bias, ANY_REGLU if self.gated else ANY_NONE)
-            return y if out is None else out.copy_(y)
-        if partial and self.ops.partials_fit(x.shape[0], *self.w.shape):
-            return self.ops.gemm_partials(x, self.w)
-        epi = EPI_REGLU if self.gated else (EPI_NONE if self.bias is None else EPI_BIAS)
-        return self.ops.gemm(x, self.w, bias=self.bias, epi=epi, out=out)
-
-
-class RecurrenceMixer:
-    @staticmethod
-    def padded(s: GatedRecurrence) -> tuple[int, int]:
-        """(channels of a block, of all blocks): a block a multiple of 16, all of them of 64."""
-        bw = _up(s.width // s.blocks, max(16, TILE // math.gcd(s.blocks, TILE)))
-        return bw, s.blocks * bw
-
-    @classmethod
-    def state(cls, s: GatedRecurrence, act) -> LayerState:
-        _, C = cls.padded(s)
-        return LayerState({"rec": ((C,), torch.float32), "conv": ((s.conv - 1, C), act)})
-
-    @staticmethod
-    def tensors(s: GatedRecurrence, h: int) -> dict:
-        w, b = s.width, s.width // s.blocks
-        return {"y": (w, h), "y.b": (w,), "x": (w, h), "x.b": (w,), "conv": (w, s.conv), "conv.b": (w,),
-                "ra": (s.blocks, b, b), "ra.b": (s.blocks, b), "ri": (s.blocks, b, b), "ri.b": (s.blocks, b),
-                "lam": (w,), "o": (h, w)}
-
-    def __init__(self, ops, s: GatedRecurrence, w, hp: int, eps: float, act):
-        self.ops, self.s = ops, s
-        bw, C = self.padded(s)
-        self.C = C
-        b0 = s.width // s.blocks
-
-        def chan(t):  # leading dimension: channels -> blocks of bw
-            return _pad(t.reshape(s.blocks, b0, *t.shape[1:]), -1, bw, *[-1] * (t.dim() - 1)).reshape(C, *t.shape[1:])
-        self.proj = Linear(ops, torch.cat([_pad(chan(w["y"]), -1, hp), _pad(chan(w["x"]), -1, hp)]), act,
-                           torch.cat([chan(w["y.b"]), chan(w["x.b"])]))
-        self.conv_w = chan(w["conv"]).float().t().contiguous()
-        self.conv_b = chan(w["conv.b"]).float()
-        ra, ri = (_pad(w[k], -1, bw, bw) for k in ("ra", "ri"))
-        self.gate_w = torch.stack([interleave_gate_up(a, i) for a, i in zip(ra, ri)]).to(act).contiguous()
-        rb, ib = (_pad(w[k], -1, bw).reshape(-1, 1) for k in ("ra.b", "ri.b"))
-        self.gate_b = interleave_gate_up(rb, ib).reshape(s.blocks, 2 * bw).float().contiguous()
-        lam = w["lam"].double()
-        self.lam = chan((-8.0 * torch.nn.functional.softplus(lam, threshold=700.0)).float())
-        self.out = Linear(ops, _pad(chan(w["o"].t()).t(), hp, -1), act)
-
-    def __call__(self, h, m: SeqBatch, st: dict):
-        o, C = self.ops, self.C
-        yx = self.proj(h)
-        gate, x = yx[:, :C], yx[:, C:]
-        u = o.causal_conv(x, self.conv_w, self.conv_b, st["conv"], m, silu=False)
-        decay, drive = o.rglru_gates(u, self.gate_w, self.gate_b, self.lam)
-        return self.out(o.gated_scan(decay, drive, gate, st["rec"], x, st["conv"], m), partial=True)
-
-
-class AttentionMixer:
-    @staticmethod
-    def padded(s: SigmoidAttention) -> int:
-        d = _up(s.dim, 32 if s.heads % 2 == 0 else 64)
-        return d if d <= 128 or d > 256 else _up(d, 64)
-
-    @classmethod
-    def state(cls, s: SigmoidAttention, act) -> LayerState:
-        return LayerState(page={"k": ((s.kv_heads, PAGE, cls.padded(s)), act),
-                                "k_rms": ((s.kv_heads, PAGE), torch.float32)})
-
-    @staticmethod
-    def tensors(s: SigmoidAttention, h: int) -> dict:
-        return {"q": (s.heads * s.dim, h), "k": (s.kv_heads * s.dim, h), "q.norm": (s.dim,), "k.norm": (s.dim,),
-                "pb": (s.heads,), "g": (s.heads, h), "o": (h, s.heads * s.dim)}
-
-    def __init__(self, ops, s: SigmoidAttention, w, hp: int, eps: float, act):
-        self.ops, self.s, self.eps = ops, s, eps
-        D = self.padded(s)
-
-        def heads(t, n):  # rows of n heads -> heads of D
-            return _pad(t.reshape(n, s.dim, -1), -1, D, hp).reshape(n * D, hp)
-        qkg = torch.cat([heads(w["q"], s.heads), heads(w["k"], s.kv_heads), _pad(w["g"], -1, hp)])
-        self.proj = Linear(ops, _pad(qkg, _up(qkg.shape[0]), -1), act)
-        self.qk_w = _pad(w["q.norm"].float() * w["k.norm"].float(), D)
-        self.pb = w["pb"].float().contiguous()
-        wo = w["o"].reshape(-1, s.heads, s.dim)
-        self.out = Linear(ops, _pad(wo, hp, -1, D).reshape(hp, s.heads * D), act)
-
-    def __call__(self, h, m: SeqBatch, st: dict):
-        s = self.s
-        a = self.ops.sigmoid_attn(self.proj(h), st["k"], st["k_rms"], self.pb, self.qk_w, m, s.heads, s.kv_heads, s.dim,
-                                  s.scale, self.eps, s.q_temp)
-        return self.out(a, partial=True)
-
-
-class ScanMixer:
-    @classmethod
-    def state(cls, s: SelectiveScan, act) -> LayerState:
-        C = _up(s.inner)
-        return LayerState({"ssm": ((C, s.state), torch.float32), "conv": ((s.conv - 1, C), act)})
-
-    @staticmethod
-    def tensors(s: SelectiveScan, h: int) -> dict:
-        n = s.inner
-        return {"in": (2 * n, h), "conv": (n, s.conv), "conv.b": (n,), "x": (s.dt_rank + 2 * s.state, n),
-                "dt": (n, s.dt_rank), "dt.b": (n,), "A_log": (n, s.state), "D": (n,), "o": (h, n)}
-
-    def __init__(self, ops, s: SelectiveScan, w, hp: int, eps: float, act):
-        self.ops, self.s = ops, s
-        n, C = s.inner, _up(s.inner)
-        self.C = C
-        self.proj = Linear(ops, torch.cat([_pad(w["in"][:n], C, hp), _pad(w["in"][n:], C, hp)]), act)
-        self.conv_w = _pad(w["conv"], C, -1).float().t().contiguous()
-        self.conv_b = _pad(w["conv.b"], C).float()
-        self.low = Linear(ops, _pad(w["x"], _up(s.dt_rank + 2 * s.state), C), act)
-        # the step sizes' operand is the first columns of [dt | B | C]; zero weights meet the rest
-        self.dt_k = _up(s.dt_rank)
-        self.dt_w = _pad(w["dt"], C, self.dt_k).to(act).contiguous()
-        self.dt_b = _pad(w["dt.b"], C).float()
-        self.A = _pad((-torch.exp(w["A_log"].double()) * math.log2(math.e)).float(), C, -1)
-        self.D = _pad(w["D"], C).float()
-        self.out = Linear(ops, _pad(w["o"], hp, C), act)
-
-    def __call__(self, h, m: SeqBatch, st: dict):
-        o, C, s = self.ops, self.C, self.s
-        xz = self.proj(h)
-        x, z = xz[:, :C], xz[:, C:]
-        xc = o.causal_conv(x, self.conv_w, self.conv_b, st["conv"], m, silu=True)
-        low = self.low(xc)
-        dt = o.gemm_any(low[:, :self.dt_k], self.dt_w, self.dt_b, ANY_SOFTPLUS)
-        y = o.selective_scan(xc, dt, low, s.dt_rank, s.dt_rank + s.state, z, self.A, self.D, st["ssm"], x, st["conv"], m)
-        return self.out(y, partial=True)
-
-
-MIXERS = {GatedRecurrence: RecurrenceMixer, SigmoidAttention: AttentionMixer, SelectiveScan: ScanMixer}
 
 
 def tensor_shapes(cfg: HybridConfig) -> dict[str, tuple]:
     """Name -> shape of every tensor of a checkpoint of this configuration."""
-    h = cfg.hidden
+    h, parallel = cfg.hidden, cfg.block == "parallel"
     out = {"embed": (cfg.vocab, h)}
+    if cfg.loop:
+        out["loop.step"] = (cfg.loop.times, h)
     for i, s in enumerate(cfg.spec):
         if s.weights_of is not None:
             continue
-        out.update({f"l{i}.norm1": (h,), f"l{i}.shift": (h,)})
-        out.update({f"l{i}.mix.{k}": v for k, v in MIXERS[type(s.mixer)].tensors(s.mixer, h).items()})
+        p = f"l{i}."
+        out.update({p + "norm1": (h,), p + ("ls1" if parallel else "shift"): (h,)})
+        out.update({f"{p}mix.{k}": v for k, v in MIXERS[type(s.mixer)].tensors(s.mixer, h).items()})
         if s.ff:
-            out.update({f"l{i}.norm2": (h,), f"l{i}.mlp.gate": (s.ff, h), f"l{i}.mlp.up": (s.ff, h),
-                        f"l{i}.mlp.down": (h, s.ff)})
-    out.update({"final.norm": (h,), "head": (cfg.vocab, h)})
+            out.update({p + ("ls2" if parallel else "norm2"): (h,), p + "mlp.gate": (s.ff, h), p + "mlp.up": (s.ff, h),
+                        p + "mlp.down": (h, s.ff)})
+            if parallel:
+                out.update({p + "mlp.gate.b": (s.ff,), p + "mlp.up.b": (s.ff,), p + "mlp.down.b": (h,)})
+    out["final.norm"] = (h,)
+    if not parallel:
+        out["head"] = (cfg.vocab, h)
     return out
 
 
@@ -225,7 +68,7 @@ def random_weights(cfg: HybridConfig, device="cpu", seed: int = 0) -> dict[str, 
     for name, shape in tensor_shapes(cfg).items():
         key = name.rsplit(".", 1)[-1] if not name.endswith((".b", ".norm")) else ".".join(name.split(".")[-2:])
         t = torch.empty(shape, dtype=torch.float32, device=dev)
-        if key in ("norm1", "norm2", "final.norm", "q.norm", "k.norm", "D"):
+        if key in ("norm1", "norm2", "final.norm", "q.norm", "k.norm", "D", "mix.norm", "dq.norm", "dkv.norm"):
             t.normal_(1.0, 0.1, generator=gen)
         elif key == "shift":
             t.uniform_(0.0, 0.6, generator=gen)
@@ -233,8 +76,10 @@ def random_weights(cfg: HybridConfig, device="cpu", seed: int = 0) -> dict[str, 
             t.uniform_(-5.0, -1.0, generator=gen)
         elif key == "A_log":
             t.uniform_(0.0, math.log(16.0), generator=gen)
-        elif key == "dt.b":
+        elif key in ("dt.b", "dt_bias"):
             t.uniform_(-5.0, -2.0, generator=gen)
+        elif key in ("ls1", "ls2"):
+            t.normal_(0.3, 0.05, generator=gen)
         elif key == "pb":
             t.normal_(-3.0, 0.5, generator=gen)
         elif key == "conv":
@@ -248,10 +93,13 @@ def random_weights(cfg: HybridConfig, device="cpu", seed: int = 0) -> dict[str, 
 
 
 def layer_states(cfg: HybridConfig, act=torch.bfloat16) -> list[LayerState]:
-    """What every layer keeps per sequence: its mixer's state and the token shift's previous row."""
+    """What every layer run keeps per sequence: its mixer's state and, in postnorm blocks, the token shift's
+    previous row."""
+    per = [MIXERS[type(s.mixer)].state(s.mixer, act) for s in (cfg.spec[r.layer] for r in cfg.runs)]
+    if cfg.block == "parallel":
+        return per
     shift = {"shift": ((_up(cfg.hidden),), torch.float32)}
-    per = [MIXERS[type(s.mixer)].state(s.mixer, act) for s in cfg.spec]
-    return [LayerState({**p.slot, **shift}, p.page) for p in per]
+    return [LayerState({**p.slot, **shift}, p.page, p.tables) for p in per]
 
 
 def cache_bytes(cfg: HybridConfig, slots: int, max_seq: int, act=torch.bfloat16) -> int:
@@ -272,25 +120,40 @@ def prefill_bytes_per_token(cfg: HybridConfig) -> int:
             return RecurrenceMixer.padded(m)[1] * (2 * 2 + 2 + 2 * 4 + 2)
         if isinstance(m, SelectiveScan):
             return _up(m.inner) * (2 * 2 + 2 + 4 + 2) + 2 * _up(m.dt_rank + 2 * m.state)
+        if isinstance(m, ChannelDelta):
+            K, V = DeltaMixer.padded(m)
+            return 2 * 2 * (2 * m.kv_heads * K + m.heads * V) + m.heads * (4 * K + 3 * 2 * V)
+        if isinstance(m, LatentAttention):
+            Q, L, R, D, V = LatentMixer.padded(m)
+            return 2 * (2 * Q + 2 * (L + R) + m.heads * (2 * D + 3 * V))
         return AttentionMixer.padded(m) * 2 * (2 * m.heads + m.kv_heads)
-    return 12 * _up(cfg.hidden) + max(max(mixer(s.mixer), 2 * _up(s.ff)) for s in cfg.spec)
+    return 12 * _up(cfg.hidden) + max(mixer(s.mixer) + 2 * _up(s.ff) if cfg.block == "parallel" else
+                                    max(mixer(s.mixer), 2 * _up(s.ff)) for s in cfg.spec)
 
 
 class _Layer:
-    """One layer's packed weights (shared by the layers that use them)."""
+    """One layer's packed weights (shared by the runs that use them)."""
 
     def __init__(self, ops, cfg: HybridConfig, i: int, raw: dict, hp: int, act):
         s, pre = cfg.spec[i], f"l{i}."
+        self.parallel = cfg.block == "parallel"
         mix = {k[len(pre) + 4:]: v for k, v in raw.items() if k.startswith(pre + "mix.")}
         self.mixer = MIXERS[type(s.mixer)](ops, s.mixer, mix, hp, cfg.eps, act)
-        self.norm1 = _pad(raw[pre + "norm1"], hp).float()
-        self.shift = _pad(raw[pre + "shift"], hp).float()
-        self.norm2 = self.gate_up = self.down = None
+
+        def vec(name):
+            return _pad(raw[pre + name], hp).float()
+        self.norm1 = vec("norm1")
+        self.shift, self.scale1 = (None, vec("ls1")) if self.parallel else (vec("shift"), None)
+        self.norm2 = self.scale2 = self.down_bias = self.gate_up = self.down = None
         if s.ff:
-            f = _up(s.ff)
-            self.norm2 = _pad(raw[pre + "norm2"], hp).float()
-            self.gate_up = Linear(ops, interleave_gate_up(_pad(raw[pre + "mlp.gate"], f, hp),
-                                                          _pad(raw[pre + "mlp.up"], f, hp)), act, relu_gated=True)
+            f, bias = _up(s.ff), None
+            if self.parallel:
+                bias = interleave_gate_up(*(_pad(raw[pre + f"mlp.{k}.b"], f)[:, None] for k in ("gate", "up")))[:, 0]
+                self.scale2, self.down_bias = vec("ls2"), vec("mlp.down.b")
+            else:
+                self.norm2 = vec("norm2")
+            w = interleave_gate_up(_pad(raw[pre + "mlp.gate"], f, hp), _pad(raw[pre + "mlp.up"], f, hp))
+            self.gate_up = Linear(ops, w, act, bias, gated="silu" if self.parallel else "relu")
             self.down = Linear(ops, _pad(raw[pre + "mlp.down"], hp, f), act)
 
 
@@ -321,10 +184,15 @@ class HybridDecoder:
         raw = {k: v.to(self.device) for k, v in weights.items()}
         self.hp = hp = _up(cfg.hidden)
         own = {i: _Layer(self.ops, cfg, i, raw, hp, act) for i, s in enumerate(cfg.spec) if s.weights_of is None}
-        self.layers = [own[i if s.weights_of is None else s.weights_of] for i, s in enumerate(cfg.spec)]
-        self.embed = _pad(raw["embed"], -1, hp).to(act).contiguous()
+        self.layers = [own[r.weights] for r in cfg.runs]
         self.final_norm = _pad(raw["final.norm"], hp).float()
-        self.head = Linear(self.ops, _pad(raw["head"], _up(cfg.vocab), hp), act)
+        self.pass_vec = _pad(raw["loop.step"], -1, hp).float() if cfg.loop else None
+        if cfg.block == "parallel":
+            self.head = Linear(self.ops, _pad(raw["embed"], _up(cfg.vocab), hp), act)
+            self.embed = self.head.w[:cfg.vocab]
+        else:
+            self.embed = _pad(raw["embed"], -1, hp).to(act).contiguous()
+            self.head = Linear(self.ops, _pad(raw["head"], _up(cfg.vocab), hp), act)
         self.cache: StateCache | None = None
 
     def _check(self, weights: dict) -> None:
@@ -350,10 +218,13 @@ class HybridDecoder:
     # ------------------------------------------------------------- step
     def _forward(self, m: SeqBatch, ids) -> torch.Tensor:
         """The residual stream after the last layer [T, Dp] of a batch; updates pages and state."""
+        m = m.on(self.cache.table)
+        return self._parallel_blocks(m, ids) if self.cfg.block == "parallel" else self._postnorm_blocks(m, ids)
+
+    def _postnorm_blocks(self, m: SeqBatch, ids) -> torch.Tensor:
         c, o, st, layers = self.cfg, self.ops, self.cache.layers, self.layers
         kw = dict(eps=c.eps, alpha=c.alpha, act=self.act)
         shift = [dict(mu=L.shift, prev=s["shift"]) for L, s in zip(layers, st)] + [dict(want_h=False)]
-        m = m.on(self.cache.table)
         x, h = o.stream_step(m, c.hidden, ids=ids, table=self.embed, act=self.act, **shift[0])
         for i, L in enumerate(layers):
             if self.layer_hook is not None:
@@ -365,8 +236,28 @@ class HybridDecoder:
                 x, h = o.stream_step(m, c.hidden, x=x, y=L.down(L.gate_up(h), partial=True), w=L.norm2, **shift[i + 1], **kw)
         return x
 
+    def _parallel_blocks(self, m: SeqBatch, ids) -> torch.Tensor:
+        c, o, st, layers, runs = self.cfg, self.ops, self.cache.layers, self.layers, self.cfg.runs
+        emb = dict(ids=ids, table=self.embed, embed_scale=c.embed_scale)
+
+        def before(i):  # what the stream gains ahead of run i, and the norm run i reads it through
+            if i == len(runs):
+                return {}
+            t = runs[i].loop_pass
+            return dict(w=layers[i].norm1, vec=None if t is None else self.pass_vec[t], **(emb if t else {}))
+        x, h = o.stream_add(m.T, c.hidden, c.eps, self.act, **{**before(0), **emb})
+        for i, L in enumerate(layers):
+            if self.layer_hook is not None:
+                self.layer_hook(i)
+            parts = [(L.mixer(h, m, st[i], partial="own" if L.gate_up else True), L.scale1, None)]
+            if L.gate_up:
+                parts.append((L.down(L.gate_up(h), partial=True), L.scale2, L.down_bias))
+            x, h = o.stream_add(m.T, c.hidden, c.eps, self.act, x=x, parts=parts, **before(i + 1))
+        return x
+
     def _logits(self, x, rows=None, out=None):
-        h = self.ops.stream_final(x, self.final_norm, self.cfg.eps, self.cfg.hidden, self.act, rows)
+        h = self.ops.stream_final(x, self.final_norm, self.cfg.eps, self.cfg.hidden, self.act, rows,
+                                  center=self.cfg.block == "parallel")
         return self.head(h, out=out)[:, :self.cfg.vocab]
 
     def step(self, m: SeqBatch, ids, rows=None) -> torch.Tensor | None:
@@ -410,9 +301,13 @@ class HybridDecoder:
         c = self.cfg
         tot = 0.0
         for n in lens:
-            for s in c.spec:
+            for s in (c.spec[r.layer] for r in c.runs):
                 tot += 2.0 * n * (s.mixer.param_count(c.hidden) + 3 * c.hidden * s.ff)
                 if isinstance(s.mixer, SigmoidAttention):
                     tot += 2.0 * s.mixer.heads * s.mixer.dim * n * n
+                elif isinstance(s.mixer, LatentAttention):
+                    tot += s.mixer.heads * (s.mixer.dim + s.mixer.rot_dim + s.mixer.vdim) * n * n
+                elif isinstance(s.mixer, ChannelDelta):
+                    tot += 6.0 * n * s.mixer.heads * s.mixer.dim * s.mixer.vdim
             tot += 2.0 * c.hidden * c.vocab
         return tot

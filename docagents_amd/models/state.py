@@ -2,7 +2,7 @@
 with a sequence and fixed-size slots for what does not.
 
 A layer declares what it keeps (``LayerState``): slot tensors (recurrent states, convolution inputs, the
-token shift's previous row) are allocated [slots, ...], page tensors (keys) [pages, ...]. A sequence owns one
+token shift's previous row) are allocated [slots, ...], page tensors (keys, latents) [pages, ...]. A sequence owns one
 slot and as many pages as its tokens need; ``table[slot, i]`` is the page of its tokens 64 i .. 64 i + 63,
 shared by every layer. Nothing is cleared when a slot or page changes hands: the kernels start a sequence's
 state at position 0 themselves, and read no key beyond a sequence's own tokens.
@@ -19,10 +19,28 @@ from ..ops.seq_batch import PAGE
 
 
 @dataclass(frozen=True)
+class RotaryTable:
+    """cos and sin of position * base^(-2 i / dims), i < dims / 2, for every position a sequence can reach: fp32
+    [positions, dims / 2, 2], from angles in double precision."""
+    dims: int
+    base: float
+
+    def bytes(self, positions: int) -> int:
+        return positions * self.dims * 4
+
+    def build(self, positions: int, device) -> torch.Tensor:
+        f = self.base ** (-2.0 * torch.arange(self.dims // 2, dtype=torch.float64) / self.dims)
+        a = torch.arange(positions, dtype=torch.float64)[:, None] * f
+        return torch.stack([a.cos(), a.sin()], -1).float().to(device)
+
+
+@dataclass(frozen=True)
 class LayerState:
-    """Shapes (without the leading slot / page dimension) and dtypes by name."""
+    """Shapes (without the leading slot / page dimension) and dtypes by name; tables over positions by name, each
+    built once for all layers that name an equal one."""
     slot: dict = field(default_factory=dict)
     page: dict = field(default_factory=dict)
+    tables: dict = field(default_factory=dict)
 
     @staticmethod
     def _bytes(spec: dict) -> int:
@@ -46,7 +64,9 @@ class StateCache:
         self.pages = pages_for(tokens) if tokens else slots * self.row_pages
         make = lambda spec, n: {k: torch.zeros((n, *shape), dtype=dt, device=self.device)  # noqa: E731
                                 for k, (shape, dt) in spec.items()}
-        self.layers = [{**make(s.slot, slots), **make(s.page, self.pages)} for s in layers]
+        self.tables = {t: t.build(self.row_pages * PAGE, self.device) for s in layers for t in s.tables.values()}
+        self.layers = [{**make(s.slot, slots), **make(s.page, self.pages), **{k: self.tables[t] for k, t in s.tables.items()}}
+                       for s in layers]
         self.table = torch.zeros((slots, self.row_pages), dtype=torch.int32, device=self.device)
         self.free = list(range(slots - 1, -1, -1))
         self.free_pages = list(range(self.pages - 1, -1, -1))
@@ -55,7 +75,8 @@ class StateCache:
     @staticmethod
     def bytes_for(layers: list[LayerState], slots: int, max_seq: int, tokens: int | None = None) -> int:
         pages = pages_for(tokens) if tokens else slots * pages_for(max_seq)
-        return sum(s.bytes(slots, pages) for s in layers)
+        tables = {t for s in layers for t in s.tables.values()}
+        return sum(s.bytes(slots, pages) for s in layers) + sum(t.bytes(pages_for(max_seq) * PAGE) for t in tables)
 
     # ------------------------------------------------------------------ ownership
     def fits(self, tokens: list[int]) -> bool:

@@ -36,7 +36,7 @@ ARCH = os.environ.get("DA_OFFLOAD_ARCH", "gfx950")
 _PART_SOURCES = {
     "gemm": ("gemm.hip", "gemm256.hip", "gemm4w.hip", "gemm8p.hip", "gemm_dk.hip"),
     "token": ("norm.hip", "rope_sample.hip"),
-    "hybrid": ("gemm_any.hip", "paged_attn.hip", "recurrent.hip", "stream_norm.hip"),
+    "hybrid": ("delta.hip", "gemm_any.hip", "latent_attn.hip", "paged_attn.hip", "recurrent.hip", "stream_norm.hip"),
 }
 PARTS = (*_PART_SOURCES, "kernels")
 

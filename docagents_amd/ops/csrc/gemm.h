@@ -6,7 +6,7 @@ enum Epi : int {
   EPI_NONE = 0,
   EPI_BIAS = 1,
   EPI_GELU = 2,       // bias (optional) + exact GELU (BERT)
-  EPI_SWIGLU = 3,     // W rows interleaved in 16-row (gate, up) groups; out N/2 = silu(g)*u
+  EPI_SWIGLU = 3,     // W rows interleaved in 16-row (gate, up) groups; out N/2 = silu(g)*u (bias optional)
   EPI_RESID = 4,      // bias (optional) + residual add
   EPI_PARTIAL = 5,    // fp32 split-K partial to workspace
   EPI_REGLU = 7,      // launchers only: EPI_SWIGLU's layout with relu(g)*u (args carry relu = 1)

@@ -168,10 +168,17 @@ gemm_bf16_kernel(GemmArgs p) {
       const int gm = row0 + rr;
       if (gm >= p.M || gout >= ncols_out) continue;
       const float* srow = st + rr * SLD + grp * 32 + within;
+      const bf16_t* gb = p.bias ? p.bias + col0 + grp * 32 + within : nullptr;
       unsigned packed[4];
 #pragma unroll
       for (int e = 0; e < 8; e += 2) {
         float g0 = srow[e], g1 = srow[e + 1], u0 = srow[16 + e], u1 = srow[16 + e + 1];
+        if (gb) {
+          g0 += bf2f(gb[e]);
+          g1 += bf2f(gb[e + 1]);
+          u0 += bf2f(gb[16 + e]);
+          u1 += bf2f(gb[16 + e + 1]);
+        }
         packed[e / 2] = pack_bf2(gate_act(g0, p.relu) * u0, gate_act(g1, p.relu) * u1);
       }
       *(u32x4_t*)(p.C + (size_t)gm * p.ldc + gout) = u32x4_t{packed[0], packed[1], packed[2], packed[3]};
@@ -247,7 +254,9 @@ gemm_splitk_reduce(const float* __restrict__ ws, int splits, int M, int N, int e
       sum_rows8(ws + (size_t)m * N + gc, splits, (size_t)M * N, g);
       sum_rows8(ws + (size_t)m * N + gc + 16, splits, (size_t)M * N, u);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) v[e] = gate_act(g[e] * inv, relu) * (u[e] * inv);
+      for (int e = 0; e < 8; ++e)
+        v[e] = gate_act(fmaf(g[e], inv, bias ? bf2f(bias[gc + e]) : 0.f), relu) *
+               fmaf(u[e], inv, bias ? bf2f(bias[gc + 16 + e]) : 0.f);
     } else {
       sum_rows8(ws + (size_t)m * N + oc, splits, (size_t)M * N, v);
 #pragma unroll
@@ -379,7 +388,9 @@ gemv_kernel(GemmArgs p) {
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
       const int o = g * 16 + 2 * t + j;
-      if (o < p.N / 2) p.C[o] = f2bf(gate_act(acc[j], p.relu) * acc[2 + j]);
+      if (o >= p.N / 2) continue;
+      const float gb = p.bias ? bf2f(p.bias[rows[j]]) : 0.f, ub = p.bias ? bf2f(p.bias[rows[2 + j]]) : 0.f;
+      p.C[o] = f2bf(gate_act(acc[j] + gb, p.relu) * (acc[2 + j] + ub));
     }
   } else {
 #pragma unroll

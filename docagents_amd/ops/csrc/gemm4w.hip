@@ -285,6 +285,18 @@ gemm4w_kernel(GemmArgs p) {
   if constexpr (SW) {
     // W rows interleaved in 16-row (gate, up) groups: j = 2q is gate, 2q + 1 up of the wave's
     // output columns q*16 + 4 fg .. + 3
+    if (p.bias) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const int gc = min(n0 + wn * 128 + j * 16 + fg * 4, p.N - 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float b = T::to_f(p.bias[gc + e]);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) acc[i][j][e] += b;
+        }
+      }
+    }
 #pragma unroll
     for (int i = 0; i < 8; ++i)
 #pragma unroll

@@ -289,6 +289,21 @@ gemm8p_kernel(GemmArgs p) {
     if constexpr (EPI == EPI_SWIGLU) {
       // W rows interleaved in 16-row (gate, up) groups: j = 0 is gate, j = 1 is up of output columns
       // (n0 + jh*128 + wn*32) / 2 + 4 efg + q
+      if (p.bias) {
+#pragma unroll
+        for (int jh_ = 0; jh_ < 2; ++jh_)
+#pragma unroll
+          for (int j = 0; j < 2; ++j)
+#pragma unroll
+            for (int q = 0; q < 4; ++q) {
+              const int gc = n0 + jh_ * 128 + wn * 32 + j * 16 + efg * 4 + q;
+              const float b = gc < p.N ? T::to_f(p.bias[gc]) : 0.f;
+#pragma unroll
+              for (int ih = 0; ih < 2; ++ih)
+#pragma unroll
+                for (int i = 0; i < MI; ++i) acc[ih][jh_][i][j][q] += b;
+            }
+      }
 #pragma unroll
       for (int ih = 0; ih < 2; ++ih)
 #pragma unroll

@@ -10,23 +10,44 @@
 
 enum AnyEpi : int {
   ANY_NONE = 0,      // + bias
-  ANY_SOFTPLUS = 1,  // softplus(x + bias), fp32 out
+  ANY_SOFTPLUS = 1,  // softplus(x + bias), times a coefficient per column where lam is given
   ANY_REGLU = 2,     // W rows interleaved in 16-row (gate, up) groups: relu(g) * u
   ANY_RGLRU = 3,     // W rows interleaved in 16-row (recurrence, input) gate groups of one block
+  ANY_SWIGLU = 4,    // as ANY_REGLU: silu(g) * u
+  ANY_ACT = 5,       // C in the operands' type, times sigmoid(u) where u is given
 };
+constexpr bool any_paired(int epi) { return epi == ANY_REGLU || epi == ANY_RGLRU || epi == ANY_SWIGLU; }
 
 struct AnyArgs {
   const void* A; const void* W; void* C; const float* bias;
   int M, N, K, lda, ldc;
   long long sA, sW, sC, sBias;  // strides between the products of a batch, in elements
-  // ANY_RGLRU: decay factors and driving terms of the recurrence, from the gates and its input u
+  // ANY_RGLRU: decay factors and driving terms of the recurrence, from the gates and its input u.
+  // ANY_SOFTPLUS: lam [N] (nullable). ANY_ACT: u [M][ldu] (nullable), columns z N .. of product z
   const void* u; const float* lam; float* decay; float* drive; int ldu, ldg;
 };
 
 // Four neighbouring outputs of row m, columns n .. n + 3 (past N: not stored).
-template <int EPI>
+template <typename T, int EPI>
 __device__ __forceinline__ void any_block(const AnyArgs& p, int z, int m, int n, f32x4_t v) {
   if (n >= p.N) return;
+  if constexpr (EPI == ANY_ACT) {
+    T* o = (T*)p.C + z * p.sC + (size_t)m * p.ldc + n;
+    const T* g = p.u ? (const T*)p.u + (size_t)m * p.ldu + (size_t)z * p.N + n : nullptr;
+    if ((p.N & 3) == 0 && (p.ldc & 3) == 0) {
+      if (g) {
+        const f32x4_t u = Act<T>::load4(g);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] *= sigmoid32(u[e]);
+      }
+      Act<T>::store4(o, v);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (n + e < p.N) o[e] = Act<T>::from_f(g ? v[e] * sigmoid32(Act<T>::to_f(g[e])) : v[e]);
+    }
+    return;
+  }
   const float* bias = p.bias ? p.bias + z * p.sBias : nullptr;
   float* o = (float*)p.C + z * p.sC + (size_t)m * p.ldc + n;
   const bool vec = (p.N & 3) == 0 && (p.ldc & 3) == 0;
@@ -38,7 +59,7 @@ __device__ __forceinline__ void any_block(const AnyArgs& p, int z, int m, int n,
   }
   if constexpr (EPI == ANY_SOFTPLUS)
 #pragma unroll
-    for (int e = 0; e < 4; ++e) v[e] = softplus32(v[e]);
+    for (int e = 0; e < 4; ++e) v[e] = softplus32(v[e]) * (p.lam ? p.lam[min(n + e, p.N - 1)] : 1.f);
   if (vec) {
     *(f32x4_t*)o = v;
   } else {
@@ -71,9 +92,9 @@ __device__ __forceinline__ void any_pair(const AnyArgs& p, int z, int m, int nb,
   }
   const int col = nb / 2 + 4 * fg;
   f32x4_t r, d;
-  if constexpr (EPI == ANY_REGLU) {
+  if constexpr (EPI == ANY_REGLU || EPI == ANY_SWIGLU) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) r[e] = fmaxf(x[e], 0.f) * y[e];
+    for (int e = 0; e < 4; ++e) r[e] = (EPI == ANY_REGLU ? fmaxf(x[e], 0.f) : silu32(x[e])) * y[e];
     *(f32x4_t*)((float*)p.C + z * p.sC + (size_t)m * p.ldc + col) = r;
   } else {
     const int ch = z * (p.N / 2) + col;
@@ -174,7 +195,7 @@ __global__ void __launch_bounds__(256) gemm_any_kernel(AnyArgs p) {
   for (int i = 0; i < F; ++i) {
     const int m = m0 + wm * WT + i * 16 + fr;
     if (m >= p.M) continue;
-    if constexpr (EPI == ANY_REGLU || EPI == ANY_RGLRU) {
+    if constexpr (any_paired(EPI)) {
 #pragma unroll
       for (int jp = 0; jp < F / 2; ++jp) {
         const int nb = n0 + wn * WT + jp * 32;
@@ -186,7 +207,7 @@ __global__ void __launch_bounds__(256) gemm_any_kernel(AnyArgs p) {
       }
     } else {
 #pragma unroll
-      for (int j = 0; j < F; ++j) any_block<EPI>(p, z, m, n0 + wn * WT + j * 16 + 4 * fg, acc[i][j]);
+      for (int j = 0; j < F; ++j) any_block<T, EPI>(p, z, m, n0 + wn * WT + j * 16 + 4 * fg, acc[i][j]);
     }
   }
 }
@@ -268,9 +289,12 @@ __global__ void __launch_bounds__(256) gemm_walk_kernel(AnyArgs p) {
                     Act<bf16_t>::load4((const bf16_t*)(sA + ml * rowb) + nb / 2 + 4 * fg), v[i][0], v[i][1]);
       } else {
 #pragma unroll
-        for (int j = 0; j < 2; ++j)
+        for (int j = 0; j < 2; ++j) {
+          f32x4_t f{1.f, 1.f, 1.f, 1.f};
+          if (p.lam && nb + 16 * j < p.N) f = *(const f32x4_t*)(p.lam + nb + 16 * j + 4 * fg);
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[i][j][e] = softplus32(v[i][j][e]);
+          for (int e = 0; e < 4; ++e) v[i][j][e] = softplus32(v[i][j][e]) * f[e];
+        }
       }
     }
     __syncthreads();  // the A tile has been read
@@ -330,7 +354,7 @@ static int launch_any_t(const AnyArgs& a, int batch, hipStream_t s) {
 }
 
 // A [M, lda] and W [batch][N, K] of bf16 (f32 = 0) or fp32 (f32 = 1) elements with 16-byte aligned
-// rows, K a multiple of 16 bytes. The result is fp32.
+// rows, K a multiple of 16 bytes. The result is fp32, with ANY_ACT of the operands' type.
 DA_EXPORT int da_gemm_any(const void* A, int lda, const void* W, void* C, int ldc, const void* bias, int M, int N,
                           int K, int f32, int epi, int batch, long long sA, long long sW, long long sC,
                           long long sBias, const void* u, int ldu, const void* lam, void* decay, void* drive, int ldg,
@@ -338,9 +362,10 @@ DA_EXPORT int da_gemm_any(const void* A, int lda, const void* W, void* C, int ld
   const int e16 = f32 ? 4 : 8;
   if (M < 1 || N < 1 || K < 1 || batch < 1 || K % e16 || lda % e16 || sA % e16 || sW % e16 || (M + 63) / 64 > 65535)
     return (int)hipErrorInvalidValue;
-  if ((epi == ANY_REGLU || epi == ANY_RGLRU) && N % 32) return (int)hipErrorInvalidValue;
+  if (any_paired(epi) && N % 32) return (int)hipErrorInvalidValue;
   if (epi == ANY_RGLRU && (!u || !lam || !decay || !drive || ldu % 4 || ldg % 4)) return (int)hipErrorInvalidValue;
   if (epi != ANY_RGLRU && !C) return (int)hipErrorInvalidValue;
+  if (epi == ANY_ACT && (sC % 4 || (u && ldu % 4))) return (int)hipErrorInvalidValue;
   AnyArgs a{};
   a.A = A; a.W = W; a.C = C; a.bias = (const float*)bias;
   a.M = M; a.N = N; a.K = K; a.lda = lda; a.ldc = ldc;
@@ -354,6 +379,8 @@ DA_EXPORT int da_gemm_any(const void* A, int lda, const void* W, void* C, int ld
     ANY_CASE(ANY_SOFTPLUS)
     ANY_CASE(ANY_REGLU)
     ANY_CASE(ANY_RGLRU)
+    ANY_CASE(ANY_SWIGLU)
+    ANY_CASE(ANY_ACT)
     default: return (int)hipErrorInvalidValue;
   }
 #undef ANY_CASE

@@ -212,7 +212,8 @@ gemm_dk_kernel(DkArgs p) {
         const float gt = red[0][m][gc + e] + red[1][m][gc + e] + red[2][m][gc + e] + red[3][m][gc + e];
         const float up = red[0][m][gc + 16 + e] + red[1][m][gc + 16 + e] + red[2][m][gc + 16 + e] +
                          red[3][m][gc + 16 + e];
-        v[e] = gate_act(gt, p.relu) * up;
+        const int bc = min(n0 + gc + e, p.N - 17);  // a ragged last tile's empty groups are not stored
+        v[e] = gate_act(gt + (p.bias ? bf2f(p.bias[bc]) : 0.f), p.relu) * (up + (p.bias ? bf2f(p.bias[bc + 16]) : 0.f));
       }
       const int oc = n0 / 2 + 16 * g + 8 * hh;
       if (m < Mb && oc < p.N / 2) {  // a ragged last tile (N % BN == 32) holds one gate/up group

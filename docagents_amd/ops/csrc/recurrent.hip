@@ -15,37 +15,9 @@
 // batches of single tokens a thread's reads are its own: there the convolution replaces it).
 #include "seq.h"
 
-struct ConvState {
-  const void* x; int ldx;   // the convolution's inputs
-  void* state; int taps, C; // [slots][taps - 1][C], oldest first
-};
-
-// The last taps - 1 inputs of portion b's channel c, after its n tokens (the slot's older ones where the
-// portion is shorter; one thread per channel, old entries are read before they are overwritten).
-template <typename T>
-__device__ __forceinline__ void conv_state_store(const ConvState& s, const SeqMeta& m, int b, int c) {
-  if (!s.state) return;
-  const int s0 = m.cu[b], n = m.cu[b + 1] - s0, keep = s.taps - 1;
-  const bool start = m.pos0[b] == 0;
-  T* st = (T*)s.state + (size_t)m.slot[b] * keep * s.C + c;
-  const T* x = (const T*)s.x + c;
-  constexpr int U = 4;
-  for (int i0 = 0; i0 < keep; i0 += U) {
-    T v[U];
-#pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const int i = min(i0 + u, keep - 1), j = n - keep + i;
-      v[u] = j >= 0 ? x[(size_t)(s0 + j) * s.ldx] : (start ? Act<T>::from_f(0.f) : st[(size_t)(i + n) * s.C]);
-    }
-#pragma unroll
-    for (int u = 0; u < U; ++u)
-      if (i0 + u < keep) st[(size_t)(i0 + u) * s.C] = v[u];
-  }
-}
-
 // ------------------------------------------------------------------------------- convolution
 struct ConvArgs {
-  const void* x; const float* w; const float* bias; void* state; void* y;  // w [taps][C]
+  const void* x; const float* w; const float* bias; void* state; void* y;  // w [taps][C], bias nullable
   int ldx, ldy, C, taps;
   int update;  // single tokens only: replace the state
   SeqMeta m;
@@ -66,7 +38,8 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
   const int t0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * CONV_RUN;
   if (c >= a.C || t0 >= a.m.T) return;
   const int t1 = min(t0 + CONV_RUN, a.m.T);
-  const f32x4_t bias = *(const f32x4_t*)(a.bias + c);
+  f32x4_t bias{0.f, 0.f, 0.f, 0.f};
+  if (a.bias) bias = *(const f32x4_t*)(a.bias + c);
   auto emit = [&](int t, f32x4_t v) {
     if constexpr (SILU) {
 #pragma unroll

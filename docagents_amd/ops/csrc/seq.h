@@ -88,3 +88,32 @@ template <typename T> __device__ __forceinline__ float act_gelu_tanh(float x) {
   if constexpr (sizeof(T) == 4) return gelu_tanh32(x);
   return x * __builtin_amdgcn_rcpf(1.f + __expf(-1.5957691216057308f * (x + 0.044715f * x * x * x)));
 }
+
+// The state of a short causal convolution, replaced by the launch of the recurrence behind it.
+struct ConvState {
+  const void* x; int ldx;   // the convolution's inputs
+  void* state; int taps, C; // [slots][taps - 1][C], oldest first
+};
+
+// The last taps - 1 inputs of portion b's channel c, after its n tokens (the slot's older ones where the
+// portion is shorter; one thread per channel, old entries are read before they are overwritten).
+template <typename T>
+__device__ __forceinline__ void conv_state_store(const ConvState& s, const SeqMeta& m, int b, int c) {
+  if (!s.state) return;
+  const int s0 = m.cu[b], n = m.cu[b + 1] - s0, keep = s.taps - 1;
+  const bool start = m.pos0[b] == 0;
+  T* st = (T*)s.state + (size_t)m.slot[b] * keep * s.C + c;
+  const T* x = (const T*)s.x + c;
+  constexpr int U = 4;
+  for (int i0 = 0; i0 < keep; i0 += U) {
+    T v[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int i = min(i0 + u, keep - 1), j = n - keep + i;
+      v[u] = j >= 0 ? x[(size_t)(s0 + j) * s.ldx] : (start ? Act<T>::from_f(0.f) : st[(size_t)(i + n) * s.C]);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (i0 + u < keep) st[(size_t)(i0 + u) * s.C] = v[u];
+  }
+}

@@ -260,7 +260,7 @@ def gemm(a: torch.Tensor, w: torch.Tensor, bias=None, epi: int = EPI_NONE, resid
     _req(out.shape == (M, nout) and out.stride(1) == 1 and out.stride(0) % 8 == 0, "bad out")
     if bias is not None:
         _bf16_cuda(bias, "bias"); _req(bias.numel() == N and bias.is_contiguous(), "bias must be [N]")
-        _req(epi in (EPI_BIAS, EPI_GELU, EPI_RESID), "bias only with BIAS/GELU/RESID epilogues")
+        _req(epi in (EPI_BIAS, EPI_GELU, EPI_RESID, *GATED), "bias only with BIAS/GELU/RESID/gated epilogues")
     ldr = 0
     if epi == EPI_RESID:
         _req(resid is not None, "EPI_RESID needs resid")
@@ -1124,5 +1124,6 @@ def pool_l2norm_f16(h, cu_seqlens, mode: int = 0, out32=None, out16=None):
 
 
 # the batch-of-portions ops (recurrent mixers, paged attention, 32-bit residual stream)
-from .seq_kernels import (causal_conv, gated_scan, gemm_any, gemm_partials, partials_fit,  # noqa: E402,F401
-                          rglru_gates, selective_scan, sigmoid_attn, stream_final, stream_step)
+from .seq_kernels import (causal_conv, delta_rule, gated_scan, gemm_any, gemm_heads, gemm_partials,  # noqa: E402,F401
+                          latent_attn, latent_flash_fits, latent_prep, partials_fit, rglru_gates, selective_scan,
+                          sigmoid_attn, stream_add, stream_final, stream_step)

@@ -541,5 +541,6 @@ def flash_attn_f16(q, k, v, cu_seqlens, max_seqlen, H, Hkv, D, causal=False, sca
 
 
 # the batch-of-portions ops (recurrent mixers, paged attention, 32-bit residual stream)
-from .seq_reference import (causal_conv, gated_scan, gemm_any, gemm_partials, partials_fit,  # noqa: E402,F401
-                            rglru_gates, selective_scan, sigmoid_attn, stream_final, stream_step)
+from .seq_reference import (causal_conv, delta_rule, gated_scan, gemm_any, gemm_heads, gemm_partials,  # noqa: E402,F401
+                            latent_attn, latent_flash_fits, latent_prep, partials_fit, rglru_gates, selective_scan,
+                            sigmoid_attn, stream_add, stream_final, stream_step)

@@ -1,5 +1,5 @@
-"""Bindings of the batch-of-portions kernels (``csrc/stream_norm.hip``, ``recurrent.hip``,
-``paged_attn.hip``, ``gemm_any.hip``). Re-exported by ``kernels``; the fp32 oracles with the same
+"""Bindings of the batch-of-portions kernels (``csrc/stream_norm.hip``, ``recurrent.hip``, ``delta.hip``,
+``paged_attn.hip``, ``latent_attn.hip``, ``gemm_any.hip``). Re-exported by ``kernels``; the fp32 oracles with the same
 signatures are in ``seq_reference``. Activations are bf16, or fp32 in the fp32 precision; the residual
 stream, recurrent state, decays, step sizes and attention weights are fp32 in both."""
 from __future__ import annotations
@@ -18,7 +18,17 @@ K._SIGS.update({
     "da_gemm_partials": [c_void_p, c_int, c_void_p] + [c_int] * 5 + [c_void_p, c_void_p],
     "da_stream_step": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_float, c_float, c_int, c_int]
                       + [c_void_p] * 5 + _META + [c_int, c_int, c_void_p],
-    "da_stream_final": [c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_void_p, c_int, c_int, c_void_p],
+    "da_stream_final": [c_void_p, c_void_p, c_void_p, c_float, c_int, c_int, c_int, c_void_p, c_int, c_int, c_void_p],
+    "da_stream_add": [c_void_p] + [c_void_p, c_int, c_void_p, c_void_p] * 2 + [c_void_p, c_void_p, c_int, c_float]
+                     + [c_void_p, c_void_p, c_float, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p],
+    "da_delta_rule": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int] + [c_int] * 4
+                     + [c_float, c_float, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_int, c_int]
+                     + _META + [c_int, c_void_p],
+    "da_latent_prep": [c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p,
+                       c_void_p, c_int, c_void_p, c_int, c_void_p, c_int] + _META + [c_int, c_void_p],
+    "da_latent_attn": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p,
+                       c_void_p, c_int] + [c_int] * 6 + [c_float, c_void_p, c_void_p, c_int, c_int, c_int] + _META
+                      + [c_int, c_void_p],
     "da_causal_conv": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int] + _META
                       + [c_int, c_void_p],
     "da_selective_scan": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_int]
@@ -31,10 +41,11 @@ K._SIGS.update({
                        + _META + [c_int, c_void_p],
 })
 K._PART_OF.update({n: "hybrid" for n in ("da_gemm_any", "da_stream_step", "da_stream_final", "da_causal_conv",
-                                         "da_selective_scan", "da_gated_scan", "da_sigmoid_attn")})
+                                         "da_selective_scan", "da_gated_scan", "da_sigmoid_attn", "da_stream_add", "da_delta_rule",
+                                         "da_latent_prep", "da_latent_attn")})
 
 ACTS = (torch.bfloat16, torch.float32)
-ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_RGLRU = 0, 1, 2, 3
+ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_RGLRU, ANY_SWIGLU, ANY_ACT = 0, 1, 2, 3, 4, 5
 
 
 def _act(t, name, dtype=None):
@@ -65,19 +76,40 @@ def _scratch(m: SeqBatch, waves: int, fill: int, device, *shapes):
     return ws, [*map(_ptr, ws), _ptr(ck), _ptr(base), tot, n]
 
 
-def gemm_any(a, w, bias=None, epi: int = ANY_NONE):
+def gemm_any(a, w, bias=None, epi: int = ANY_NONE, coef=None):
     """fp32 [M, N'] = epi(a[M, K] @ w[N, K]^T + bias), a and w both bf16 or both fp32, bias fp32; any M and
-    N, K a multiple of 16 bytes. ANY_SOFTPLUS: softplus; ANY_REGLU: w rows interleaved by 16 (gate, up)."""
+    N, K a multiple of 16 bytes. ANY_SOFTPLUS: softplus, times coef (fp32 [N]) if given; ANY_REGLU / ANY_SWIGLU: w
+    rows interleaved by 16 (gate, up)."""
     f32 = _act(a, "a")
     _act(w, "w", a.dtype)
     M, Kd = a.shape
     N = w.shape[0]
-    _req(w.is_contiguous() and Kd == w.shape[1] and epi in (ANY_NONE, ANY_SOFTPLUS, ANY_REGLU), "gemm_any")
+    _req(w.is_contiguous() and Kd == w.shape[1] and epi in (ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_SWIGLU), "gemm_any")
     if bias is not None:
         _f32(bias, "bias", N)
-    out = torch.empty((M, N // 2 if epi == ANY_REGLU else N), dtype=torch.float32, device=a.device)
+    if coef is not None:
+        _f32(coef, "coef", N)
+        _req(epi == ANY_SOFTPLUS, "coef goes with softplus")
+    out = torch.empty((M, N // 2 if epi in (ANY_REGLU, ANY_SWIGLU) else N), dtype=torch.float32, device=a.device)
     _check(lib().da_gemm_any(_ptr(a), a.stride(0), _ptr(w), _ptr(out), out.stride(0), _ptr(bias), M, N, Kd, f32, epi, 1, 0,
-                             0, 0, 0, None, 0, None, None, None, 0, _stream()), "gemm_any")
+                             0, 0, 0, None, 0, _ptr(coef), None, None, 0, _stream()), "gemm_any")
+    return out
+
+
+def gemm_heads(a, w, stride: int, gate=None):
+    """Per head i: a[:, i * stride : + K] @ w[i]^T for w [H, N, K] -> [M, H * N] in the activation type, times
+    sigmoid(gate [M, H * N]) if given."""
+    f32 = _act(a, "a")
+    _act(w, "w", a.dtype)
+    (H, N, Kd), M = w.shape, a.shape[0]
+    _req(w.is_contiguous() and a.shape[1] >= (H - 1) * stride + Kd and stride >= Kd and N % 4 == 0, "gemm_heads operands")
+    out = torch.empty((M, H * N), dtype=a.dtype, device=a.device)
+    if gate is not None:
+        _act(gate, "gate", a.dtype)
+        _req(gate.shape == out.shape and gate.stride(0) % 4 == 0, "gate")
+    _check(lib().da_gemm_any(_ptr(a), a.stride(0), _ptr(w), _ptr(out), out.stride(0), None, M, N, Kd, f32, ANY_ACT, H, stride,
+                             N * Kd, N, 0, _ptr(gate), 0 if gate is None else gate.stride(0), None, None, None, 0,
+                             _stream()), "gemm_heads")
     return out
 
 
@@ -87,9 +119,9 @@ def partials_fit(M: int, N: int, Kd: int) -> bool:
     return 1 < M <= 128 and not (M <= K.DK_SPLITK_ABOVE and Kd % 256 == 0)
 
 
-def gemm_partials(a, w):
+def gemm_partials(a, w, own: bool = False):
     """bf16 a[M, K] @ w[N, K]^T as fp32 partials [splits, M, N] (their sum is the product), in the shared workspace:
-    valid until the next product."""
+    valid until the next product (own: in a buffer of their own)."""
     K._bf16_cuda(a, "a"); K._bf16_cuda(w, "w")
     M, Kd = a.shape
     N = w.shape[0]
@@ -97,7 +129,8 @@ def gemm_partials(a, w):
          and a.stride(0) % 8 == 0 and a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0, "gemm_partials operands")
     tile = 9 if M > 64 else K._decode_tile(M)
     splits = K._auto_splits(M, N, Kd)
-    ws = K._workspace(splits * M * N * 4, a.device)
+    n = splits * M * N * 4
+    ws = torch.empty(n, dtype=torch.uint8, device=a.device) if own else K._workspace(n, a.device)
     _check(lib().da_gemm_partials(_ptr(a), a.stride(0), _ptr(w), M, N, Kd, tile, splits, _ptr(ws), _stream()),
            "gemm_partials")
     return ws[:splits * M * N * 4].view(torch.float32).view(splits, M, N)
@@ -156,27 +189,66 @@ def stream_step(m: SeqBatch, dim: int, eps: float = 0.0, alpha: float = 1.0, ids
     return xo, ho
 
 
-def stream_final(x, w, eps: float, dim: int, act, rows=None):
-    """RMSNorm of the (selected: rows int64) stream rows in the activation type."""
+def stream_add(T: int, dim: int, eps: float, act, x=None, parts=(), ids=None, table=None, embed_scale: float = 1.0,
+               vec=None, w=None):
+    """One update of the fp32 residual stream [T, Dp]: x' = x + sum of scale (y + bias) over ``parts`` (at most two;
+    y [T, Dp] in the activation type or fp32 partials [splits, T, Dp], scale and bias fp32 [Dp], bias or None)
+    + table[ids] * embed_scale + vec; h = LayerNorm(x') w over ``dim`` of the padded columns, in the activation type
+    (w None: none). -> (x', h)."""
+    _req(len(parts) <= 2, "stream parts")
+    ref = x if x is not None else table
+    Dp, dev, f32 = ref.shape[-1], ref.device, int(act == torch.float32)
+    _req(Dp % 4 == 0 and dim <= Dp <= 16384, "stream columns")
+    if x is not None:
+        _f32(x, "x", T * Dp)
+    args = []
+    for y, scale, bias in (*parts, *[(None, None, None)] * (2 - len(parts))):
+        splits = 0
+        if y is not None:
+            splits = y.shape[0] if y.dim() == 3 else 0
+            _act(y, "y", torch.float32 if splits else act)
+            _req(y.is_contiguous() and y.shape[-2:] == (T, Dp), "y rows")
+            _f32(scale, "scale", Dp)
+            if bias is not None:
+                _f32(bias, "bias", Dp)
+        args += [_ptr(y), splits, _ptr(scale), _ptr(bias)]
+    if ids is not None:
+        _act(table, "table", act)
+        _req(table.is_contiguous() and table.shape[1] == Dp, "table")
+        _req(ids.dtype == torch.int32 and ids.is_contiguous() and ids.numel() >= T and ids.is_cuda, "ids")
+    for t, name in ((vec, "vec"), (w, "w")):
+        if t is not None:
+            _f32(t, name, Dp)
+    xo = torch.empty((T, Dp), dtype=torch.float32, device=dev)
+    ho = None if w is None else torch.empty((T, Dp), dtype=act, device=dev)
+    _check(lib().da_stream_add(_ptr(x), *args, _ptr(ids), _ptr(table) if ids is not None else None,
+                               0 if ids is None else table.shape[0], float(embed_scale), _ptr(vec), _ptr(w), float(eps), T,
+                               dim, Dp, _ptr(xo), _ptr(ho), f32, _stream()), "stream_add")
+    return xo, ho
+
+
+def stream_final(x, w, eps: float, dim: int, act, rows=None, center: bool = False):
+    """RMSNorm (center: LayerNorm) of the (selected: rows int64) stream rows in the activation type."""
     _f32(x, "x")
     _f32(w, "w", x.shape[1])
     if rows is not None:
         _req(rows.dtype == torch.int64 and rows.is_contiguous() and rows.is_cuda, "rows int64")
     n = x.shape[0] if rows is None else rows.numel()
     y = torch.empty((n, x.shape[1]), dtype=act, device=x.device)
-    _check(lib().da_stream_final(_ptr(x), _ptr(rows), _ptr(w), float(eps), dim, x.shape[1], _ptr(y), n,
+    _check(lib().da_stream_final(_ptr(x), _ptr(rows), _ptr(w), float(eps), dim, x.shape[1], int(center), _ptr(y), n,
                                  int(act == torch.float32), _stream()), "stream_final")
     return y
 
 
 def causal_conv(x, w, bias, state, m: SeqBatch, silu: bool):
     """Per-channel causal convolution over each portion: x [T, C] (row view), w fp32 [taps, C] (last row: the
-    current token), bias fp32 [C], state [slots, taps - 1, C]: the inputs before the portion, replaced here in
+    current token), bias fp32 [C] or None, state [slots, taps - 1, C]: the inputs before the portion, replaced here in
     batches of single tokens and by the recurrence's op otherwise."""
     f32 = _act(x, "x")
     taps, C = w.shape
     _f32(w, "w")
-    _f32(bias, "bias", C)
+    if bias is not None:
+        _f32(bias, "bias", C)
     _req(x.shape == (m.T, C) and x.stride(0) % 4 == 0 and C % 4 == 0, "conv input")
     _req(state.dtype == x.dtype and state.is_contiguous() and state.shape[1:] == (taps - 1, C), "conv state")
     y = torch.empty((m.T, C), dtype=x.dtype, device=x.device)
@@ -269,3 +341,79 @@ def sigmoid_attn(qkg, kc, kr, pb, qk_w, m: SeqBatch, H: int, G: int, dim: int, s
                                  pps if part is not None else -(-m.max_ctx // PAGE), m.max_len, int(m.singles), *_meta(m),
                                  f32, _stream()), "sigmoid_attn")
     return out
+
+
+def delta_rule(qkv, decay, beta, state, conv_x, conv_state, m: SeqBatch, H: int, G: int, q_scale: float, unit_eps: float,
+               norm):
+    """Gated delta rule: qkv [T, 2 G K + H V] (after the convolution), decay fp32 [T, H K] (log2 of each key channel's
+    decay), beta [T, >= H] before its sigmoid, state fp32 [slots, H, V, K], updated (and conv_state, see
+    ``selective_scan``). norm = (weight fp32 [V], gate [T, H V], true channels of a value head, eps): every head's
+    read-out is RMS-normed, weighted and gated. -> [T, H V] in the activation type."""
+    weight, gate, dim, eps = norm
+    f32 = _act(qkv, "qkv")
+    _act(beta, "beta", qkv.dtype)
+    _act(gate, "gate", qkv.dtype)
+    _, H2, V, Kd = state.shape
+    C = 2 * G * Kd + H * V
+    _f32(state, "state")
+    _f32(decay, "decay", m.T * H * Kd)
+    _f32(weight, "weight", V)
+    _req(H2 == H and qkv.shape == (m.T, C) and qkv.stride(0) % 4 == 0 and beta.shape[0] == m.T and beta.shape[1] >= H
+         and gate.shape == (m.T, H * V) and gate.stride(0) % 4 == 0 and V % 4 == 0, "delta_rule shapes")
+    o = torch.empty((m.T, H * V), dtype=qkv.dtype, device=qkv.device)
+    _check(lib().da_delta_rule(_ptr(qkv), qkv.stride(0), _ptr(decay), _ptr(beta), beta.stride(0), _ptr(state), _ptr(o), H * V,
+                               H, G, Kd, V, float(q_scale), float(unit_eps), _ptr(weight), _ptr(gate), gate.stride(0), dim,
+                               float(eps), *_conv_args(conv_x, conv_state, C, qkv.dtype, m), C, *_meta(m), f32, _stream()),
+           "delta_rule")
+    return o
+
+
+def _latent_pages(pages, rot, m: SeqBatch, rot_dim: int):
+    t = m.table
+    _act(pages, "pages")
+    _f32(rot, "rot")
+    _req(pages.is_contiguous() and pages.dim() == 3 and pages.shape[1] == PAGE, "pages")
+    _req(t is not None and t.is_cuda and t.dtype == torch.int32 and t.is_contiguous() and t.dim() == 2, "page table")
+    _req(rot.shape[1:] == (rot_dim // 2, 2) and rot.shape[0] >= t.shape[1] * PAGE, "rotary table")
+    _req(m.max_ctx <= t.shape[1] * PAGE, f"context {m.max_ctx} exceeds the page table ({t.shape[1]} pages)")
+    return t
+
+
+def latent_prep(x, q_w, q_dim: int, c_w, c_dim: int, rot_dim: int, eps: float, pages, rot, m: SeqBatch):
+    """x [T, >= Q + L + R] = [query latent | latent | key part]: the query latent RMS-normed (weight q_w fp32 [Q], over
+    q_dim columns) is returned; the latent, normed likewise, and the key part, rotated, go to the token's row of
+    ``pages`` [pages, 64, L + R]. rot: fp32 [positions, rot_dim / 2, 2]."""
+    f32 = _act(x, "x", pages.dtype)
+    Q, L, W = q_w.numel(), c_w.numel(), pages.shape[2]
+    _f32(q_w, "q_w")
+    _f32(c_w, "c_w")
+    t = _latent_pages(pages, rot, m, rot_dim)
+    _req(x.shape[0] == m.T and x.shape[1] >= Q + W and x.stride(0) % 4 == 0 and Q % 4 == 0 and L % 4 == 0 and W > L, "x")
+    cq = torch.empty((m.T, Q), dtype=x.dtype, device=x.device)
+    _check(lib().da_latent_prep(_ptr(x), x.stride(0), _ptr(q_w), Q, q_dim, _ptr(c_w), L, c_dim, W - L, rot_dim, float(eps),
+                                _ptr(cq), _ptr(pages), pages.shape[0], _ptr(t), t.shape[1], _ptr(rot), rot.shape[0],
+                                *_meta(m), f32, _stream()), "latent_prep")
+    return cq
+
+
+def latent_attn(q, ql, pages, rot, sink, m: SeqBatch, H: int, rot_at: int, rot_dim: int, L: int, scale: float):
+    """Attention in the latent space: ql [T, H L] queries against the latents, q [T, H D] the queries whose rotated part
+    (before rotation) starts at column rot_at of a head; sink fp32 [H] -> sum of weight * latent, [T, H L]."""
+    f32 = _act(q, "q", pages.dtype)
+    _act(ql, "ql", pages.dtype)
+    _f32(sink, "sink", H)
+    t = _latent_pages(pages, rot, m, rot_dim)
+    D, W = q.shape[1] // H, pages.shape[2]
+    _req(q.shape == (m.T, H * D) and ql.shape == (m.T, H * L) and rot_at + rot_dim <= D and L + rot_dim <= W, "query columns")
+    _req(L <= 1152 and W <= 1216, f"latents of {W} columns")
+    out = torch.empty((m.T, H * L), dtype=q.dtype, device=q.device)
+    part, ml, nsplit, pps = None, None, 1, -(-m.max_ctx // PAGE)
+    _check(lib().da_latent_attn(_ptr(q), q.stride(0), _ptr(ql), ql.stride(0), _ptr(pages), pages.shape[0], _ptr(t), t.shape[1],
+                                _ptr(rot), rot.shape[0], _ptr(sink), _ptr(out), out.stride(0), H, D, rot_at, rot_dim, L, W - L,
+                                float(scale), _ptr(part), _ptr(ml), nsplit, pps, m.max_len, *_meta(m), f32, _stream()),
+           "latent_attn")
+    return out
+
+
+def latent_flash_fits(D: int, V: int) -> bool:
+    return False

@@ -9,7 +9,7 @@ import torch.nn.functional as F
 
 from .seq_batch import PAGE, SeqBatch
 
-ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_RGLRU = 0, 1, 2, 3
+ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_RGLRU, ANY_SWIGLU = 0, 1, 2, 3, 4
 
 
 def _portions(m: SeqBatch):
@@ -24,23 +24,29 @@ def _ungroup(y):
     return yy[..., 0, :].flatten(-2), yy[..., 1, :].flatten(-2)
 
 
-def gemm_any(a, w, bias=None, epi: int = ANY_NONE):
+def gemm_any(a, w, bias=None, epi: int = ANY_NONE, coef=None):
     y = a.float() @ w.float().t()
     if bias is not None:
         y = y + bias
     if epi == ANY_SOFTPLUS:
-        return F.softplus(y)
-    if epi == ANY_REGLU:
+        return F.softplus(y) if coef is None else F.softplus(y) * coef
+    if epi in (ANY_REGLU, ANY_SWIGLU):
         g, u = _ungroup(y)
-        return F.relu(g) * u
+        return (F.relu(g) if epi == ANY_REGLU else F.silu(g)) * u
     return y
+
+
+def gemm_heads(a, w, stride: int, gate=None):
+    H, N, K = w.shape
+    y = torch.cat([a[:, i * stride:i * stride + K].float() @ w[i].float().t() for i in range(H)], 1)
+    return (y if gate is None else y * torch.sigmoid(gate.float())).to(a.dtype)
 
 
 def partials_fit(M: int, N: int, K: int) -> bool:
     return False
 
 
-def gemm_partials(a, w):
+def gemm_partials(a, w, own: bool = False):
     return (a.float() @ w.float().t())[None]
 
 
@@ -76,8 +82,31 @@ def stream_step(m: SeqBatch, dim: int, eps: float = 0.0, alpha: float = 1.0, ids
     return (xo if want_x else None), (h.to(act) if want_h else None)
 
 
-def stream_final(x, w, eps: float, dim: int, act, rows=None):
+def _layer_norm(x, w, eps: float, dim: int):
+    v = x[:, :dim] - x[:, :dim].mean(-1, keepdim=True)
+    out = torch.zeros_like(x)
+    out[:, :dim] = v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w[:dim]
+    return out
+
+
+def stream_add(T: int, dim: int, eps: float, act, x=None, parts=(), ids=None, table=None, embed_scale: float = 1.0,
+               vec=None, w=None):
+    out = None if x is None else x.clone()
+    for y, scale, bias in parts:
+        y = y.sum(0) if y.dim() == 3 else y.float()
+        out = out + (y if bias is None else y + bias) * scale
+    if ids is not None:
+        e = table[ids.long()].float() * embed_scale
+        out = e if out is None else out + e
+    if vec is not None:
+        out = out + vec
+    return out, None if w is None else _layer_norm(out, w, eps, dim).to(act)
+
+
+def stream_final(x, w, eps: float, dim: int, act, rows=None, center: bool = False):
     v = x if rows is None else x[rows]
+    if center:
+        return _layer_norm(v, w, eps, dim).to(act)
     return (v / torch.sqrt(v.pow(2).sum(-1, keepdim=True) / dim + eps) * w).to(act)
 
 
@@ -87,7 +116,7 @@ def causal_conv(x, w, bias, state, m: SeqBatch, silu: bool):
     for t0, t1, s, p in _portions(m):
         old = state[s].float() if p > 0 else torch.zeros(taps - 1, x.shape[1])
         full = torch.cat([old, x[t0:t1].float()])
-        y[t0:t1] = bias + sum(w[k] * full[k:k + t1 - t0] for k in range(taps))
+        y[t0:t1] = (0 if bias is None else bias) + sum(w[k] * full[k:k + t1 - t0] for k in range(taps))
     return (F.silu(y) if silu else y).to(x.dtype)
 
 
@@ -150,4 +179,71 @@ def sigmoid_attn(qkg, kc, kr, pb, qk_w, m: SeqBatch, H: int, G: int, dim: int, s
         wt = torch.sigmoid(sc) * torch.ones(n, p + n).tril(p)
         o = (wt @ ks).transpose(0, 1) * torch.sigmoid(gate)[..., None]
         out[t0:t1] = o.reshape(n, H * D).to(qkg.dtype)
+    return out
+
+
+def delta_rule(qkv, decay, beta, state, conv_x, conv_state, m: SeqBatch, H: int, G: int, q_scale: float, unit_eps: float,
+               norm):
+    weight, gate, dim, eps = norm
+    _, _, V, K = state.shape
+    g = H // G
+    T = qkv.shape[0]
+    unit = lambda x: x / torch.sqrt(x.pow(2).sum(-1, keepdim=True) + unit_eps)  # noqa: E731
+    q = (unit(qkv[:, :G * K].float().view(T, G, K)) * q_scale).repeat_interleave(g, 1)
+    k = unit(qkv[:, G * K:2 * G * K].float().reshape(T, G, K)).repeat_interleave(g, 1)
+    v = qkv[:, 2 * G * K:].float().reshape(T, H, V)
+    b, a = torch.sigmoid(beta[:, :H].float()), torch.exp2(decay.view(T, H, K))
+    y = torch.empty(T, H, V)
+    for t0, t1, s, p in _portions(m):
+        S = state[s].clone() if p > 0 else torch.zeros_like(state[s])
+        for t in range(t0, t1):
+            S = S * a[t][:, None]
+            u = b[t][:, None] * (v[t] - (S @ k[t][:, :, None])[..., 0])
+            S = S + u[:, :, None] * k[t][:, None]
+            y[t] = (S @ q[t][:, :, None])[..., 0]
+        state[s] = S
+        _save_conv(conv_x, conv_state, t0, t1, s, p)
+    y = y.to(qkv.dtype).float()
+    y = y / torch.sqrt(y.pow(2).sum(-1, keepdim=True) / dim + eps) * weight
+    return (y.flatten(1) * torch.sigmoid(gate.float())).to(qkv.dtype)
+
+
+def latent_flash_fits(D: int, V: int) -> bool:
+    return False
+
+
+def _turn(x, cs, R: int):
+    """The first R columns of x [..., n] turned by the angles whose cos and sin are cs [..., R / 2, 2]."""
+    h = R // 2
+    u, v, c, s = x[..., :h], x[..., h:R], cs[..., 0], cs[..., 1]
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., R:]], -1)
+
+
+def latent_prep(x, q_w, q_dim: int, c_w, c_dim: int, rot_dim: int, eps: float, pages, rot, m: SeqBatch):
+    Q, L, W = q_w.numel(), c_w.numel(), pages.shape[2]
+    rms = lambda v, n: v / torch.sqrt(v.pow(2).sum(-1, keepdim=True) / n + eps)  # noqa: E731
+    cq = rms(x[:, :Q].float(), q_dim) * q_w
+    c = rms(x[:, Q:Q + L].float(), c_dim) * c_w
+    kr = x[:, Q + L:Q + W].float()
+    table = m.table.tolist()
+    for t0, t1, s, p in _portions(m):
+        row = torch.cat([c[t0:t1], _turn(kr[t0:t1], rot[p:p + t1 - t0], rot_dim)], 1).to(pages.dtype)
+        for i in range(t1 - t0):
+            pages[table[s][(p + i) // PAGE], (p + i) % PAGE] = row[i]
+    return cq.to(x.dtype)
+
+
+def latent_attn(q, ql, pages, rot, sink, m: SeqBatch, H: int, rot_at: int, rot_dim: int, L: int, scale: float):
+    D = q.shape[1] // H
+    out = torch.empty((m.T, H * L), dtype=q.dtype)
+    table = m.table.tolist()
+    for t0, t1, s, p in _portions(m):
+        n = t1 - t0
+        qr = q[t0:t1].float().view(n, H, D)[:, :, rot_at:rot_at + rot_dim]
+        qr = _turn(qr, rot[p:p + n, None], rot_dim).to(q.dtype).float()
+        c = pages[table[s][:(p + n + PAGE - 1) // PAGE]].float().flatten(0, 1)[:p + n]
+        sc = ql[t0:t1].float().view(n, H, L) @ c[:, :L].t() + qr @ c[:, L:L + rot_dim].t()
+        sc = (sc * scale).masked_fill(torch.ones(n, p + n).triu(p + 1)[:, None].bool(), -math.inf)
+        w = torch.softmax(torch.cat([sc, sink[None, :, None].expand(n, H, 1)], -1), -1)[..., :-1]
+        out[t0:t1] = (w @ c[:, :L]).reshape(n, H * L).to(q.dtype)
     return out
