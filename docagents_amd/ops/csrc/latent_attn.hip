@@ -188,6 +188,449 @@ static int launch_lat_any_t(const LatArgs& a, hipStream_t s) {
   return launch_lat_any<T, 16, 72>(a, s);
 }
 
+// ------------------------------------------------------------------------------- matrix cores, absorbed
+// 16 query rows per workgroup, 4 waves, one page per step. A wave loads its 16 keys of the page in the score
+// product's operand layout straight to registers (S^T = K Q^T on 16x16x32 MFMAs), and leaves their latents in LDS for
+// the transposing reads of the sum, O^T += C^T P^T, in which it owns a quarter of the latent's columns for all keys of the
+// page. The next page's loads are in flight during the sum. A weight enters the second product as two bf16 terms (its
+// rounding and the remainder), so its fp32 value counts to about 16 bits.
+template <int L> struct LD {
+  static constexpr int VSTR = L == 64 ? 192 : L * 2 + 64;  // bytes of a latent in LDS
+  static constexpr int PSTR = PAGE * 2 + 16;               // bytes of a row's weights
+  static constexpr int OFF_P = PAGE * VSTR, OFF_MX = OFF_P + 2 * 16 * PSTR, BYTES = OFF_MX + 4 * 16 * 4;
+};
+
+__device__ __forceinline__ unsigned split_lo(unsigned hi, float a, float b) {
+  return pack_bf2(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
+}
+
+template <int L, int R>
+__global__ void __launch_bounds__(256, 2) latent_mfma_kernel(LatArgs a, int rtiles, int ntiles) {
+  using C = LD<L>;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  constexpr int W = L + R, NDS = W / 32, NLS = L / 32, NDB = L / 64;
+  // the row tiles of one split of a portion follow each other on one XCD: its pages are read from HBM once
+  const int id = xcd_remap(blockIdx.x, ntiles);
+  const int rt = id % rtiles, split = id / rtiles % a.nsplit, b = id / rtiles / a.nsplit;
+  const int s0 = a.m.cu[b], n = a.m.cu[b + 1] - s0, rows = n * a.H;
+  if (rt * 16 >= rows) return;
+  const int pos0 = a.m.pos0[b], slot = a.m.slot[b];
+  const int klast = pos0 + min(rt * 16 + 15, rows - 1) / a.H;  // last key of the tile
+  const int p0 = split * a.pps, p1 = min(p0 + a.pps, klast / PAGE + 1);
+  if (p0 >= p1) return;
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, fr = lane & 15, fg = lane >> 4;
+  const int row = rt * 16 + fr, rc = min(row, rows - 1), tok = rc / a.H, hd = rc % a.H;
+  const int qpos = pos0 + tok;
+  char* sV = smem;
+  char* sP = smem + C::OFF_P;
+  float* sM = (float*)(smem + C::OFF_MX);
+
+  bf16x8_t qf[NDS];
+  const bf16_t* ql = (const bf16_t*)a.ql + (size_t)(s0 + tok) * a.ldl + (size_t)hd * L + fg * 8;
+#pragma unroll
+  for (int ds = 0; ds < NLS; ++ds) qf[ds] = *(const bf16x8_t*)(ql + ds * 32);
+  const bf16_t* qr = (const bf16_t*)a.q + (size_t)(s0 + tok) * a.ldq + (size_t)hd * a.D + a.ra;
+  const float* cs = a.rot + (size_t)min(qpos, a.npos - 1) * a.rdim;
+#pragma unroll
+  for (int ds = NLS; ds < NDS; ++ds)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) qf[ds][e] = (short)f2bf(rotated<bf16_t>(qr, cs, a.rdim, (ds - NLS) * 32 + fg * 8 + e));
+  const float c2 = a.scale * LOG2E;
+
+  bf16x8_t kf[NDS];
+  const int key = wv * 16 + fr;  // the key of a page this lane loads
+  auto load_page = [&](int p) {
+    const bf16_t* kp = (const bf16_t*)a.pages + ((size_t)lat_page(a, slot, p) * PAGE + key) * W + fg * 8;
+    const bool in = p * PAGE + key <= klast;  // rows past it may hold anything: read as zero
+#pragma unroll
+    for (int ds = 0; ds < NDS; ++ds) {
+      const u32x4_t v = *(const u32x4_t*)(kp + ds * 32);
+      kf[ds] = __builtin_bit_cast(bf16x8_t, in ? v : u32x4_t{0, 0, 0, 0});
+    }
+  };
+  f32x4_t oacc[NDB];
+#pragma unroll
+  for (int i = 0; i < NDB; ++i) oacc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float mx = -1e30f, sum = 0.f;  // of row fr: common to the waves; over this lane's keys
+  load_page(p0);
+  for (int p = p0; p < p1; ++p) {
+    f32x4_t s{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ds = 0; ds < NDS; ++ds) s = mfma16(kf[ds], qf[ds], s);
+    float top = -1e30f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      s[e] = p * PAGE + wv * 16 + fg * 4 + e <= qpos ? s[e] * c2 : -INFINITY;
+      top = fmaxf(top, s[e]);
+    }
+    top = fmaxf(top, __shfl_xor(top, 16, 64));
+    top = fmaxf(top, __shfl_xor(top, 32, 64));
+    if (fg == 0) sM[wv * 16 + fr] = top;
+    __syncthreads();  // maxima written; every wave is done with the last page's latents and weights
+#pragma unroll
+    for (int ds = 0; ds < NLS; ++ds) *(bf16x8_t*)(sV + key * C::VSTR + ds * 64 + fg * 16) = kf[ds];
+    if (p + 1 < p1) load_page(p + 1);
+    const float mnew = fmaxf(mx, fmaxf(fmaxf(sM[fr], sM[16 + fr]), fmaxf(sM[32 + fr], sM[48 + fr])));
+    const float f = __builtin_amdgcn_exp2f(mx - mnew);
+    mx = mnew;
+    sum *= f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      s[e] = __builtin_amdgcn_exp2f(s[e] - mnew);
+      sum += s[e];
+    }
+    const unsigned h0 = pack_bf2(s[0], s[1]), h1 = pack_bf2(s[2], s[3]);
+    char* pp = sP + fr * C::PSTR + (wv * 16 + fg * 4) * 2;
+    *(u32x2_t*)pp = u32x2_t{h0, h1};
+    *(u32x2_t*)(pp + 16 * C::PSTR) = u32x2_t{split_lo(h0, s[0], s[1]), split_lo(h1, s[2], s[3])};
+#pragma unroll
+    for (int i = 0; i < NDB; ++i) oacc[i] *= f;
+    __syncthreads();
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
+      // k slot 8 fg + j of the product holds key 32 half + 16 (j / 4) + 4 fg + j % 4
+      const char* pr = sP + fr * C::PSTR + (half * 32 + fg * 4) * 2;
+      const u32x2_t ha = *(const u32x2_t*)pr, hb = *(const u32x2_t*)(pr + 32);
+      const u32x2_t la = *(const u32x2_t*)(pr + 16 * C::PSTR), lb = *(const u32x2_t*)(pr + 16 * C::PSTR + 32);
+      const bf16x8_t bh = __builtin_bit_cast(bf16x8_t, u32x4_t{ha[0], ha[1], hb[0], hb[1]});
+      const bf16x8_t bl = __builtin_bit_cast(bf16x8_t, u32x4_t{la[0], la[1], lb[0], lb[1]});
+      const int vrow = half * 32 + 4 * fg + (fr >> 2);
+#pragma unroll
+      for (int db = 0; db < NDB; ++db) {
+        const char* vp = sV + vrow * C::VSTR + ((wv * NDB + db) * 16 + 4 * (fr & 3)) * 2;
+        const s16x4_t lo = lds_read_tr16(vp), up = lds_read_tr16(vp + 16 * C::VSTR);
+        const bf16x8_t va = bf16x8_t{lo[0], lo[1], lo[2], lo[3], up[0], up[1], up[2], up[3]};
+        oacc[db] = mfma16(va, bh, oacc[db]);
+        oacc[db] = mfma16(va, bl, oacc[db]);
+      }
+    }
+  }
+  sum += __shfl_xor(sum, 16, 64);
+  sum += __shfl_xor(sum, 32, 64);
+  __syncthreads();
+  if (fg == 0) sM[wv * 16 + fr] = sum;
+  __syncthreads();
+  sum = sM[fr] + sM[16 + fr] + sM[32 + fr] + sM[48 + fr];
+  if (row >= rows) return;
+  if (a.nsplit > 1) {
+    const size_t at = ((size_t)b * a.rows + row) * a.nsplit + split;
+    if (wv == 0 && fg == 0) *(f32x2_t*)(a.part_ml + at * 2) = f32x2_t{mx, sum};
+#pragma unroll
+    for (int db = 0; db < NDB; ++db) *(f32x4_t*)(a.part + at * L + (wv * NDB + db) * 16 + fg * 4) = oacc[db];
+  } else {
+    const float sink = a.sink[hd] * LOG2E, m2 = fmaxf(mx, sink);
+    const float f = __builtin_amdgcn_exp2f(mx - m2), inv = f / fmaf(sum, f, __builtin_amdgcn_exp2f(sink - m2));
+    bf16_t* o = (bf16_t*)a.out + (size_t)(s0 + tok) * a.ldo + (size_t)hd * L;
+#pragma unroll
+    for (int db = 0; db < NDB; ++db) Act<bf16_t>::store4(o + (wv * NDB + db) * 16 + fg * 4, oacc[db] * inv);
+  }
+}
+
+// The splits of a row put together, and the sink. L / 4 threads (64 at least).
+__global__ void latent_combine_kernel(LatArgs a) {
+  const int row = blockIdx.x, b = blockIdx.y, s0 = a.m.cu[b], n = a.m.cu[b + 1] - s0;
+  if (row >= n * a.H) return;
+  const int tok = row / a.H, hd = row % a.H;
+  const int used = min(a.nsplit, ((a.m.pos0[b] + tok) / PAGE + a.pps) / a.pps);  // splits that hold keys the row sees
+  const size_t at = ((size_t)b * a.rows + row) * a.nsplit;
+  const float sink = a.sink[hd] * LOG2E;
+  float m = sink;
+  for (int s = 0; s < used; ++s) m = fmaxf(m, a.part_ml[(at + s) * 2]);
+  float sum = __builtin_amdgcn_exp2f(sink - m);
+  const int c = threadIdx.x * 4;
+  f32x4_t v{0.f, 0.f, 0.f, 0.f};
+  for (int q = 0; q < used; q += 8) {
+    f32x4_t x[8];
+    f32x2_t ml[8];
+#pragma unroll
+    for (int s = 0; s < 8; ++s) {
+      const size_t i = at + min(q + s, used - 1);
+      x[s] = *(const f32x4_t*)(a.part + i * a.L + min(c, a.L - 4));
+      ml[s] = *(const f32x2_t*)(a.part_ml + i * 2);
+    }
+#pragma unroll
+    for (int s = 0; s < 8; ++s) {
+      const float f = q + s < used ? __builtin_amdgcn_exp2f(ml[s][0] - m) : 0.f;
+      sum = fmaf(ml[s][1], f, sum);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = fmaf(x[s][e], f, v[e]);
+    }
+  }
+  if (c < a.L) Act<bf16_t>::store4((bf16_t*)a.out + (size_t)(s0 + tok) * a.ldo + (size_t)hd * a.L + c, v * (1.f / sum));
+}
+
+template <int L, int R>
+static int launch_lat_mfma(const LatArgs& a, hipStream_t s) {
+  static const hipError_t e = hipFuncSetAttribute((const void*)latent_mfma_kernel<L, R>,
+                                                  hipFuncAttributeMaxDynamicSharedMemorySize, LD<L>::BYTES);
+  if (e != hipSuccess) return (int)e;
+  const int rtiles = (a.rows + 15) / 16;
+  const long long tiles = (long long)rtiles * a.nsplit * a.m.B;
+  if (tiles > 0x7fffffffll) return (int)hipErrorInvalidValue;
+  latent_mfma_kernel<L, R><<<(int)tiles, 256, LD<L>::BYTES, s>>>(a, rtiles, (int)tiles);
+  if (a.nsplit > 1) latent_combine_kernel<<<dim3(a.rows, a.m.B), L < 256 ? 64 : L / 4, 0, s>>>(a);
+  DA_LAUNCH_CHECK();
+}
+static bool lat_mfma_dims(int L, int R) { return (L == 64 || L == 128 || L == 256 || L == 512) && (R == 32 || R == 64); }
+static int launch_lat_mfma_t(const LatArgs& a, hipStream_t s) {
+#define LAT_CASE(LL, RR) \
+  if (a.L == LL && a.R == RR) return launch_lat_mfma<LL, RR>(a, s);
+  LAT_CASE(64, 32) LAT_CASE(64, 64) LAT_CASE(128, 32) LAT_CASE(128, 64)
+  LAT_CASE(256, 32) LAT_CASE(256, 64) LAT_CASE(512, 32) LAT_CASE(512, 64)
+#undef LAT_CASE
+  return (int)hipErrorInvalidValue;
+}
+
+// ------------------------------------------------------------------------------- matrix cores, expanded
+// A page of a portion's context per workgroup: its cache rows to row cctx[b] + position of a packed matrix.
+__global__ void __launch_bounds__(256) latent_gather_kernel(LatArgs a, const int* cctx, bf16_t* lat) {
+  const int b = blockIdx.y, p = blockIdx.x, W = a.L + a.R, c0 = cctx[b];
+  const int n = min(PAGE, cctx[b + 1] - c0 - p * PAGE);
+  if (n <= 0) return;
+  const u32x4_t* src = (const u32x4_t*)((const bf16_t*)a.pages + (size_t)lat_page(a, a.m.slot[b], p) * PAGE * W);
+  u32x4_t* dst = (u32x4_t*)(lat + (size_t)(c0 + p * PAGE) * W);
+  for (int i = threadIdx.x; i < n * W / 8; i += 256) dst[i] = src[i];
+}
+
+struct FlashArgs {
+  LatArgs a;                  // q, rot, sink, out [T][H V], m
+  const int* cctx;            // rows of portion b's context in lat / kv: cctx[b] + position
+  const bf16_t* lat;          // [contexts][L + R]
+  const bf16_t* kv; int ldkv; // [contexts][H][d keys | V values]
+  const bf16_t* gate; int ldg;
+  int qtiles;
+};
+
+// 128 query rows (tokens) of one head per workgroup (4 waves x 32), 64 keys per step: S^T = K Q^T on 32x32x16 MFMAs, a
+// lane owns one query and 32 of the step's keys; its weights stay in registers as the B operand of O^T += V^T P^T. The
+// next step's keys are in flight while this one's are used.
+template <int D, int V> struct LF {
+  static constexpr int KSTR = D * 2 + 16;
+  static constexpr int VSTR = (V % 64 == 32) ? V * 2 : (V == 64 ? 192 : V * 2 + 64);
+  static constexpr int KB = PAGE * KSTR, BYTES = KB + PAGE * VSTR;
+};
+
+template <int D, int V>
+__global__ void __launch_bounds__(256, 2) latent_flash_kernel(FlashArgs p, int ntiles) {
+  using C = LF<D, V>;
+  const LatArgs& a = p.a;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  constexpr int NDS = D / 16, NDB = V / 32, KP = D / 32, VP = V / 32;  // MFMA steps, blocks; 16-byte pieces per thread
+  // a head's tiles follow each other on one XCD (they read the same keys), the longest first
+  const int id = xcd_remap(blockIdx.x, ntiles);
+  const int qt = p.qtiles - 1 - id % p.qtiles, hd = id / p.qtiles % a.H, b = id / p.qtiles / a.H;
+  const int s0 = a.m.cu[b], n = a.m.cu[b + 1] - s0;
+  if (qt * 128 >= n) return;
+  const int pos0 = a.m.pos0[b], c0 = p.cctx[b], nctx = p.cctx[b + 1] - c0;
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, qr = lane & 31, hi = lane >> 5;
+  const int tok = qt * 128 + wv * 32 + qr, tc = min(tok, n - 1), qpos = pos0 + tc;
+  const int wfirst = pos0 + min(qt * 128 + wv * 32, n - 1), wlast = pos0 + min(qt * 128 + wv * 32 + 31, n - 1);
+  const int klast = min(pos0 + min(qt * 128 + 127, n - 1), nctx - 1), nt = klast / PAGE + 1;
+  const int d = a.ra, W = a.L + a.R;
+
+  bf16x8_t qf[NDS];
+  const bf16_t* qp = (const bf16_t*)a.q + (size_t)(s0 + tc) * a.ldq + (size_t)hd * a.D;
+  const float* cs = a.rot + (size_t)min(qpos, a.npos - 1) * a.rdim;
+#pragma unroll
+  for (int ds = 0; ds < NDS; ++ds) {
+    const int c = ds * 16 + hi * 8;
+    if (c < d) {
+      qf[ds] = *(const bf16x8_t*)(qp + c);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) qf[ds][e] = (short)f2bf(rotated<bf16_t>(qp + d, cs, a.rdim, c - d + e));
+    }
+  }
+  const float c2 = a.scale * LOG2E;
+
+  u32x4_t kreg[KP], vreg[VP];
+  auto load = [&](int t) {
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int pc = tid + 256 * i, r = pc / (D / 8), c = pc % (D / 8) * 8;
+      const int k = min(t * PAGE + r, klast);
+      const bf16_t* src = c < d ? p.kv + (size_t)(c0 + k) * p.ldkv + (size_t)hd * (d + V) + c
+                                : p.lat + (size_t)(c0 + k) * W + a.L + min(c - d, a.R - 8);
+      kreg[i] = *(const u32x4_t*)src;
+      if (c >= d + a.R) kreg[i] = u32x4_t{0, 0, 0, 0};
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int pc = tid + 256 * i, r = pc / (V / 8), c = pc % (V / 8) * 8;
+      vreg[i] = *(const u32x4_t*)(p.kv + (size_t)(c0 + min(t * PAGE + r, klast)) * p.ldkv + (size_t)hd * (d + V) + d + c);
+    }
+  };
+  auto store = [&]() {
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int pc = tid + 256 * i;
+      *(u32x4_t*)(smem + pc / (D / 8) * C::KSTR + pc % (D / 8) * 16) = kreg[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int pc = tid + 256 * i;
+      *(u32x4_t*)(smem + C::KB + pc / (V / 8) * C::VSTR + pc % (V / 8) * 16) = vreg[i];
+    }
+  };
+  f32x16_t oacc[NDB];
+#pragma unroll
+  for (int i = 0; i < NDB; ++i)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) oacc[i][e] = 0.f;
+  float mx = a.sink[hd] * LOG2E, sum = 1.f;
+
+  load(0);
+  for (int t = 0; t < nt; ++t) {
+    __syncthreads();
+    store();
+    __syncthreads();
+    if (t + 1 < nt) load(t + 1);
+    const int kb = t * PAGE;
+    if (kb > wlast) continue;
+    f32x16_t s[2];
+#pragma unroll
+    for (int hh = 0; hh < 2; ++hh) {
+#pragma unroll
+      for (int e = 0; e < 16; ++e) s[hh][e] = 0.f;
+#pragma unroll
+      for (int ds = 0; ds < NDS; ++ds) {
+        const bf16x8_t kf = *(const bf16x8_t*)(smem + (hh * 32 + qr) * C::KSTR + ds * 32 + hi * 16);
+        s[hh] = mfma32(kf, qf[ds], s[hh]);
+      }
+    }
+    if (kb + PAGE - 1 > wfirst) {
+#pragma unroll
+      for (int hh = 0; hh < 2; ++hh)
+#pragma unroll
+        for (int e = 0; e < 16; ++e)
+          if (kb + hh * 32 + 8 * (e >> 2) + 4 * hi + (e & 3) > qpos) s[hh][e] = -INFINITY;
+    }
+    float top = s[0][0];
+#pragma unroll
+    for (int e = 1; e < 16; ++e) top = fmaxf(top, s[0][e]);
+#pragma unroll
+    for (int e = 0; e < 16; ++e) top = fmaxf(top, s[1][e]);
+    top = max_xhalf(top) * c2;
+    if (__any(top > mx)) {
+      const float mnew = fmaxf(mx, top), f = __builtin_amdgcn_exp2f(mx - mnew);
+      mx = mnew;
+      sum *= f;
+#pragma unroll
+      for (int i = 0; i < NDB; ++i)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) oacc[i][e] *= f;
+    }
+    float ps = 0.f;
+#pragma unroll
+    for (int hh = 0; hh < 2; ++hh)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) {
+        s[hh][e] = __builtin_amdgcn_exp2f(fmaf(s[hh][e], c2, -mx));
+        ps += s[hh][e];
+      }
+    sum += sum_xhalf(ps);
+#pragma unroll
+    for (int kc = 0; kc < 4; ++kc) {
+      const int hh = kc >> 1, cb = (kc & 1) * 8;
+      u32x4_t wh, wl;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float x = s[hh][cb + 2 * e], y = s[hh][cb + 2 * e + 1];
+        wh[e] = pack_bf2(x, y);
+        wl[e] = split_lo(wh[e], x, y);
+      }
+      const bf16x8_t bh = __builtin_bit_cast(bf16x8_t, wh), bl = __builtin_bit_cast(bf16x8_t, wl);
+      const int g4 = lane >> 4, li = lane & 15;
+      const int vrow = kc * 16 + 4 * (g4 >> 1) + (li >> 2);
+#pragma unroll
+      for (int db = 0; db < NDB; ++db) {
+        const char* vp = smem + C::KB + vrow * C::VSTR + (db * 32 + 16 * (g4 & 1) + 4 * (li & 3)) * 2;
+        const s16x4_t lo = lds_read_tr16(vp), up = lds_read_tr16(vp + 8 * C::VSTR);
+        const bf16x8_t va = bf16x8_t{lo[0], lo[1], lo[2], lo[3], up[0], up[1], up[2], up[3]};
+        oacc[db] = mfma32(va, bh, oacc[db]);
+        oacc[db] = mfma32(va, bl, oacc[db]);
+      }
+    }
+  }
+  if (tok >= n) return;
+  const float inv = 1.f / sum;
+  const bf16_t* g = p.gate + (size_t)(s0 + tok) * p.ldg + (size_t)hd * V;
+  bf16_t* o = (bf16_t*)a.out + (size_t)(s0 + tok) * a.ldo + (size_t)hd * V;
+#pragma unroll
+  for (int db = 0; db < NDB; ++db)
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int c = db * 32 + 8 * q + 4 * hi;
+      const f32x4_t gt = Act<bf16_t>::load4(g + c);
+      f32x4_t y;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] = oacc[db][4 * q + e] * inv * sigmoid32(gt[e]);
+      Act<bf16_t>::store4(o + c, y);
+    }
+}
+
+template <int D, int V>
+static int launch_lat_flash(const FlashArgs& p, hipStream_t s) {
+  static const hipError_t e = hipFuncSetAttribute((const void*)latent_flash_kernel<D, V>,
+                                                  hipFuncAttributeMaxDynamicSharedMemorySize, LF<D, V>::BYTES);
+  if (e != hipSuccess) return (int)e;
+  const long long tiles = (long long)p.qtiles * p.a.H * p.a.m.B;
+  if (tiles > 0x7fffffffll) return (int)hipErrorInvalidValue;
+  latent_flash_kernel<D, V><<<(int)tiles, 256, LF<D, V>::BYTES, s>>>(p, (int)tiles);
+  DA_LAUNCH_CHECK();
+}
+template <int D>
+static int launch_lat_flash_v(const FlashArgs& p, int V, hipStream_t s) {
+  switch (V) {
+    case 32: return launch_lat_flash<D, 32>(p, s);
+    case 64: return launch_lat_flash<D, 64>(p, s);
+    case 96: return launch_lat_flash<D, 96>(p, s);
+    case 128: return launch_lat_flash<D, 128>(p, s);
+    default: return (int)hipErrorInvalidValue;
+  }
+}
+
+// lat [contexts][L + R] <- the cache rows of every portion's context (positions 0 .. its last token), packed at cctx.
+DA_EXPORT int da_latent_gather(void* pages, int npages, const void* table, int max_pages, int L, int R, const void* cctx,
+                               int max_ctx, void* lat, const void* cu, const void* slot, const void* pos0, const void* seq,
+                               int T, int B, void* stream) {
+  if (T < 1 || B < 1 || B > 65535 || max_ctx < 1 || (L + R) % 8 || npages < 1 || max_pages < 1 ||
+      (max_ctx + PAGE - 1) / PAGE > max_pages)
+    return (int)hipErrorInvalidValue;
+  LatArgs a{};
+  a.pages = pages; a.table = (const int*)table; a.max_pages = max_pages; a.npages = npages; a.L = L; a.R = R;
+  a.m = SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B};
+  latent_gather_kernel<<<dim3((max_ctx + PAGE - 1) / PAGE, B), 256, 0, (hipStream_t)stream>>>(a, (const int*)cctx,
+                                                                                             (bf16_t*)lat);
+  DA_LAUNCH_CHECK();
+}
+
+// Attention (bf16) over keys and values expanded from the latents: kv [contexts][H][d | V], rotated key parts at column L
+// of lat; times sigmoid(gate). D in {64, 96, 128, 192, 256} >= d + the rotated part, V in {32, 64, 96, 128}.
+DA_EXPORT int da_latent_flash(const void* q, int ldq, const void* lat, const void* kv, int ldkv, const void* gate, int ldg,
+                              const void* rot, int npos, const void* sink, void* out, int ldo, int H, int D, int d, int rdim,
+                              int L, int R, int V, float scale, const void* cctx, int max_len, const void* cu,
+                              const void* slot, const void* pos0, const void* seq, int T, int B, void* stream) {
+  if (T < 1 || B < 1 || H < 1 || d < 8 || d % 8 || rdim < 2 || rdim % 2 || rdim > R || d + rdim > D || L % 8 || R < 8 || R % 8 ||
+      ldq % 8 || ldkv % 8 || ldkv < H * (d + V) || ldg % 4 || ldo % 4 || npos < 1 || max_len < 1)
+    return (int)hipErrorInvalidValue;
+  FlashArgs p{};
+  p.a.q = q; p.a.ldq = ldq; p.a.rot = (const float*)rot; p.a.npos = npos; p.a.sink = (const float*)sink;
+  p.a.out = out; p.a.ldo = ldo; p.a.H = H; p.a.D = D; p.a.ra = d; p.a.rdim = rdim; p.a.L = L; p.a.R = R; p.a.scale = scale;
+  p.a.m = SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B};
+  p.cctx = (const int*)cctx; p.lat = (const bf16_t*)lat; p.kv = (const bf16_t*)kv; p.ldkv = ldkv;
+  p.gate = (const bf16_t*)gate; p.ldg = ldg; p.qtiles = (max_len + 127) / 128;
+  hipStream_t s = (hipStream_t)stream;
+  switch (D) {
+    case 64: return launch_lat_flash_v<64>(p, V, s);
+    case 96: return launch_lat_flash_v<96>(p, V, s);
+    case 128: return launch_lat_flash_v<128>(p, V, s);
+    case 192: return launch_lat_flash_v<192>(p, V, s);
+    case 256: return launch_lat_flash_v<256>(p, V, s);
+    default: return (int)hipErrorInvalidValue;
+  }
+}
+
 // x [T][ldx] = [query latent Q | latent L | key part R] before their norms and rotation -> cq [T][Q], and the token's
 // cache row. rot fp32 [npos][rdim / 2][2]. Every count of columns a multiple of 4.
 DA_EXPORT int da_latent_prep(const void* x, int ldx, const void* qw, int Q, int qdim, const void* cw, int L, int cdim, int R,
@@ -226,5 +669,6 @@ DA_EXPORT int da_latent_attn(const void* q, int ldq, const void* ql, int ldl, vo
             SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B}, (float*)part,
             (float*)part_ml, nsplit, pps, max_len * H};
   hipStream_t s = (hipStream_t)stream;
-  return f32 ? launch_lat_any_t<float>(a, s) : launch_lat_any_t<bf16_t>(a, s);
+  if (f32) return launch_lat_any_t<float>(a, s);
+  return lat_mfma_dims(L, R) ? launch_lat_mfma_t(a, s) : launch_lat_any_t<bf16_t>(a, s);
 }

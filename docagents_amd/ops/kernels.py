@@ -1125,5 +1125,5 @@ def pool_l2norm_f16(h, cu_seqlens, mode: int = 0, out32=None, out16=None):
 
 # the batch-of-portions ops (recurrent mixers, paged attention, 32-bit residual stream)
 from .seq_kernels import (causal_conv, delta_rule, gated_scan, gemm_any, gemm_heads, gemm_partials,  # noqa: E402,F401
-                          latent_attn, latent_flash_fits, latent_prep, partials_fit, rglru_gates, selective_scan,
-                          sigmoid_attn, stream_add, stream_final, stream_step)
+                          latent_attn, latent_flash, latent_flash_fits, latent_gather, latent_prep, partials_fit, rglru_gates,
+                          selective_scan, sigmoid_attn, stream_add, stream_final, stream_step)

@@ -36,15 +36,19 @@ K._SIGS.update({
                          + [c_void_p] * 4 + [c_int] * 3 + _META + [c_int, c_void_p],
     "da_gated_scan": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p,
                       c_int] + [c_void_p] * 4 + [c_int] * 2 + _META + [c_int, c_void_p],
+    "da_latent_gather": [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p] + _META + [c_void_p],
+    "da_latent_flash": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p,
+                        c_int] + [c_int] * 7 + [c_float, c_void_p, c_int] + _META + [c_void_p],
     "da_sigmoid_attn": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float,
                         c_float, c_float, K.ctypes.c_double] + [c_int] * 4 + [c_void_p, c_int, c_void_p] + [c_int] * 4
                        + _META + [c_int, c_void_p],
 })
 K._PART_OF.update({n: "hybrid" for n in ("da_gemm_any", "da_stream_step", "da_stream_final", "da_causal_conv",
                                          "da_selective_scan", "da_gated_scan", "da_sigmoid_attn", "da_stream_add", "da_delta_rule",
-                                         "da_latent_prep", "da_latent_attn")})
+                                         "da_latent_prep", "da_latent_attn", "da_latent_gather", "da_latent_flash")})
 
 ACTS = (torch.bfloat16, torch.float32)
+LATENT_MFMA = (64, 128, 256, 512)  # latents the matrix-core attention takes (with a key part of 32 or 64 columns)
 ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_RGLRU, ANY_SWIGLU, ANY_ACT = 0, 1, 2, 3, 4, 5
 
 
@@ -407,7 +411,15 @@ def latent_attn(q, ql, pages, rot, sink, m: SeqBatch, H: int, rot_at: int, rot_d
     _req(q.shape == (m.T, H * D) and ql.shape == (m.T, H * L) and rot_at + rot_dim <= D and L + rot_dim <= W, "query columns")
     _req(L <= 1152 and W <= 1216, f"latents of {W} columns")
     out = torch.empty((m.T, H * L), dtype=q.dtype, device=q.device)
-    part, ml, nsplit, pps = None, None, 1, -(-m.max_ctx // PAGE)
+    part, ml, rows, pages_ctx = None, None, m.max_len * H, -(-m.max_ctx // PAGE)
+    nsplit, pps = 1, pages_ctx
+    if not f32 and L in LATENT_MFMA and W - L in (32, 64):
+        want = max(1, min(-(-1024 // (m.B * -(-rows // 16))), -(-pages_ctx // 2)))  # ~1024 workgroups, >= 2 pages each
+        pps = -(-pages_ctx // want)
+        nsplit = -(-pages_ctx // pps)
+    if nsplit > 1:
+        part = torch.empty((m.B, rows, nsplit, L), dtype=torch.float32, device=q.device)
+        ml = torch.empty((m.B, rows, nsplit, 2), dtype=torch.float32, device=q.device)
     _check(lib().da_latent_attn(_ptr(q), q.stride(0), _ptr(ql), ql.stride(0), _ptr(pages), pages.shape[0], _ptr(t), t.shape[1],
                                 _ptr(rot), rot.shape[0], _ptr(sink), _ptr(out), out.stride(0), H, D, rot_at, rot_dim, L, W - L,
                                 float(scale), _ptr(part), _ptr(ml), nsplit, pps, m.max_len, *_meta(m), f32, _stream()),
@@ -416,4 +428,37 @@ def latent_attn(q, ql, pages, rot, sink, m: SeqBatch, H: int, rot_at: int, rot_d
 
 
 def latent_flash_fits(D: int, V: int) -> bool:
-    return False
+    """Whether ``latent_flash`` takes (padded) query / key heads of D columns and value heads of V."""
+    return D in (64, 96, 128, 192, 256) and V in (32, 64, 96, 128)
+
+
+def latent_gather(pages, m: SeqBatch):
+    """The cache rows of every portion's context (its tokens included), packed one portion after another."""
+    t, (cctx, n) = m.table, m.context()
+    _act(pages, "pages", torch.bfloat16)
+    _req(pages.is_contiguous() and t is not None and t.dtype == torch.int32 and t.is_contiguous(), "pages")
+    W = pages.shape[2]
+    lat = torch.empty((n, W), dtype=pages.dtype, device=pages.device)
+    _check(lib().da_latent_gather(_ptr(pages), pages.shape[0], _ptr(t), t.shape[1], W, 0, _ptr(cctx),
+                                  int((m.starts + m.lens).max()), _ptr(lat), *_meta(m), _stream()), "latent_gather")
+    return lat
+
+
+def latent_flash(q, lat, kv, gate, rot, sink, m: SeqBatch, H: int, d: int, rot_dim: int, L: int, V: int, scale: float):
+    """Attention over expanded keys and values (bf16): q [T, H D] (d plain columns of a head, then the rotated ones before
+    rotation), lat from ``latent_gather`` (rotated key parts at column L), kv [contexts, H (d + V)], gate [T, H V]
+    -> softmax(with sink) values * sigmoid(gate), [T, H V]."""
+    for x, name in ((q, "q"), (lat, "lat"), (kv, "kv"), (gate, "gate")):
+        _act(x, name, torch.bfloat16)
+    cctx, n = m.context()
+    D, W = q.shape[1] // H, lat.shape[1]
+    _f32(rot, "rot")
+    _f32(sink, "sink", H)
+    _req(latent_flash_fits(D, V) and q.shape == (m.T, H * D) and d % 8 == 0 and d + rot_dim <= D, "query columns")
+    _req(lat.shape[0] == n and lat.is_contiguous() and kv.shape == (n, H * (d + V)) and W - L >= rot_dim, "keys")
+    _req(gate.shape == (m.T, H * V) and rot.shape[1:] == (rot_dim // 2, 2), "gate / rotary table")
+    out = torch.empty((m.T, H * V), dtype=q.dtype, device=q.device)
+    _check(lib().da_latent_flash(_ptr(q), q.stride(0), _ptr(lat), _ptr(kv), kv.stride(0), _ptr(gate), gate.stride(0),
+                                 _ptr(rot), rot.shape[0], _ptr(sink), _ptr(out), out.stride(0), H, D, d, rot_dim, L, W - L,
+                                 V, float(scale), _ptr(cctx), m.max_len, *_meta(m), _stream()), "latent_flash")
+    return out
