@@ -1,19 +1,11 @@
 """Small Binupel configurations, checkpoints and step schedules shared by the tests."""
-import json
-
-import numpy as np
-import pytest
 import torch
 
 import binupel_oracle as oracle
 from docagents_amd.models import make_decoder
 from docagents_amd.models.configs import checkpoint_config
-from docagents_amd.ops.seq_batch import pack_batch
+from seq_cases import checkpoint, row_errors
 
-CPU = pytest.param("cpu", "fp32", id="cpu-fp32")
-GPU32 = pytest.param("cuda", "fp32", id="gpu-fp32", marks=pytest.mark.gpu)
-GPU16 = pytest.param("cuda", "bf16", id="gpu-bf16", marks=pytest.mark.gpu)
-WHERE = [CPU, GPU32, GPU16]
 # rms error of a row of logits / rms of the logits; "ones" (alpha = 1, a stack run twice, one-channel states)
 # amplifies bf16 roundings: the same model in torch on the CPU is off by up to 6.4e-2
 TOL = {"fp32": 5e-5, "bf16": 3e-2}
@@ -104,13 +96,6 @@ def weights(cfg, seed=0, dtype=torch.bfloat16):
     return out
 
 
-def checkpoint(path, cfg, w):
-    from safetensors.torch import save_file
-    (path / "config.json").write_text(json.dumps(cfg))
-    save_file({k: v.contiguous() for k, v in w.items()}, str(path / "model.safetensors"))
-    return str(path)
-
-
 def build(tmp_path, name, device, dtype, seed=0, edit=None):
     """(model loaded from a checkpoint folder, config, weights); edit(weights) may change them first."""
     cfg = CONFIGS[name] if isinstance(name, str) else name
@@ -118,43 +103,6 @@ def build(tmp_path, name, device, dtype, seed=0, edit=None):
     if edit:
         edit(w)
     return make_decoder(checkpoint_config(checkpoint(tmp_path, cfg, w)), device, dtype=dtype), cfg, w
-
-
-def tokens(cfg, n, seed):
-    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).tolist()
-
-
-def run(model, requests, schedule, slots=4, max_seq=None, pool=None):
-    """requests: id -> tokens; schedule: steps of [(id, count), ...]. Every position's logits, per request, from the
-    model's step on its state cache. A request's slot and pages are given back at its last token."""
-    longest = max(len(t) for t in requests.values())
-    cache = model.alloc_cache(slots, max_seq or longest, tokens=pool)
-    at, slot, out = {}, {}, {i: [] for i in requests}
-    for step in schedule:
-        ids, lens, sl, p0 = [], [], [], []
-        for i, n in step:
-            if i not in slot:
-                slot[i], at[i] = cache.acquire(1, [0])[0], 0
-            cache.extend([slot[i]], [at[i] + n])
-            ids += requests[i][at[i]:at[i] + n]
-            lens.append(n), sl.append(slot[i]), p0.append(at[i])
-            at[i] += n
-        m, tok = pack_batch(lens, sl, p0, model.device, ids)
-        lg = model.step(m, tok, torch.arange(m.T, device=model.device)).float().cpu()
-        row = 0
-        for (i, n) in step:
-            out[i].append(lg[row:row + n])
-            row += n
-            if at[i] == len(requests[i]):
-                cache.release([slot.pop(i)])
-    assert sorted(cache.free) == list(range(slots)) and sorted(cache.free_pages) == list(range(cache.pages))
-    return {i: torch.cat(v) for i, v in out.items()}
-
-
-def row_errors(got, want):
-    d = got.double() - want.double()
-    d = d - d.mean(-1, keepdim=True)
-    return d.pow(2).mean(-1).sqrt() / want.double().pow(2).mean().sqrt()
 
 
 def check(got, want, dtype, what=""):

@@ -9,8 +9,7 @@ import pytest
 import torch
 
 import binupel_oracle as oracle
-from binupel_cases import (CONFIGS, CPU, GPU16, GPU32, TOL, WHERE, att, build, check, checkpoint, config, expect, rec,
-                           row_errors, run, ssm, tokens, weights)
+from binupel_cases import CONFIGS, TOL, att, build, check, config, expect, rec, ssm, weights
 from docagents_amd.engine.generator import ContinuousScheduler, Generator
 from docagents_amd.engine.replay import replay
 from docagents_amd.models import make_decoder
@@ -19,59 +18,8 @@ from docagents_amd.models.configs import DECODERS, HybridConfig, binupel_config,
 from docagents_amd.models.state import LayerState, StateCache
 from docagents_amd.ops import get_ops
 from docagents_amd.ops.seq_batch import PAGE, pack_batch
-
-@pytest.fixture(autouse=True, scope="module")
-def one_thread():
-    """The plain implementation's many tiny operations run faster without a thread pool."""
-    n = torch.get_num_threads()
-    torch.set_num_threads(1)
-    yield
-    torch.set_num_threads(n)
-
-
-ACT = {"fp32": torch.float32, "bf16": torch.bfloat16}
-
-
-def close(got, want, dtype, scale=1.0):
-    got, want = got.double().cpu(), want.double()
-    tol = {"fp32": 2e-5, "bf16": 1.5e-2}[dtype] * scale
-    err = (got - want).abs().max() / want.abs().max()
-    assert err < tol, f"off by {float(err):.3g} of the largest value"
-
-
-def rand(seed, *shape, std=1.0):
-    return std * torch.randn(shape, generator=torch.Generator().manual_seed(seed))
-
-
-class Portions:
-    """Three sequences of unequal lengths, fed to an op in portions; want() is the oracle's whole sequences."""
-
-    def __init__(self, device, dtype, lens=(150, 3, 70), cuts=((2, 64, 70, 1, 13), (1, 2), (66, 1, 3))):
-        self.device, self.act, self.lens, self.cuts = device, ACT[dtype], lens, cuts
-        self.slots = [2, 0, 3]
-
-    def __iter__(self):
-        """(batch, rows of every sequence in it as (sequence, first, last))"""
-        at = [0] * len(self.lens)
-        for k in range(max(len(c) for c in self.cuts)):
-            ids = [i for i, c in enumerate(self.cuts) if k < len(c)]
-            n = [self.cuts[i][k] for i in ids]
-            m, _ = pack_batch(n, [self.slots[i] for i in ids], [at[i] for i in ids], self.device)
-            spans = [(i, at[i], at[i] + c) for i, c in zip(ids, n)]
-            for i, c in zip(ids, n):
-                at[i] += c
-            yield m, spans
-
-    def pack(self, seqs, spans):
-        return torch.cat([seqs[i][a:b] for i, a, b in spans]).to(self.device, self.act).contiguous()
-
-    def stored(self, seqs):
-        """What an op sees of values kept in the activation type."""
-        return [s.to(self.act).double() for s in seqs]
-
-    def state(self, *shape, dtype=None):
-        """Slots that hold another sequence's leftovers."""
-        return torch.full((4, *shape), 7.0, dtype=dtype or torch.float32, device=self.device)
+from seq_cases import (ACT, CPU, GPU16, GPU32, WHERE, Portions, checkpoint, close, mixed_schedule, one_thread,  # noqa: F401
+                       rand, row_errors, run, tokens)
 
 
 # ---------------------------------------------------------------------------------- mechanisms alone
@@ -387,25 +335,6 @@ def test_token_by_token_equals_the_prompt(tmp_path, name, device, dtype):
     model, cfg, w = build(tmp_path, name, device, dtype, seed=3)
     req = {"a": tokens(cfg, 140, 6)}
     check(run(model, req, [[("a", 1)]] * 140)["a"], expect(cfg, w, req["a"]), dtype, name)
-
-
-def mixed_schedule(lens, seed):
-    """Up to four live requests a step, portions of 2..70 beside single tokens, requests left out of steps."""
-    rng = np.random.default_rng(seed)
-    left, live, todo, sched = dict(lens), [], list(lens), []
-    while todo or live:
-        while len(live) < 4 and todo and (not live or rng.random() < 0.6):
-            live.append(todo.pop(0))
-        step = []
-        for i in live:
-            if rng.random() < 0.8:
-                c = min(left[i], 1 if rng.random() < 0.5 else int(rng.integers(2, 70)))
-                step.append((i, c))
-                left[i] -= c
-        live = [i for i in live if left[i]]
-        if step:
-            sched.append(step)
-    return sched
 
 
 @pytest.mark.parametrize("device,dtype", WHERE)

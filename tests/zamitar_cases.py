@@ -2,13 +2,13 @@
 import torch
 
 import zamitar_oracle as oracle
-from binupel_cases import checkpoint, row_errors
 from docagents_amd.models import make_decoder
 from docagents_amd.models.configs import checkpoint_config
+from seq_cases import checkpoint, row_errors
 
 # rms error of a row of logits / rms of the logits
-TOL = {"fp32": 3e-5, "bf16": 3e-2}
-TOL16 = {"deep": 6e-2}  # eleven layer runs
+TOL = {"fp32": 3e-5, "bf16": 1e-2}
+TOL16 = {"ones": 3e-2}  # norms over five channels
 
 
 def delta(heads, kv, dim, vdim, conv=4):
@@ -34,8 +34,8 @@ CONFIGS = {
     # no width a multiple of a tile, query / key heads shared, layers without feed-forward, a loop in the middle
     "odd": config(90, 203, [(latent(5, 24, 8, 40, 36, 50), None), (delta(6, 2, 20, 28, 3), 100),
                             (latent(3, 12, 20, 16, 70, 33), 52), (delta(4, 4, 40, 72, 2), None)], loop=(1, 3, 3)),
-    # one head, one tap, no loop
-    "ones": config(64, 97, [(delta(1, 1, 32, 64, 1), 64), (latent(1, 32, 2, 32, 1, 1), None), (delta(2, 1, 1, 1, 2), 33)],
+    # one head, one tap, one rotated pair, no loop (no norm over one channel: its sign would flip on rounding)
+    "ones": config(64, 97, [(delta(1, 1, 32, 64, 1), 64), (latent(1, 32, 2, 32, 6, 5), None), (delta(2, 1, 4, 6, 2), 33)],
                    eps=1e-3, scale=1.0),
     # wide heads and latents, many query heads, everything looped
     "wide": config(130, 151, [(delta(6, 3, 128, 96, 6), 96), (latent(20, 128, 64, 128, 96, 300), 80)], loop=(0, 2, 2)),
