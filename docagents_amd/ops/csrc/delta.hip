@@ -115,9 +115,9 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
 
   fetch(t0);
   for (int t = t0; t < t1; t += DT) {
-    __syncthreads();
+    lds_barrier();
     stage();
-    __syncthreads();
+    lds_barrier();
     if (t + DT < t1) fetch(t + DT);
     const int n = min(DT, t1 - t);
     for (int r = 0; r < n; ++r) {
@@ -181,21 +181,24 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
 //   U  = T (V / rk - (kappa 2^G) S)                                 rows u_t rk_t: what the tokens write
 //   o  = rq ((chi 2^G) S + tril(Q) U)
 //   S <- 2^G_end S + (kappa 2^(G_end - G))^T U
-// A workgroup of 8 waves walks a head's chunks; it forms the operands together (in LDS, as MFMA fragments), then each wave
-// runs 16 columns of V and S by itself, S staying in its accumulators.
+// delta_prep: a wave per chunk and head forms what does not depend on S (kappa 2^G, chi 2^G, kappa 2^(G_end - G), T, Q), as
+// MFMA fragments in scratch memory. delta_apply: a wave walks its portion's chunks with 16 columns of V and S by itself,
+// S staying in its accumulators; the waves of a workgroup share the next chunk's fragments, in flight to LDS meanwhile.
 //
 // Every fp32 operand enters its product as two bf16 terms (its rounding and the remainder), three of their four
-// products taken: about 16 bits, accumulated in fp32. The solve of T's blocks is in fp32.
+// products taken: about 16 bits, accumulated in fp32. The solve of T is in fp32.
 //
-// M and Q: rows of an 8-token block are scaled by 2^(G_t - m) and columns by 2^(m - G_j), m the cumulative decay at the
-// block's middle, so no factor leaves the range of an exponent as long as a token's decay is at least 2^-24; stronger ones
-// count as that there (less than the rounding of what they are added to).
-constexpr int CT = 32;                          // tokens of a chunk
-constexpr int FG_B = 272, FRAG = 4 * FG_B;      // bytes: a fragment's four lane rows, padded apart; a fragment
+// Products of 16-token blocks scale rows by 2^(G_t - m) and columns by 2^(m - G_j): m between the blocks off the
+// diagonal (no factor above 1), the block's start on it. Where a channel decays by more than 2^100 within a block, rows go
+// by 8 tokens with m in their middle and a token's decay limited to 2^-24 (a stronger one leaves less than the rounding
+// of what it is added to), so that no factor leaves the range of an exponent.
+constexpr int CT = 32;  // tokens of a chunk
 
-// Operand with rows of 16 (lane fr) and 32 k values: k sits at lane row (k % 16) / 4, element (k / 16) * 4 + k % 4, the
-// order in which an accumulator's rows become the other operand.
-__device__ __forceinline__ int frag_at(int fr, int k) { return (k & 15) / 4 * FG_B + fr * 16 + ((k >> 4) * 4 + (k & 3)) * 2; }
+struct ChunkArgs {
+  DeltaArgs a;
+  ChunkMeta ch;         // chunks of CT tokens of all portions
+  char* frags;          // [chunks][H][NF KB]
+};
 
 struct Split { bf16x8_t hi, lo; };
 __device__ __forceinline__ unsigned lo_of(unsigned hi, float a, float b) {
@@ -211,46 +214,285 @@ __device__ __forceinline__ f32x4_t mma3(const Split& a, const Split& b, f32x4_t 
   c = mfma16(a.hi, b.lo, c);
   return mfma16(a.hi, b.hi, c);
 }
-__device__ __forceinline__ Split frag_load(const char* p, int lane) {
-  p += (lane >> 4) * FG_B + (lane & 15) * 16;
-  return {*(const bf16x8_t*)p, *(const bf16x8_t*)(p + FRAG)};
-}
 
-template <int KB> struct DC {                   // K = 32 KB key channels
-  static constexpr int K = 32 * KB, OP = 4 * KB * FRAG;  // an operand of 32 tokens x K, both terms
-  static constexpr int KP = 0, QP = OP, KM = 2 * OP, AK = 3 * OP, AQ = 4 * OP, BK = 5 * OP;
-  static constexpr int TF = 6 * OP, QF = TF + 4 * FRAG;  // T and Q: 2 row blocks, both terms
-  static constexpr int SM = QF + 4 * FRAG;               // diag(b) M: fp32 [32][36]
-  static constexpr int SD = SM + 32 * 36 * 4;            // solve: fp32 [3][16][17]
-  static constexpr int TOT = SD + 3 * 16 * 17 * 4;       // decay sums of 4 tokens: fp32 [2][8][K] (as they are, limited)
-  static constexpr int MID = TOT + 2 * 8 * K * 4;        // fp32 [4][K]
-  static constexpr int END = MID + 4 * K * 4;            // 2^G_end: fp32 [K]
-  static constexpr int TOK = END + K * 4;                // per token, two chunks: rk, rq, b
-  static constexpr int BYTES = TOK + 2 * 3 * CT * 4;
+// A fragment is 1 KB, lane l's 16 bytes at 16 l. Its lane (fr, fg) holds row fr and the 8 k values 16 u + 4 fg + e (u < 2,
+// e < 4) of 32: the order in which an accumulator's rows become the other operand. An operand's two terms follow each other.
+template <int KB> struct DC {  // K = 32 KB key channels; offsets in fragments
+  static constexpr int K = 32 * KB;
+  static constexpr int KP = 0, QP = 4 * KB;            // kappa 2^G, chi 2^G: [token block][32 channels]
+  static constexpr int KM = 8 * KB;                    // (kappa 2^(G_end - G))^T: [16 channels][tokens]
+  static constexpr int TF = 12 * KB, QF = TF + 4;      // T, Q: [token block][tokens]
+  static constexpr int VEC = QF + 4;                   // fp32: 2^G_end [K], rk [32], rq [32]
+  static constexpr int NF = VEC + 1;
 };
 
+struct Vec8 { f32x4_t u[2]; };  // a lane's 8 channels (or tokens), 16 u + 4 fg + e
+__device__ __forceinline__ Split split8(const Vec8& v) { return split8(v.u[0], v.u[1]); }
+#define V8(expr)                                                                         \
+  [&] {                                                                                  \
+    Vec8 r_;                                                                             \
+    _Pragma("unroll") for (int u = 0; u < 2; ++u)                                        \
+        _Pragma("unroll") for (int e = 0; e < 4; ++e) r_.u[u][e] = (expr);                \
+    return r_;                                                                           \
+  }()
+
+template <int D> __device__ __forceinline__ float row_shr(float v) {  // lane fr - D of the 16, 0 before the first
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x110 | D, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float row_scan(float v) {  // inclusive sums over the 16 lanes
+  v += row_shr<1>(v);
+  v += row_shr<2>(v);
+  v += row_shr<4>(v);
+  return v + row_shr<8>(v);
+}
+template <int L> __device__ __forceinline__ float row_lane(float v) {  // lane L of the 16
+  return __int_as_float(__builtin_amdgcn_ds_swizzle(__float_as_int(v), L << 5 | 0x10));
+}
+
+// LDS of a wave, used in turn: two terms of 32 tokens x 32 channels to be transposed; the solve.
+struct PrepLds {
+  static constexpr int ROW = 80;                                     // bytes of a token's 32 channels
+  static constexpr int SM = 0, SQ = 32 * 36 * 4, SD = 2 * SQ;        // fp32 [32][36] twice, [3][16][17]
+  static constexpr int TOK = SD + 3 * 16 * 17 * 4, BYTES = TOK + 32 * 4;  // b
+};
+static_assert(2 * 32 * PrepLds::ROW <= PrepLds::TOK, "the staged tile shares the solve's space");
+
 template <int KB>
-__global__ void __launch_bounds__(512, 2) delta_chunk_kernel(DeltaArgs a) {
+__global__ void __launch_bounds__(256, 2) delta_prep_kernel(ChunkArgs p) {
   using C = DC<KB>;
+  const DeltaArgs& a = p.a;
+  __shared__ __attribute__((aligned(16))) char smem[4 * PrepLds::BYTES];
+  constexpr int K = C::K;
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, fr = lane & 15, fg = lane >> 4;
+  const int item = blockIdx.x * 4 + wv;
+  if (item >= p.ch.n * a.H) return;  // the waves share nothing: no barriers below
+  const int ci = item / a.H, h = item % a.H, hk = h / (a.H / a.G);
+  const int b = p.ch.ck[2 * ci], s1 = a.m.cu[b + 1], t0 = a.m.cu[b] + p.ch.ck[2 * ci + 1] * CT;
+  if (s1 - a.m.cu[b] < a.below) return;
+  char* lds = smem + wv * PrepLds::BYTES;
+  char* out = p.frags + (size_t)item * C::NF * 1024 + lane * 16;
+  float* vec = (float*)(p.frags + ((size_t)item * C::NF + C::VEC) * 1024);
+  auto wait_own = [] {  // this wave's LDS writes are read back by itself
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_wave_barrier();
+  };
+  auto put = [&](int f, const Split& v) {
+    *(bf16x8_t*)(out + f * 1024) = v.hi;
+    *(bf16x8_t*)(out + (f + 1) * 1024) = v.lo;
+  };
+
+  // rows of this lane's two tokens
+  const bf16_t *xq[2], *xk[2];
+  const float* xg[2];
+  bool in[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int t = t0 + 16 * i + fr;
+    in[i] = t < s1;
+    const size_t row = min(t, s1 - 1);
+    xq[i] = (const bf16_t*)a.x + row * a.ldx + hk * K + 4 * fg;
+    xk[i] = xq[i] + a.G * K;
+    xg[i] = a.decay + row * a.H * K + (size_t)h * K + 4 * fg;
+  }
+  struct Raw { u32x2_t q[2][2], k[2][2]; f32x4_t g[2][2]; };
+  auto load = [&](int ks) {
+    Raw r;
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        r.q[i][u] = *(const u32x2_t*)(xq[i] + ks * 32 + 16 * u);
+        r.k[i][u] = *(const u32x2_t*)(xk[i] + ks * 32 + 16 * u);
+        r.g[i][u] = *(const f32x4_t*)(xg[i] + ks * 32 + 16 * u);
+      }
+    return r;
+  };
+  f32x4_t M[3], Q[3];  // blocks (0, 0), (1, 1), (1, 0)
+#pragma unroll
+  for (int i = 0; i < 3; ++i) M[i] = Q[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float nk[2] = {0.f, 0.f}, nq[2] = {0.f, 0.f};
+
+  Raw next = load(0);
+#pragma unroll 1
+  for (int ks = 0; ks < KB; ++ks) {
+    const Raw r = next;
+    if (ks + 1 < KB) next = load(ks + 1);
+    Vec8 k[2], q[2], g[2], L[2], P[2], E[2], eT[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      auto half = [&](const u32x2_t& w, int e) {
+        return in[i] ? __uint_as_float(e & 1 ? w[e >> 1] & 0xffff0000u : w[e >> 1] << 16) : 0.f;
+      };
+      k[i] = V8(half(r.k[i][u], e));
+      q[i] = V8(half(r.q[i][u], e));
+      g[i] = V8(in[i] ? r.g[i][u][e] : 0.f);
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          nk[i] = fmaf(k[i].u[u][e], k[i].u[u][e], nk[i]);
+          nq[i] = fmaf(q[i].u[u][e], q[i].u[u][e], nq[i]);
+        }
+      L[i] = V8(row_scan(g[i].u[u][e]));
+      const Vec8 T = V8(row_lane<15>(L[i].u[u][e]));
+      P[i] = V8(__builtin_amdgcn_exp2f(L[i].u[u][e]));                  // from the block's start
+      E[i] = V8(k[i].u[u][e] * __builtin_amdgcn_exp2f(T.u[u][e] - L[i].u[u][e]));  // kappa to the block's end
+      eT[i] = V8(row_lane<15>(P[i].u[u][e]));
+      const Vec8 ka = V8(k[i].u[u][e] * P[i].u[u][e]), qa = V8(q[i].u[u][e] * P[i].u[u][e]);
+      const Split sk = split8(ka), sq = split8(qa);
+      if (i == 0) {
+        put(C::KP + ks * 2, sk);
+        put(C::QP + ks * 2, sq);
+      } else {
+        const Split B = split8(E[0]);
+        M[2] = mma3(sk, B, M[2]);
+        Q[2] = mma3(sq, B, Q[2]);
+        put(C::KP + (KB + ks) * 2, split8(V8(ka.u[u][e] * eT[0].u[u][e])));
+        put(C::QP + (KB + ks) * 2, split8(V8(qa.u[u][e] * eT[0].u[u][e])));
+      }
+      float lowest = 0.f;
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) lowest = fminf(lowest, T.u[u][e]);
+      if (!__any(lowest < -100.f)) {
+        const Split B = split8(V8(k[i].u[u][e] * __builtin_amdgcn_exp2f(-L[i].u[u][e])));
+        M[i] = mma3(sk, B, M[i]);
+        Q[i] = mma3(sq, B, Q[i]);
+      } else {
+        const Vec8 l = V8(row_scan(fmaxf(g[i].u[u][e], -24.f)));
+        const Vec8 m0 = V8(row_lane<3>(l.u[u][e])), m1 = V8(row_lane<11>(l.u[u][e]));
+        const bool up = fr >= 8;
+        const Vec8 to = V8(__builtin_amdgcn_exp2f(l.u[u][e] - (up ? m1.u[u][e] : m0.u[u][e])));
+        const Vec8 col = V8(k[i].u[u][e] * __builtin_amdgcn_exp2f((up ? m1.u[u][e] : m0.u[u][e]) - l.u[u][e]));
+        // the step between the middles in two: the factor alone may underflow where the product does not
+        const Vec8 half_step = V8(up ? 1.f : __builtin_amdgcn_exp2f(0.5f * (m1.u[u][e] - m0.u[u][e])));
+        // rows 0 .. 7 against columns 0 .. 7, then rows 8 .. 15 against all
+        Split B = split8(V8(up ? 0.f : col.u[u][e]));
+        M[i] = mma3(split8(V8(up ? 0.f : k[i].u[u][e] * to.u[u][e])), B, M[i]);
+        Q[i] = mma3(split8(V8(up ? 0.f : q[i].u[u][e] * to.u[u][e])), B, Q[i]);
+        B = split8(V8(col.u[u][e] * half_step.u[u][e] * half_step.u[u][e]));
+        M[i] = mma3(split8(V8(up ? k[i].u[u][e] * to.u[u][e] : 0.f)), B, M[i]);
+        Q[i] = mma3(split8(V8(up ? q[i].u[u][e] * to.u[u][e] : 0.f)), B, Q[i]);
+      }
+    }
+    if (fr == 0)
+#pragma unroll
+      for (int u = 0; u < 2; ++u) *(f32x4_t*)(vec + ks * 32 + 16 * u + 4 * fg) = eT[0].u[u] * eT[1].u[u];
+    // kappa to the chunk's end, transposed: rows are channels
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const Split v = split8(i ? E[1] : V8(E[0].u[u][e] * eT[1].u[u][e]));
+      char* w = lds + (16 * i + fr) * PrepLds::ROW + fg * 8;
+      const u32x4_t hi = __builtin_bit_cast(u32x4_t, v.hi), lo = __builtin_bit_cast(u32x4_t, v.lo);
+      *(u32x2_t*)w = u32x2_t{hi[0], hi[1]};
+      *(u32x2_t*)(w + 32) = u32x2_t{hi[2], hi[3]};
+      w += 32 * PrepLds::ROW;
+      *(u32x2_t*)w = u32x2_t{lo[0], lo[1]};
+      *(u32x2_t*)(w + 32) = u32x2_t{lo[2], lo[3]};
+    }
+    wait_own();
+#pragma unroll
+    for (int c = 0; c < 2; ++c)
+#pragma unroll
+      for (int part = 0; part < 2; ++part) {
+        const char* v = lds + (part * 32 + 4 * fg + (fr >> 2)) * PrepLds::ROW + (c * 16 + 4 * (fr & 3)) * 2;
+        const s16x4_t x = lds_read_tr16(v), y = lds_read_tr16(v + 16 * PrepLds::ROW);
+        *(bf16x8_t*)(out + (C::KM + (2 * ks + c) * 2 + part) * 1024) =
+            bf16x8_t{x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+      }
+    wait_own();
+  }
+
+  // norms and write strengths of the tokens
+  float* sM = (float*)(lds + PrepLds::SM);
+  float* sQ = (float*)(lds + PrepLds::SQ);
+  float* sD = (float*)(lds + PrepLds::SD);
+  float* sB = (float*)(lds + PrepLds::TOK);
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    nk[i] += __shfl_xor(nk[i], 16, 64);
+    nk[i] = sum_xhalf(nk[i]) + a.eps;
+    nq[i] += __shfl_xor(nq[i], 16, 64);
+    nq[i] = sum_xhalf(nq[i]) + a.eps;
+    if (fg == 0) {
+      vec[K + 16 * i + fr] = 1.f / sqrtf(nk[i]);
+      vec[K + CT + 16 * i + fr] = a.q_scale / sqrtf(nq[i]);
+      const float bt = bf2f(((const bf16_t*)a.beta)[(size_t)min(t0 + 16 * i + fr, s1 - 1) * a.ldb + h]);
+      sB[16 * i + fr] = in[i] ? sigmoid32(bt) / nk[i] : 0.f;
+    }
+  }
+  wait_own();
+#pragma unroll
+  for (int i = 0; i < 3; ++i) {
+    const int r0 = i ? 16 : 0, c0 = i == 1 ? 16 : 0;
+    const f32x4_t bt = *(const f32x4_t*)(sB + r0 + 4 * fg);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      sM[(r0 + 4 * fg + e) * 36 + c0 + fr] = M[i][e] * bt[e];
+      sQ[(r0 + 4 * fg + e) * 36 + c0 + fr] = Q[i][e];
+    }
+  }
+  wait_own();
+  // the diagonal blocks' inverses by columns: lanes fg & 1 == blk take block blk, column fr
+  const int blk = fg & 1;
+  float x[16];
+#pragma unroll
+  for (int r = 0; r < 16; ++r) {
+    float v = r == fr ? 1.f : 0.f;
+    const float* Lr = sM + (blk * 16 + r) * 36 + blk * 16;
+#pragma unroll
+    for (int i = 0; i < r; ++i) v = fmaf(-Lr[i], x[i], v);
+    x[r] = v;
+  }
+  if (fg < 2)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) sD[(blk * 16 + r) * 17 + fr] = x[r];
+  // Q's lower triangle as fragments
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int r = 16 * i + fr;
+    put(C::QF + i * 2, split8(V8(16 * u + 4 * fg + e <= r ? sQ[r * 36 + 16 * u + 4 * fg + e] : 0.f)));
+  }
+  wait_own();
+  f32x4_t y{0.f, 0.f, 0.f, 0.f}, z = y;  // the block below the diagonal: -D1 (L10 D0)
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    y = __builtin_amdgcn_mfma_f32_16x16x4f32(sM[(16 + fr) * 36 + 4 * i + fg], sD[(4 * i + fg) * 17 + fr], y, 0, 0, 0);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) sD[(32 + 4 * fg + e) * 17 + fr] = y[e];
+  wait_own();
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    z = __builtin_amdgcn_mfma_f32_16x16x4f32(sD[(16 + fr) * 17 + 4 * i + fg], sD[(32 + 4 * i + fg) * 17 + fr], z, 0, 0, 0);
+  const float bc = sB[fr], bd = sB[blk * 16 + fr];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) sQ[(16 + 4 * fg + e) * 36 + fr] = -z[e] * bc;
+  if (fg < 2)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) sQ[(blk * 16 + r) * 36 + blk * 16 + fr] = x[r] * bd;
+  wait_own();
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int r = 16 * i + fr;
+    put(C::TF + i * 2, split8(V8(16 * u + 4 * fg + e <= r ? sQ[r * 36 + 16 * u + 4 * fg + e] : 0.f)));
+  }
+}
+
+typedef __attribute__((address_space(1))) const void* frag_g_t;
+typedef __attribute__((address_space(3))) void* frag_l_t;
+
+template <int KB>
+__global__ void __launch_bounds__(512, 2) delta_apply_kernel(ChunkArgs p) {
+  using C = DC<KB>;
+  const DeltaArgs& a = p.a;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  constexpr int K = C::K, LP = KB == 1 ? 16 : KB == 2 ? 32 : 64;  // lanes of a token: a channel pair each
-  const int b = blockIdx.z, h = blockIdx.y, hk = h / (a.H / a.G);
+  constexpr int K = C::K;
+  const int b = blockIdx.z, h = blockIdx.y;
   const int t0 = a.m.cu[b], t1 = a.m.cu[b + 1];
   if (t1 - t0 < a.below) return;
-  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, fr = lane & 15, fg = lane >> 4;
-  const int pair = tid % LP, grp = tid / LP;                // staging: two channels of the chunk's tokens 4 grp ..
-  const bool on = grp < 8 && 2 * pair < K;
-  const int ch = min(2 * pair, K - 2);
-  float* sM = (float*)(smem + C::SM);
-  float* sD = (float*)(smem + C::SD);
-  float* sT = (float*)(smem + C::TOT);
-  float* sMid = (float*)(smem + C::MID);
-  float* sEnd = (float*)(smem + C::END);
-
-  for (int i = tid; i < 8 * FRAG / 16; i += 512) *(u32x4_t*)(smem + C::TF + i * 16) = u32x4_t{0, 0, 0, 0};
-
-  // this wave's columns
-  const int col = blockIdx.x * 128 + wv * 16 + fr, colc = min(col, a.V - 1);
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, nw = blockDim.x >> 6, fr = lane & 15, fg = lane >> 4;
+  const int col = blockIdx.x * nw * 16 + wv * 16 + fr, colc = min(col, a.V - 1);
   const bool live = col < a.V;
   float* st = a.state + (((size_t)a.m.slot[b] * a.H + h) * a.V + colc) * K + 4 * fg;
   f32x4_t S[2 * KB];
@@ -260,215 +502,53 @@ __global__ void __launch_bounds__(512, 2) delta_chunk_kernel(DeltaArgs a) {
     S[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     if (stored) S[i] = *(const f32x4_t*)(st + 16 * i);
   }
-
-  unsigned rk[4], rq[4];
-  f32x2_t rg[4];
-  bf16_t rv[8], rb = 0;
-  auto fetch = [&](int t) {
-    const bf16_t* x = (const bf16_t*)a.x;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const size_t row = min(t + 4 * min(grp, 7) + i, t1 - 1);
-      rq[i] = *(const unsigned*)(x + row * a.ldx + hk * K + ch);
-      rk[i] = *(const unsigned*)(x + row * a.ldx + (a.G + hk) * K + ch);
-      rg[i] = *(const f32x2_t*)(a.decay + row * a.H * K + (size_t)h * K + ch);
-    }
+  const char* src = p.frags + ((size_t)p.ch.base[b] * a.H + h) * C::NF * 1024 + lane * 16;
+  const size_t stride = (size_t)a.H * C::NF * 1024;
+  auto issue = [&](int k) {
+    char* dst = smem + (k & 1) * C::NF * 1024;
+    for (int f = wv; f < C::NF; f += nw)
+      __builtin_amdgcn_global_load_lds((frag_g_t)(src + k * stride + f * 1024), (frag_l_t)(dst + f * 1024), 16, 0, 0);
+  };
+  bf16_t rv[8];
+  auto load_v = [&](int t) {
 #pragma unroll
     for (int i = 0; i < 8; ++i)
-      rv[i] = x[(size_t)min(t + (i >> 2) * 16 + 4 * fg + (i & 3), t1 - 1) * a.ldx + 2 * a.G * K + h * a.V + colc];
-    if (pair < 4) rb = ((const bf16_t*)a.beta)[(size_t)min(t + 4 * min(grp, 7) + pair, t1 - 1) * a.ldb + h];
+      rv[i] = ((const bf16_t*)a.x)[(size_t)min(t + (i >> 2) * 16 + 4 * fg + (i & 3), t1 - 1) * a.ldx + 2 * a.G * K + h * a.V + colc];
   };
-
-  fetch(t0);
-  for (int t = t0, par = 0; t < t1; t += CT, par ^= 1) {
-    float* tok_rk = (float*)(smem + C::TOK) + par * 3 * CT;
-    float *tok_rq = tok_rk + CT, *tok_b = tok_rq + CT;
-    // ---- sums of this thread's 4 tokens, norms of the tokens; tokens past the end are zero and decay nothing
-    f32x2_t kap[4], chi[4], g[4], gl[4];
-    f32x2_t vv[4];  // V / rk comes later: V of the wave's columns, rows 4 fg + (0..3) of both token blocks
-    float nk[4], nq[4];
+  f32x4_t O[2];
+  auto store_o = [&](int t) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const bool in = on && t + 4 * grp + i < t1;
-      kap[i] = in ? f32x2_t{__uint_as_float(rk[i] << 16), __uint_as_float(rk[i] & 0xffff0000u)} : f32x2_t{0.f, 0.f};
-      chi[i] = in ? f32x2_t{__uint_as_float(rq[i] << 16), __uint_as_float(rq[i] & 0xffff0000u)} : f32x2_t{0.f, 0.f};
-#pragma unroll
-      for (int e = 0; e < 2; ++e) {
-        const float d = in ? rg[i][e] : 0.f;
-        g[i][e] = (i ? g[i - 1][e] : 0.f) + d;
-        gl[i][e] = (i ? gl[i - 1][e] : 0.f) + fmaxf(d, -24.f);
-      }
-      nk[i] = fmaf(kap[i][0], kap[i][0], kap[i][1] * kap[i][1]);
-      nq[i] = fmaf(chi[i][0], chi[i][0], chi[i][1] * chi[i][1]);
-    }
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      vv[i] = f32x2_t{bf2f(rv[i]), bf2f(rv[4 + i])};
-      nk[i] = lanes_sum<16>(nk[i]);
-      nq[i] = lanes_sum<16>(nq[i]);
-      if constexpr (LP > 16) {
-        nk[i] += __shfl_xor(nk[i], 16, 64);
-        nq[i] += __shfl_xor(nq[i], 16, 64);
-      }
-      if constexpr (LP > 32) {
-        nk[i] = sum_xhalf(nk[i]);
-        nq[i] = sum_xhalf(nq[i]);
-      }
-    }
-    if (grp < 8) {
-      if (on) {
-        *(f32x2_t*)(sT + grp * K + ch) = g[3];
-        *(f32x2_t*)(sT + (8 + grp) * K + ch) = gl[3];
-      }
-      if (pair < 4) {
-        const float k2 = pair == 0 ? nk[0] : pair == 1 ? nk[1] : pair == 2 ? nk[2] : nk[3];
-        const float q2 = pair == 0 ? nq[0] : pair == 1 ? nq[1] : pair == 2 ? nq[2] : nq[3];
-        const int i = 4 * grp + pair;
-        const float r2 = 1.f / (k2 + a.eps);
-        tok_rk[i] = sqrtf(r2);
-        tok_rq[i] = a.q_scale / sqrtf(q2 + a.eps);
-        tok_b[i] = t + i < t1 ? sigmoid32(bf2f(rb)) * r2 : 0.f;
-      }
-    }
-    __syncthreads();
-    // ---- the operands
-    if (on) {
-      f32x2_t base{0.f, 0.f}, basel{0.f, 0.f}, mid{0.f, 0.f}, end{0.f, 0.f};
-#pragma unroll
-      for (int i = 0; i < 8; ++i) {
-        const f32x2_t v = *(const f32x2_t*)(sT + i * K + ch), vl = *(const f32x2_t*)(sT + (8 + i) * K + ch);
-        end += v;
-        if (i < grp) base += v, basel += vl;
-        if (i <= (grp & ~1)) mid += vl;  // the first half of this thread's block of 8
-      }
-      if (!(grp & 1)) *(f32x2_t*)(sMid + grp / 2 * K + ch) = mid;
-      if (grp == 0)
-        *(f32x2_t*)(sEnd + ch) = f32x2_t{__builtin_amdgcn_exp2f(end[0]), __builtin_amdgcn_exp2f(end[1])};
-      const int ks = ch >> 5, blk = grp >> 2;
-      char* row = smem + ((blk * KB + ks) * 2) * FRAG;
-      f32x2_t km[4];
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        f32x2_t kp, qp, ak, aq, bk;
-#pragma unroll
-        for (int e = 0; e < 2; ++e) {
-          const float G = base[e] + g[i][e], Gm = basel[e] + gl[i][e] - mid[e];
-          const float P = __builtin_amdgcn_exp2f(G), E = __builtin_amdgcn_exp2f(Gm);
-          kp[e] = kap[i][e] * P;
-          qp[e] = chi[i][e] * P;
-          ak[e] = kap[i][e] * E;
-          aq[e] = chi[i][e] * E;
-          bk[e] = kap[i][e] * __builtin_amdgcn_exp2f(-Gm);
-          km[i][e] = kap[i][e] * __builtin_amdgcn_exp2f(end[e] - G);
-        }
-        const int at = frag_at((4 * grp + i) & 15, ch & 31);
-        auto put = [&](int op, const f32x2_t& v) {
-          const unsigned hi = pack_bf2(v[0], v[1]);
-          *(unsigned*)(row + op + at) = hi;
-          *(unsigned*)(row + op + FRAG + at) = lo_of(hi, v[0], v[1]);
-        };
-        put(C::KP, kp);
-        put(C::QP, qp);
-        put(C::AK, ak);
-        put(C::AQ, aq);
-        put(C::BK, bk);
-      }
-#pragma unroll
-      for (int e = 0; e < 2; ++e) {  // rows: channels; k: tokens
-        char* p = smem + C::KM + ((ch + e) >> 4) * 2 * FRAG + frag_at((ch + e) & 15, 4 * grp);
-        const unsigned h0 = pack_bf2(km[0][e], km[1][e]), h1 = pack_bf2(km[2][e], km[3][e]);
-        *(u32x2_t*)p = u32x2_t{h0, h1};
-        *(u32x2_t*)(p + FRAG) = u32x2_t{lo_of(h0, km[0][e], km[1][e]), lo_of(h1, km[2][e], km[3][e])};
-      }
-    }
-    if (t + CT < t1) fetch(t + CT);
-    __syncthreads();
-    // ---- M and Q, 8 x 8 blocks by the middle that their rows are scaled to. Waves 0, 1: blocks on the diagonal; 2, 3: below
-    // it within 16 tokens; 4, 5: rows 16 .. 23 and 24 .. 31 against columns 0 .. 15
-    if (wv < 6) {
-      const int rblk = wv < 4 ? wv & 1 : 1, cblk = wv < 4 ? wv & 1 : 0;
-      const int rsub = wv < 2 ? -1 : wv < 4 ? 2 * rblk + 1 : wv - 2;  // the rows' block of 8 that this wave fills
-      f32x4_t m{0.f, 0.f, 0.f, 0.f}, q = m;
-#pragma unroll
-      for (int ks = 0; ks < KB; ++ks) {
-        Split B = frag_load(smem + C::BK + (cblk * KB + ks) * 2 * FRAG, lane);
-        if (rsub >= 0) {  // column fr is scaled to its own block's middle: to the rows'
-          const int c = ks * 32 + 4 * fg;
-          f32x4_t v[2];
-#pragma unroll
-          for (int u = 0; u < 2; ++u) {
-            const f32x4_t to = *(const f32x4_t*)(sMid + rsub * K + c + 16 * u);
-            const f32x4_t from = *(const f32x4_t*)(sMid + (cblk * 2 + (fr >> 3)) * K + c + 16 * u);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-              // in two steps: the factor alone may underflow where the product does not
-              const float f = __builtin_amdgcn_exp2f(0.5f * fminf(to[e] - from[e], 0.f));
-              v[u][e] = (bf2f((bf16_t)B.hi[4 * u + e]) + bf2f((bf16_t)B.lo[4 * u + e])) * f * f;
-            }
-          }
-          B = split8(v[0], v[1]);
-        }
-        m = mma3(frag_load(smem + C::AK + (rblk * KB + ks) * 2 * FRAG, lane), B, m);
-        q = mma3(frag_load(smem + C::AQ + (rblk * KB + ks) * 2 * FRAG, lane), B, q);
-      }
-      const int j = cblk * 16 + fr;
+    for (int i = 0; i < 2; ++i)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        const int r = rblk * 16 + 4 * fg + e;
-        const bool mine = rsub < 0 ? r / 8 == j / 8 : r / 8 == rsub && (wv >= 4 || j / 8 == rsub - 1);
-        if (!mine) continue;
-        sM[r * 36 + j] = j < r ? m[e] * tok_b[r] : 0.f;
-        const float v = j <= r ? q[e] : 0.f;
-        const bf16_t hi = f2bf(v);
-        char* p = smem + C::QF + rblk * 2 * FRAG + frag_at(r & 15, j);
-        *(bf16_t*)p = hi;
-        *(bf16_t*)(p + FRAG) = f2bf(v - bf2f(hi));
+        const int tt = t + 16 * i + 4 * fg + e;
+        if (live && tt < t1) ((bf16_t*)a.o)[(size_t)tt * a.ldo + h * a.V + col] = f2bf(O[i][e]);
       }
+  };
+  issue(0);
+  load_v(t0);
+  for (int t = t0, k = 0; t < t1; t += CT, ++k) {
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    lds_barrier();  // this chunk's fragments are there; every wave is done with the last chunk's
+    const char* buf = smem + (k & 1) * C::NF * 1024;
+    const float* vec = (const float*)(buf + C::VEC * 1024);
+    f32x4_t X[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const f32x4_t r = *(const f32x4_t*)(vec + K + 16 * i + 4 * fg);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) X[i][e] = t + 16 * i + 4 * fg + e < t1 ? bf2f(rv[4 * i + e]) * __builtin_amdgcn_rcpf(r[e]) : 0.f;
     }
-    __syncthreads();
-    // ---- T by wave 0, while the others begin with the products of the state
-    if (wv == 0) {
-      const int blk = fg & 1;
-      const float* L = sM + blk * 16 * 36 + blk * 16;
-      float x[16];
-#pragma unroll
-      for (int r = 0; r < 16; ++r) {
-        float v = r == fr ? 1.f : 0.f;
-#pragma unroll
-        for (int i = 0; i < r; ++i) v = fmaf(-L[r * 36 + i], x[i], v);
-        x[r] = v;
-      }
-      auto put = [&](int r, int j, float v) {  // T[r][j]
-        const bf16_t hi = f2bf(v);
-        char* p = smem + C::TF + (r >> 4) * 2 * FRAG + frag_at(r & 15, j);
-        *(bf16_t*)p = hi;
-        *(bf16_t*)(p + FRAG) = f2bf(v - bf2f(hi));
-      };
-      if (fg < 2) {
-        const float bj = tok_b[blk * 16 + fr];
-#pragma unroll
-        for (int r = 0; r < 16; ++r) {
-          sD[(blk * 16 + r) * 17 + fr] = x[r];
-          put(blk * 16 + r, blk * 16 + fr, x[r] * bj);
-        }
-      }
-      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // this wave's own LDS writes are read back by it alone
-      __builtin_amdgcn_wave_barrier();
-      f32x4_t y{0.f, 0.f, 0.f, 0.f}, z = y;
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        y = __builtin_amdgcn_mfma_f32_16x16x4f32(sM[(16 + fr) * 36 + 4 * i + fg], sD[(4 * i + fg) * 17 + fr], y, 0, 0, 0);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) sD[(32 + 4 * fg + e) * 17 + fr] = y[e];
-      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-      __builtin_amdgcn_wave_barrier();
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        z = __builtin_amdgcn_mfma_f32_16x16x4f32(sD[(16 + fr) * 17 + 4 * i + fg], sD[(32 + 4 * i + fg) * 17 + fr], z, 0, 0, 0);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) put(16 + 4 * fg + e, fr, -z[e] * tok_b[fr]);
+    if (k) store_o(t - CT);
+    if (t + CT < t1) {
+      issue(k + 1);
+      load_v(t + CT);
     }
-    f32x4_t R[2], O[2];
+    auto frag = [&](int f) {
+      const char* q = buf + f * 1024 + lane * 16;
+      return Split{*(const bf16x8_t*)q, *(const bf16x8_t*)(q + 1024)};
+    };
+    f32x4_t R[2];
 #pragma unroll
     for (int i = 0; i < 2; ++i) R[i] = O[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -476,54 +556,43 @@ __global__ void __launch_bounds__(512, 2) delta_chunk_kernel(DeltaArgs a) {
       const Split B = split8(S[2 * ks], S[2 * ks + 1]);
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
-        R[i] = mma3(frag_load(smem + C::KP + (i * KB + ks) * 2 * FRAG, lane), B, R[i]);
-        O[i] = mma3(frag_load(smem + C::QP + (i * KB + ks) * 2 * FRAG, lane), B, O[i]);
+        R[i] = mma3(frag(C::KP + (i * KB + ks) * 2), B, R[i]);
+        O[i] = mma3(frag(C::QP + (i * KB + ks) * 2), B, O[i]);
       }
     }
-    __syncthreads();
-    // ---- what the tokens write, what they read, the state after them
-    f32x4_t X[2], U[2];
+    Split B = split8(X[0] - R[0], X[1] - R[1]);
+    f32x4_t U[2];
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const f32x4_t r = *(const f32x4_t*)(tok_rk + 16 * i + 4 * fg);
-#pragma unroll
-      for (int e = 0; e < 4; ++e)
-        X[i][e] = t + 16 * i + 4 * fg + e < t1 ? vv[e][i] * __builtin_amdgcn_rcpf(r[e]) - R[i][e] : 0.f;
-      U[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    }
-    Split B = split8(X[0], X[1]);
-#pragma unroll
-    for (int i = 0; i < 2; ++i) U[i] = mma3(frag_load(smem + C::TF + i * 2 * FRAG, lane), B, U[i]);
+    for (int i = 0; i < 2; ++i) U[i] = mma3(frag(C::TF + i * 2), B, f32x4_t{0.f, 0.f, 0.f, 0.f});
     B = split8(U[0], U[1]);
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      O[i] = mma3(frag_load(smem + C::QF + i * 2 * FRAG, lane), B, O[i]);
-      const f32x4_t r = *(const f32x4_t*)(tok_rq + 16 * i + 4 * fg);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int tt = t + 16 * i + 4 * fg + e;
-        if (live && tt < t1) ((bf16_t*)a.o)[(size_t)tt * a.ldo + h * a.V + col] = f2bf(O[i][e] * r[e]);
-      }
-    }
+    for (int i = 0; i < 2; ++i) O[i] = mma3(frag(C::QF + i * 2), B, O[i]) * *(const f32x4_t*)(vec + K + CT + 16 * i + 4 * fg);
 #pragma unroll
     for (int i = 0; i < 2 * KB; ++i) {
-      S[i] *= *(const f32x4_t*)(sEnd + 16 * i + 4 * fg);
-      S[i] = mma3(frag_load(smem + C::KM + i * 2 * FRAG, lane), B, S[i]);
+      S[i] *= *(const f32x4_t*)(vec + 16 * i + 4 * fg);
+      S[i] = mma3(frag(C::KM + i * 2), B, S[i]);
     }
   }
+  store_o(t0 + (t1 - t0 - 1) / CT * CT);
   if (live)
 #pragma unroll
     for (int i = 0; i < 2 * KB; ++i) *(f32x4_t*)(st + 16 * i) = S[i];
-  const int wg = blockIdx.y * gridDim.x + blockIdx.x, step = gridDim.x * gridDim.y * 512;
-  for (int c = wg * 512 + tid; c < a.conv.C; c += step) conv_state_store<bf16_t>(a.conv, a.m, b, c);
+  const int wg = blockIdx.y * gridDim.x + blockIdx.x, step = gridDim.x * gridDim.y * blockDim.x;
+  for (int c = wg * blockDim.x + threadIdx.x; c < a.conv.C; c += step) conv_state_store<bf16_t>(a.conv, a.m, b, c);
 }
 
 template <int KB>
-static int launch_delta_chunk(const DeltaArgs& a, hipStream_t s) {
-  static const hipError_t e = hipFuncSetAttribute((const void*)delta_chunk_kernel<KB>,
-                                                  hipFuncAttributeMaxDynamicSharedMemorySize, DC<KB>::BYTES);
+static int launch_delta_chunk(const ChunkArgs& p, hipStream_t s) {
+  constexpr int lds = 2 * DC<KB>::NF * 1024;
+  static const hipError_t e = hipFuncSetAttribute((const void*)delta_apply_kernel<KB>,
+                                                  hipFuncAttributeMaxDynamicSharedMemorySize, lds);
   if (e != hipSuccess) return (int)e;
-  delta_chunk_kernel<KB><<<dim3((a.V + 127) / 128, a.H, a.m.B), 512, DC<KB>::BYTES, s>>>(a);
+  const DeltaArgs& a = p.a;
+  delta_prep_kernel<KB><<<(p.ch.n * a.H + 3) / 4, 256, 0, s>>>(p);
+  // a head's columns on one CU where the heads fill the chip, else spread over more
+  int nw = 8;
+  while (nw > 2 && (long long)a.m.B * a.H * ((a.V + 16 * nw - 1) / (16 * nw)) < 256) nw /= 2;
+  delta_apply_kernel<KB><<<dim3((a.V + 16 * nw - 1) / (16 * nw), a.H, a.m.B), 64 * nw, lds, s>>>(p);
   DA_LAUNCH_CHECK();
 }
 
@@ -582,22 +651,22 @@ static int launch_delta(const DeltaArgs& a, hipStream_t s) {
 }
 
 template <typename T>
-static int launch_delta_t(const DeltaArgs& a0, int min_len, int max_len, int chunk_from, const void* w, const void* gate, int ldg, int dim,
-                          float eps, hipStream_t s) {
-  DeltaArgs a = a0;
+static int launch_delta_t(const ChunkArgs& p0, int min_len, const void* w, const void* gate, int ldg, int dim, float eps,
+                          hipStream_t s) {
+  ChunkArgs p = p0;
+  DeltaArgs& a = p.a;
   int err = 0;
-  a.below = 0x7fffffff;
-  if constexpr (sizeof(T) == 2) {
-    if (max_len >= chunk_from && a.K <= 128) {
-      a.below = chunk_from;
-      switch (a.K) {
-        case 32: err = launch_delta_chunk<1>(a, s); break;
-        case 64: err = launch_delta_chunk<2>(a, s); break;
-        case 96: err = launch_delta_chunk<3>(a, s); break;
-        default: err = launch_delta_chunk<4>(a, s); break;
-      }
-      if (err) return err;
+  if (sizeof(T) == 2 && p.ch.n) {
+    switch (a.K) {
+      case 32: err = launch_delta_chunk<1>(p, s); break;
+      case 64: err = launch_delta_chunk<2>(p, s); break;
+      case 96: err = launch_delta_chunk<3>(p, s); break;
+      case 128: err = launch_delta_chunk<4>(p, s); break;
+      default: return (int)hipErrorInvalidValue;
     }
+    if (err) return err;
+  } else {
+    a.below = 0x7fffffff;
   }
   if (min_len < a.below) switch (a.K) {
 #define DELTA_CASE(LN, N) \
@@ -621,18 +690,22 @@ static int launch_delta_t(const DeltaArgs& a0, int min_len, int max_len, int chu
 // x [T][ldx] (activation type): G query heads, G key heads of K channels, H value heads of V; decay fp32 [T][H K];
 // K = 32 n (n <= 8), 64 n (n <= 8) or 128 n (n <= 8); V % 4 == 0. norm weight w fp32 [V], gate [T][ldg]; dim: the
 // channels a value head really has. conv: as the other recurrences' (state null: kept by the convolution's launch).
-// min_len / max_len: shortest and longest portion; bf16 portions of chunk_from tokens or more run in chunks where K <= 128.
+// min_len: shortest portion. Chunk list ck / base (n_chunks of them, 32 tokens each, of all portions) and scratch frags
+// [n_chunks][H][(3 K / 8 + 9) KB]: bf16 portions of chunk_from tokens or more run in chunks (K 32, 64, 96 or 128).
 DA_EXPORT int da_delta_rule(const void* x, int ldx, const void* decay, const void* beta, int ldb, void* state, void* o,
                             int ldo, int H, int G, int K, int V, float q_scale, float unit_eps, const void* w,
                             const void* gate, int ldg, int dim, float eps, const void* conv_x, int ld_conv,
-                            void* conv_state, int taps, int conv_c, int min_len, int max_len, int chunk_from, const void* cu,
+                            void* conv_state, int taps, int conv_c, int min_len, int chunk_from, const void* ck,
+                            const void* base, int n_chunks, void* frags, const void* cu,
                             const void* slot, const void* pos0, const void* seq, int T, int B, int f32, void* stream) {
   if (T < 1 || B < 1 || B > 65535 || G < 1 || H % G || H > 65535 || V < 4 || V % 4 ||
-      ldx % 4 || ldo % 4 || ldg % 4 || dim < 1 || dim > V || taps < 1 || min_len < 1 || max_len < min_len || chunk_from < 1 || ldx % 2 || (long long)T * H > 0x7fffffffll / 4)
+      ldx % 4 || ldo % 4 || ldg % 4 || dim < 1 || dim > V || taps < 1 || min_len < 1 || chunk_from < 1 || n_chunks < 0 || (n_chunks && (!ck || !base || !frags)) ||
+      (long long)n_chunks * H > 0x7fffffffll / 4 || ldx % 2 || (long long)T * H > 0x7fffffffll / 4)
     return (int)hipErrorInvalidValue;
-  DeltaArgs a{x, ldx, (const float*)decay, beta, ldb, (float*)state, o, ldo, H, G, K, V, q_scale, unit_eps, 0,
-              ConvState{conv_x, ld_conv, conv_state, taps, conv_c},
-              SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B}};
-  return f32 ? launch_delta_t<float>(a, min_len, max_len, chunk_from, w, gate, ldg, dim, eps, (hipStream_t)stream)
-             : launch_delta_t<bf16_t>(a, min_len, max_len, chunk_from, w, gate, ldg, dim, eps, (hipStream_t)stream);
+  ChunkArgs p{DeltaArgs{x, ldx, (const float*)decay, beta, ldb, (float*)state, o, ldo, H, G, K, V, q_scale, unit_eps, chunk_from,
+                        ConvState{conv_x, ld_conv, conv_state, taps, conv_c},
+                        SeqMeta{(const int*)cu, (const int*)slot, (const int*)pos0, (const int*)seq, T, B}},
+              ChunkMeta{(const int*)ck, (const int*)base, n_chunks, CT}, (char*)frags};
+  return f32 ? launch_delta_t<float>(p, min_len, w, gate, ldg, dim, eps, (hipStream_t)stream)
+             : launch_delta_t<bf16_t>(p, min_len, w, gate, ldg, dim, eps, (hipStream_t)stream);
 }

@@ -266,7 +266,7 @@ __global__ void __launch_bounds__(256, 2) latent_mfma_kernel(LatArgs a, int rtil
     top = fmaxf(top, __shfl_xor(top, 16, 64));
     top = fmaxf(top, __shfl_xor(top, 32, 64));
     if (fg == 0) sM[wv * 16 + fr] = top;
-    __syncthreads();  // maxima written; every wave is done with the last page's latents and weights
+    lds_barrier();  // maxima written; every wave is done with the last page's latents and weights
 #pragma unroll
     for (int ds = 0; ds < NLS; ++ds) *(bf16x8_t*)(sV + key * C::VSTR + ds * 64 + fg * 16) = kf[ds];
     if (p + 1 < p1) load_page(p + 1);
@@ -285,7 +285,7 @@ __global__ void __launch_bounds__(256, 2) latent_mfma_kernel(LatArgs a, int rtil
     *(u32x2_t*)(pp + 16 * C::PSTR) = u32x2_t{split_lo(h0, s[0], s[1]), split_lo(h1, s[2], s[3])};
 #pragma unroll
     for (int i = 0; i < NDB; ++i) oacc[i] *= f;
-    __syncthreads();
+    lds_barrier();
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
       // k slot 8 fg + j of the product holds key 32 half + 16 (j / 4) + 4 fg + j % 4
@@ -307,9 +307,9 @@ __global__ void __launch_bounds__(256, 2) latent_mfma_kernel(LatArgs a, int rtil
   }
   sum += __shfl_xor(sum, 16, 64);
   sum += __shfl_xor(sum, 32, 64);
-  __syncthreads();
+  lds_barrier();
   if (fg == 0) sM[wv * 16 + fr] = sum;
-  __syncthreads();
+  lds_barrier();
   sum = sM[fr] + sM[16 + fr] + sM[32 + fr] + sM[48 + fr];
   if (row >= rows) return;
   if (a.nsplit > 1) {
@@ -481,9 +481,9 @@ __global__ void __launch_bounds__(256, 2) latent_flash_kernel(FlashArgs p, int n
 
   load(0);
   for (int t = 0; t < nt; ++t) {
-    __syncthreads();
+    lds_barrier();
     store();
-    __syncthreads();
+    lds_barrier();
     if (t + 1 < nt) load(t + 1);
     const int kb = t * PAGE;
     if (kb > wlast) continue;

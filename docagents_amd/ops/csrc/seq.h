@@ -47,6 +47,14 @@ template <> struct Act<float> {
   __device__ static __forceinline__ void store2(float* p, float a, float b) { *(f32x2_t*)p = f32x2_t{a, b}; }
 };
 
+// Workgroup barrier for LDS alone: this wave's LDS accesses are done, its global loads stay in flight
+// (__syncthreads() waits for those too).
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
 // Elementary functions good to a few fp32 ulp on the hardware's 1-ulp exp2 / log2 / rcp / sqrt (the library
 // forms spend most of their instructions on cases that cannot occur here: the epilogues and scans that
 // use these run at their instruction count).

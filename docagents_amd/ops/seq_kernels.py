@@ -22,8 +22,8 @@ K._SIGS.update({
     "da_stream_add": [c_void_p] + [c_void_p, c_int, c_void_p, c_void_p] * 2 + [c_void_p, c_void_p, c_int, c_float]
                      + [c_void_p, c_void_p, c_float, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p],
     "da_delta_rule": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int] + [c_int] * 4
-                     + [c_float, c_float, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p, c_int, c_void_p] + [c_int] * 5
-                     + _META + [c_int, c_void_p],
+                     + [c_float, c_float, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p, c_int, c_void_p] + [c_int] * 4
+                     + [c_void_p, c_void_p, c_int, c_void_p] + _META + [c_int, c_void_p],
     "da_latent_prep": [c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int, c_int, c_float, c_void_p,
                        c_void_p, c_int, c_void_p, c_int, c_void_p, c_int] + _META + [c_int, c_void_p],
     "da_latent_attn": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p,
@@ -48,7 +48,8 @@ K._PART_OF.update({n: "hybrid" for n in ("da_gemm_any", "da_stream_step", "da_st
                                          "da_latent_prep", "da_latent_attn", "da_latent_gather", "da_latent_flash")})
 
 ACTS = (torch.bfloat16, torch.float32)
-DELTA_CHUNK_FROM = 33  # tokens from which a portion's delta rule runs in chunks on the matrix cores (bf16)
+DELTA_CHUNK = 32       # tokens of a chunk of the delta rule on the matrix cores (bf16)
+DELTA_CHUNK_FROM = 33  # tokens from which a portion runs in chunks
 LATENT_MFMA = (64, 128, 256, 512)  # latents the matrix-core attention takes (with a key part of 32 or 64 columns)
 ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_RGLRU, ANY_SWIGLU, ANY_ACT = 0, 1, 2, 3, 4, 5
 
@@ -348,6 +349,11 @@ def sigmoid_attn(qkg, kc, kr, pb, qk_w, m: SeqBatch, H: int, G: int, dim: int, s
     return out
 
 
+def delta_chunk_bytes(K: int) -> int:
+    """Scratch of a chunk and head (fragments of 1 KB)."""
+    return (3 * K // 8 + 9) * 1024
+
+
 def delta_rule(qkv, decay, beta, state, conv_x, conv_state, m: SeqBatch, H: int, G: int, q_scale: float, unit_eps: float,
                norm):
     """Gated delta rule: qkv [T, 2 G K + H V] (after the convolution), decay fp32 [T, H K] (log2 of each key channel's
@@ -366,11 +372,16 @@ def delta_rule(qkv, decay, beta, state, conv_x, conv_state, m: SeqBatch, H: int,
     _req(H2 == H and qkv.shape == (m.T, C) and qkv.stride(0) % 4 == 0 and beta.shape[0] == m.T and beta.shape[1] >= H
          and gate.shape == (m.T, H * V) and gate.stride(0) % 4 == 0 and V % 4 == 0, "delta_rule shapes")
     o = torch.empty((m.T, H * V), dtype=qkv.dtype, device=qkv.device)
+    ck = base = frags = None
+    n = 0
+    if not f32 and Kd <= 128 and m.max_len >= DELTA_CHUNK_FROM:
+        ck, base, n = m.chunks(DELTA_CHUNK)
+        frags = torch.empty(n * H * delta_chunk_bytes(Kd), dtype=torch.uint8, device=qkv.device)
     _check(lib().da_delta_rule(_ptr(qkv), qkv.stride(0), _ptr(decay), _ptr(beta), beta.stride(0), _ptr(state), _ptr(o), H * V,
                                H, G, Kd, V, float(q_scale), float(unit_eps), _ptr(weight), _ptr(gate), gate.stride(0), dim,
                                float(eps), *_conv_args(conv_x, conv_state, C, qkv.dtype, m), C,
-                               1 if m.lens is None else int(m.lens.min()), m.max_len, DELTA_CHUNK_FROM, *_meta(m),
-                               f32, _stream()), "delta_rule")
+                               1 if m.lens is None else int(m.lens.min()), DELTA_CHUNK_FROM, _ptr(ck), _ptr(base), n,
+                               _ptr(frags), *_meta(m), f32, _stream()), "delta_rule")
     return o
 
 
