@@ -183,7 +183,8 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
 //   S <- 2^G_end S + (kappa 2^(G_end - G))^T U
 // delta_prep: a wave per chunk and head forms what does not depend on S (kappa 2^G, chi 2^G, kappa 2^(G_end - G), T, Q), as
 // MFMA fragments in scratch memory. delta_apply: a wave walks its portion's chunks with 16 columns of V and S by itself,
-// S staying in its accumulators; the waves of a workgroup share the next chunk's fragments, in flight to LDS meanwhile.
+// S staying in its accumulators; the waves of a workgroup share the fragments, which are on their way to LDS one and
+// two chunks ahead.
 //
 // Every fp32 operand enters its product as two bf16 terms (its rounding and the remainder), three of their four
 // products taken: about 16 bits, accumulated in fp32. The solve of T is in fp32.
@@ -224,6 +225,8 @@ template <int KB> struct DC {  // K = 32 KB key channels; offsets in fragments
   static constexpr int TF = 12 * KB, QF = TF + 4;      // T, Q: [token block][tokens]
   static constexpr int VEC = QF + 4;                   // fp32: 2^G_end [K], rk [32], rq [32]
   static constexpr int NF = VEC + 1;
+  // delta_apply: what the state is multiplied by first, and the rest
+  static constexpr int NA = KM, NB = NF - KM;
 };
 
 struct Vec8 { f32x4_t u[2]; };  // a lane's 8 channels (or tokens), 16 u + 4 fg + e
@@ -482,17 +485,31 @@ __global__ void __launch_bounds__(256, 2) delta_prep_kernel(ChunkArgs p) {
 typedef __attribute__((address_space(1))) const void* frag_g_t;
 typedef __attribute__((address_space(3))) void* frag_l_t;
 
-template <int KB>
-__global__ void __launch_bounds__(512, 2) delta_apply_kernel(ChunkArgs p) {
+template <int N> __device__ __forceinline__ void vm_wait() {  // all but this wave's last N memory operations are done
+  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
+}
+
+// LDS of NW waves: part A of three chunks (two with 8 waves, whose V takes the space), part B of two; V of the workgroup's
+// columns of two.
+template <int KB, int NW> struct DL {
   using C = DC<KB>;
+  static constexpr int AHEAD = NW == 8 ? 1 : 2, B = (AHEAD + 1) * C::NA, VB = CT * 16 * NW * 2;  // chunks; fragments; bytes
+  static constexpr int V = (B + 2 * C::NB) * 1024, BYTES = V + 2 * VB;
+  static_assert(BYTES <= 160 * 1024, "LDS");
+};
+
+template <int KB, int NW>  // NW waves
+__global__ void __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) delta_apply_kernel(ChunkArgs p) {
+  using C = DC<KB>;
+  using D = DL<KB, NW>;
   const DeltaArgs& a = p.a;
   extern __shared__ __attribute__((aligned(16))) char smem[];
   constexpr int K = C::K;
   const int b = blockIdx.z, h = blockIdx.y;
   const int t0 = a.m.cu[b], t1 = a.m.cu[b + 1];
   if (t1 - t0 < a.below) return;
-  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, nw = blockDim.x >> 6, fr = lane & 15, fg = lane >> 4;
-  const int col = blockIdx.x * nw * 16 + wv * 16 + fr, colc = min(col, a.V - 1);
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, fr = lane & 15, fg = lane >> 4;
+  const int col = blockIdx.x * NW * 16 + wv * 16 + fr, colc = min(col, a.V - 1);
   const bool live = col < a.V;
   float* st = a.state + (((size_t)a.m.slot[b] * a.H + h) * a.V + colc) * K + 4 * fg;
   f32x4_t S[2 * KB];
@@ -504,96 +521,163 @@ __global__ void __launch_bounds__(512, 2) delta_apply_kernel(ChunkArgs p) {
   }
   const char* src = p.frags + ((size_t)p.ch.base[b] * a.H + h) * C::NF * 1024 + lane * 16;
   const size_t stride = (size_t)a.H * C::NF * 1024;
-  auto issue = [&](int k) {
-    char* dst = smem + (k & 1) * C::NF * 1024;
-    for (int f = wv; f < C::NF; f += nw)
-      __builtin_amdgcn_global_load_lds((frag_g_t)(src + k * stride + f * 1024), (frag_l_t)(dst + f * 1024), 16, 0, 0);
-  };
-  bf16_t rv[8];
-  auto load_v = [&](int t) {
+  const int nc = (t1 - t0 + CT - 1) / CT;
+  // a chunk's two parts to LDS, PA and PB instructions a wave (chunks past the last one: that one again, unread)
+  constexpr int PA = (C::NA + NW - 1) / NW, PB = (C::NB + NW - 1) / NW;
+  auto issue_a = [&](int k) {
+    const char* from = src + min(k, nc - 1) * stride;
+    char* to = smem + k % (D::AHEAD + 1) * C::NA * 1024;
 #pragma unroll
-    for (int i = 0; i < 8; ++i)
-      rv[i] = ((const bf16_t*)a.x)[(size_t)min(t + (i >> 2) * 16 + 4 * fg + (i & 3), t1 - 1) * a.ldx + 2 * a.G * K + h * a.V + colc];
+    for (int i = 0; i < PA; ++i) {
+      const int f = min(wv + i * NW, C::NA - 1);
+      __builtin_amdgcn_global_load_lds((frag_g_t)(from + f * 1024), (frag_l_t)(to + f * 1024), 16, 0, 0);
+    }
+  };
+  auto issue_b = [&](int k) {
+    const char* from = src + min(k, nc - 1) * stride + C::KM * 1024;
+    char* to = smem + (D::B + (k & 1) * C::NB) * 1024;
+#pragma unroll
+    for (int i = 0; i < PB; ++i) {
+      const int f = min(wv + i * NW, C::NB - 1);
+      __builtin_amdgcn_global_load_lds((frag_g_t)(from + f * 1024), (frag_l_t)(to + f * 1024), 16, 0, 0);
+    }
+  };
+  // V's tokens x columns, one instruction a wave: 16 bytes a lane, 2 NW lanes a token
+  auto issue_v = [&](int k) {
+    const int i = wv * 64 + lane, c = min(blockIdx.x * NW * 16 + i % (2 * NW) * 8, a.V - 8);
+    const bf16_t* from = (const bf16_t*)a.x + (size_t)min(t0 + min(k, nc - 1) * CT + i / (2 * NW), t1 - 1) * a.ldx + 2 * a.G * K +
+                         h * a.V + c;
+    __builtin_amdgcn_global_load_lds((frag_g_t)from, (frag_l_t)(smem + D::V + (k & 1) * D::VB + wv * 1024), 16, 0, 0);
   };
   f32x4_t O[2];
   auto store_o = [&](int t) {
+    if (!live) return;
+    bf16_t* o = (bf16_t*)a.o + (size_t)(t + 4 * fg) * a.ldo + h * a.V + col;
+    if (t + CT <= t1) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i)
+      for (int i = 0; i < 8; ++i) o[(size_t)((i >> 2) * 16 + (i & 3)) * a.ldo] = f2bf(O[i >> 2][i & 3]);
+    } else {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int tt = t + 16 * i + 4 * fg + e;
-        if (live && tt < t1) ((bf16_t*)a.o)[(size_t)tt * a.ldo + h * a.V + col] = f2bf(O[i][e]);
-      }
+      for (int i = 0; i < 8; ++i)
+        if (t + 4 * fg + (i >> 2) * 16 + (i & 3) < t1) o[(size_t)((i >> 2) * 16 + (i & 3)) * a.ldo] = f2bf(O[i >> 2][i & 3]);
+    }
   };
-  issue(0);
-  load_v(t0);
-  for (int t = t0, k = 0; t < t1; t += CT, ++k) {
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  issue_a(0);
+  issue_b(0);
+  issue_v(0);
+  if (D::AHEAD == 2) issue_a(1);
+  // LDS reads run a step ahead of the products that use them; the scheduling barriers keep them there.
+  for (int k = 0; k < nc; ++k) {
+    const int t = t0 + k * CT;
+    vm_wait<D::AHEAD == 2 ? PA : 0>();  // all but the next chunk's part A
     lds_barrier();  // this chunk's fragments are there; every wave is done with the last chunk's
-    const char* buf = smem + (k & 1) * C::NF * 1024;
-    const float* vec = (const float*)(buf + C::VEC * 1024);
-    f32x4_t X[2];
-#pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const f32x4_t r = *(const f32x4_t*)(vec + K + 16 * i + 4 * fg);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) X[i][e] = t + 16 * i + 4 * fg + e < t1 ? bf2f(rv[4 * i + e]) * __builtin_amdgcn_rcpf(r[e]) : 0.f;
-    }
-    if (k) store_o(t - CT);
-    if (t + CT < t1) {
-      issue(k + 1);
-      load_v(t + CT);
-    }
+    const char* bufa = smem + k % (D::AHEAD + 1) * C::NA * 1024;
+    const char* bufb = smem + (D::B + (k & 1) * C::NB - C::KM) * 1024;
+    const float* vec = (const float*)(bufb + C::VEC * 1024);
     auto frag = [&](int f) {
-      const char* q = buf + f * 1024 + lane * 16;
+      const char* q = (f < C::NA ? bufa : bufb) + f * 1024 + lane * 16;
       return Split{*(const bf16x8_t*)q, *(const bf16x8_t*)(q + 1024)};
     };
+    Split kp[2][2], qp[2][2], tf[2], qf[2], km[4];
+    auto load_ks = [&](int ks) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        kp[ks & 1][i] = frag(C::KP + (i * KB + ks) * 2);
+        qp[ks & 1][i] = frag(C::QP + (i * KB + ks) * 2);
+      }
+    };
+    load_ks(0);
+    f32x4_t rk[2], rq[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      rk[i] = *(const f32x4_t*)(vec + K + 16 * i + 4 * fg);
+      rq[i] = *(const f32x4_t*)(vec + K + CT + 16 * i + 4 * fg);
+    }
+    if (k) store_o(t - CT);
+    issue_b(k + 1);
+    issue_v(k + 1);
+    issue_a(k + D::AHEAD);
     f32x4_t R[2];
 #pragma unroll
     for (int i = 0; i < 2; ++i) R[i] = O[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int ks = 0; ks < KB; ++ks) {
+      if (ks + 1 < KB) {
+        load_ks(ks + 1);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 2; ++i) {
+          tf[i] = frag(C::TF + i * 2);
+          qf[i] = frag(C::QF + i * 2);
+        }
+      }
+      __builtin_amdgcn_sched_barrier(0);
       const Split B = split8(S[2 * ks], S[2 * ks + 1]);
 #pragma unroll
       for (int i = 0; i < 2; ++i) {
-        R[i] = mma3(frag(C::KP + (i * KB + ks) * 2), B, R[i]);
-        O[i] = mma3(frag(C::QP + (i * KB + ks) * 2), B, O[i]);
+        R[i] = mma3(kp[ks & 1][i], B, R[i]);
+        O[i] = mma3(qp[ks & 1][i], B, O[i]);
       }
+      __builtin_amdgcn_sched_barrier(0);
     }
-    Split B = split8(X[0] - R[0], X[1] - R[1]);
-    f32x4_t U[2];
+    constexpr int PRE = 2 * KB < 4 ? 2 * KB : 4;
+    f32x4_t end[2 * KB];
 #pragma unroll
-    for (int i = 0; i < 2; ++i) U[i] = mma3(frag(C::TF + i * 2), B, f32x4_t{0.f, 0.f, 0.f, 0.f});
+    for (int i = 0; i < PRE; ++i) km[i] = frag(C::KM + i * 2);
+#pragma unroll
+    for (int i = 0; i < 2 * KB; ++i) end[i] = *(const f32x4_t*)(vec + 16 * i + 4 * fg);
+    const bf16_t* vl = (const bf16_t*)(smem + D::V + (k & 1) * D::VB) + 4 * fg * 16 * NW + wv * 16 + fr;
+    unsigned rv[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) rv[i] = vl[((i >> 2) * 16 + (i & 3)) * 16 * NW];
+    __builtin_amdgcn_sched_barrier(0);
+    f32x4_t X[2], U[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        X[i][e] = t + 16 * i + 4 * fg + e < t1 ? fmaf(__uint_as_float(rv[4 * i + e] << 16), __builtin_amdgcn_rcpf(rk[i][e]), -R[i][e]) : 0.f;
+    Split B = split8(X[0], X[1]);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) U[i] = mma3(tf[i], B, f32x4_t{0.f, 0.f, 0.f, 0.f});
     B = split8(U[0], U[1]);
 #pragma unroll
-    for (int i = 0; i < 2; ++i) O[i] = mma3(frag(C::QF + i * 2), B, O[i]) * *(const f32x4_t*)(vec + K + CT + 16 * i + 4 * fg);
+    for (int i = 0; i < 2 * KB; ++i) S[i] *= end[i];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) O[i] = mma3(qf[i], B, O[i]) * rq[i];
 #pragma unroll
     for (int i = 0; i < 2 * KB; ++i) {
-      S[i] *= *(const f32x4_t*)(vec + 16 * i + 4 * fg);
-      S[i] = mma3(frag(C::KM + i * 2), B, S[i]);
+      S[i] = mma3(km[i % PRE], B, S[i]);
+      if (i + PRE < 2 * KB) km[i % PRE] = frag(C::KM + (i + PRE) * 2);
     }
   }
-  store_o(t0 + (t1 - t0 - 1) / CT * CT);
+  store_o(t0 + (nc - 1) * CT);
   if (live)
 #pragma unroll
     for (int i = 0; i < 2 * KB; ++i) *(f32x4_t*)(st + 16 * i) = S[i];
-  const int wg = blockIdx.y * gridDim.x + blockIdx.x, step = gridDim.x * gridDim.y * blockDim.x;
-  for (int c = wg * blockDim.x + threadIdx.x; c < a.conv.C; c += step) conv_state_store<bf16_t>(a.conv, a.m, b, c);
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // no transfer to LDS outlives its workgroup
+  const int wg = blockIdx.y * gridDim.x + blockIdx.x, step = gridDim.x * gridDim.y * 64 * NW;
+  for (int c = wg * 64 * NW + threadIdx.x; c < a.conv.C; c += step) conv_state_store<bf16_t>(a.conv, a.m, b, c);
 }
 
+template <int KB, int NW>
+static int launch_delta_apply(const ChunkArgs& p, hipStream_t s) {
+  static const hipError_t e = hipFuncSetAttribute((const void*)delta_apply_kernel<KB, NW>,
+                                                  hipFuncAttributeMaxDynamicSharedMemorySize, DL<KB, NW>::BYTES);
+  if (e != hipSuccess) return (int)e;
+  const DeltaArgs& a = p.a;
+  delta_apply_kernel<KB, NW><<<dim3((a.V + 16 * NW - 1) / (16 * NW), a.H, a.m.B), 64 * NW, DL<KB, NW>::BYTES, s>>>(p);
+  DA_LAUNCH_CHECK();
+}
 template <int KB>
 static int launch_delta_chunk(const ChunkArgs& p, hipStream_t s) {
-  constexpr int lds = 2 * DC<KB>::NF * 1024;
-  static const hipError_t e = hipFuncSetAttribute((const void*)delta_apply_kernel<KB>,
-                                                  hipFuncAttributeMaxDynamicSharedMemorySize, lds);
-  if (e != hipSuccess) return (int)e;
   const DeltaArgs& a = p.a;
   delta_prep_kernel<KB><<<(p.ch.n * a.H + 3) / 4, 256, 0, s>>>(p);
   // a head's columns on one CU where the heads fill the chip, else spread over more
-  int nw = 8;
-  while (nw > 2 && (long long)a.m.B * a.H * ((a.V + 16 * nw - 1) / (16 * nw)) < 256) nw /= 2;
-  delta_apply_kernel<KB><<<dim3((a.V + 16 * nw - 1) / (16 * nw), a.H, a.m.B), 64 * nw, lds, s>>>(p);
-  DA_LAUNCH_CHECK();
+  const long long heads = (long long)a.m.B * a.H;
+  if (heads * ((a.V + 127) / 128) >= 256) return launch_delta_apply<KB, 8>(p, s);
+  if (heads * ((a.V + 63) / 64) >= 256) return launch_delta_apply<KB, 4>(p, s);
+  return launch_delta_apply<KB, 2>(p, s);
 }
 
 // o / rms(o) * w * sigmoid(gate), in place, per head: `lanes` lanes a head.
@@ -656,7 +740,7 @@ static int launch_delta_t(const ChunkArgs& p0, int min_len, const void* w, const
   ChunkArgs p = p0;
   DeltaArgs& a = p.a;
   int err = 0;
-  if (sizeof(T) == 2 && p.ch.n) {
+  if (sizeof(T) == 2 && p.ch.n && a.V % 8 == 0 && a.ldx % 8 == 0) {
     switch (a.K) {
       case 32: err = launch_delta_chunk<1>(p, s); break;
       case 64: err = launch_delta_chunk<2>(p, s); break;
