@@ -325,6 +325,54 @@ __global__ void __launch_bounds__(256) gemm_walk_kernel(AnyArgs p) {
   }
 }
 
+// Few rows (16 RT at most), bf16: 32 columns per workgroup, its waves take turns at the 32-k steps, operands straight from
+// memory to registers with U steps in flight, and their sums meet in LDS: one or two memory round trips in all.
+template <int EPI, int RT>
+__global__ void __launch_bounds__(256) gemm_rows_kernel(AnyArgs p) {
+  constexpr int U = 4, SR = 36;  // steps in flight; floats of a staged row
+  __shared__ __attribute__((aligned(16))) float part[4][RT * 16 * SR];
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, fr = lane & 15, fg = lane >> 4;
+  const int n0 = blockIdx.x * 32, z = blockIdx.z;
+  const bf16_t* A = (const bf16_t*)p.A + z * p.sA;
+  const bf16_t* W = (const bf16_t*)p.W + z * p.sW;
+  f32x4_t acc[RT][2];
+#pragma unroll
+  for (int i = 0; i < RT; ++i) acc[i][0] = acc[i][1] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = wv * 32; k0 < p.K; k0 += 128 * U) {
+    bf16x8_t fa[U][RT], fw[U][2];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = min(k0 + 128 * u + fg * 8, p.K - 8);
+#pragma unroll
+      for (int i = 0; i < RT; ++i) fa[u][i] = *(const bf16x8_t*)(A + (size_t)min(i * 16 + fr, p.M - 1) * p.lda + k);
+#pragma unroll
+      for (int j = 0; j < 2; ++j) fw[u][j] = *(const bf16x8_t*)(W + (size_t)min(n0 + j * 16 + fr, p.N - 1) * p.K + k);
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const bool in = k0 + 128 * u + fg * 8 < p.K;
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const bf16x8_t w = in ? fw[u][j] : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+        for (int i = 0; i < RT; ++i) acc[i][j] = mfma16(w, in ? fa[u][i] : bf16x8_t{0, 0, 0, 0, 0, 0, 0, 0}, acc[i][j]);
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < RT; ++i)
+#pragma unroll
+    for (int j = 0; j < 2; ++j) *(f32x4_t*)(part[wv] + (i * 16 + fr) * SR + j * 16 + 4 * fg) = acc[i][j];
+  __syncthreads();
+  for (int i = tid; i < RT * 16 * 8; i += 256) {
+    const int m = i >> 3, c = (i & 7) * 4, at = m * SR + c;
+    if (m >= p.M) continue;
+    const f32x4_t v = (*(const f32x4_t*)(part[0] + at) + *(const f32x4_t*)(part[1] + at)) +
+                      (*(const f32x4_t*)(part[2] + at) + *(const f32x4_t*)(part[3] + at));
+    any_block<bf16_t, EPI>(p, z, m, n0 + c, v);
+  }
+}
+
 template <typename T, int EPI, int BT>
 static int launch_any(const AnyArgs& a, int batch, hipStream_t s) {
   constexpr int lds = 4 * BT * ANY_ROWB;
@@ -349,6 +397,14 @@ static int launch_any_t(const AnyArgs& a, int batch, hipStream_t s) {
       DA_LAUNCH_CHECK();
     }
   }
+  if constexpr (sizeof(T) == 2 && !any_paired(EPI) && EPI != ANY_NONE)
+    if (a.M <= 64) {
+      const dim3 grid((a.N + 31) / 32, 1, batch);
+      if (a.M <= 16) gemm_rows_kernel<EPI, 1><<<grid, 256, 0, s>>>(a);
+      else if (a.M <= 32) gemm_rows_kernel<EPI, 2><<<grid, 256, 0, s>>>(a);
+      else gemm_rows_kernel<EPI, 4><<<grid, 256, 0, s>>>(a);
+      DA_LAUNCH_CHECK();
+    }
   const long tiles = (long)((a.N + 127) / 128) * ((a.M + 127) / 128) * batch;
   return a.N % 128 == 0 && tiles >= 512 ? launch_any<T, EPI, 128>(a, batch, s) : launch_any<T, EPI, 64>(a, batch, s);
 }

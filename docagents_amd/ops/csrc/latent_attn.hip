@@ -27,11 +27,14 @@ struct LatArgs {
   int rows;                                      // rows (tokens x heads) of the longest portion
 };
 
-__device__ __forceinline__ int lat_page(const LatArgs& a, int slot, int i) {
-  const int p = a.table[(size_t)slot * a.max_pages + min(i, a.max_pages - 1)];
-  DA_ASSERT(p >= 0 && p < a.npages);
-  return min(max(p, 0), a.npages - 1);
+__device__ __forceinline__ int lat_entry(const LatArgs& a, int slot, int i) {
+  return a.table[(size_t)slot * a.max_pages + min(i, a.max_pages - 1)];
 }
+__device__ __forceinline__ int lat_page_of(const LatArgs& a, int entry) {
+  DA_ASSERT(entry >= 0 && entry < a.npages);
+  return min(max(entry, 0), a.npages - 1);
+}
+__device__ __forceinline__ int lat_page(const LatArgs& a, int slot, int i) { return lat_page_of(a, lat_entry(a, slot, i)); }
 
 // ------------------------------------------------------------------------------- norms, rotation, page write
 struct LatPrepArgs {
@@ -42,44 +45,59 @@ struct LatPrepArgs {
   float eps;
 };
 
-// A wave per token: the query latent normed to its own matrix, the cached latent normed and the key part rotated to
-// the token's page.
+// Two waves per token: one norms the query latent to its own matrix; the other norms the cached latent and rotates the
+// key part, both to the token's page.
 template <typename T>
 __global__ void __launch_bounds__(256) latent_prep_kernel(LatPrepArgs p) {
   const LatArgs& a = p.a;
-  const int t = blockIdx.x * 4 + (threadIdx.x >> 6), l = threadIdx.x & 63;
+  const int item = blockIdx.x * 4 + (threadIdx.x >> 6), t = item >> 1, l = threadIdx.x & 63;
   if (t >= a.m.T) return;
-  const int b = a.m.seq[t], pos = a.m.pos0[b] + t - a.m.cu[b];
   const T* x = (const T*)p.x + (size_t)t * p.ldx;
-  const int W = a.L + a.R;
-  T* page = (T*)a.pages + ((size_t)lat_page(a, a.m.slot[b], pos / PAGE) * PAGE + pos % PAGE) * W;
-  auto norm = [&](const T* src, T* dst, const float* w, int n, int dim) {
+  auto norm = [&](const T* src, T* out, const float* w, int n, int dim) {
+    constexpr int U = 6;  // pieces of 256 columns kept in registers
+    f32x4_t v[U], g[U];
     float ss = 0.f;
-    for (int c = l * 4; c < n; c += 256) {
-      const f32x4_t v = Act<T>::load4(src + c);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
+    for (int i = 0; i < U; ++i) {
+      const int c = min((i * 64 + l) * 4, n - 4);
+      v[i] = Act<T>::load4(src + c);
+      g[i] = *(const f32x4_t*)(w + c);
+    }
+#pragma unroll
+    for (int i = 0; i < U; ++i)
+      if ((i * 64 + l) * 4 < n)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = fmaf(v[i][e], v[i][e], ss);
+    for (int c = (U * 64 + l) * 4; c < n; c += 256) {
+      const f32x4_t y = Act<T>::load4(src + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss = fmaf(y[e], y[e], ss);
     }
     const float inv = 1.f / sqrtf(wave_sum(ss) / dim + p.eps);
-    for (int c = l * 4; c < n; c += 256) {
-      f32x4_t v = Act<T>::load4(src + c);
-      const f32x4_t g = *(const f32x4_t*)(w + c);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] *= inv * g[e];
-      Act<T>::store4(dst + c, v);
-    }
+    for (int i = 0; i < U; ++i)
+      if ((i * 64 + l) * 4 < n) Act<T>::store4(out + (i * 64 + l) * 4, v[i] * inv * g[i]);
+    for (int c = (U * 64 + l) * 4; c < n; c += 256)
+      Act<T>::store4(out + c, Act<T>::load4(src + c) * inv * *(const f32x4_t*)(w + c));
   };
-  norm(x, (T*)p.cq + (size_t)t * p.Q, p.qw, p.Q, p.qdim);
-  norm(x + p.Q, page, p.cw, a.L, p.cdim);
+  if (!(item & 1)) {
+    norm(x, (T*)p.cq + (size_t)t * p.Q, p.qw, p.Q, p.qdim);
+    return;
+  }
+  const int b = a.m.seq[t], pos = a.m.pos0[b] + t - a.m.cu[b];
   const T* kr = x + p.Q + a.L;
   const int half = a.rdim / 2;
   const float* cs = a.rot + (size_t)min(pos, a.npos - 1) * a.rdim;
-  for (int c = l; c < a.R; c += 64) {
-    float v = Act<T>::to_f(kr[c]);
-    if (c < half) v = v * cs[2 * c] - Act<T>::to_f(kr[c + half]) * cs[2 * c + 1];
-    else if (c < a.rdim) v = v * cs[2 * (c - half)] + Act<T>::to_f(kr[c - half]) * cs[2 * (c - half) + 1];
-    page[a.L + c] = Act<T>::from_f(v);
-  }
+  auto turned = [&](int c) {  // loads first: column c, its partner, their angle
+    const int i = min(c, a.rdim - 1), j = i < half ? i : i - half;
+    const float v = Act<T>::to_f(kr[c]), w = Act<T>::to_f(kr[i < half ? i + half : j]), co = cs[2 * j], si = cs[2 * j + 1];
+    return c >= a.rdim ? v : c < half ? v * co - w * si : v * co + w * si;
+  };
+  const float first = turned(min(l, a.R - 1));
+  T* page = (T*)a.pages + ((size_t)lat_page(a, a.m.slot[b], pos / PAGE) * PAGE + pos % PAGE) * (a.L + a.R);
+  if (l < a.R) page[a.L + l] = Act<T>::from_f(first);
+  for (int c = l + 64; c < a.R; c += 64) page[a.L + c] = Act<T>::from_f(turned(c));
+  norm(x + p.Q, page, p.cw, a.L, p.cdim);
 }
 
 // Element c of a query head's rotated part at position pos (zero past it). Rounded to the activation type, as the
@@ -91,6 +109,39 @@ __device__ __forceinline__ float rotated(const T* qr, const float* cs, int rdim,
   if (c < half) v = Act<T>::to_f(qr[c]) * cs[2 * c] - Act<T>::to_f(qr[c + half]) * cs[2 * c + 1];
   else if (c < rdim) v = Act<T>::to_f(qr[c]) * cs[2 * (c - half)] + Act<T>::to_f(qr[c - half]) * cs[2 * (c - half) + 1];
   return Act<T>::to_f(Act<T>::from_f(v));
+}
+
+// Elements c .. c + 7 (c a multiple of 8), with loads that do not wait for each other.
+__device__ __forceinline__ bf16x8_t rotated8(const bf16_t* qr, const float* cs, int rdim, int c) {
+  const int half = rdim / 2;
+  float x[8], y[8], co[8], si[8];  // elements, what they are paired with, angles
+  if (half % 8 == 0) {
+    const int a = min(c, rdim - 8), j = a < half ? a : a - half;
+    const bf16x8_t u = *(const bf16x8_t*)(qr + a), v = *(const bf16x8_t*)(qr + (a < half ? a + half : j));
+    f32x4_t t[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) t[i] = *(const f32x4_t*)(cs + 2 * j + 4 * i);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      x[e] = bf2f((bf16_t)u[e]);
+      y[e] = bf2f((bf16_t)v[e]);
+      co[e] = t[e >> 1][2 * (e & 1)];
+      si[e] = t[e >> 1][2 * (e & 1) + 1];
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int a = min(c + e, rdim - 1), j = a < half ? a : a - half;
+      x[e] = bf2f(qr[a]);
+      y[e] = bf2f(qr[a < half ? a + half : j]);
+      co[e] = cs[2 * j];
+      si[e] = cs[2 * j + 1];
+    }
+  }
+  bf16x8_t r;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) r[e] = (short)f2bf(c + e < rdim ? fmaf(x[e], co[e], c + e < half ? -y[e] * si[e] : y[e] * si[e]) : 0.f);
+  return r;
 }
 
 // ------------------------------------------------------------------------------- any size, fp32 arithmetic
@@ -232,31 +283,31 @@ __global__ void __launch_bounds__(256, 2) latent_mfma_kernel(LatArgs a, int rtil
   const bf16_t* qr = (const bf16_t*)a.q + (size_t)(s0 + tok) * a.ldq + (size_t)hd * a.D + a.ra;
   const float* cs = a.rot + (size_t)min(qpos, a.npos - 1) * a.rdim;
 #pragma unroll
-  for (int ds = NLS; ds < NDS; ++ds)
-#pragma unroll
-    for (int e = 0; e < 8; ++e) qf[ds][e] = (short)f2bf(rotated<bf16_t>(qr, cs, a.rdim, (ds - NLS) * 32 + fg * 8 + e));
+  for (int ds = NLS; ds < NDS; ++ds) qf[ds] = rotated8(qr, cs, a.rdim, (ds - NLS) * 32 + fg * 8);
   const float c2 = a.scale * LOG2E;
 
   bf16x8_t kf[NDS];
   const int key = wv * 16 + fr;  // the key of a page this lane loads
-  auto load_page = [&](int p) {
-    const bf16_t* kp = (const bf16_t*)a.pages + ((size_t)lat_page(a, slot, p) * PAGE + key) * W + fg * 8;
-    const bool in = p * PAGE + key <= klast;  // rows past it may hold anything: read as zero
+  auto load_page = [&](int p, int entry) {
+    // rows past the last key may hold anything: that key's instead (their weights are zero)
+    const bf16_t* kp = (const bf16_t*)a.pages + ((size_t)lat_page_of(a, entry) * PAGE + min(key, klast - p * PAGE)) * W + fg * 8;
 #pragma unroll
-    for (int ds = 0; ds < NDS; ++ds) {
-      const u32x4_t v = *(const u32x4_t*)(kp + ds * 32);
-      kf[ds] = __builtin_bit_cast(bf16x8_t, in ? v : u32x4_t{0, 0, 0, 0});
-    }
+    for (int ds = 0; ds < NDS; ++ds) kf[ds] = *(const bf16x8_t*)(kp + ds * 32);
   };
   f32x4_t oacc[NDB];
 #pragma unroll
   for (int i = 0; i < NDB; ++i) oacc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float mx = -1e30f, sum = 0.f;  // of row fr: common to the waves; over this lane's keys
-  load_page(p0);
+  load_page(p0, lat_entry(a, slot, p0));
+  int next = lat_entry(a, slot, p0 + 1);
   for (int p = p0; p < p1; ++p) {
-    f32x4_t s{0.f, 0.f, 0.f, 0.f};
+    f32x4_t s{0.f, 0.f, 0.f, 0.f}, s1 = s;
 #pragma unroll
-    for (int ds = 0; ds < NDS; ++ds) s = mfma16(kf[ds], qf[ds], s);
+    for (int ds = 0; ds < NDS; ds += 2) {
+      s = mfma16(kf[ds], qf[ds], s);
+      if (ds + 1 < NDS) s1 = mfma16(kf[ds + 1], qf[ds + 1], s1);
+    }
+    s += s1;
     float top = -1e30f;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
@@ -269,7 +320,10 @@ __global__ void __launch_bounds__(256, 2) latent_mfma_kernel(LatArgs a, int rtil
     lds_barrier();  // maxima written; every wave is done with the last page's latents and weights
 #pragma unroll
     for (int ds = 0; ds < NLS; ++ds) *(bf16x8_t*)(sV + key * C::VSTR + ds * 64 + fg * 16) = kf[ds];
-    if (p + 1 < p1) load_page(p + 1);
+    if (p + 1 < p1) {
+      load_page(p + 1, next);
+      next = lat_entry(a, slot, p + 2);
+    }
     const float mnew = fmaxf(mx, fmaxf(fmaxf(sM[fr], sM[16 + fr]), fmaxf(sM[32 + fr], sM[48 + fr])));
     const float f = __builtin_amdgcn_exp2f(mx - mnew);
     mx = mnew;
@@ -434,11 +488,10 @@ __global__ void __launch_bounds__(256, 2) latent_flash_kernel(FlashArgs p, int n
 #pragma unroll
   for (int ds = 0; ds < NDS; ++ds) {
     const int c = ds * 16 + hi * 8;
-    if (c < d) {
-      qf[ds] = *(const bf16x8_t*)(qp + c);
-    } else {
-#pragma unroll
-      for (int e = 0; e < 8; ++e) qf[ds][e] = (short)f2bf(rotated<bf16_t>(qp + d, cs, a.rdim, c - d + e));
+    if (ds * 16 < d) qf[ds] = *(const bf16x8_t*)(qp + min(c, d - 8));
+    if (ds * 16 + 8 >= d) {
+      const bf16x8_t r = rotated8(qp + d, cs, a.rdim, max(c - d, 0));
+      qf[ds] = c < d ? qf[ds] : r;
     }
   }
   const float c2 = a.scale * LOG2E;
@@ -451,8 +504,7 @@ __global__ void __launch_bounds__(256, 2) latent_flash_kernel(FlashArgs p, int n
       const int k = min(t * PAGE + r, klast);
       const bf16_t* src = c < d ? p.kv + (size_t)(c0 + k) * p.ldkv + (size_t)hd * (d + V) + c
                                 : p.lat + (size_t)(c0 + k) * W + a.L + min(c - d, a.R - 8);
-      kreg[i] = *(const u32x4_t*)src;
-      if (c >= d + a.R) kreg[i] = u32x4_t{0, 0, 0, 0};
+      kreg[i] = *(const u32x4_t*)src;  // past d + R: any key's columns, the queries are zero there
     }
 #pragma unroll
     for (int i = 0; i < VP; ++i) {
@@ -556,12 +608,17 @@ __global__ void __launch_bounds__(256, 2) latent_flash_kernel(FlashArgs p, int n
   const float inv = 1.f / sum;
   const bf16_t* g = p.gate + (size_t)(s0 + tok) * p.ldg + (size_t)hd * V;
   bf16_t* o = (bf16_t*)a.out + (size_t)(s0 + tok) * a.ldo + (size_t)hd * V;
+  u32x2_t gates[NDB][4];  // loaded ahead of the stores, which they might alias
+#pragma unroll
+  for (int db = 0; db < NDB; ++db)
+#pragma unroll
+    for (int q = 0; q < 4; ++q) gates[db][q] = *(const u32x2_t*)(g + db * 32 + 8 * q + 4 * hi);
 #pragma unroll
   for (int db = 0; db < NDB; ++db)
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
       const int c = db * 32 + 8 * q + 4 * hi;
-      const f32x4_t gt = Act<bf16_t>::load4(g + c);
+      const f32x4_t gt = Act<bf16_t>::load4((const bf16_t*)&gates[db][q]);
       f32x4_t y;
 #pragma unroll
       for (int e = 0; e < 4; ++e) y[e] = oacc[db][4 * q + e] * inv * sigmoid32(gt[e]);
@@ -648,8 +705,8 @@ DA_EXPORT int da_latent_prep(const void* x, int ldx, const void* qw, int Q, int 
   p.x = x; p.ldx = ldx; p.qw = (const float*)qw; p.cw = (const float*)cw; p.cq = cq;
   p.Q = Q; p.qdim = qdim; p.cdim = cdim; p.eps = eps;
   hipStream_t s = (hipStream_t)stream;
-  if (f32) latent_prep_kernel<float><<<(T + 3) / 4, 256, 0, s>>>(p);
-  else latent_prep_kernel<bf16_t><<<(T + 3) / 4, 256, 0, s>>>(p);
+  if (f32) latent_prep_kernel<float><<<(T + 1) / 2, 256, 0, s>>>(p);
+  else latent_prep_kernel<bf16_t><<<(T + 1) / 2, 256, 0, s>>>(p);
   DA_LAUNCH_CHECK();
 }
 
