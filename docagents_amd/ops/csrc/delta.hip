@@ -680,8 +680,8 @@ static int launch_delta_chunk(const ChunkArgs& p, hipStream_t s) {
   return launch_delta_apply<KB, 2>(p, s);
 }
 
-// o / rms(o) * w * sigmoid(gate), in place, per head: `lanes` lanes a head.
-template <typename T>
+// o / rms(o) * w * sigmoid(gate), in place, per head: `lanes` lanes a head, U pieces of 4 columns of theirs in registers.
+template <typename T, int U>
 __global__ void __launch_bounds__(256)
 head_norm_kernel(T* o, int ldo, const T* gate, int ldg, const float* w, int T_, int H, int V, int dim, float eps, int lanes) {
   const int item = blockIdx.x * (256 / lanes) + threadIdx.x / lanes, l = threadIdx.x % lanes;
@@ -689,7 +689,6 @@ head_norm_kernel(T* o, int ldo, const T* gate, int ldg, const float* w, int T_, 
   const int it = live ? item : T_ * H - 1, t = it / H, h = it % H;
   T* r = o + (size_t)t * ldo + (size_t)h * V;
   const T* gr = gate + (size_t)t * ldg + (size_t)h * V;
-  constexpr int U = 4;
   f32x4_t v[U], g[U];
   float ss = 0.f;
 #pragma unroll
@@ -766,8 +765,9 @@ static int launch_delta_t(const ChunkArgs& p0, int min_len, const void* w, const
   int lanes = 4;
   while (lanes < 64 && lanes * 4 < a.V) lanes *= 2;
   const int per = 256 / lanes;
-  head_norm_kernel<T><<<(unsigned)(((size_t)a.m.T * a.H + per - 1) / per), 256, 0, s>>>(
-      (T*)a.o, a.ldo, (const T*)gate, ldg, (const float*)w, a.m.T, a.H, a.V, dim, eps, lanes);
+  auto norm = a.V <= 4 * lanes ? head_norm_kernel<T, 1> : head_norm_kernel<T, 4>;
+  norm<<<(unsigned)(((size_t)a.m.T * a.H + per - 1) / per), 256, 0, s>>>((T*)a.o, a.ldo, (const T*)gate, ldg, (const float*)w,
+                                                                        a.m.T, a.H, a.V, dim, eps, lanes);
   DA_LAUNCH_CHECK();
 }
 

@@ -45,6 +45,8 @@ struct LatPrepArgs {
   float eps;
 };
 
+template <int K> struct Pieces { static constexpr int N = K; };
+
 // Two waves per token: one norms the query latent to its own matrix; the other norms the cached latent and rotates the
 // key part, both to the token's page.
 template <typename T>
@@ -53,8 +55,8 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatPrepArgs p) {
   const int item = blockIdx.x * 4 + (threadIdx.x >> 6), t = item >> 1, l = threadIdx.x & 63;
   if (t >= a.m.T) return;
   const T* x = (const T*)p.x + (size_t)t * p.ldx;
-  auto norm = [&](const T* src, T* out, const float* w, int n, int dim) {
-    constexpr int U = 6;  // pieces of 256 columns kept in registers
+  auto norm = [&](auto pieces, const T* src, T* out, const float* w, int n, int dim) {
+    constexpr int U = decltype(pieces)::N;  // pieces of 256 columns kept in registers
     f32x4_t v[U], g[U];
     float ss = 0.f;
 #pragma unroll
@@ -81,7 +83,7 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatPrepArgs p) {
       Act<T>::store4(out + c, Act<T>::load4(src + c) * inv * *(const f32x4_t*)(w + c));
   };
   if (!(item & 1)) {
-    norm(x, (T*)p.cq + (size_t)t * p.Q, p.qw, p.Q, p.qdim);
+    norm(Pieces<6>{}, x, (T*)p.cq + (size_t)t * p.Q, p.qw, p.Q, p.qdim);
     return;
   }
   const int b = a.m.seq[t], pos = a.m.pos0[b] + t - a.m.cu[b];
@@ -97,7 +99,7 @@ __global__ void __launch_bounds__(256) latent_prep_kernel(LatPrepArgs p) {
   T* page = (T*)a.pages + ((size_t)lat_page(a, a.m.slot[b], pos / PAGE) * PAGE + pos % PAGE) * (a.L + a.R);
   if (l < a.R) page[a.L + l] = Act<T>::from_f(first);
   for (int c = l + 64; c < a.R; c += 64) page[a.L + c] = Act<T>::from_f(turned(c));
-  norm(x + p.Q, page, p.cw, a.L, p.cdim);
+  norm(Pieces<2>{}, x + p.Q, page, p.cw, a.L, p.cdim);
 }
 
 // Element c of a query head's rotated part at position pos (zero past it). Rounded to the activation type, as the
@@ -443,7 +445,16 @@ __global__ void __launch_bounds__(256) latent_gather_kernel(LatArgs a, const int
   if (n <= 0) return;
   const u32x4_t* src = (const u32x4_t*)((const bf16_t*)a.pages + (size_t)lat_page(a, a.m.slot[b], p) * PAGE * W);
   u32x4_t* dst = (u32x4_t*)(lat + (size_t)(c0 + p * PAGE) * W);
-  for (int i = threadIdx.x; i < n * W / 8; i += 256) dst[i] = src[i];
+  const int pieces = n * W / 8;
+  constexpr int U = 6;
+  for (int i0 = threadIdx.x; i0 < pieces; i0 += 256 * U) {
+    u32x4_t v[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) v[u] = src[min(i0 + 256 * u, pieces - 1)];
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (i0 + 256 * u < pieces) dst[i0 + 256 * u] = v[u];
+  }
 }
 
 struct FlashArgs {

@@ -60,10 +60,12 @@ __global__ void __launch_bounds__(256) causal_conv_kernel(ConvArgs a) {
 #pragma unroll
       for (int i = 0; i < CONV_RUN + TAPS - 1; ++i) {
         const int t = min(t0 + i - (TAPS - 1), t1 - 1);
-        x[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-        if (t >= s0) x[i] = Act<T>::load4((const T*)a.x + (size_t)t * a.ldx + c);
-        else if (stored) x[i] = Act<T>::load4(st + (size_t)(TAPS - 1 + t - s0) * a.C);
+        const T* in = (const T*)a.x + (size_t)max(t, s0) * a.ldx + c;
+        x[i] = Act<T>::load4(t < s0 && stored ? st + (size_t)(TAPS - 1 + t - s0) * a.C : in);
       }
+#pragma unroll
+      for (int i = 0; i + 1 < TAPS; ++i)
+        if (t0 + i - (TAPS - 1) < s0 && !stored) x[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int i = 0; i < CONV_RUN; ++i) {
         if (t0 + i >= t1) break;

@@ -50,6 +50,7 @@ K._PART_OF.update({n: "hybrid" for n in ("da_gemm_any", "da_stream_step", "da_st
 ACTS = (torch.bfloat16, torch.float32)
 DELTA_CHUNK = 32       # tokens of a chunk of the delta rule on the matrix cores (bf16)
 DELTA_CHUNK_FROM = 33  # tokens from which a portion runs in chunks
+LATENT_WGS, LATENT_MIN_PAGES = 512, 2  # of single tokens: about so many workgroups, so many pages each
 LATENT_MFMA = (64, 128, 256, 512)  # latents the matrix-core attention takes (with a key part of 32 or 64 columns)
 ANY_NONE, ANY_SOFTPLUS, ANY_REGLU, ANY_RGLRU, ANY_SWIGLU, ANY_ACT = 0, 1, 2, 3, 4, 5
 
@@ -427,7 +428,7 @@ def latent_attn(q, ql, pages, rot, sink, m: SeqBatch, H: int, rot_at: int, rot_d
     part, ml, rows, pages_ctx = None, None, m.max_len * H, -(-m.max_ctx // PAGE)
     nsplit, pps = 1, pages_ctx
     if not f32 and L in LATENT_MFMA and W - L in (32, 64):
-        want = max(1, min(-(-1024 // (m.B * -(-rows // 16))), -(-pages_ctx // 2)))  # ~1024 workgroups, >= 2 pages each
+        want = max(1, min(-(-LATENT_WGS // (m.B * -(-rows // 16))), -(-pages_ctx // LATENT_MIN_PAGES)))
         pps = -(-pages_ctx // want)
         nsplit = -(-pages_ctx // pps)
     if nsplit > 1:
