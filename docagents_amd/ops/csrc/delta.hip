@@ -636,7 +636,8 @@ __global__ void __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) delta_apply_kernel(C
     for (int i = 0; i < 2; ++i)
 #pragma unroll
       for (int e = 0; e < 4; ++e)
-        X[i][e] = t + 16 * i + 4 * fg + e < t1 ? fmaf(__uint_as_float(rv[4 * i + e] << 16), __builtin_amdgcn_rcpf(rk[i][e]), -R[i][e]) : 0.f;
+        X[i][e] = t + 16 * i + 4 * fg + e < t1
+                      ? fmaf(__uint_as_float(rv[4 * i + e] << 16), __builtin_amdgcn_rcpf(rk[i][e]), -R[i][e]) : 0.f;
     Split B = split8(X[0], X[1]);
 #pragma unroll
     for (int i = 0; i < 2; ++i) U[i] = mma3(tf[i], B, f32x4_t{0.f, 0.f, 0.f, 0.f});
@@ -783,8 +784,9 @@ DA_EXPORT int da_delta_rule(const void* x, int ldx, const void* decay, const voi
                             const void* base, int n_chunks, void* frags, const void* cu,
                             const void* slot, const void* pos0, const void* seq, int T, int B, int f32, void* stream) {
   if (T < 1 || B < 1 || B > 65535 || G < 1 || H % G || H > 65535 || V < 4 || V % 4 ||
-      ldx % 4 || ldo % 4 || ldg % 4 || dim < 1 || dim > V || taps < 1 || min_len < 1 || chunk_from < 1 || n_chunks < 0 || (n_chunks && (!ck || !base || !frags)) ||
-      (long long)n_chunks * H > 0x7fffffffll / 4 || ldx % 2 || (long long)T * H > 0x7fffffffll / 4)
+      ldx % 4 || ldo % 4 || ldg % 4 || dim < 1 || dim > V || taps < 1 || min_len < 1 || chunk_from < 1 || n_chunks < 0 ||
+      (n_chunks && (!ck || !base || !frags)) || (long long)n_chunks * H > 0x7fffffffll / 4 ||
+      (long long)T * H > 0x7fffffffll / 4)
     return (int)hipErrorInvalidValue;
   ChunkArgs p{DeltaArgs{x, ldx, (const float*)decay, beta, ldb, (float*)state, o, ldo, H, G, K, V, q_scale, unit_eps, chunk_from,
                         ConvState{conv_x, ld_conv, conv_state, taps, conv_c},

@@ -4,8 +4,9 @@
 // product feeds a recurrence (step sizes, gates), which must not be rounded to 16 bits; everything
 // else runs on gemm.hip's kernels. The fp32 precision runs every product here.
 //
-// BT x BT tile (64, or 128 where the rows fill the chip), 4 waves of a quarter each, K in 128-byte slices through double-buffered LDS (rows padded to 144
-// bytes: conflict-free 16-byte reads), the next slice's loads in flight while this one is multiplied.
+// BT x BT tile (64, or 128 where the rows fill the chip), 4 waves of a quarter each, K in 128-byte slices through
+// double-buffered LDS (rows padded to 144 bytes: conflict-free 16-byte reads), the next slice's loads in flight while this
+// one is multiplied.
 #include "seq.h"
 
 enum AnyEpi : int {
@@ -387,8 +388,10 @@ static int launch_any(const AnyArgs& a, int batch, hipStream_t s) {
 template <typename T, int EPI>
 static int launch_any_t(const AnyArgs& a, int batch, hipStream_t s) {
   if constexpr (sizeof(T) == 2 && (EPI == ANY_SOFTPLUS || EPI == ANY_RGLRU)) {
-    if (a.M >= 1024 && a.K <= 256 && a.K % 32 == 0 && a.N % 16 == 0 && a.ldc % 4 == 0 && (EPI != ANY_RGLRU || (a.A == a.u && a.sA == a.N / 2 && a.K == a.N / 2))) {
-      const int row = a.K * 2 + 16 > 272 ? a.K * 2 + 16 : 272, lds = 64 * (a.K * 2 + 16 + row), nt = (a.N + 63) / 64 * batch, mt = (a.M + 63) / 64;
+    if (a.M >= 1024 && a.K <= 256 && a.K % 32 == 0 && a.N % 16 == 0 && a.ldc % 4 == 0 &&
+        (EPI != ANY_RGLRU || (a.A == a.u && a.sA == a.N / 2 && a.K == a.N / 2))) {
+      const int row = a.K * 2 + 16 > 272 ? a.K * 2 + 16 : 272, lds = 64 * (a.K * 2 + 16 + row);
+      const int nt = (a.N + 63) / 64 * batch, mt = (a.M + 63) / 64;
       static const hipError_t e = hipFuncSetAttribute((const void*)gemm_walk_kernel<EPI>,
                                                       hipFuncAttributeMaxDynamicSharedMemorySize, 128 * 528);
       if (e != hipSuccess) return (int)e;

@@ -142,7 +142,10 @@ __device__ __forceinline__ bf16x8_t rotated8(const bf16_t* qr, const float* cs, 
   }
   bf16x8_t r;
 #pragma unroll
-  for (int e = 0; e < 8; ++e) r[e] = (short)f2bf(c + e < rdim ? fmaf(x[e], co[e], c + e < half ? -y[e] * si[e] : y[e] * si[e]) : 0.f);
+  for (int e = 0; e < 8; ++e) {
+    const float s = c + e < half ? -si[e] : si[e];
+    r[e] = (short)f2bf(c + e < rdim ? fmaf(x[e], co[e], y[e] * s) : 0.f);
+  }
   return r;
 }
 
@@ -476,7 +479,7 @@ template <int D, int V> struct LF {
 };
 
 template <int D, int V>
-__global__ void __launch_bounds__(256, 2) latent_flash_kernel(FlashArgs p, int ntiles) {
+__global__ void __launch_bounds__(256, D + V > 320 ? 1 : 2) latent_flash_kernel(FlashArgs p, int ntiles) {
   using C = LF<D, V>;
   const LatArgs& a = p.a;
   extern __shared__ __attribute__((aligned(16))) char smem[];

@@ -26,12 +26,14 @@ HOT_NO_SCRATCH = {  # mangled-name prefixes of the kernels the flagship bench ru
                  "_Z18gemm_splitk_reduce", "_Z23splitk_reduce_resid_ssq"],
     "gemm8p.hip": ["_Z13gemm8p_kernelILi6ELi256E", "_Z13gemm8p_kernelILi3ELi256E", "_Z13gemm8p_kernelILi4ELi256E"],
     "gemm_dk.hip": ["_Z14gemm_dk_kernel"],
-    "gemm_any.hip": ["_Z15gemm_any_kernelIt", "_Z16gemm_walk_kernel"],
+    "delta.hip": ["_Z17delta_scan_kernelIt", "_Z17delta_prep_kernel", "_Z18delta_apply_kernel", "_Z16head_norm_kernelIt"],
+    "gemm_any.hip": ["_Z15gemm_any_kernelIt", "_Z16gemm_walk_kernel", "_Z16gemm_rows_kernel"],
+    "latent_attn.hip": ["_Z18latent_prep_kernelIt", "_Z18latent_mfma_kernel", "_Z19latent_flash_kernel"],
     "paged_attn.hip": ["_Z19sigmoid_attn_kernelILi64E", "_Z19sigmoid_attn_kernelILi128E", "_Z21sigmoid_decode_kernelILi128E",
                        "_Z16attn_prep_kernelIt"],
     "recurrent.hip": ["_Z15sel_scan_kernelItLi8E", "_Z15sel_scan_kernelItLi4E", "_Z15gru_scan_kernelIt",
                       "_Z18causal_conv_kernelItLi4E"],
-    "stream_norm.hip": ["_Z13stream_kernelItLi1E", "_Z13stream_kernelItLi4E"],
+    "stream_norm.hip": ["_Z13stream_kernelItLi1E", "_Z13stream_kernelItLi4E", "_Z17stream_add_kernelIt"],
     "vecsearch.hip": ["_Z24topk_dense_stream_kernel", "_Z20topk_dense_mq_kernel"],  # the shard scans
 }
 NO_SERIAL_LOAD_LOOPS = {"gemm.hip": ["_Z18gemm_splitk_reduce", "_Z23splitk_reduce_resid_ssq",

@@ -87,7 +87,7 @@ def test_causal_conv_without_bias(device, dtype, taps):
 
 
 @pytest.mark.parametrize("device,dtype", WHERE)
-@pytest.mark.parametrize("M,N,K", [(1, 64, 64), (5, 96, 128), (130, 200, 64), (1500, 192, 128)])
+@pytest.mark.parametrize("M,N,K", [(1, 64, 64), (5, 96, 128), (23, 40, 64), (64, 72, 192), (130, 200, 64), (1500, 192, 128)])
 def test_log_decays(device, dtype, M, N, K):
     """The low-rank projection's epilogue: softplus times a rate per column, in fp32 at every size of the decay."""
     a, w, b = rand(1, M, K).to(ACT[dtype]), rand(2, N, K, std=K ** -0.5).to(ACT[dtype]), rand(3, N) - 2
@@ -99,7 +99,8 @@ def test_log_decays(device, dtype, M, N, K):
 
 
 @pytest.mark.parametrize("device,dtype", WHERE)
-@pytest.mark.parametrize("M,H,N,K,stride", [(1, 3, 64, 40, 64), (37, 5, 40, 128, 128), (200, 2, 128, 24, 32), (700, 16, 256, 64, 96)])
+@pytest.mark.parametrize("M,H,N,K,stride", [(1, 3, 64, 40, 64), (16, 2, 44, 1160, 1160), (18, 2, 24, 520, 528), (37, 5, 40, 128, 128),
+                                               (64, 2, 36, 640, 640), (200, 2, 128, 24, 32), (700, 16, 256, 64, 96)])
 def test_products_per_head(device, dtype, M, H, N, K, stride):
     if M == 700 and device == "cpu":
         pytest.skip("the large tile, on the GPU")
@@ -407,28 +408,29 @@ def test_sink_takes_its_share(device, dtype, expand):
     close(got[:, 2], v[2].expand(n, 32), dtype)
 
 
+@pytest.mark.parametrize("Q,qd,L,cd", [(64, 40, 64, 50), (1664, 1650, 640, 630)])
 @pytest.mark.parametrize("device,dtype", WHERE)
-def test_latents_reach_their_pages(device, dtype):
+def test_latents_reach_their_pages(device, dtype, Q, qd, L, cd):
     """Norms and rotation of what is cached, page by page, and the normed query latent."""
-    act, Q, L, R, rot, n = ACT[dtype], 64, 64, 32, 10, 150
+    act, R, rot, n = ACT[dtype], 32, 10, 150
     ops = get_ops(device)
     x = rand(1, n, Q + L + R + 8).to(act)
-    x[:, Q + 50:Q + L], x[:, Q + L + rot:Q + L + R] = 0, 0
-    x[:, 40:Q] = 0
-    qw, cw = torch.nn.functional.pad(rand(2, 40), (0, 24)), torch.nn.functional.pad(rand(3, 50), (0, 14))
+    x[:, Q + cd:Q + L], x[:, Q + L + rot:Q + L + R] = 0, 0
+    x[:, qd:Q] = 0
+    qw, cw = torch.nn.functional.pad(rand(2, qd), (0, Q - qd)), torch.nn.functional.pad(rand(3, cd), (0, L - cd))
     table = torch.tensor([[5, 0, 3], [1, 4, 2]], dtype=torch.int32, device=device)
     pool = torch.zeros(6, PAGE, L + R, dtype=act, device=device)
     rt = RotaryTable(rot, 300.0).build(3 * PAGE, device)
     got = []
     for a, b in ((0, 65), (65, 66), (66, 150)):
         m, _ = pack_batch([b - a], [1], [a], device)
-        got.append(ops.latent_prep(x[a:b].to(device), qw.to(device), 40, cw.to(device), 50, rot, 0.1, pool, rt, m.on(table)))
+        got.append(ops.latent_prep(x[a:b].to(device), qw.to(device), qd, cw.to(device), cd, rot, 0.1, pool, rt, m.on(table)))
     xd = x.double()
-    close(torch.cat(got)[:, :40], oracle.rms(xd[:, :40], 0.1) * qw[:40].double(), dtype)
+    close(torch.cat(got)[:, :qd], oracle.rms(xd[:, :qd], 0.1) * qw[:qd].double(), dtype)
     rows = pool[[1, 4, 2]].flatten(0, 1)[:n].double().cpu()
-    close(rows[:, :50], oracle.rms(xd[:, Q:Q + 50], 0.1) * cw[:50].double(), dtype)
+    close(rows[:, :cd], oracle.rms(xd[:, Q:Q + cd], 0.1) * cw[:cd].double(), dtype)
     close(rows[:, L:L + rot], oracle.rotate(xd[:, Q + L:Q + L + rot], range(n), 300.0, rot), dtype)
-    assert not rows[:, 50:L].any() and not rows[:, L + rot:].any() and not pool[[0, 3, 5]].any()
+    assert not rows[:, cd:L].any() and not rows[:, L + rot:].any() and not pool[[0, 3, 5]].any()
 
 
 # ---------------------------------------------------------------------------------- whole models
