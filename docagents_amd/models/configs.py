@@ -147,8 +147,8 @@ class HybridLayer:
 
 @dataclass(frozen=True)
 class LayerLoop:
-    """Layers start .. stop - 1 run ``times`` times in a row. A pass begins by adding its own learned vector to the
-    stream, and every pass but the first the embedding output too."""
+    """Layers ``start`` up to, not including, ``stop`` are passed through ``times`` times. A pass opens by adding a learned
+    vector of its own to the stream; later passes also add the scaled embeddings again."""
     start: int
     stop: int
     times: int

@@ -1,7 +1,7 @@
 // Gated delta rule with a decay per key channel, over a batch of portions (SeqMeta), state per sequence slot.
 //
-// Per token and head, S [K][V] in fp32 (stored [V][K]), a = exp2(log decay) per key channel:
-//   S <- a S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+// Per token and head, S [K][V] in fp32 (stored [V][K]), D = diag(exp2(log decay)) over the key channels:
+//   u = beta (v - k^T D S),  S' = D S + k u,  o = q^T S'      (v, u, o: rows of V)
 // with q and k made unit vectors (q scaled), then o / rms(o) * w * sigmoid(gate).
 //
 // delta_scan: token by token on the vector ALUs, in fp32. The columns of S do not depend on each other: a group of LN
